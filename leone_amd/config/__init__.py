@@ -4,3 +4,4 @@ from .pamevik import PamevikConfig
 from .zukinex import ZukinexConfig
 from .fosulix import FosulixConfig
 from .nogidra import NogidraConfig
+from .reverax import ReveraxConfig

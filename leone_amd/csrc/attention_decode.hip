@@ -40,6 +40,7 @@
 // it has to supply as P^T for the second product.
 #include "common.h"
 #include "leone_hip.h"
+#include "score_shape.h"
 
 #include <math.h>
 #include <type_traits>
@@ -129,14 +130,15 @@ struct ScoreBias {
     int temp_every = 0;
 };
 
-template <int kD16, bool kFused>
+// kShaped: capped scores, sinks, results turned back (ScoreShape); without it none of that is in the kernel.
+template <int kD16, bool kFused, bool kShaped>
 __global__ void __launch_bounds__(kDecodeThreads, kD16 <= 4 ? 3 : kD16 <= 8 ? 2 : 1)
 attention_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pool,
                         const bf16_t* __restrict__ v_pool, const int* __restrict__ positions,
                         const int* __restrict__ row_entry, const int* __restrict__ block_table, int max_blocks,
                         float* __restrict__ part_acc, float* __restrict__ part_ml, bf16_t* __restrict__ out,
                         int q_heads, int kv_heads, int page_shift, float to_log2, int window, int splits,
-                        FromProjection from, int keep_first, ScoreBias bias) {
+                        FromProjection from, int keep_first, ScoreBias bias, ScoreShape shape) {
     constexpr int kD = kD16 * 16;
     constexpr int kSteps = (kD16 + 1) / 2;           // 32-element steps of the q.k product
     extern __shared__ float smem[];                   // [waves][columns][kD] accumulators, then m and l
@@ -159,6 +161,8 @@ attention_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__
     // this lane's column is query head kvh * group + col0 + c
     const float to_log2_row = bias.temp_every > 0
         ? to_log2 * (1.0f + bias.temp_coef * logf(static_cast<float>(n / bias.temp_every + 1))) : to_log2;
+    const float cap_log2 = shape.cap * 1.4426950408889634f;                // capped scores, in units of log2
+    const float to_cap = kShaped && shape.cap > 0.f ? to_log2_row / cap_log2 : 0.f;
     const float slope_log2 = (bias.slopes && c < cols) ? bias.slopes[kvh * group + col0 + c] * 1.4426950408889634f : 0.f;
     const int* table = block_table + static_cast<long>(row_entry[row]) * max_blocks;
     const int t_begin = lo / kTileKeys, t_end = (n + kTileKeys - 1) / kTileKeys;
@@ -453,8 +457,9 @@ attention_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
             const int key = run0 + j;
-            const float raw = j < 4 ? sa[j & 3] : sb[j & 3];
-            sc[j] = (full || in_reach(key)) ? fmaf(raw, to_log2_row, slope_log2 * static_cast<float>(key - (n - 1))) : -INFINITY;
+            float raw = j < 4 ? sa[j & 3] : sb[j & 3];
+            if (kShaped && shape.cap > 0.f) raw = cap_log2 * tanh_fast(raw * to_cap);
+            sc[j] = (full || in_reach(key)) ? fmaf(raw, kShaped && shape.cap > 0.f ? 1.0f : to_log2_row, slope_log2 * static_cast<float>(key - (n - 1))) : -INFINITY;
             tile_max = fmaxf(tile_max, sc[j]);
         }
         tile_max = fmaxf(tile_max, __shfl_xor(tile_max, 16, kWave));
@@ -523,22 +528,28 @@ attention_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__
     __syncthreads();
     for (int i = threadIdx.x; i < cols * kD; i += kDecodeThreads) {
         const int col = i / kD, d = i % kD;
+        const int partner = kShaped && shape.turn_cos != nullptr && splits == 1 ? turn_partner(d, kD / 2, shape.turn_pairing) : d;
         float top = -INFINITY;
 #pragma unroll
         for (int w = 0; w < kDecodeWaves; ++w) top = fmaxf(top, sm_m[w * cols + col]);
-        float num = 0.f, den = 0.f;
+        float num = 0.f, den = 0.f, num_partner = 0.f;
         if (top != -INFINITY) {
 #pragma unroll
             for (int w = 0; w < kDecodeWaves; ++w) {
                 const float mw = sm_m[w * cols + col];
                 const float wgt = mw == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(mw - top);
                 num += sm_acc[(w * cols + col) * kD + d] * wgt;
+                if (kShaped) num_partner += sm_acc[(w * cols + col) * kD + partner] * wgt;
                 den += sm_l[w * cols + col] * wgt;
             }
         }
-        const long rh = static_cast<long>(row) * q_heads + kvh * group + col0 + col;
+        const int head = kvh * group + col0 + col;
+        const long rh = static_cast<long>(row) * q_heads + head;
         if (splits == 1) {                            // nothing to merge with: this is the result
-            out[rh * kD + d] = from_float<bf16_t>(num / den);
+            if (kShaped && shape.sinks != nullptr) den += __builtin_amdgcn_exp2f(shape.sinks[head] * 1.4426950408889634f - top);
+            float value = num / den;
+            if (kShaped && shape.turn_cos != nullptr) value = turned_back(value, num_partner / den, d, kD, n - 1, shape);
+            out[rh * kD + d] = from_float<bf16_t>(value);
             continue;
         }
         const long slot = rh * splits + split;
@@ -555,9 +566,11 @@ attention_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__
 constexpr int kReduceThreads = 128;
 constexpr int kMaxSplits = 256;
 
+template <bool kShaped>
 __global__ void __launch_bounds__(kReduceThreads)
 attention_reduce_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
-                        bf16_t* __restrict__ out, int head_dim, int splits) {
+                        bf16_t* __restrict__ out, int head_dim, int splits, const int* __restrict__ positions, int q_heads,
+                        ScoreShape shape) {
     __shared__ float weight[kMaxSplits];
     __shared__ float wave_top[kReduceThreads / kWave];
     const long rh = blockIdx.x;                      // row * q_heads + head
@@ -573,6 +586,27 @@ attention_reduce_kernel(const float* __restrict__ part_acc, const float* __restr
     __syncthreads();
     float den = 0.f;
     for (int s = 0; s < splits; ++s) den += ml[2 * s + 1] * weight[s];
+    if constexpr (kShaped) {
+        // the sink counts once, whatever the splits; a result that is turned back needs both elements of its pairs
+        if (shape.sinks != nullptr) den += __builtin_amdgcn_exp2f(shape.sinks[rh % q_heads] * 1.4426950408889634f - top);
+        if (shape.turn_cos != nullptr) {
+            const long pos = positions[rh / q_heads];
+            for (int d = threadIdx.x; d < head_dim; d += kReduceThreads) {
+                if (!turn_is_first(d, head_dim / 2, shape.turn_pairing)) continue;
+                const int e = turn_partner(d, head_dim / 2, shape.turn_pairing);
+                float u = 0.f, v = 0.f;
+                for (int s = 0; s < splits; ++s) {
+                    const float* acc = part_acc + (rh * splits + s) * head_dim;
+                    u += acc[d] * weight[s];
+                    v += acc[e] * weight[s];
+                }
+                u /= den, v /= den;
+                out[rh * head_dim + d] = from_float<bf16_t>(turned_back(u, v, d, head_dim, pos, shape));
+                out[rh * head_dim + e] = from_float<bf16_t>(turned_back(v, u, e, head_dim, pos, shape));
+            }
+            return;
+        }
+    }
     for (int d = threadIdx.x; d < head_dim; d += kReduceThreads) {
         float num = 0.f;
         for (int s = 0; s < splits; ++s) num += part_acc[(rh * splits + s) * head_dim + d] * weight[s];
@@ -592,31 +626,37 @@ static void launch_decode(const void* q, const void* k_pool, const void* v_pool,
                           const int* row_entry, const int* block_table, int max_blocks, float* part_acc,
                           float* part_ml, void* out, int rows, int q_heads, int kv_heads, int page_shift, float scale,
                           int window, int splits, const FromProjection* from, int keep_first, ScoreBias bias,
-                          hipStream_t stream) {
+                          const ScoreShape& shape, hipStream_t stream) {
     const int group = q_heads / kv_heads;
     dim3 grid(rows, kv_heads * ((group + 15) / 16), splits);
     const size_t smem = decode_smem_bytes(kD16 * 16, group, max_blocks);
     const float to_log2 = scale * 1.4426950408889634f;
     if constexpr (kD16 % 4 == 0) {
         if (from != nullptr) {
-            attention_decode_kernel<kD16, true><<<grid, kDecodeThreads, smem, stream>>>(
+            attention_decode_kernel<kD16, true, false><<<grid, kDecodeThreads, smem, stream>>>(
                 nullptr, static_cast<const bf16_t*>(k_pool), static_cast<const bf16_t*>(v_pool), positions, row_entry,
                 block_table, max_blocks, part_acc, part_ml, static_cast<bf16_t*>(out), q_heads, kv_heads, page_shift,
-                to_log2, window, splits, *from, keep_first, bias);
+                to_log2, window, splits, *from, keep_first, bias, ScoreShape{});
             return;
         }
     }
-    attention_decode_kernel<kD16, false><<<grid, kDecodeThreads, smem, stream>>>(
-        static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pool), static_cast<const bf16_t*>(v_pool),
-        positions, row_entry, block_table, max_blocks, part_acc, part_ml, static_cast<bf16_t*>(out), q_heads, kv_heads,
-        page_shift, to_log2, window, splits, FromProjection{}, keep_first, bias);
+#define LEONE_DECODE_LAUNCH(SHAPED)                                                                                          \
+    attention_decode_kernel<kD16, false, SHAPED><<<grid, kDecodeThreads, smem, stream>>>(                                    \
+        static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pool), static_cast<const bf16_t*>(v_pool),               \
+        positions, row_entry, block_table, max_blocks, part_acc, part_ml, static_cast<bf16_t*>(out), q_heads, kv_heads,      \
+        page_shift, to_log2, window, splits, FromProjection{}, keep_first, bias, shape)
+    if (shape.any()) LEONE_DECODE_LAUNCH(true);
+    else LEONE_DECODE_LAUNCH(false);
+#undef LEONE_DECODE_LAUNCH
 }
 
 static int decode_checked(const void* q, void* out, const void* k_pool, const void* v_pool, const int* positions,
                           const int* row_entry, const int* block_table, int max_blocks, float* part_acc,
                           float* part_ml, int rows, int q_heads, int kv_heads, int head_dim, int page_tokens,
                           float scale, int window, int splits, const FromProjection* from, int keep_first,
-                          hipStream_t stream, ScoreBias bias = ScoreBias{}) {
+                          hipStream_t stream, ScoreBias bias = ScoreBias{}, const ScoreShape& shape = ScoreShape{}) {
+    if (check_score_shape("attention_decode", shape, head_dim)) return 1;
+    LEONE_REQUIRE(!from || !shape.any(), "attention_decode: capped scores, sinks and turned values come with finished queries");
     LEONE_REQUIRE(bias.temp_every >= 0, "attention_decode: the query factor's period %d must not be negative", bias.temp_every);
     LEONE_REQUIRE(keep_first >= 0, "attention_decode: keep_first %d must not be negative", keep_first);
     LEONE_REQUIRE((q || from) && out && k_pool && v_pool && positions && row_entry && block_table,
@@ -641,7 +681,7 @@ static int decode_checked(const void* q, void* out, const void* k_pool, const vo
 #define LEONE_DECODE_CASE(N)                                                                                      \
     case N:                                                                                                       \
         launch_decode<N>(q, k_pool, v_pool, positions, row_entry, block_table, max_blocks, part_acc, part_ml,     \
-                         out, rows, q_heads, kv_heads, page_shift, scale, window, splits, from, keep_first, bias, stream); \
+                         out, rows, q_heads, kv_heads, page_shift, scale, window, splits, from, keep_first, bias, shape, stream); \
         break;
     switch (head_dim / 16) {
         LEONE_DECODE_CASE(1) LEONE_DECODE_CASE(2) LEONE_DECODE_CASE(3) LEONE_DECODE_CASE(4)
@@ -655,8 +695,12 @@ static int decode_checked(const void* q, void* out, const void* k_pool, const vo
 #undef LEONE_DECODE_CASE
     LEONE_LAUNCH_CHECK("attention_decode");
     if (splits > 1) {                                 // a single split has written the result itself
-        attention_reduce_kernel<<<rows * q_heads, kReduceThreads, 0, stream>>>(
-            part_acc, part_ml, static_cast<bf16_t*>(out), head_dim, splits);
+        if (shape.any())
+            attention_reduce_kernel<true><<<rows * q_heads, kReduceThreads, 0, stream>>>(
+                part_acc, part_ml, static_cast<bf16_t*>(out), head_dim, splits, positions, q_heads, shape);
+        else
+            attention_reduce_kernel<false><<<rows * q_heads, kReduceThreads, 0, stream>>>(
+                part_acc, part_ml, static_cast<bf16_t*>(out), head_dim, splits, positions, q_heads, shape);
         LEONE_LAUNCH_CHECK("attention_reduce");
     }
     return 0;
@@ -696,6 +740,20 @@ extern "C" int leone_attention_decode_biased(const void* q, void* out, const voi
     return decode_checked(q, out, k_pool, v_pool, positions, row_entry, block_table, max_blocks, part_acc, part_ml, rows,
                           q_heads, kv_heads, head_dim, page_tokens, scale, window, splits, nullptr, keep_first, stream,
                           ScoreBias{slopes, temp_coef, temp_every});
+}
+
+// The same with what score_shape.h describes: cap (0: none), sinks, and the tables that turn results back (null: none).
+extern "C" int leone_attention_decode_shaped(const void* q, void* out, const void* k_pool, const void* v_pool,
+                                             const int* positions, const int* row_entry, const int* block_table,
+                                             int max_blocks, float* part_acc, float* part_ml, int rows, int q_heads,
+                                             int kv_heads, int head_dim, int page_tokens, float scale, int window,
+                                             int splits, int keep_first, const float* slopes, float temp_coef,
+                                             int temp_every, float cap, const float* sinks, const float* turn_cos,
+                                             const float* turn_sin, int turn_positions, int turn_pairing, hipStream_t stream) {
+    return decode_checked(q, out, k_pool, v_pool, positions, row_entry, block_table, max_blocks, part_acc, part_ml, rows,
+                          q_heads, kv_heads, head_dim, page_tokens, scale, window, splits, nullptr, keep_first, stream,
+                          ScoreBias{slopes, temp_coef, temp_every},
+                          ScoreShape{cap, sinks, turn_cos, turn_sin, turn_positions, turn_pairing});
 }
 
 // The same for a step in which every row is another request, taking the fused q/k/v projection instead of

@@ -37,6 +37,7 @@
 #include "common.h"
 #include "leone_hip.h"
 #include "prefill_order.h"
+#include "score_shape.h"
 
 #include <math.h>
 
@@ -66,14 +67,15 @@ __host__ __device__ constexpr int stage_runs(int head_dim) { return (head_dim / 
 
 // tiles: [n_groups][4][3] = (entry, first row of the tile in the step, rows in the tile); a tile has at
 // most 32 rows, 0 rows marks an unused place; the tiles of a group belong to one entry.
-template <int kD16>
+// kShaped: capped scores, sinks, results turned back (ScoreShape); without it none of that is in the kernel.
+template <int kD16, bool kShaped>
 __global__ void __launch_bounds__(kPrefillThreads, 2)
 attention_prefill_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out, const bf16_t* __restrict__ k_pool,
                          const bf16_t* __restrict__ v_pool, const int* __restrict__ positions,
                          const int* __restrict__ tiles, int n_groups, const int* __restrict__ block_table,
                          int max_blocks, int q_heads, int kv_heads, int page_shift, float scale, int window,
                          float* __restrict__ part_acc, float* __restrict__ part_ml, int splits, int keep_first,
-                         const float* __restrict__ slopes, float temp_coef, int temp_every) {
+                         const float* __restrict__ slopes, float temp_coef, int temp_every, ScoreShape shape) {
     constexpr int kD = kD16 * 16;
     constexpr int kRuns = kD / 8;                      // 16-byte runs of one key
     constexpr int kDT = (kD + 31) / 32;                // 32-row tiles of the second product's result
@@ -330,11 +332,17 @@ attention_prefill_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
             for (int v = 0; v < 16; ++v) sc[v] += sc_odd[v];
         }
         // lane (j, h): sc[v] is row j's score of key key0 + 8 h + v (v < 8) or key0 + 16 + 8 h + v - 8
+        if (kShaped && shape.cap > 0.f) {                      // in units of the raw dot product, like everything before to_log2
+            const float to_cap = row_factor * scale / shape.cap, from_cap = shape.cap / scale;
+#pragma unroll
+            for (int v = 0; v < 16; ++v) sc[v] = from_cap * tanh_fast(sc[v] * to_cap);
+        }
         if (biased) {
+            const float factor = kShaped && shape.cap > 0.f ? 1.0f : row_factor;
 #pragma unroll
             for (int v = 0; v < 16; ++v) {
                 const int key = key0 + 8 * h + (v & 7) + 16 * (v >> 3);
-                sc[v] = fmaf(sc[v], row_factor, slope_raw * static_cast<float>(key - row_pos));
+                sc[v] = fmaf(sc[v], factor, slope_raw * static_cast<float>(key - row_pos));
             }
         }
         if (!full) {                                           // the same for the whole wave
@@ -440,7 +448,41 @@ attention_prefill_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
         return;
     }
     if (!row_ok) return;
-    const float inv = poisoned ? __builtin_nanf("") : 1.0f / l_row;
+    float l_all = l_row;
+    if (kShaped && shape.sinks != nullptr) l_all += __builtin_amdgcn_exp2f(shape.sinks[head] * 1.44269504088896340736f - m_ref);
+    const float inv = poisoned ? __builtin_nanf("") : 1.0f / l_all;
+    if (kShaped && shape.turn_cos != nullptr) {
+        // Results turned back by the row's own angles.  Half a head is a multiple of 8 elements, so an element's partner
+        // is the same lane's: eight elements e, 8 of them further by half.
+        constexpr int kEights = kD / 8, kHalfEights = kEights / 2;
+        const long tpos = row_pos < shape.turn_positions ? row_pos : shape.turn_positions - 1;
+        const float* cs = shape.turn_cos + tpos * (kD / 2);
+        const float* sn = shape.turn_sin + tpos * (kD / 2);
+        if (shape.turn_pairing == 0) {
+#pragma unroll
+            for (int e = 0; e < kHalfEights; ++e) {
+                const int f = e + kHalfEights;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const float c = cs[8 * e + 4 * h + i], n = sn[8 * e + 4 * h + i];
+                    const float u = acc[e / 4][4 * (e % 4) + i], v = acc[f / 4][4 * (f % 4) + i];
+                    acc[e / 4][4 * (e % 4) + i] = u * c + v * n;
+                    acc[f / 4][4 * (f % 4) + i] = v * c - u * n;
+                }
+            }
+        } else {
+#pragma unroll
+            for (int e = 0; e < kEights; ++e)
+#pragma unroll
+                for (int i = 0; i < 4; i += 2) {
+                    const int m = (8 * e + 4 * h + i) / 2;
+                    const float c = cs[m], n = sn[m];
+                    const float u = acc[e / 4][4 * (e % 4) + i], v = acc[e / 4][4 * (e % 4) + i + 1];
+                    acc[e / 4][4 * (e % 4) + i] = u * c + v * n;
+                    acc[e / 4][4 * (e % 4) + i + 1] = v * c - u * n;
+                }
+        }
+    }
     bf16_t* orow = out + (static_cast<long>(tile_row0 + j) * q_heads + head) * kD;
 #pragma unroll
     for (int dt = 0; dt < kDT; ++dt)
@@ -469,7 +511,7 @@ constexpr int kMaxPrefillSplits = 32;
 __global__ void __launch_bounds__(kMergeThreads)
 attention_prefill_merge_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
                                bf16_t* __restrict__ out, const int* __restrict__ tiles, int q_heads, int head_dim,
-                               int splits) {
+                               int splits, const int* __restrict__ positions, ScoreShape shape) {
     const int* tile = tiles + 3 * static_cast<long>(blockIdx.x / kMergeBlocksPerTile);
     const int row0 = tile[1], rows = tile[2], head = blockIdx.y;
     const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
@@ -497,24 +539,44 @@ attention_prefill_merge_kernel(const float* __restrict__ part_acc, const float* 
                 }
             }
         }
+        if (shape.sinks != nullptr) den += __builtin_amdgcn_exp2f(shape.sinks[head] * 1.44269504088896340736f - top);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) num[i] /= den;
+        if (shape.turn_cos != nullptr) {
+            float turned[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int d = lane + kWave * i;
+                const int e = d < head_dim ? turn_partner(d, head_dim / 2, shape.turn_pairing) : 0;
+                float partner = 0.f;
+#pragma unroll
+                for (int k = 0; k < 4; ++k) {                     // every lane takes part in every exchange
+                    const float got = __shfl(num[k], e % kWave, kWave);
+                    if (e / kWave == k) partner = got;
+                }
+                turned[i] = d < head_dim ? turned_back(num[i], partner, d, head_dim, positions[row0 + r], shape) : 0.f;
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i) num[i] = turned[i];
+        }
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int d = lane + kWave * i;
-            if (d < head_dim) out[rh * head_dim + d] = from_float<bf16_t>(num[i] / den);
+            if (d < head_dim) out[rh * head_dim + d] = from_float<bf16_t>(num[i]);
         }
     }
 }
 
-template <int kD16>
+template <int kD16, bool kShaped>
 static int launch_prefill(const void* q, void* out, const void* k_pool, const void* v_pool, const int* positions,
                           const int* tiles, int n_groups, const int* block_table, int max_blocks, int q_heads,
                           int kv_heads, int page_shift, float scale, int window, float* part_acc, float* part_ml,
                           int splits, int keep_first, const float* slopes, float temp_coef, int temp_every,
-                          hipStream_t stream) {
+                          const ScoreShape& shape, hipStream_t stream) {
     const size_t shared = 2 * static_cast<size_t>(stage_runs(16 * kD16)) * sizeof(uint4) + static_cast<size_t>(max_blocks) * sizeof(int);
     static size_t allowed = 48 * 1024;                 // what a kernel may use without asking
     if (shared > allowed) {
-        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&attention_prefill_kernel<kD16>),
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&attention_prefill_kernel<kD16, kShaped>),
                                                  hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(shared));
         if (e != hipSuccess) {
             set_error("attention_prefill: %zu bytes of shared memory were refused: %s", shared, hipGetErrorString(e));
@@ -522,10 +584,10 @@ static int launch_prefill(const void* q, void* out, const void* k_pool, const vo
         }
         allowed = shared;
     }
-    attention_prefill_kernel<kD16><<<dim3(n_groups * q_heads, splits), kPrefillThreads, shared, stream>>>(
+    attention_prefill_kernel<kD16, kShaped><<<dim3(n_groups * q_heads, splits), kPrefillThreads, shared, stream>>>(
         static_cast<const bf16_t*>(q), static_cast<bf16_t*>(out), static_cast<const bf16_t*>(k_pool),
         static_cast<const bf16_t*>(v_pool), positions, tiles, n_groups, block_table, max_blocks, q_heads, kv_heads,
-        page_shift, scale, window, part_acc, part_ml, splits, keep_first, slopes, temp_coef, temp_every);
+        page_shift, scale, window, part_acc, part_ml, splits, keep_first, slopes, temp_coef, temp_every, shape);
     return 0;
 }
 
@@ -576,6 +638,21 @@ extern "C" int leone_attention_prefill_biased(const void* q, void* out, const vo
                                               float scale, int window, float* part_acc, float* part_ml, int splits,
                                               int keep_first, const float* slopes, float temp_coef, int temp_every,
                                               hipStream_t stream) {
+    return leone_attention_prefill_shaped(q, out, k_pool, v_pool, positions, tiles, n_groups, block_table, max_blocks, q_heads,
+                                          kv_heads, head_dim, page_tokens, scale, window, part_acc, part_ml, splits, keep_first,
+                                          slopes, temp_coef, temp_every, 0.f, nullptr, nullptr, nullptr, 0, 0, stream);
+}
+
+// The same with what score_shape.h describes: cap (0: none), sinks, and the tables that turn results back (null: none).
+extern "C" int leone_attention_prefill_shaped(const void* q, void* out, const void* k_pool, const void* v_pool,
+                                              const int* positions, const int* tiles, int n_groups, const int* block_table,
+                                              int max_blocks, int q_heads, int kv_heads, int head_dim, int page_tokens,
+                                              float scale, int window, float* part_acc, float* part_ml, int splits,
+                                              int keep_first, const float* slopes, float temp_coef, int temp_every, float cap,
+                                              const float* sinks, const float* turn_cos, const float* turn_sin,
+                                              int turn_positions, int turn_pairing, hipStream_t stream) {
+    const ScoreShape shape{cap, sinks, turn_cos, turn_sin, turn_positions, turn_pairing};
+    if (check_score_shape("attention_prefill", shape, head_dim)) return 1;
     LEONE_REQUIRE(temp_every >= 0, "attention_prefill: the query factor's period %d must not be negative", temp_every);
     LEONE_REQUIRE(keep_first >= 0 && (keep_first == 0 || window == 0 || splits == 1),
                   "attention_prefill: kept first keys (%d) beside a window come with one range of keys, not %d", keep_first, splits);
@@ -600,9 +677,15 @@ extern "C" int leone_attention_prefill_biased(const void* q, void* out, const vo
     int status = 0;
 #define LEONE_PREFILL_CASE(N)                                                                                      \
     case N:                                                                                                        \
-        status = launch_prefill<N>(q, out, k_pool, v_pool, positions, tiles, n_groups, block_table, max_blocks,    \
-                                   q_heads, kv_heads, page_shift, scale, window, part_acc, part_ml, splits,        \
-                                   keep_first, slopes, temp_coef, temp_every, stream);                             \
+        status = shape.any()                                                                                       \
+                     ? launch_prefill<N, true>(q, out, k_pool, v_pool, positions, tiles, n_groups, block_table,    \
+                                               max_blocks, q_heads, kv_heads, page_shift, scale, window, part_acc, \
+                                               part_ml, splits, keep_first, slopes, temp_coef, temp_every, shape,  \
+                                               stream)                                                             \
+                     : launch_prefill<N, false>(q, out, k_pool, v_pool, positions, tiles, n_groups, block_table,   \
+                                                max_blocks, q_heads, kv_heads, page_shift, scale, window, part_acc, \
+                                                part_ml, splits, keep_first, slopes, temp_coef, temp_every, shape, \
+                                                stream);                                                           \
         break;
     switch (head_dim / 16) {
         LEONE_PREFILL_CASE(1) LEONE_PREFILL_CASE(2) LEONE_PREFILL_CASE(3) LEONE_PREFILL_CASE(4)
@@ -617,7 +700,7 @@ extern "C" int leone_attention_prefill_biased(const void* q, void* out, const vo
     if (splits > 1) {
         attention_prefill_merge_kernel<<<dim3(n_groups * kPrefillWaves * kMergeBlocksPerTile, q_heads), kMergeThreads, 0,
                                          stream>>>(
-            part_acc, part_ml, static_cast<bf16_t*>(out), tiles, q_heads, head_dim, splits);
+            part_acc, part_ml, static_cast<bf16_t*>(out), tiles, q_heads, head_dim, splits, positions, shape);
         LEONE_LAUNCH_CHECK("attention_prefill_merge");
     }
     return 0;

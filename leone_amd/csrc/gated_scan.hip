@@ -8,6 +8,9 @@
 //                 dt_t = softplus(pre_t + bias),  f_t = exp(-exp(rate_log) * dt_t)  for every key channel of the head,
 //                 S_t = f_t S_(t-1) + (dt_t B_t) x_t^T,   o_t = S_t^T C_t + skip * x_t
 //                 with B and C shared by the heads of a group (head h reads group h / (heads / groups))
+//   time_mix_scan the same walk for a memory whose decays come ready made and whose current token counts by a weight of its
+//                 own until it is written: o_t = (S_(t-1) + diag(bonus) k_t v_t^T)^T r_t, then S_t = diag(w_t) S_(t-1) + k_t v_t^T
+//                 (the read-out of the old state plus v_t times the row's sum of bonus * k * r, which is made once a row)
 //   gated_chain   chains the end states of chunks that were walked side by side (see below).
 //
 // The layout is that of the other matrix-memory recurrences: a workgroup of four waves owns a run of columns of one
@@ -63,9 +66,15 @@ struct GatedScanArgs {
     long step_stride;
     int step_off;
     AnyVec step_bias, rate_log, skip;   // [heads] each
+    // the time-mixing form: r, k and v at proj, k_at and v_at (all of `stride`, head h at h * dim or h * vdim), the decays
+    // w at decay [rows, heads * dim]
+    const float* k_at = nullptr;
+    const float* v_at = nullptr;
+    const float* decay = nullptr;
+    AnyVec bonus{};                     // [heads * dim]
 };
 
-enum GsKind : int { kGsGated = 0, kGsStateSpace = 1 };
+enum GsKind : int { kGsGated = 0, kGsStateSpace = 1, kGsTimeMix = 2 };
 
 template <bool kTrack, int kKind>
 __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p, int groups) {
@@ -101,6 +110,7 @@ __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p,
         for (int i = 0; i < kGsLaneRows; ++i) carried[i] = 1.f;
     }
 
+    __shared__ float s_now[kKind == kGsTimeMix ? kGsTokens : 1];   // the time-mixing form: a row's sum of bonus * k * r
     __shared__ float s_dt[kGsTokens], s_decay[kGsTokens];   // the state-space form: a row's step size and decay, made once
     for (int t0 = 0; t0 < n; t0 += kGsTokens) {
         const int here = min(kGsTokens, n - t0);
@@ -124,6 +134,14 @@ __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p,
                     fv = s_decay[t];
                     kv = p.no_input ? 0.f : s_dt[t] * base[p.k_off + shared_head * p.dim + i];
                 }
+            } else if (kKind == kGsTimeMix) {
+                if (i < p.dim) {
+                    const long r = first + t0 + t;
+                    const int ch = head * p.dim + i;
+                    qv = p.proj[r * p.stride + ch];
+                    fv = p.decay[r * p.heads * p.dim + ch];
+                    kv = p.no_input ? 0.f : p.k_at[r * p.stride + ch];
+                }
             } else if (i < p.dim) {
                 const float* base = p.proj + static_cast<long>(first + t0 + t) * p.stride;
                 const float qp = base[p.q_off + head * p.dim + i];
@@ -139,6 +157,19 @@ __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p,
             sk[idx] = kv;
         }
         __syncthreads();
+        if constexpr (kKind == kGsTimeMix) {
+            // sixteen threads a row
+            for (int t = tid / 16; t < here; t += blockDim.x / 16) {
+                float sum = 0.f;
+                if (!p.no_input)
+                    for (int i = tid % 16; i < p.dim; i += 16)
+                        sum = fmaf(load_any(p.bonus, head * p.dim + i) * sk[t * dkp + i], sq[t * dkp + i], sum);
+#pragma unroll
+                for (int off = 8; off > 0; off >>= 1) sum += __shfl_xor(sum, off, kWave);
+                if (tid % 16 == 0) s_now[t] = sum;
+            }
+            __syncthreads();
+        }
         if (col[0] < p.vdim) {                                  // the lanes of a column are in or out together
             for (int t = 0; t < here; ++t) {
                 const long row = first + t0 + t;
@@ -149,15 +180,17 @@ __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p,
 #pragma unroll
                 for (int c = 0; c < kGsLaneCols; ++c) {
                     acc[c] = 0.f;
-                    v[c] = (!p.no_input && col[c] < p.vdim) ? p.proj[row * p.stride + p.v_off + head * p.vdim + col[c]] : 0.f;
+                    const float* v_row = kKind == kGsTimeMix ? p.v_at + row * p.stride : p.proj + row * p.stride + p.v_off;
+                    v[c] = (!p.no_input && col[c] < p.vdim) ? v_row[head * p.vdim + col[c]] : 0.f;
                 }
 #pragma unroll
                 for (int i = 0; i < kGsLaneRows; ++i) {
                     const float f = ft[i], k = kt[i], q = qt[i];
 #pragma unroll
                     for (int c = 0; c < kGsLaneCols; ++c) {
+                        if constexpr (kKind == kGsTimeMix) acc[c] = fmaf(S[c][i], q, acc[c]);       // the state before this row
                         S[c][i] = fmaf(f, S[c][i], k * v[c]);
-                        acc[c] = fmaf(S[c][i], q, acc[c]);
+                        if constexpr (kKind != kGsTimeMix) acc[c] = fmaf(S[c][i], q, acc[c]);
                     }
                     if constexpr (kTrack) carried[i] *= f;
                 }
@@ -166,7 +199,9 @@ __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p,
                     for (int off = per_wave; off < kWave; off <<= 1) acc[c] += __shfl_xor(acc[c], off, kWave);
                     if (part == 0 && col[c] < p.vdim) {
                         float* dst = p.out + (row * p.heads + head) * p.vdim + col[c];
-                        const float read = kKind == kGsStateSpace ? fmaf(skip, v[c], acc[c]) : acc[c];
+                        const float read = kKind == kGsStateSpace ? fmaf(skip, v[c], acc[c])
+                                           : kKind == kGsTimeMix  ? fmaf(s_now[t], v[c], acc[c])
+                                                                  : acc[c];
                         *dst = p.accumulate ? *dst + read : read;
                     }
                 }
@@ -288,6 +323,36 @@ extern "C" int leone_state_space_scan(const float* xbc, long stride, int x_off, 
     if (gate_product) gated_scan_kernel<true, kGsStateSpace><<<grid, waves * kWave, shared, stream>>>(a, groups);
     else gated_scan_kernel<false, kGsStateSpace><<<grid, waves * kWave, shared, stream>>>(a, groups);
     LEONE_LAUNCH_CHECK("state_space_scan");
+    return 0;
+}
+
+// The time-mixing form.  r, k, v float [rows, stride] (heads * dim, heads * dim and heads * vdim columns), decay float
+// [rows, heads * dim], bonus [heads * dim] of bonus_dtype.  States, segments, products and out as for leone_gated_scan.
+extern "C" int leone_time_mix_scan(const float* r, const float* k, const float* v, long stride, const float* decay,
+                                   const void* bonus, int bonus_dtype, int no_input, int accumulate, const int* segments,
+                                   int n_segments, const float* state_in, long in_stride, float* state_out, long out_stride,
+                                   float* decay_product, float* out, int heads, int dim, int vdim, hipStream_t stream) {
+    LEONE_REQUIRE(r && k && v && decay && bonus && segments && out, "time_mix_scan: null pointer");
+    LEONE_REQUIRE(bonus_dtype == kF32 || bonus_dtype == kBF16, "time_mix_scan: unknown element type");
+    LEONE_REQUIRE(n_segments > 0 && heads > 0 && heads <= 65535 && dim > 0 && vdim > 0, "time_mix_scan: %d segments, %d heads of %d x %d",
+                  n_segments, heads, dim, vdim);
+    LEONE_REQUIRE(dim <= kGsMaxDim, "time_mix_scan: heads of %d key channels, the kernel takes up to %d", dim, kGsMaxDim);
+    const long per_slot = static_cast<long>(heads) * dim * vdim;
+    LEONE_REQUIRE((!state_in || in_stride >= per_slot) && (!state_out || out_stride >= per_slot),
+                  "time_mix_scan: states of %ld floats do not fit", per_slot);
+    LEONE_REQUIRE(stride >= static_cast<long>(heads) * (dim > vdim ? dim : vdim), "time_mix_scan: rows of %ld do not hold the heads", stride);
+    const AnyVec none{nullptr, bonus_dtype};
+    GatedScanArgs a{r, stride, 0, 0, 0, none, none, 0, no_input, accumulate, reinterpret_cast<const GsSegment*>(segments),
+                    state_in, in_stride, state_out, out_stride, decay_product, out, heads, dim, vdim, heads, 0, nullptr, 0, 0,
+                    none, none, none, k, v, decay, AnyVec{bonus, bonus_dtype}};
+    const int groups = gs_lane_groups(dim);
+    const int per_wave = (kWave / groups) * kGsLaneCols;         // as for the state-space form: no wave stands idle
+    const int waves = ceil_div(vdim, per_wave) < kGsThreads / kWave ? ceil_div(vdim, per_wave) : kGsThreads / kWave;
+    const dim3 grid(n_segments, heads, ceil_div(vdim, waves * per_wave));
+    const size_t shared = 3 * kGsTokens * groups * kGsLaneRows * sizeof(float);
+    if (decay_product) gated_scan_kernel<true, kGsTimeMix><<<grid, waves * kWave, shared, stream>>>(a, groups);
+    else gated_scan_kernel<false, kGsTimeMix><<<grid, waves * kWave, shared, stream>>>(a, groups);
+    LEONE_LAUNCH_CHECK("time_mix_scan");
     return 0;
 }
 

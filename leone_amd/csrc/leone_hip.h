@@ -389,4 +389,56 @@ int leone_residual_norm(float* x, const float* delta, int planes, long plane, fl
                         float eps, void* y, int y_dtype, const int* rows, int n_rows, int hidden, hipStream_t stream);
 int leone_depth_mix(float* x, const float* delta, int planes, long plane, float scale, float* history, long slot_stride,
                     int count, const void* weight, int weight_dtype, long total, hipStream_t stream);
+// The attention kernels with a cap on the scores (0: none), a sink a head in the denominator and results turned back by the
+// row's own angles (null: none); see score_shape.h.
+int leone_attention_rows_shaped(const void* q, void* out, const void* k_pool, const void* v_pool, int dtype, const int* positions,
+                                const int* row_entry, const int* block_table, int max_blocks, int rows, int q_heads, int kv_heads,
+                                int head_dim, int v_dim, int page_tokens, float scale, int window, const float* gate,
+                                long gate_stride, int keep_first, int gate_each, const float* slopes, float temp_coef,
+                                int temp_every, float cap, const float* sinks, const float* turn_cos, const float* turn_sin,
+                                int turn_positions, int turn_pairing, hipStream_t stream);
+int leone_attention_decode_shaped(const void* q, void* out, const void* k_pool, const void* v_pool, const int* positions,
+                                  const int* row_entry, const int* block_table, int max_blocks, float* part_acc, float* part_ml,
+                                  int rows, int q_heads, int kv_heads, int head_dim, int page_tokens, float scale, int window,
+                                  int splits, int keep_first, const float* slopes, float temp_coef, int temp_every, float cap,
+                                  const float* sinks, const float* turn_cos, const float* turn_sin, int turn_positions,
+                                  int turn_pairing, hipStream_t stream);
+int leone_attention_prefill_shaped(const void* q, void* out, const void* k_pool, const void* v_pool, const int* positions,
+                                   const int* tiles, int n_groups, const int* block_table, int max_blocks, int q_heads,
+                                   int kv_heads, int head_dim, int page_tokens, float scale, int window, float* part_acc,
+                                   float* part_ml, int splits, int keep_first, const float* slopes, float temp_coef,
+                                   int temp_every, float cap, const float* sinks, const float* turn_cos, const float* turn_sin,
+                                   int turn_positions, int turn_pairing, hipStream_t stream);
+// Attention whose heads' scaled scores are mixed by talk [q_heads, q_heads] before the softmax.
+int leone_attention_rows_talk(const void* q, void* out, const void* k_pool, const void* v_pool, int dtype, const void* talk,
+                              int talk_dtype, const int* positions, const int* row_entry, const int* block_table, int max_blocks,
+                              int rows, int q_heads, int kv_heads, int head_dim, int v_dim, int page_tokens, float scale,
+                              int window, hipStream_t stream);
+// leone_qk_norm_rope_write for projections that still get a bias [all heads' columns], values that are turned by their
+// position, and heads of which only the first norm_count elements exist (the rest are zeros that do not count in a norm).
+int leone_qk_norm_rope_write_turned(const void* qkv, int qkv_dtype, int qkv_planes, long qkv_plane, void* q_out, void* k_pool,
+                                    void* v_pool, int dtype, const void* q_gain, const void* k_gain, int gain_dtype, float eps,
+                                    const float* cos_table, const float* sin_table, int table_positions, int rotary_dim,
+                                    int pairing, const int* positions, const int* row_entry, const int* block_table,
+                                    int max_blocks, int rows, int q_heads, int kv_heads, int head_dim, int page_tokens,
+                                    int write_cache, int v_dim, long row_width, const void* bias, int bias_dtype,
+                                    const float* v_cos, const float* v_sin, int v_positions, int v_pairing, int norm_count,
+                                    hipStream_t stream);
+// x += sum_t factor_t * scale_t * rows_t (up to four results, each float in planes, with an optional vector), then up to two
+// RMS norms of the new rows in equal groups of columns, each with its own gain (see branch_norm.hip).
+int leone_branch_norm(float* x, const void* const* term_rows, const int* term_planes, const long* term_plane,
+                      const float* term_factor, const void* const* term_scale, const int* term_scale_dtype, int terms,
+                      const void* const* gains, const int* gain_dtypes, void* const* outs, int norms, int out_dtype, float eps,
+                      int groups, const int* rows, int n_rows, int hidden, hipStream_t stream);
+// The token before beside the token itself, decays from a low-rank product, and the memory they drive (see time_mix.hip and
+// gated_scan.hip).
+int leone_token_mix(const void* h, int dtype, const void* mu, int mu_dtype, int mixes, const float* state, float* state_out,
+                    const int* spans, int entries, const int* row_entry, void* out, int rows, int hidden, int single_rows,
+                    hipStream_t stream);
+int leone_low_rank_decay(const float* low, long low_stride, const void* w2, int w2_dtype, const void* w0, int w0_dtype, float* out,
+                         int rows, int channels, int rank, hipStream_t stream);
+int leone_time_mix_scan(const float* r, const float* k, const float* v, long stride, const float* decay, const void* bonus,
+                        int bonus_dtype, int no_input, int accumulate, const int* segments, int n_segments, const float* state_in,
+                        long in_stride, float* state_out, long out_stride, float* decay_product, float* out, int heads, int dim,
+                        int vdim, hipStream_t stream);
 }

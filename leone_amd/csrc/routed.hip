@@ -7,8 +7,9 @@
 //   moe_plan     the (row, place) pairs of every expert gathered into tiles of pairs of one expert.
 //   route_plan   both in one launch of one workgroup, for steps of few rows; experts that every row takes with
 //                weight 1 (a shared expert cut to the experts' size) may stand behind the routed ones.
-//   moe_product  gated: act(W_gate x) * (W_up x) of every pair, by its expert's matrices; else W_down of that, times
-//                the pair's weight, float.  Three kernels: any type and size (float sums of 8-element runs a lane);
+//   moe_product  gated: act(W_gate x) * (W_up x) of every pair, by its expert's matrices; plain (experts without a gate):
+//                act(W_up x), or act(W_up (weight x)) where the pair's weight multiplies what the expert reads; else
+//                W_down of that, times the pair's weight if there is one, float.  Three kernels: any type and size (float sums of 8-element runs a lane);
 //                bfloat16 on the matrix cores from registers (tiles of 16 or 64 pairs); bfloat16 on the matrix cores
 //                through shared memory (tiles of 128 pairs x 128 rows).
 //   moe_combine  a row's pairs summed in the order of its places; a router output beyond the experts with
@@ -305,14 +306,18 @@ __device__ inline void load8f<bf16_t>(const bf16_t* __restrict__ p, int k, int l
 
 // A tile's pairs against kMoeCols rows of its expert's matrices: a wave takes kColsPerWave rows, its lanes runs of
 // eight elements of the inner size; sums over the lanes at the end.
-//   kGated: w = [experts][2][n][k] (gate rows, then up rows), y[pair][col] = act(gate) * up in T
-//   else:   w = [experts][n][k], y[pair][col] = weight[pair] * product in float
-// x: kGated: row pair / top of [rows][k]; else row pair of [pairs][k].
-template <typename T, bool kGated>
+//   kMoeGated: w = [experts][2][n][k] (gate rows, then up rows), y[pair][col] = act(gate) * up in T
+//   kMoePlain: w = [experts][n][k], y[pair][col] = act(weight[pair] * product) in T (a product of weight[pair] * x)
+//   kMoeDown:  w = [experts][n][k], y[pair][col] = weight[pair] * product in float
+// x: kMoeDown: row pair of [pairs][k]; else row pair / top of [rows][k].  Without weights they count as 1.
+enum MoeMode : int { kMoeDown = 0, kMoeGated = 1, kMoePlain = 2 };
+
+template <typename T, int kMode>
 __global__ void __launch_bounds__(kMoeThreads)
 moe_product_kernel(const T* __restrict__ x, const T* __restrict__ w, void* __restrict__ y, const float* __restrict__ pair_weight,
                    const int* __restrict__ tile_expert, const int* __restrict__ tile_pairs, int top, int n, int k, int act,
                    float limit, int runs) {
+    constexpr bool kGated = kMode == kMoeGated;
     const int tile = blockIdx.x;
     const int e = tile_expert[tile];
     if (e < 0) return;
@@ -337,7 +342,7 @@ moe_product_kernel(const T* __restrict__ x, const T* __restrict__ w, void* __res
 #pragma unroll
         for (int p = 0; p < kTilePairs; ++p) {
             if (pair[p] >= 0) {
-                load8f<T>(x + static_cast<long>(kGated ? pair[p] / top : pair[p]) * k, at, k, runs != 0, xv[p]);
+                load8f<T>(x + static_cast<long>(kMode != kMoeDown ? pair[p] / top : pair[p]) * k, at, k, runs != 0, xv[p]);
             } else {
 #pragma unroll
                 for (int i = 0; i < 8; ++i) xv[p][i] = 0.f;
@@ -384,8 +389,11 @@ moe_product_kernel(const T* __restrict__ x, const T* __restrict__ w, void* __res
         if (col < n && which >= 0) {
             if constexpr (kGated)
                 static_cast<T*>(y)[static_cast<long>(which) * n + col] = from_float<T>(glu_value(mine, mine2, act, limit));
+            else if constexpr (kMode == kMoePlain)
+                static_cast<T*>(y)[static_cast<long>(which) * n + col] =
+                    from_float<T>(plain_act(pair_weight ? mine * pair_weight[which] : mine, act));
             else
-                static_cast<float*>(y)[static_cast<long>(which) * n + col] = mine * pair_weight[which];
+                static_cast<float*>(y)[static_cast<long>(which) * n + col] = pair_weight ? mine * pair_weight[which] : mine;
         }
     }
 }
@@ -407,11 +415,12 @@ __device__ inline moe_bf16x8 moe_zero8() {
     return __builtin_bit_cast(moe_bf16x8, z);
 }
 
-template <int kPB, int kRT, bool kGated>
+template <int kPB, int kRT, int kMode>
 __global__ void __launch_bounds__(kMoeThreads)
 moe_product_mfma_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, void* __restrict__ y,
                         const float* __restrict__ pair_weight, const int* __restrict__ tile_expert,
                         const int* __restrict__ tile_pairs, int top, int n, int k, int act, float limit) {
+    constexpr bool kGated = kMode == kMoeGated;
     // kPB blocks of 16 pairs a tile; kRT blocks of 16 rows a wave (a workgroup takes 64 * kRT rows): the more of
     // both, the fewer times the rows of the matrix and of x are fetched again by other workgroups.
     constexpr int kTile = 16 * kPB;
@@ -427,7 +436,7 @@ moe_product_mfma_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__
 #pragma unroll
     for (int b = 0; b < kPB; ++b) {
         pair[b] = tile_pairs[static_cast<long>(tile) * kTile + 16 * b + c];
-        xrow[b] = x + static_cast<long>(pair[b] < 0 ? 0 : (kGated ? pair[b] / top : pair[b])) * k;
+        xrow[b] = x + static_cast<long>(pair[b] < 0 ? 0 : (kMode != kMoeDown ? pair[b] / top : pair[b])) * k;
     }
     const long matrix = static_cast<long>(n) * k;
     bool row_ok[kRT];
@@ -483,7 +492,7 @@ moe_product_mfma_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__
 #pragma unroll
     for (int b = 0; b < kPB; ++b) {
         if (pair[b] < 0) continue;
-        const float scale = kGated ? 1.f : pair_weight[pair[b]];
+        const float scale = kGated || !pair_weight ? 1.f : pair_weight[pair[b]];
 #pragma unroll
         for (int t = 0; t < kRT; ++t) {
 #pragma unroll
@@ -493,6 +502,8 @@ moe_product_mfma_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__
                 if constexpr (kGated)
                     static_cast<bf16_t*>(y)[static_cast<long>(pair[b]) * n + r] =
                         from_float<bf16_t>(glu_value(acc[t][b][j], acc2[t][b][j], act, limit));
+                else if constexpr (kMode == kMoePlain)
+                    static_cast<bf16_t*>(y)[static_cast<long>(pair[b]) * n + r] = from_float<bf16_t>(plain_act(acc[t][b][j] * scale, act));
                 else
                     static_cast<float*>(y)[static_cast<long>(pair[b]) * n + r] = acc[t][b][j] * scale;
             }
@@ -511,11 +522,12 @@ constexpr int kBigPairs = 128;
 constexpr int kBigRows = 128;
 constexpr int kBigChunk = 64;
 
-template <bool kGated>
+template <int kMode>
 __global__ void __launch_bounds__(kMoeThreads, 2)
 moe_product_tiled_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, void* __restrict__ y,
                          const float* __restrict__ pair_weight, const int* __restrict__ tile_expert,
                          const int* __restrict__ tile_pairs, int top, int n, int k, int act, float limit, int n_tiles, int n_blocks) {
+    constexpr bool kGated = kMode == kMoeGated;
     constexpr int kWRows = kGated ? 2 * kBigRows : kBigRows;          // rows of the matrix in a chunk
     constexpr int kXPieces = kBigPairs * 8 / kMoeThreads;             // 16-byte pieces of x a thread brings per chunk
     constexpr int kWPieces = kWRows * 8 / kMoeThreads;
@@ -547,7 +559,7 @@ moe_product_tiled_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict_
 #pragma unroll
     for (int i = 0; i < kXPieces; ++i) {
         const int pair = my_pairs[tid / 8 + 32 * i];
-        x_from[i] = pair < 0 ? nullptr : x + static_cast<long>(kGated ? pair / top : pair) * k + 8 * part;
+        x_from[i] = pair < 0 ? nullptr : x + static_cast<long>(kMode != kMoeDown ? pair / top : pair) * k + 8 * part;
     }
 #pragma unroll
     for (int i = 0; i < kWPieces; ++i) {
@@ -613,17 +625,24 @@ moe_product_tiled_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict_
     for (int tb = 0; tb < 4; ++tb) {
         const int pair = my_pairs[64 * wp + 16 * tb + c];
         if (pair < 0) continue;
-        const float scale = kGated ? 1.f : pair_weight[pair];
+        const float scale = kGated || !pair_weight ? 1.f : pair_weight[pair];
 #pragma unroll
         for (int ta = 0; ta < 4; ++ta) {
             const int r = row_base + 64 * wr + 16 * ta + 4 * g;
             if (r >= n) continue;
             float v0, v1, v2, v3;
-            if constexpr (kGated) {
-                v0 = glu_value(acc[ta][tb][0], acc2[ta][tb][0], act, limit);
-                v1 = glu_value(acc[ta][tb][1], acc2[ta][tb][1], act, limit);
-                v2 = glu_value(acc[ta][tb][2], acc2[ta][tb][2], act, limit);
-                v3 = glu_value(acc[ta][tb][3], acc2[ta][tb][3], act, limit);
+            if constexpr (kMode != kMoeDown) {
+                if constexpr (kGated) {
+                    v0 = glu_value(acc[ta][tb][0], acc2[ta][tb][0], act, limit);
+                    v1 = glu_value(acc[ta][tb][1], acc2[ta][tb][1], act, limit);
+                    v2 = glu_value(acc[ta][tb][2], acc2[ta][tb][2], act, limit);
+                    v3 = glu_value(acc[ta][tb][3], acc2[ta][tb][3], act, limit);
+                } else {
+                    v0 = plain_act(acc[ta][tb][0] * scale, act);
+                    v1 = plain_act(acc[ta][tb][1] * scale, act);
+                    v2 = plain_act(acc[ta][tb][2] * scale, act);
+                    v3 = plain_act(acc[ta][tb][3] * scale, act);
+                }
                 bf16_t* to = static_cast<bf16_t*>(y) + static_cast<long>(pair) * n + r;
                 if (r + 3 < n && n % 4 == 0) {
                     uint2 packed;
@@ -749,51 +768,56 @@ extern "C" int leone_moe_plan(const int* chosen, int pairs, int experts, int* ti
 }
 
 // gated != 0: x [rows, k], w [experts, 2, n, k], y [pairs, n] of dtype = act(gate) * up (act: GateAct).
-// gated == 0: x [pairs, k], w [experts, n, k], y float32 [pairs, n] = pair_weight[pair] * product.
+// gated == 0: x [pairs, k], w [experts, n, k], y float32 [pairs, n] = pair_weight[pair] * product (null: 1).
+// gated == 2: x [rows, k], w [experts, n, k], y [pairs, n] of dtype = act(pair_weight[pair] * product) (null: 1).
 // tile: pairs a tile holds, as leone_moe_plan was told: leone_moe_tile_pairs() for the kernel that takes any type and
 // size; 16 or 64 for the matrix-core kernel (bfloat16, n and k multiples of 8).
 extern "C" int leone_moe_product(const void* x, const void* w, void* y, const float* pair_weight, int dtype, int gated,
                                  const int* tile_expert, const int* tile_pairs, int max_tiles, int tile, int top, int n, int k,
                                  int act, float limit, hipStream_t stream) {
+    LEONE_REQUIRE(gated >= kMoeDown && gated <= kMoePlain, "moe_product: unknown kind of product %d", gated);
+    LEONE_REQUIRE(act == kGateSilu || act == kGateGeluTanh || (act == kGateClampedSwish && limit > 0.f && gated != kMoePlain) ||
+                      (act == kActReluSquared && gated != kMoeGated),
+                  "moe_product: unknown activation %d (limit %g)", act, limit);
     if (tile != kTilePairs) {
         LEONE_REQUIRE(tile == 16 || tile == 64 || tile == 128, "moe_product: tiles of %d pairs", tile);
         LEONE_REQUIRE(dtype == kBF16 && k % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0,
                       "moe_product: the matrix-core kernel takes bfloat16 with an inner size that is a multiple of 8, not %d", k);
-        LEONE_REQUIRE(x && w && y && tile_expert && tile_pairs && (gated || pair_weight), "moe_product: null pointer");
+        LEONE_REQUIRE(x && w && y && tile_expert && tile_pairs, "moe_product: null pointer");
         LEONE_REQUIRE(max_tiles > 0 && top > 0 && n > 0 && k > 0, "moe_product: %d tiles, sizes %d x %d", max_tiles, n, k);
-        LEONE_REQUIRE(act == kGateSilu || act == kGateGeluTanh || (act == kGateClampedSwish && limit > 0.f), "moe_product: unknown activation %d (limit %g)", act, limit);
         const dim3 cores(max_tiles, ceil_div(n, tile == 128 ? 128 : 64));
         LEONE_REQUIRE(cores.y <= 65535, "moe_product: %d rows of a matrix are too many", n);
 #define LEONE_MOE_CORES(PB, RT, G)                                                                                      \
     moe_product_mfma_kernel<PB, RT, G><<<cores, kMoeThreads, 0, stream>>>(static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(w), \
                                                                           y, pair_weight, tile_expert, tile_pairs, top, n, k, act, limit)
         if (tile == 16) {
-            if (gated) LEONE_MOE_CORES(1, 1, true);
-            else LEONE_MOE_CORES(1, 1, false);
+            if (gated == kMoeGated) LEONE_MOE_CORES(1, 1, kMoeGated);
+            else if (gated == kMoePlain) LEONE_MOE_CORES(1, 1, kMoePlain);
+            else LEONE_MOE_CORES(1, 1, kMoeDown);
         } else if (tile == 64) {
-            if (gated) LEONE_MOE_CORES(4, 1, true);
-            else LEONE_MOE_CORES(4, 1, false);
+            if (gated == kMoeGated) LEONE_MOE_CORES(4, 1, kMoeGated);
+            else if (gated == kMoePlain) LEONE_MOE_CORES(4, 1, kMoePlain);
+            else LEONE_MOE_CORES(4, 1, kMoeDown);
         } else {
             const long places = static_cast<long>(cores.x) * cores.y;
             LEONE_REQUIRE(places + 7 <= 0x7fffffffL, "moe_product: too many tiles");
             const int grid = static_cast<int>((places + 7) / 8 * 8);
-            if (gated)
-                moe_product_tiled_kernel<true><<<grid, kMoeThreads, 0, stream>>>(static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(w),
-                                                                                 y, pair_weight, tile_expert, tile_pairs, top, n, k, act, limit,
-                                                                                 static_cast<int>(cores.x), static_cast<int>(cores.y));
-            else
-                moe_product_tiled_kernel<false><<<grid, kMoeThreads, 0, stream>>>(static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(w),
-                                                                                  y, pair_weight, tile_expert, tile_pairs, top, n, k, act, limit,
-                                                                                  static_cast<int>(cores.x), static_cast<int>(cores.y));
+#define LEONE_MOE_TILED(MODE)                                                                                               \
+    moe_product_tiled_kernel<MODE><<<grid, kMoeThreads, 0, stream>>>(static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(w), \
+                                                                     y, pair_weight, tile_expert, tile_pairs, top, n, k, act, limit, \
+                                                                     static_cast<int>(cores.x), static_cast<int>(cores.y))
+            if (gated == kMoeGated) LEONE_MOE_TILED(kMoeGated);
+            else if (gated == kMoePlain) LEONE_MOE_TILED(kMoePlain);
+            else LEONE_MOE_TILED(kMoeDown);
+#undef LEONE_MOE_TILED
         }
 #undef LEONE_MOE_CORES
         LEONE_LAUNCH_CHECK("moe_product");
         return 0;
     }
     LEONE_REQUIRE(dtype == kF32 || dtype == kBF16, "moe_product: unknown element type %d", dtype);
-    LEONE_REQUIRE(x && w && y && tile_expert && tile_pairs && (gated || pair_weight), "moe_product: null pointer");
+    LEONE_REQUIRE(x && w && y && tile_expert && tile_pairs, "moe_product: null pointer");
     LEONE_REQUIRE(max_tiles > 0 && top > 0 && n > 0 && k > 0, "moe_product: %d tiles, sizes %d x %d", max_tiles, n, k);
-    LEONE_REQUIRE(act == kGateSilu || act == kGateGeluTanh || (act == kGateClampedSwish && limit > 0.f), "moe_product: unknown activation %d (limit %g)", act, limit);
     const uintptr_t run = 8 * (dtype == kF32 ? sizeof(float) : sizeof(bf16_t));
     const int runs = k % 8 == 0 && reinterpret_cast<uintptr_t>(x) % run == 0 && reinterpret_cast<uintptr_t>(w) % run == 0;
     const dim3 grid(max_tiles, ceil_div(n, kMoeCols));
@@ -802,11 +826,13 @@ extern "C" int leone_moe_product(const void* x, const void* w, void* y, const fl
     moe_product_kernel<T, G><<<grid, kMoeThreads, 0, stream>>>(static_cast<const T*>(x), static_cast<const T*>(w), y, pair_weight, \
                                                                tile_expert, tile_pairs, top, n, k, act, limit, runs)
     if (dtype == kF32) {
-        if (gated) LEONE_MOE(float, true);
-        else LEONE_MOE(float, false);
+        if (gated == kMoeGated) LEONE_MOE(float, kMoeGated);
+        else if (gated == kMoePlain) LEONE_MOE(float, kMoePlain);
+        else LEONE_MOE(float, kMoeDown);
     } else {
-        if (gated) LEONE_MOE(bf16_t, true);
-        else LEONE_MOE(bf16_t, false);
+        if (gated == kMoeGated) LEONE_MOE(bf16_t, kMoeGated);
+        else if (gated == kMoePlain) LEONE_MOE(bf16_t, kMoePlain);
+        else LEONE_MOE(bf16_t, kMoeDown);
     }
 #undef LEONE_MOE
     LEONE_LAUNCH_CHECK("moe_product");

@@ -244,6 +244,16 @@ __global__ void rope_table_kernel(float* __restrict__ cos_out, float* __restrict
 constexpr int kMaxPairsPerLane = 4;  // head_dim up to 512
 enum RopePairing : int { kPairHalfSplit = 0, kPairAdjacent = 1 };
 
+// What else may happen to the heads: a bias on the projection (all heads' columns; null: none), value heads that are turned
+// by their own position over their whole size (null tables: none), and heads of which only the first norm_count elements
+// exist (0: all), the rest being zeros that do not count in a norm.
+struct HeadExtras {
+    AnyVec bias;
+    const float* v_cos;
+    const float* v_sin;
+    int v_positions, v_pairing, norm_count;
+};
+
 template <typename TIn, typename T>
 __global__ void qk_norm_rope_write_kernel(
     const TIn* __restrict__ qkv, int planes, long plane, T* __restrict__ q_out, T* __restrict__ k_pool, T* __restrict__ v_pool,
@@ -251,7 +261,7 @@ __global__ void qk_norm_rope_write_kernel(
     const float* __restrict__ sin_table, int table_positions, const int* __restrict__ positions,
     const int* __restrict__ row_entry, const int* __restrict__ block_table, int max_blocks,
     int q_heads, int kv_heads, int head_dim, int page_tokens, int write_cache, int rotary_half, int pairing,
-    int v_dim, long row_width) {
+    int v_dim, long row_width, HeadExtras extra) {
     const int row = blockIdx.x;
     const int head = blockIdx.y * (blockDim.x / kWave) + threadIdx.x / kWave;
     const int lane = threadIdx.x % kWave;
@@ -285,6 +295,11 @@ __global__ void qk_norm_rope_write_kernel(
         return kind == 0 ? d : kind == 1 ? key_offset(token, d, page_tokens) : value_offset(token, d, size);
     };
 
+    const bool turn_values = !is_q && !is_k && extra.v_cos != nullptr;
+    if (turn_values) {                           // the pairs are the values' own, over their whole size
+        rotary_half = half;
+        pairing = extra.v_pairing;
+    }
     // the two elements of pair p
     auto first = [&](int p) { return pairing == kPairHalfSplit && p < rotary_half ? p : 2 * p; };
     auto second = [&](int p) { return pairing == kPairHalfSplit && p < rotary_half ? p + rotary_half : 2 * p + 1; };
@@ -300,6 +315,10 @@ __global__ void qk_norm_rope_write_kernel(
                 a[i] += to_float(src[s * plane + first(p)]);
                 b[i] += to_float(src[s * plane + second(p)]);
             }
+            if (extra.bias.ptr) {
+                a[i] += load_any(extra.bias, head_at + first(p));
+                b[i] += load_any(extra.bias, head_at + second(p));
+            }
             // rounded as a product stored in the outputs' type would be: the same bits whichever way it came
             a[i] = to_float(from_float<T>(a[i]));
             b[i] = to_float(from_float<T>(b[i]));
@@ -307,7 +326,20 @@ __global__ void qk_norm_rope_write_kernel(
             ss = fmaf(b[i], b[i], ss);
         }
     }
-    if (!is_q && !is_k) {  // value head: plain copy
+    if (turn_values) {
+        const long at = static_cast<long>(pos < extra.v_positions ? pos : extra.v_positions - 1) * half;
+#pragma unroll
+        for (int i = 0; i < kMaxPairsPerLane; ++i) {
+            const int p = lane + i * kWave;
+            if (p < half) {
+                const float c = extra.v_cos[at + p], s = extra.v_sin[at + p];
+                const float u = a[i], v = b[i];
+                a[i] = u * c - v * s;
+                b[i] = u * s + v * c;
+            }
+        }
+    }
+    if (!is_q && !is_k) {  // value head: copied
 #pragma unroll
         for (int i = 0; i < kMaxPairsPerLane; ++i) {
             const int p = lane + i * kWave;
@@ -322,7 +354,7 @@ __global__ void qk_norm_rope_write_kernel(
     float inv = 1.f;
     if (gain.ptr) {
         ss = wave_sum(ss);
-        inv = 1.0f / sqrtf(ss / static_cast<float>(head_dim) + eps);
+        inv = 1.0f / sqrtf(ss / static_cast<float>(extra.norm_count > 0 ? extra.norm_count : head_dim) + eps);
     }
     const bool rotate = cos_table != nullptr;
     const int tpos = pos < table_positions ? pos : table_positions - 1;  // host checks the bound
@@ -732,6 +764,27 @@ extern "C" int leone_qk_norm_rope_write(const void* qkv, int qkv_dtype, int qkv_
                                         const int* positions, const int* row_entry, const int* block_table,
                                         int max_blocks, int rows, int q_heads, int kv_heads, int head_dim,
                                         int page_tokens, int write_cache, int v_dim, long row_width, hipStream_t stream) {
+    return leone_qk_norm_rope_write_turned(qkv, qkv_dtype, qkv_planes, qkv_plane, q_out, k_pool, v_pool, dtype, q_gain, k_gain,
+                                           gain_dtype, eps, cos_table, sin_table, table_positions, rotary_dim, pairing, positions,
+                                           row_entry, block_table, max_blocks, rows, q_heads, kv_heads, head_dim, page_tokens,
+                                           write_cache, v_dim, row_width, nullptr, kF32, nullptr, nullptr, 0, 0, 0, stream);
+}
+
+extern "C" int leone_qk_norm_rope_write_turned(const void* qkv, int qkv_dtype, int qkv_planes, long qkv_plane, void* q_out,
+                                               void* k_pool, void* v_pool, int dtype, const void* q_gain, const void* k_gain,
+                                               int gain_dtype, float eps, const float* cos_table, const float* sin_table,
+                                               int table_positions, int rotary_dim, int pairing, const int* positions,
+                                               const int* row_entry, const int* block_table, int max_blocks, int rows,
+                                               int q_heads, int kv_heads, int head_dim, int page_tokens, int write_cache,
+                                               int v_dim, long row_width, const void* bias, int bias_dtype, const float* v_cos,
+                                               const float* v_sin, int v_positions, int v_pairing, int norm_count,
+                                               hipStream_t stream) {
+    const HeadExtras extra{AnyVec{bias, bias_dtype}, v_cos, v_sin, v_positions, v_pairing, norm_count};
+    const bool plain = !bias && !v_cos && norm_count <= 0;
+    LEONE_REQUIRE(!bias || bias_dtype == kF32 || bias_dtype == kBF16, "qk_norm_rope_write: unknown type of the bias");
+    LEONE_REQUIRE((v_cos == nullptr) == (v_sin == nullptr) && (!v_cos || v_positions > 0) && norm_count <= head_dim &&
+                      (v_pairing == kPairHalfSplit || v_pairing == kPairAdjacent),
+                  "qk_norm_rope_write: the values' rotation needs two tables and a known pairing, a norm at most the head's elements");
     if (v_dim <= 0) v_dim = head_dim;
     const long heads_width = static_cast<long>(q_heads + kv_heads) * head_dim + static_cast<long>(kv_heads) * v_dim;
     if (row_width <= 0) row_width = heads_width;
@@ -770,7 +823,7 @@ extern "C" int leone_qk_norm_rope_write(const void* qkv, int qkv_dtype, int qkv_
                          (!write_cache || (reinterpret_cast<uintptr_t>(k_pool) % run_bytes == 0 && page_tokens % 8 == 0));
     const bool tables_aligned = (!q_gain || (reinterpret_cast<uintptr_t>(q_gain) % 32 == 0 && reinterpret_cast<uintptr_t>(k_gain) % 32 == 0)) &&
                                 (!cos_table || (reinterpret_cast<uintptr_t>(cos_table) % 32 == 0 && reinterpret_cast<uintptr_t>(sin_table) % 32 == 0));
-    if (whole_head && v_dim == head_dim && row_width == heads_width && head_dim % 16 == 0 && head_dim <= 128 && aligned && tables_aligned && static_cast<long>(rows) * (q_heads + 2 * kv_heads) * 8 < 0x7fffffffL * 256) {
+    if (plain && whole_head && v_dim == head_dim && row_width == heads_width && head_dim % 16 == 0 && head_dim <= 128 && aligned && tables_aligned && static_cast<long>(rows) * (q_heads + 2 * kv_heads) * 8 < 0x7fffffffL * 256) {
 #define LEONE_RUNS_ARGS                                                                                             \
     qkv, qkv_planes, qkv_plane, q_out, k_pool, v_pool, qg, kg, eps, cos_table, sin_table, table_positions, positions, \
         row_entry, block_table, max_blocks, rows, q_heads, kv_heads, page_tokens, write_cache, stream
@@ -797,7 +850,7 @@ extern "C" int leone_qk_norm_rope_write(const void* qkv, int qkv_dtype, int qkv_
         static_cast<const TIN*>(qkv), qkv_planes, qkv_plane, static_cast<T*>(q_out), static_cast<T*>(k_pool),       \
         static_cast<T*>(v_pool), qg, kg, eps, cos_table, sin_table, table_positions, positions, row_entry,          \
         block_table, max_blocks, q_heads, kv_heads, head_dim, page_tokens, write_cache, cos_table ? rotary_dim / 2 : 0, pairing, \
-        v_dim, row_width)
+        v_dim, row_width, extra)
     if (dtype == kF32) LEONE_QK_ANY(float, float);
     else if (qkv_dtype == kF32) LEONE_QK_ANY(float, bf16_t);
     else LEONE_QK_ANY(bf16_t, bf16_t);

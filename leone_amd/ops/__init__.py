@@ -234,14 +234,18 @@ def qk_norm_rope_write(qkv: torch.Tensor, q_heads: int, kv_heads: int, head_dim:
                        k_pool: Optional[torch.Tensor], v_pool: Optional[torch.Tensor], write_cache: bool = True,
                        out: Optional[torch.Tensor] = None, out_dtype: Optional[torch.dtype] = None,
                        pairing: str = "half_split", value_dim: Optional[int] = None,
-                       queries_only: bool = False) -> torch.Tensor:
+                       queries_only: bool = False, bias: Optional[torch.Tensor] = None,
+                       value_rotation: Optional[tuple] = None, norm_count: int = 0) -> torch.Tensor:
     """Splits the fused projection, normalises and rotates q and k heads, writes k and v into the cache.
     ``qkv`` is ``[rows, width]`` of the cache's type, or float32 (also as planes ``[p, rows, width]`` whose
     sum, in order, is meant: a product cut along K) with ``out_dtype`` naming the type of q and the cache.
     The rotation's shape comes with its tables (``_rotation_shape``): their width says how much of a head is
     rotated, ``pairing`` which elements go together.  ``value_dim``: the value heads' own size (then a row may
     also hold further columns behind the heads, which are left alone).  ``queries_only``: the rows hold the query
-    heads (and perhaps further columns) but no key and value heads: a layer that reads another layer's cache."""
+    heads (and perhaps further columns) but no key and value heads: a layer that reads another layer's cache.
+    ``bias`` (a vector over all heads' columns) is added first.  ``value_rotation`` = (cos, sin, pairing): value heads
+    are turned by their own position over their whole size before they are cached.  ``norm_count``: only so many
+    elements of a head exist (the rest are zeros that do not count in the heads' norms; 0: all)."""
     planes = qkv.shape[0] if qkv.dim() == 3 else 1
     rows, width = qkv.shape[-2:]
     kind = out_dtype or qkv.dtype
@@ -270,7 +274,18 @@ def qk_norm_rope_write(qkv: torch.Tensor, q_heads: int, kv_heads: int, head_dim:
     gain_code = _code(q_gain, "q gain") if q_gain is not None else F32
     if q_gain is not None and (k_gain is None or k_gain.dtype != q_gain.dtype):
         raise KernelError("qk_norm_rope_write: q and k gains must come together in one type")
-    call("leone_qk_norm_rope_write", _dev(qkv, "qkv"), _code(qkv, "qkv"), planes, rows * width,
+    v_cos = v_sin = None
+    v_positions = v_pairing = 0
+    if value_rotation is not None:
+        v_cos, v_sin = value_rotation[:2]
+        v_positions, v_dims, v_pairing = _rotation_shape("qk_norm_rope_write values", value_dim, v_cos, v_sin, value_rotation[2])
+        if v_dims != value_dim:
+            raise KernelError(f"qk_norm_rope_write: values of {value_dim} elements are turned whole, the tables cover {v_dims}")
+    if not 0 <= norm_count <= head_dim:
+        raise KernelError(f"qk_norm_rope_write: {norm_count} of {head_dim} elements in a head's norm")
+    if bias is not None and bias.numel() != (q_heads * head_dim if queries_only else heads_width):
+        raise KernelError(f"qk_norm_rope_write: a bias of {bias.numel()} for heads of {heads_width} columns")
+    call("leone_qk_norm_rope_write_turned", _dev(qkv, "qkv"), _code(qkv, "qkv"), planes, rows * width,
          _dev(out, "q out", kind),
          _dev(k_pool if write_cache else None, "k pool", kind),
          _dev(v_pool if write_cache else None, "v pool", kind), _CODES[kind],
@@ -279,8 +294,31 @@ def qk_norm_rope_write(qkv: torch.Tensor, q_heads: int, kv_heads: int, head_dim:
          rotary_dim, pairing_code, _dev(positions, "positions", torch.int32, (rows,)),
          _dev(row_entry if write_cache else None, "row map", torch.int32, (rows,)),
          _dev(block_table if write_cache else None, "block table", torch.int32), max_blocks, rows, q_heads,
-         kv_heads, head_dim, page_tokens, 1 if write_cache else 0, value_dim, width, _stream())
+         kv_heads, head_dim, page_tokens, 1 if write_cache else 0, value_dim, width, _dev(bias, "bias"),
+         _code(bias, "bias") if bias is not None else F32, _dev(v_cos, "value cos", torch.float32),
+         _dev(v_sin, "value sin", torch.float32), v_positions, v_pairing, int(norm_count), _stream())
     return out
+
+
+class ScoreShape:
+    """What an attention does to its scores and results beside the mask: ``cap`` (scaled scores become cap * tanh(score /
+    cap)), ``sinks`` (float32 ``[q_heads]``: exp(sinks[h]) stands in the denominator and weighs no value) and ``turn`` =
+    (cos, sin, pairing): the cached values were turned by their positions, a row's results are turned back by its own
+    (tables float32 ``[positions, value size / 2]``)."""
+
+    def __init__(self, cap: Optional[float] = None, sinks: Optional[torch.Tensor] = None, turn: Optional[tuple] = None):
+        self.cap, self.sinks, self.turn = float(cap or 0.0), sinks, turn
+
+    def args(self, q_heads: int, value_dim: int) -> tuple:
+        cos, sin, pairing = self.turn if self.turn is not None else (None, None, "half_split")
+        positions, dims, code = _rotation_shape("attention results", value_dim, cos, sin, pairing)
+        if cos is not None and dims != value_dim:
+            raise KernelError(f"attention: results of {value_dim} elements are turned back whole, the tables cover {dims}")
+        return (self.cap, _dev(self.sinks, "sinks", torch.float32, (q_heads,)), _dev(cos, "turn cos", torch.float32),
+                _dev(sin, "turn sin", torch.float32), positions, code)
+
+
+_PLAIN_SCORES = ScoreShape()
 
 
 def _strided_rows(t: Optional[torch.Tensor], what: str, rows: int, columns: int, dtype=torch.float32):
@@ -298,14 +336,15 @@ def attention_rows(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, 
                    row_entry: torch.Tensor, block_table: torch.Tensor, q_heads: int, scale: float,
                    window: int = 0, out: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
                    keep_first: int = 0, gate_each: bool = False, slopes: Optional[torch.Tensor] = None,
-                   query_factor: Optional[tuple] = None) -> torch.Tensor:
+                   query_factor: Optional[tuple] = None, shape: Optional[ScoreShape] = None) -> torch.Tensor:
     """Each query row attends its request's cached keys up to its own position (the last ``window`` of them,
     and, whatever the window, those at positions below ``keep_first``).  The result has the values'
     size a head.  ``slopes`` float32 ``[q_heads]``: head h's score for the key at distance d is lowered by
     slopes[h] * d.  ``query_factor`` = (coef, every): the queries of a row at position p count times
     1 + coef * ln(floor((p + 1) / every) + 1).  ``gate``: float32 ``[rows, >= q_heads]`` (a view into a wider row is fine, unit stride along the
     heads): head h of row r is multiplied by sigmoid(gate[r, h]); with ``gate_each`` the gate holds a value for
-    every element of the result, ``[rows, >= q_heads * value_dim]``."""
+    every element of the result, ``[rows, >= q_heads * value_dim]``.  ``shape``: capped scores, sinks, results turned
+    back (``ScoreShape``; results are turned back before the gate)."""
     rows = q.shape[0]
     pages, kv_heads, page_tokens, head_dim, value_dim = cache_dims_kv(k_pool, v_pool)
     if q.shape[1] != q_heads * head_dim:
@@ -314,13 +353,32 @@ def attention_rows(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, 
         out = torch.empty((rows, q_heads * value_dim), dtype=q.dtype, device=q.device)
     gate_at, gate_stride = _strided_rows(gate, "attention gate", rows, q_heads * value_dim if gate_each else q_heads)
     coef, every = query_factor if query_factor is not None else (0.0, 0)
-    call("leone_attention_rows_biased", _dev(q, "attention q"), _dev(out, "attention out", q.dtype, (rows, q_heads * value_dim)),
+    call("leone_attention_rows_shaped", _dev(q, "attention q"), _dev(out, "attention out", q.dtype, (rows, q_heads * value_dim)),
          _dev(k_pool, "k pool", q.dtype), _dev(v_pool, "v pool", q.dtype), _code(q, "attention q"),
          _dev(positions, "positions", torch.int32, (rows,)), _dev(row_entry, "row map", torch.int32, (rows,)),
          _dev(block_table, "block table", torch.int32), block_table.shape[1], rows, q_heads, kv_heads, head_dim,
          value_dim, page_tokens, float(scale), int(window), gate_at, gate_stride, int(keep_first),
          1 if (gate_each and gate is not None) else 0, _dev(slopes, "slopes", torch.float32, (q_heads,)), float(coef),
-         int(every), _stream())
+         int(every), *(shape or _PLAIN_SCORES).args(q_heads, value_dim), _stream())
+    return out
+
+
+def attention_rows_talk(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, talk: torch.Tensor, positions: torch.Tensor,
+                        row_entry: torch.Tensor, block_table: torch.Tensor, q_heads: int, scale: float, window: int = 0,
+                        out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``attention_rows`` whose heads' scaled scores are mixed before the softmax: score_h <- sum_g talk[h, g] score_g over
+    all query heads g (``talk`` ``[q_heads, q_heads]``).  Any type and size."""
+    rows = q.shape[0]
+    pages, kv_heads, page_tokens, head_dim, value_dim = cache_dims_kv(k_pool, v_pool)
+    if q.shape[1] != q_heads * head_dim:
+        raise KernelError(f"attention: query width {q.shape[1]} is not {q_heads}*{head_dim}")
+    if out is None:
+        out = torch.empty((rows, q_heads * value_dim), dtype=q.dtype, device=q.device)
+    call("leone_attention_rows_talk", _dev(q, "attention q"), _dev(out, "attention out", q.dtype, (rows, q_heads * value_dim)),
+         _dev(k_pool, "k pool", q.dtype), _dev(v_pool, "v pool", q.dtype), _code(q, "attention q"),
+         _dev(talk, "talk", None, (q_heads, q_heads)), _code(talk, "talk"), _dev(positions, "positions", torch.int32, (rows,)),
+         _dev(row_entry, "row map", torch.int32, (rows,)), _dev(block_table, "block table", torch.int32), block_table.shape[1],
+         rows, q_heads, kv_heads, head_dim, value_dim, page_tokens, float(scale), int(window), _stream())
     return out
 
 
@@ -357,10 +415,11 @@ def attention_decode(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor
                      row_entry: torch.Tensor, block_table: torch.Tensor, q_heads: int, scale: float,
                      window: int = 0, max_context: int = 1, splits: Optional[int] = None,
                      out: Optional[torch.Tensor] = None, keep_first: int = 0, slopes: Optional[torch.Tensor] = None,
-                     query_factor: Optional[tuple] = None) -> torch.Tensor:
+                     query_factor: Optional[tuple] = None, shape: Optional[ScoreShape] = None) -> torch.Tensor:
     """Split-KV attention on the matrix cores (bfloat16).  ``max_context`` only steers the number of splits.
     ``keep_first``: keys at positions below it stay in sight of a windowed layer.  ``slopes`` and ``query_factor``
-    as for ``attention_rows``: scores that fall with the distance, queries that count more the further on they stand."""
+    as for ``attention_rows``: scores that fall with the distance, queries that count more the further on they stand.
+    ``shape``: capped scores, sinks, results turned back."""
     rows = q.shape[0]
     pages, kv_heads, page_tokens, head_dim = cache_dims(k_pool, v_pool)
     if q.shape[1] != q_heads * head_dim:
@@ -375,13 +434,14 @@ def attention_decode(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor
         part_acc = torch.empty((rows * q_heads * splits * head_dim,), dtype=torch.float32, device=q.device)
         part_ml = torch.empty((rows * q_heads * splits * 2,), dtype=torch.float32, device=q.device)
     coef, every = query_factor if query_factor is not None else (0.0, 0)
-    call("leone_attention_decode_biased", _dev(q, "attention q", torch.bfloat16),
+    call("leone_attention_decode_shaped", _dev(q, "attention q", torch.bfloat16),
          _dev(out, "attention out", torch.bfloat16, q.shape), _dev(k_pool, "k pool", torch.bfloat16),
          _dev(v_pool, "v pool", torch.bfloat16), _dev(positions, "positions", torch.int32, (rows,)),
          _dev(row_entry, "row map", torch.int32, (rows,)), _dev(block_table, "block table", torch.int32),
          block_table.shape[1], _dev(part_acc, "partials"), _dev(part_ml, "partial sums"), rows, q_heads, kv_heads,
          head_dim, page_tokens, float(scale), int(window), int(splits), int(keep_first) if window else 0,
-         _dev(slopes, "slopes", torch.float32, (q_heads,)), float(coef), int(every), _stream())
+         _dev(slopes, "slopes", torch.float32, (q_heads,)), float(coef), int(every),
+         *(shape or _PLAIN_SCORES).args(q_heads, head_dim), _stream())
     return out
 
 
@@ -471,9 +531,9 @@ def attention_prefill(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, 
                       positions: torch.Tensor, tiles: torch.Tensor, block_table: torch.Tensor, q_heads: int,
                       scale: float, window: int = 0, mean_keys: int = 1, splits: Optional[int] = None,
                       covered_rows: Optional[int] = None, keep_first: int = 0, slopes: Optional[torch.Tensor] = None,
-                      query_factor: Optional[tuple] = None) -> torch.Tensor:
-    """Attention for the rows that ``tiles`` covers; writes into ``out``.  ``slopes`` and ``query_factor`` as for
-    ``attention_rows``.
+                      query_factor: Optional[tuple] = None, shape: Optional[ScoreShape] = None) -> torch.Tensor:
+    """Attention for the rows that ``tiles`` covers; writes into ``out``.  ``slopes``, ``query_factor`` and
+    ``shape`` as for ``attention_rows``.
 
     ``tiles`` is int32 [n, 3]: (entry, first row, rows) with at most PREFILL_TILE_ROWS consecutive rows of one
     request each, PREFILL_GROUP_TILES to a group, all tiles of a group of the same entry, unused places with
@@ -505,13 +565,14 @@ def attention_prefill(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, 
         part_acc = torch.empty((covered * q_heads * splits * head_dim,), dtype=torch.float32, device=q.device)
         part_ml = torch.empty((covered * q_heads * splits * 2,), dtype=torch.float32, device=q.device)
     coef, every = query_factor if query_factor is not None else (0.0, 0)
-    call("leone_attention_prefill_biased", _dev(q, "attention q", torch.bfloat16),
+    call("leone_attention_prefill_shaped", _dev(q, "attention q", torch.bfloat16),
          _dev(out, "attention out", torch.bfloat16, q.shape), _dev(k_pool, "k pool", torch.bfloat16),
          _dev(v_pool, "v pool", torch.bfloat16), _dev(positions, "positions", torch.int32, (rows,)),
          _dev(tiles, "tiles", torch.int32), groups, _dev(block_table, "block table", torch.int32),
          block_table.shape[1], q_heads, kv_heads, head_dim, page_tokens, float(scale), int(window),
          _dev(part_acc, "partials"), _dev(part_ml, "partial sums"), int(splits), keep_first,
-         _dev(slopes, "slopes", torch.float32, (q_heads,)), float(coef), int(every), _stream())
+         _dev(slopes, "slopes", torch.float32, (q_heads,)), float(coef), int(every),
+         *(shape or _PLAIN_SCORES).args(q_heads, head_dim), _stream())
     return out
 
 
@@ -1540,7 +1601,8 @@ def add_normed(x: torch.Tensor, delta: Optional[torch.Tensor], gain: Optional[to
 
 ROUTER_SCORES = {"softmax": 0, "sigmoid": 1}     # how a router turns its logits into scores
 # what experts put on gate and up: a gate activation, or "clamped_swish" (gate and up held to a limit, see ``glu_value``)
-EXPERT_ACTIVATIONS = {**GATE_ACTIVATIONS, "clamped_swish": 2}
+EXPERT_ACTIVATIONS = {**GATE_ACTIVATIONS, "clamped_swish": 2}      # of experts with a gate
+PLAIN_ACTIVATIONS = {**GATE_ACTIVATIONS, "relu2": 3}                # of experts without one
 
 
 class RouterRule:
@@ -1563,11 +1625,12 @@ class RouterRule:
 _DEFAULT_RULE = RouterRule()
 
 
-def _expert_act(activation: str, limit: Optional[float]) -> tuple:
+def _expert_act(activation: str, limit: Optional[float], gated: bool = True) -> tuple:
+    known = EXPERT_ACTIVATIONS if gated else PLAIN_ACTIVATIONS
     try:
-        code = EXPERT_ACTIVATIONS[activation]
+        code = known[activation]
     except KeyError:
-        raise KernelError(f"unknown expert activation {activation!r}; known: {', '.join(EXPERT_ACTIVATIONS)}") from None
+        raise KernelError(f"unknown expert activation {activation!r}; known: {', '.join(known)}") from None
     if code == 2 and not (limit is not None and limit > 0.0):
         raise KernelError(f"the clamped activation needs a positive limit, found {limit!r}")
     return code, float(limit or 0.0)
@@ -1610,32 +1673,39 @@ def _expert_tiles(x: torch.Tensor, rows: int, top: int, experts: int, hidden: in
             torch.empty((max_tiles, tile), dtype=torch.int32, device=x.device))
 
 
-def _check_experts(x: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor):
+def _check_experts(x: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor):
+    """(rows, hidden, experts, ff, whether the experts have a gate)."""
     rows, hidden = x.shape
-    experts, two, ff, k = w_gate_up.shape
-    if two != 2 or k != hidden or tuple(w_down.shape) != (experts, hidden, ff) or w_gate_up.dtype != x.dtype or w_down.dtype != x.dtype:
-        raise KernelError(f"routed experts: matrices {tuple(w_gate_up.shape)} and {tuple(w_down.shape)} of {w_gate_up.dtype} "
+    gated = w_up.dim() == 4
+    experts, ff, k = w_up.shape[0], w_up.shape[-2], w_up.shape[-1]
+    if w_up.dim() not in (3, 4) or (gated and w_up.shape[1] != 2) or k != hidden or tuple(w_down.shape) != (experts, hidden, ff) \
+            or w_up.dtype != x.dtype or w_down.dtype != x.dtype:
+        raise KernelError(f"routed experts: matrices {tuple(w_up.shape)} and {tuple(w_down.shape)} of {w_up.dtype} "
                           f"do not fit rows {tuple(x.shape)} of {x.dtype}")
-    return rows, hidden, experts, ff
+    return rows, hidden, experts, ff, gated
 
 
-def _expert_products(x, chosen, weight, tiles, w_gate_up, w_down, activation, extra, limit=None) -> torch.Tensor:
-    rows, hidden, experts, ff = _check_experts(x, w_gate_up, w_down)
-    act, limit = _expert_act(activation, limit)
+def _expert_products(x, chosen, weight, tiles, w_up, w_down, activation, extra, limit=None, weigh_input=False) -> torch.Tensor:
+    rows, hidden, experts, ff, gated = _check_experts(x, w_up, w_down)
+    if weigh_input and gated:
+        raise KernelError("routed experts: a weight on what an expert reads goes with experts without a gate")
+    act, limit = _expert_act(activation, limit, gated)
     top = chosen.shape[1]
     pairs = rows * top
     tile, max_tiles, tile_expert, tile_pairs = tiles
     device = x.device
+    weights = _dev(weight, "weights", torch.float32, (rows, top))
     hidden_act = torch.empty((pairs, ff), dtype=x.dtype, device=device)
-    call("leone_moe_product", _dev(x, "routed rows"), _dev(w_gate_up, "expert gate/up"), _dev(hidden_act, "expert hidden"), 0,
-         _code(x, "routed rows"), 1, _dev(tile_expert, "tiles"), _dev(tile_pairs, "tile pairs"), max_tiles, tile, top, ff, hidden,
-         act, limit, _stream())
+    # the weight stands on the input's side (a product of weight * x is weight times the product) or on the result's
+    call("leone_moe_product", _dev(x, "routed rows"), _dev(w_up, "expert up"), _dev(hidden_act, "expert hidden"),
+         weights if weigh_input else 0, _code(x, "routed rows"), 1 if gated else 2, _dev(tile_expert, "tiles"),
+         _dev(tile_pairs, "tile pairs"), max_tiles, tile, top, ff, hidden, act, limit, _stream())
     pair_out = torch.empty((pairs, hidden), dtype=torch.float32, device=device)
     call("leone_moe_product", _dev(hidden_act, "expert hidden"), _dev(w_down, "expert down"), _dev(pair_out, "pair results"),
-         _dev(weight, "weights", torch.float32, (rows, top)), _code(x, "routed rows"), 0, _dev(tile_expert, "tiles"),
+         0 if weigh_input else weights, _code(x, "routed rows"), 0, _dev(tile_expert, "tiles"),
          _dev(tile_pairs, "tile pairs"), max_tiles, tile, top, hidden, ff, 0, 0.0, _stream())
     out = torch.empty((rows, hidden), dtype=torch.float32, device=device)
-    call("leone_moe_combine", _dev(pair_out, "pair results"), _dev(chosen, "chosen"), _dev(weight, "weights"),
+    call("leone_moe_combine", _dev(pair_out, "pair results"), _dev(chosen, "chosen"), weights,
          _dev(x, "routed rows"), _code(x, "routed rows"), _dev(extra, "extra", torch.float32, (rows, hidden)),
          _dev(out, "routed out"), rows, top, experts, hidden, _stream())
     return out
@@ -1643,35 +1713,37 @@ def _expert_products(x, chosen, weight, tiles, w_gate_up, w_down, activation, ex
 
 def routed_experts(x: torch.Tensor, chosen: torch.Tensor, weight: torch.Tensor, w_gate_up: torch.Tensor,
                    w_down: torch.Tensor, activation: str = "silu", extra: Optional[torch.Tensor] = None,
-                   limit: Optional[float] = None) -> torch.Tensor:
+                   limit: Optional[float] = None, weigh_input: bool = False) -> torch.Tensor:
     """Every row through the experts chosen for it: float32 ``[rows, hidden]`` = sum over a row's places of
     weight * W_down[e] (act(W_gate[e] x) * (W_up[e] x)), in the places' order; a chosen index from the number of
     experts on stands for an expert that hands the row on as it is; ``extra`` (float32 ``[rows, hidden]``) is added.
     ``w_gate_up`` is ``[experts, 2, ff, hidden]`` (gate rows, then up rows), ``w_down`` ``[experts, hidden, ff]``, both
-    of ``x``'s type.  Nothing here depends on the choice except through device arrays."""
-    rows, hidden, experts, ff = _check_experts(x, w_gate_up, w_down)
+    of ``x``'s type; experts without a gate come as ``[experts, ff, hidden]`` and compute W_down[e] act(W_up[e] x)
+    (``PLAIN_ACTIVATIONS``).  ``weigh_input`` (experts without a gate): the weight multiplies what the expert reads
+    instead of what it gives.  Nothing here depends on the choice except through device arrays."""
+    rows, hidden, experts, ff, _ = _check_experts(x, w_gate_up, w_down)
     top = chosen.shape[1]
     tiles = _expert_tiles(x, rows, top, experts, hidden, ff)
     call("leone_moe_plan", _dev(chosen, "chosen", torch.int32, (rows, top)), rows * top, experts, _dev(tiles[2], "tiles"),
          _dev(tiles[3], "tile pairs"), tiles[1], tiles[0], _stream())
-    return _expert_products(x, chosen, weight, tiles, w_gate_up, w_down, activation, extra, limit)
+    return _expert_products(x, chosen, weight, tiles, w_gate_up, w_down, activation, extra, limit, weigh_input)
 
 
 def routed_feed_forward(x: torch.Tensor, logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, group_count: int,
                         group_keep: int, w_gate_up: torch.Tensor, w_down: torch.Tensor, activation: str = "silu",
                         extra: Optional[torch.Tensor] = None, always: int = 0, rule: Optional[RouterRule] = None,
-                        limit: Optional[float] = None) -> torch.Tensor:
+                        limit: Optional[float] = None, weigh_input: bool = False) -> torch.Tensor:
     """``route_topk`` on the router's float32 ``logits`` and ``routed_experts`` with its choice; for steps of few rows
     (up to ``ROUTE_PLAN_ROWS``) the choice and the tiles are made in one launch.  ``always`` (such steps only): the
     last so many experts of the matrices are no choice of the router's but taken by every row with weight 1 (a
     shared expert cut to the experts' size rides along in the experts' launches)."""
-    rows, hidden, experts, ff = _check_experts(x, w_gate_up, w_down)
+    rows, hidden, experts, ff, _ = _check_experts(x, w_gate_up, w_down)
     total = logits.shape[1]
     if rows > ROUTE_PLAN_ROWS:
         if always:
             raise KernelError(f"routed_feed_forward: experts for every row ride along in steps of up to {ROUTE_PLAN_ROWS} rows only")
         chosen, weight = route_topk(logits, correction, top, group_count, group_keep, rule)
-        return routed_experts(x, chosen, weight, w_gate_up, w_down, activation, extra, limit)
+        return routed_experts(x, chosen, weight, w_gate_up, w_down, activation, extra, limit, weigh_input)
     if total > library().leone_route_max_outputs():
         raise KernelError(f"route_topk: {total} router outputs, the kernel takes {library().leone_route_max_outputs()}")
     if not 0 <= always < experts:
@@ -1685,7 +1757,7 @@ def routed_feed_forward(x: torch.Tensor, logits: torch.Tensor, correction: Optio
          _dev(chosen, "chosen"), _dev(weight, "weights"), rows, total, int(top), int(group_count), int(group_keep), experts,
          _dev(tiles[2], "tiles"), _dev(tiles[3], "tile pairs"), tiles[1], tiles[0], int(always),
          *(rule or _DEFAULT_RULE).args(), _stream())
-    return _expert_products(x, chosen, weight, tiles, w_gate_up, w_down, activation, extra, limit)
+    return _expert_products(x, chosen, weight, tiles, w_gate_up, w_down, activation, extra, limit, weigh_input)
 
 
 # ---- a forget gate per key channel, attention through a shared latent, the stream as a sum over depth -----------
@@ -1707,9 +1779,7 @@ def gated_scan(proj: torch.Tensor, columns: dict, f_bias: torch.Tensor, lower: t
         raise KernelError("gated_scan: the gates' bias and lower bound must share one type")
     if q_activation not in (None, "silu"):
         raise KernelError(f"gated_scan: queries pass as they are or through silu, not {q_activation!r}")
-    spans = entry_spans(step)
-    device = proj.device
-    out = torch.empty((rows, heads * vdim), dtype=torch.float32, device=device)
+    out = torch.empty((rows, heads * vdim), dtype=torch.float32, device=proj.device)
 
     def walk(segments, state_in, state_out, no_input=False, accumulate=False, product=None):
         call("leone_gated_scan", _dev(proj, "projection", torch.float32), width, columns["q"], columns["f"], columns["v"],
@@ -1720,20 +1790,7 @@ def gated_scan(proj: torch.Tensor, columns: dict, f_bias: torch.Tensor, lower: t
              _dev(state_out, "state written"), state_out.stride(0) if state_out is not None else 0,
              _dev(product, "gate products"), _dev(out, "out"), heads, dim, vdim, _stream())
 
-    plan = chunk_plan(step, *GATED_CHUNKS)
-    if plan is None:
-        walk(spans, state, state if write_state else None)
-    else:
-        chunks = plan["chunks"]
-        work = torch.empty((chunks.shape[0], heads, dim * vdim), dtype=torch.float32, device=device)
-        product = torch.empty((chunks.shape[0], heads, dim), dtype=torch.float32, device=device)
-        walk(chunks, None, work, product=product)
-        call("leone_gated_chain", _dev(plan["links"], "links", torch.int32), plan["links"].shape[0], _dev(work, "work"),
-             work.stride(0), _dev(product, "gate products"), _dev(state, "state"), state.stride(0), heads, dim, vdim,
-             1 if write_state else 0, _stream())
-        walk(plan["again"], work, None, no_input=True, accumulate=True)
-        if plan["short"].shape[0]:
-            walk(plan["short"], state, state if write_state else None)
+    _walk_rows(step, walk, state, heads, dim, vdim, write_state)
     return out
 
 
@@ -1755,9 +1812,7 @@ def state_space_scan(xbc: torch.Tensor, columns: dict, groups: int, step_size: t
     if groups <= 0 or heads % groups:
         raise KernelError(f"state_space_scan: {heads} heads do not share {groups} groups evenly")
     step_at, step_stride = _strided_rows(step_size, "step sizes", rows, heads)
-    spans = entry_spans(step)
-    device = xbc.device
-    out = torch.empty((rows, heads * vdim), dtype=torch.float32, device=device)
+    out = torch.empty((rows, heads * vdim), dtype=torch.float32, device=xbc.device)
 
     def walk(segments, state_in, state_out, no_input=False, accumulate=False, product=None):
         call("leone_state_space_scan", _dev(xbc, "x, B and C", torch.float32), width, columns["x"], columns["b"], columns["c"],
@@ -1769,21 +1824,87 @@ def state_space_scan(xbc: torch.Tensor, columns: dict, groups: int, step_size: t
              _dev(state_out, "state written"), state_out.stride(0) if state_out is not None else 0,
              _dev(product, "decay products"), _dev(out, "out"), heads, dim, vdim, _stream())
 
+    _walk_rows(step, walk, state, heads, dim, vdim, write_state)
+    return out
+
+
+def time_mix_scan(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, bonus: torch.Tensor,
+                  state: torch.Tensor, step, heads: int, dim: int, vdim: int, write_state: bool = True) -> torch.Tensor:
+    """A matrix memory with ready-made decays over every entry's rows: per head o_t = (S + diag(bonus) k_t v_t^T)^T r_t,
+    then S <- diag(decay_t) S + k_t v_t^T.  ``r``, ``k`` (``heads * dim`` columns) and ``v`` (``heads * vdim``) are float32
+    rows, possibly slices of wider rows, all with one distance from row to row; ``decay`` float32 ``[rows, heads * dim]``;
+    ``bonus`` ``[heads * dim]``; ``state`` float32 ``[slots, heads, dim * vdim]``.  Returns o float32 ``[rows, heads * vdim]``.
+    Long portions are walked in chunks side by side, as in ``gated_scan``, chained by the product of the chunk's decays."""
+    rows = r.shape[0]
+    if state.dtype != torch.float32 or state.dim() != 3 or tuple(state.shape[1:]) != (heads, dim * vdim) or not state.is_contiguous():
+        raise KernelError(f"time_mix_scan: state {tuple(state.shape)} is not [slots, {heads}, {dim * vdim}] float32")
+    r_at, stride = _strided_rows(r, "r", rows, heads * dim)
+    k_at, k_stride = _strided_rows(k, "k", rows, heads * dim)
+    v_at, v_stride = _strided_rows(v, "v", rows, heads * vdim)
+    if not stride == k_stride == v_stride:
+        raise KernelError(f"time_mix_scan: r, k and v lie {stride}, {k_stride} and {v_stride} elements apart from row to row")
+    out = torch.empty((rows, heads * vdim), dtype=torch.float32, device=r.device)
+
+    def walk(segments, state_in, state_out, no_input=False, accumulate=False, product=None):
+        call("leone_time_mix_scan", r_at, k_at, v_at, stride, _dev(decay, "decays", torch.float32, (rows, heads * dim)),
+             _dev(bonus, "bonus", None, (heads * dim,)), _code(bonus, "bonus"), 1 if no_input else 0, 1 if accumulate else 0,
+             _dev(segments, "segments", torch.int32), segments.shape[0],
+             _dev(state_in, "state read"), state_in.stride(0) if state_in is not None else 0,
+             _dev(state_out, "state written"), state_out.stride(0) if state_out is not None else 0,
+             _dev(product, "decay products"), _dev(out, "out"), heads, dim, vdim, _stream())
+
+    _walk_rows(step, walk, state, heads, dim, vdim, write_state)
+    return out
+
+
+def token_mix(h: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, step, write_state: bool = True) -> torch.Tensor:
+    """h + (h' - h) * mu[m] for every vector of ``mu`` ``[mixes, hidden]``, h' the token before of the same request: the row
+    above, the request's stored row (``state`` float32 ``[slots, hidden]``) ahead of a portion, zeros at a sequence's
+    start.  Returns ``[mixes, rows, hidden]`` in ``h``'s type and stores every entry's last row unless told not to."""
+    rows, hidden = h.shape
+    mixes = mu.shape[0]
+    if tuple(mu.shape) != (mixes, hidden) or state.dtype != torch.float32 or tuple(state.shape[1:]) != (hidden,):
+        raise KernelError(f"token_mix: mixes {tuple(mu.shape)} and state {tuple(state.shape)} for rows of {hidden}")
+    spans = entry_spans(step)
+    out = torch.empty((mixes, rows, hidden), dtype=h.dtype, device=h.device)
+    single_rows = bool(step.decode_only) and step.entry_slots.numel() == rows
+    call("leone_token_mix", _dev(h, "rows"), _code(h, "rows"), _dev(mu, "mu"), _code(mu, "mu"), mixes, _dev(state, "stored rows"),
+         state.data_ptr() if write_state else 0, _dev(spans, "spans"), spans.shape[0],
+         _dev(step.row_entry, "row map", torch.int32, (rows,)), _dev(out, "mixed rows"), rows, hidden, 1 if single_rows else 0, _stream())
+    return out
+
+
+def low_rank_decay(low: torch.Tensor, w2: torch.Tensor, w0: torch.Tensor) -> torch.Tensor:
+    """exp(-exp(w2 tanh(low) + w0)): ``low`` float32 ``[rows, >= rank]`` (a slice of wider rows is fine), ``w2``
+    ``[channels, rank]``, ``w0`` ``[channels]`` -> float32 ``[rows, channels]``, all of it float."""
+    channels, rank = w2.shape
+    rows = low.shape[0]
+    low_at, stride = _strided_rows(low, "low-rank values", rows, rank)
+    out = torch.empty((rows, channels), dtype=torch.float32, device=low.device)
+    call("leone_low_rank_decay", low_at, stride, _dev(w2, "decay matrix"), _code(w2, "decay matrix"),
+         _dev(w0, "decay base", None, (channels,)), _code(w0, "decay base"), _dev(out, "decays"), rows, channels, rank, _stream())
+    return out
+
+
+def _walk_rows(step, walk, state: torch.Tensor, heads: int, dim: int, vdim: int, write_state: bool) -> None:
+    """A recurrence S <- diag(decay) S + ... over a step's rows: ``walk(segments, state read, state written, no_input=,
+    accumulate=, product=)`` walks segments of rows in order.  Long portions go chunk by chunk side by side: every chunk
+    from zeros (leaving what it wrote and the product of its decays), the chunks chained, every chunk again from the
+    state it starts from with nothing written into it."""
     plan = chunk_plan(step, *GATED_CHUNKS)
     if plan is None:
-        walk(spans, state, state if write_state else None)
-    else:
-        chunks = plan["chunks"]
-        work = torch.empty((chunks.shape[0], heads, dim * vdim), dtype=torch.float32, device=device)
-        product = torch.empty((chunks.shape[0], heads, dim), dtype=torch.float32, device=device)
-        walk(chunks, None, work, product=product)
-        call("leone_gated_chain", _dev(plan["links"], "links", torch.int32), plan["links"].shape[0], _dev(work, "work"),
-             work.stride(0), _dev(product, "decay products"), _dev(state, "state"), state.stride(0), heads, dim, vdim,
-             1 if write_state else 0, _stream())
-        walk(plan["again"], work, None, no_input=True, accumulate=True)
-        if plan["short"].shape[0]:
-            walk(plan["short"], state, state if write_state else None)
-    return out
+        walk(entry_spans(step), state, state if write_state else None)
+        return
+    chunks = plan["chunks"]
+    work = torch.empty((chunks.shape[0], heads, dim * vdim), dtype=torch.float32, device=state.device)
+    product = torch.empty((chunks.shape[0], heads, dim), dtype=torch.float32, device=state.device)
+    walk(chunks, None, work, product=product)
+    call("leone_gated_chain", _dev(plan["links"], "links", torch.int32), plan["links"].shape[0], _dev(work, "work"),
+         work.stride(0), _dev(product, "decay products"), _dev(state, "state"), state.stride(0), heads, dim, vdim,
+         1 if write_state else 0, _stream())
+    walk(plan["again"], work, None, no_input=True, accumulate=True)
+    if plan["short"].shape[0]:
+        walk(plan["short"], state, state if write_state else None)
 
 
 def _rotation_tables(what: str, part: int, cos, sin):
@@ -1998,3 +2119,69 @@ def depth_mix(x: torch.Tensor, delta: Optional[torch.Tensor], scale: float, hist
     call("leone_depth_mix", _dev(x, "stream", torch.float32), _dev(delta, "delta"), planes, plane, float(scale),
          _dev(history, "history"), history.stride(0), int(count), _dev(weight, "depth weights"), _code(weight, "depth weights"),
          n * hidden, _stream())
+
+
+# ---- sublayers side by side on one stream -----------------------------------------------------------------------
+class MixedDelta:
+    """What several sublayers add to the stream together: the sum of factor * scale * rows over ``terms`` = (rows float32
+    ``[n, hidden]`` or planes ``[p, n, hidden]``, factor, scale vector ``[hidden]`` or None).  A norm that can takes it in
+    place of a delta (``branch_norm``); any other consumer asks for ``materialize()``."""
+
+    def __init__(self, terms):
+        self.terms = list(terms)
+
+    def materialize(self) -> torch.Tensor:
+        total = None
+        for rows, factor, scale in self.terms:
+            rows = (rows.sum(dim=0) if rows.dim() == 3 else rows).float() * float(factor)
+            rows = rows if scale is None else rows * scale.float()
+            total = rows if total is None else total + rows
+        return total
+
+
+BRANCH_TERMS = 4          # results one call adds
+BRANCH_NORMS = 2          # norms it makes
+
+
+def branch_norm(x: torch.Tensor, terms, gains, eps: float, groups: int, out_dtype: torch.dtype,
+                rows: Optional[torch.Tensor] = None) -> list:
+    """x += sum of factor * scale * rows over ``terms`` (see ``MixedDelta``) in the float32 stream, then for every gain of
+    ``gains`` the RMS norm of the new rows in ``groups`` equal groups of neighbouring columns, each over its own root mean
+    square, times the gain, in ``out_dtype``.  With ``rows`` (int32 indices) only those rows come back and the stream is
+    left as it was."""
+    n, hidden = x.shape
+    terms = list(terms)
+    while len(terms) > BRANCH_TERMS:                     # more than one launch takes: the first ones are added ahead
+        if rows is not None:
+            first = MixedDelta(terms[:len(terms) - BRANCH_TERMS + 1]).materialize()
+            terms = [(first, 1.0, None)] + terms[len(terms) - BRANCH_TERMS + 1:]
+        else:
+            branch_norm(x, terms[:BRANCH_TERMS], [], eps, groups, out_dtype)
+            terms = terms[BRANCH_TERMS:]
+    if len(gains) > BRANCH_NORMS:
+        raise KernelError(f"branch_norm: {len(gains)} norms, one launch makes {BRANCH_NORMS}")
+    n_out = n if rows is None else rows.numel()
+    outs = [torch.empty((n_out, hidden), dtype=out_dtype, device=x.device) for _ in gains]
+    if not terms and not gains:
+        return outs
+    held = []
+    for delta, factor, scale in terms:
+        delta, planes, plane = _planes(delta, n, hidden, "result")
+        held.append((delta, planes, plane, float(factor), scale))
+    t, g = max(len(held), 1), max(len(gains), 1)
+    term_rows = (ctypes.c_void_p * t)(*[_dev(d, "result") for d, *_ in held])
+    term_planes = (ctypes.c_int * t)(*[p for _, p, *_ in held])
+    term_plane = (ctypes.c_long * t)(*[p for _, _, p, *_ in held])
+    factors = (ctypes.c_float * t)(*[f for *_, f, _ in held])
+    scales = (ctypes.c_void_p * t)(*[_dev(s, "result scale", None, (hidden,)) for *_, s in held])
+    scale_codes = (ctypes.c_int * t)(*[_code(s, "result scale") if s is not None else F32 for *_, s in held])
+    gain_ptrs = (ctypes.c_void_p * g)(*[_dev(v, "gain", None, (hidden,)) for v in gains])
+    gain_codes = (ctypes.c_int * g)(*[_code(v, "gain") for v in gains])
+    out_ptrs = (ctypes.c_void_p * g)(*[_dev(y, "normed rows") for y in outs])
+
+    def at(array):
+        return ctypes.cast(array, ctypes.c_void_p)
+    call("leone_branch_norm", _dev(x, "stream", torch.float32), at(term_rows), at(term_planes), at(term_plane), at(factors),
+         at(scales), at(scale_codes), len(held), at(gain_ptrs), at(gain_codes), at(out_ptrs), len(gains), _CODES[out_dtype],
+         float(eps), int(groups), _dev(rows, "rows", torch.int32) if rows is not None else 0, n_out, hidden, _stream())
+    return outs

@@ -109,6 +109,22 @@ _PROTOTYPES = {
     "leone_latent_attention": [P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, P],
     "leone_residual_norm": [P, P, c_int, ctypes.c_long, c_float, P, c_int, c_float, P, c_int, P, c_int, c_int, P],
     "leone_depth_mix": [P, P, c_int, ctypes.c_long, c_float, P, ctypes.c_long, c_int, P, c_int, ctypes.c_long, P],
+    "leone_attention_rows_shaped": [P, P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
+                                    c_int, P, ctypes.c_long, c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, P],
+    "leone_attention_decode_shaped": [P, P, P, P, P, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
+                                      c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, P],
+    "leone_attention_prefill_shaped": [P, P, P, P, P, P, c_int, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, P, P,
+                                       c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, P],
+    "leone_attention_rows_talk": [P, P, P, P, c_int, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
+                                  c_int, P],
+    "leone_qk_norm_rope_write_turned": [P, c_int, c_int, ctypes.c_long, P, P, P, c_int, P, P, c_int, c_float, P, P, c_int, c_int,
+                                        c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, ctypes.c_long,
+                                        P, c_int, P, P, c_int, c_int, c_int, P],
+    "leone_branch_norm": [P, P, P, P, P, P, P, c_int, P, P, P, c_int, c_int, c_float, c_int, P, c_int, c_int, P],
+    "leone_token_mix": [P, c_int, P, c_int, c_int, P, P, P, c_int, P, P, c_int, c_int, c_int, P],
+    "leone_low_rank_decay": [P, ctypes.c_long, P, c_int, P, c_int, P, c_int, c_int, c_int, P],
+    "leone_time_mix_scan": [P, P, P, ctypes.c_long, P, P, c_int, c_int, c_int, P, c_int, P, ctypes.c_long, P, ctypes.c_long, P, P,
+                            c_int, c_int, c_int, P],
     "leone_delta_chain": [P, c_int, P, ctypes.c_long, P, P, ctypes.c_long, c_int, c_int, c_int, c_int, P],
 }
 

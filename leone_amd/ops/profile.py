@@ -53,6 +53,15 @@ OPERATIONS = {
     "leone_attention_rows_kept": "attention",
     "leone_attention_decode_kept": "attention",
     "leone_attention_prefill_kept": "attention",
+    "leone_attention_rows_shaped": "attention",
+    "leone_attention_decode_shaped": "attention",
+    "leone_attention_prefill_shaped": "attention",
+    "leone_attention_rows_talk": "attention",
+    "leone_qk_norm_rope_write_turned": "qknorm rope kv",
+    "leone_branch_norm": "norm",
+    "leone_token_mix": "token mix",
+    "leone_low_rank_decay": "low rank decay",
+    "leone_time_mix_scan": "time mix scan",
     "leone_route_topk": "router",
     "leone_moe_plan": "router",
     "leone_route_plan": "router",

@@ -5,7 +5,7 @@ from typing import Dict, List, Optional
 
 import torch
 
-from ..weights.loader import TensorSpec
+from ..weights.loader import VECTOR, TensorSpec
 from .. import ops
 from .base import BLOCKS, CONVS, FEED_FORWARDS, MIXERS, NORMS, Part, PartSpec
 from .context import CacheView, StepContext
@@ -240,7 +240,7 @@ class PostNormBlock(Part):
         if isinstance(pending, ops.NormedDelta) and hasattr(pending.norm, "add_behind"):
             return pending.norm.add_behind(x, pending.rows, step.dtype)
         if pending is not None:
-            delta = pending.materialize() if isinstance(pending, ops.NormedDelta) else pending
+            delta = pending.materialize() if isinstance(pending, (ops.NormedDelta, ops.ScaledDelta, ops.MixedDelta)) else pending
             x.add_(delta.sum(dim=0) if delta.dim() == 3 else delta)
         return ops.add_normed(x, None, None, 0.0, out_dtype=step.dtype)
 
@@ -314,3 +314,74 @@ class ScaledPreNormBlock(Part):
             return delta
         h = self.norm2.add_norm(x, delta, step.dtype)
         return ops.ScaledDelta(self.feed_forward.forward(h, step), self.scale)
+
+
+@BLOCKS.register("parallel_prenorm")
+class ParallelPreNormBlock(Part):
+    """Mixer and feed-forward side by side, each behind a norm of its own, both of the same stream:
+
+        x <- x + scale1 * mixer(norm1(x)) + scale2 * feed_forward(norm2(x))
+
+    with learned vectors ``scale1`` and ``scale2`` (tensor names ``[hidden]``; None: no scale).  The second sublayer is there
+    only if ``feed_forward`` is given.  Parameters: ``hidden``, ``norm1``, ``mixer``, ``scale1`` and optionally ``norm2``,
+    ``feed_forward``, ``scale2``.  The sublayers hand back float32.  Nothing is added here: the block hands on
+    ``ops.MixedDelta`` (the branches of a mixer made of several as terms of their own), and the norms that run next
+    make the sum, the stream's new rows and both norms of them in one kernel.
+    """
+
+    def __init__(self, spec: PartSpec, **context):
+        self.hidden = int(spec["hidden"])
+        self.norm1 = NORMS.build(spec["norm1"], **context)
+        self.mixer = MIXERS.build(spec["mixer"], **context)
+        self.feed_forward = FEED_FORWARDS.build(spec["feed_forward"], **context) if spec.get("feed_forward") is not None else None
+        self.norm2 = NORMS.build(spec["norm2"], **context) if spec.get("norm2") is not None else None
+        if self.feed_forward is not None and self.norm2 is None:
+            raise ValueError("a parallel_prenorm block with a feed-forward needs norm2")
+        self.scale_names = (spec.get("scale1"), spec.get("scale2") if self.feed_forward is not None else None)
+        self.scales = [None, None]
+
+    def parts(self):
+        return tuple(part for part in (self.norm1, self.mixer, self.norm2, self.feed_forward) if part is not None)
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(getattr(part, "graph_safe", False) for part in self.parts())
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        return [s for part in self.parts() for s in part.tensor_specs()] + \
+            [TensorSpec(name, (self.hidden,), VECTOR) for name in self.scale_names if name]
+
+    def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
+        for part in self.parts():
+            part.bind(tensors)
+        self.scales = [tensors.pop(name).contiguous() if name else None for name in self.scale_names]
+
+    def streamed_weights(self) -> List[torch.Tensor]:
+        return [w for part in self.parts() if hasattr(part, "streamed_weights") for w in part.streamed_weights()]
+
+    def cache_need(self):
+        return self.mixer.cache_need()
+
+    def row_tilings(self):
+        found = []
+        for part in self.parts():
+            if hasattr(part, "row_tiling"):
+                found.append(part.row_tiling())
+            if hasattr(part, "row_tilings"):
+                found += part.row_tilings()
+        return found
+
+    def forward(self, x: torch.Tensor, pending, step: StepContext, cache: Optional[CacheView]):
+        if self.feed_forward is None:
+            y1, y2 = self.norm1.add_norm(x, pending, step.dtype), None
+        elif hasattr(self.norm1, "add_norms"):
+            y1, y2 = self.norm1.add_norms(self.norm2, x, pending, step.dtype)
+        else:
+            y1 = self.norm1.add_norm(x, pending, step.dtype)
+            y2 = self.norm2.add_norm(x, None, step.dtype)
+        branches = self.mixer.branch_results(y1, step, cache) if hasattr(self.mixer, "branch_results") else \
+            [(self.mixer.forward(y1, step, cache), 1.0)]
+        terms = [(rows, factor, self.scales[0]) for rows, factor in branches]
+        if self.feed_forward is not None:
+            terms.append((self.feed_forward.forward(y2, step), 1.0, self.scales[1]))
+        return ops.MixedDelta(terms)

@@ -142,7 +142,9 @@ class RoutedGluMlp(Part):
     (a group's score is the sum of its so many best choice scores, 1 by default), ``renormalize`` (False: the weights
     are the winners' scores themselves), ``weight_scale`` (multiplies the weights), and ``activation`` "clamped_swish"
     with ``limit`` (``ops.EXPERT_ACTIVATIONS``): g = min(gate, limit), u = clamp(up, -limit, limit),
-    g sigmoid(1.702 g) (u + 1).
+    g sigmoid(1.702 g) (u + 1).  ``gated`` False: an expert has no gate and computes down_e(act(up_e y)), ``activation`` a key
+    of ``ops.PLAIN_ACTIVATIONS`` (silu, gelu_tanh, relu2: the square of relu); ``weigh_input`` (such experts only): the weight
+    multiplies what the expert reads, not what it gives.
 
     The choice lives on the device only: which rows go to which expert is worked out there, and the grids do not
     depend on it, so a recorded step replays with other choices.
@@ -160,8 +162,12 @@ class RoutedGluMlp(Part):
         if self.top > self.total or self.total % self.group_count or not 1 <= self.group_keep <= self.group_count:
             raise ValueError(f"a router of {self.total} outputs cannot choose {self.top} from {self.group_keep} of "
                              f"{self.group_count} equal groups")
-        if self.activation not in ops.EXPERT_ACTIVATIONS:
-            raise ValueError(f"unknown expert activation {self.activation!r}; known: {', '.join(ops.EXPERT_ACTIVATIONS)}")
+        self.gated, self.weigh_input = bool(p.get("gated", True)), bool(p.get("weigh_input", False))
+        known = ops.EXPERT_ACTIVATIONS if self.gated else ops.PLAIN_ACTIVATIONS
+        if self.activation not in known:
+            raise ValueError(f"unknown expert activation {self.activation!r}; known: {', '.join(known)}")
+        if self.weigh_input and (self.gated or self.identity or p.get("shared") is not None):
+            raise ValueError("a weight on what an expert reads goes with experts without a gate, no identity outputs and no shared expert")
         self.limit = float(p["limit"]) if p.get("limit") is not None else None
         if self.activation == "clamped_swish" and not (self.limit and self.limit > 0.0):
             raise ValueError(f"the clamped activation needs a positive limit, found {self.limit!r}")
@@ -178,8 +184,8 @@ class RoutedGluMlp(Part):
             specs.append(TensorSpec(self.correction_name, (self.total,), VECTOR))
         for e in range(self.experts):
             name = self.expert_name.format(e=e)
-            specs += [TensorSpec(name + ".gate", (self.intermediate, self.hidden), MATRIX),
-                      TensorSpec(name + ".up", (self.intermediate, self.hidden), MATRIX),
+            specs += [TensorSpec(name + ".gate", (self.intermediate, self.hidden), MATRIX)] if self.gated else []
+            specs += [TensorSpec(name + ".up", (self.intermediate, self.hidden), MATRIX),
                       TensorSpec(name + ".down", (self.hidden, self.intermediate), MATRIX)]
         return specs + (self.shared.tensor_specs() if self.shared is not None else [])
 
@@ -187,14 +193,16 @@ class RoutedGluMlp(Part):
         self.w_router = tensors.pop(self.router_name).contiguous()
         self.correction = tensors.pop(self.correction_name).contiguous() if self.correction_name else None
         names = [self.expert_name.format(e=e) for e in range(self.experts)]
-        # all experts side by side: [experts, 2, ff, hidden] (gate rows, then up rows) and [experts, hidden, ff]
-        gate_up = torch.stack([torch.stack([tensors.pop(n + ".gate"), tensors.pop(n + ".up")]) for n in names])
+        # all experts side by side: [experts, 2, ff, hidden] (gate rows, then up rows; without gates [experts, ff, hidden])
+        # and [experts, hidden, ff]
+        gate_up = torch.stack([torch.stack([tensors.pop(n + ".gate"), tensors.pop(n + ".up")]) if self.gated else tensors.pop(n + ".up")
+                               for n in names])
         down = torch.stack([tensors.pop(n + ".down") for n in names])
         # A shared expert of the experts' kind rides along in the experts' launches of short steps: cut into pieces of
         # the experts' size (the last filled up with zero rows, which add nothing), they stand behind the experts as
         # experts that every row takes with weight 1.
         self.always = 0
-        if isinstance(self.shared, SwiGluMlp) and self.shared.activation == self.activation:
+        if self.gated and isinstance(self.shared, SwiGluMlp) and self.shared.activation == self.activation:
             shared = {k: tensors[self.shared.names[k]] for k in ("gate", "up", "down")}
             pieces = -(-self.shared.intermediate // self.intermediate)
             pad = pieces * self.intermediate - self.shared.intermediate
@@ -227,4 +235,4 @@ class RoutedGluMlp(Part):
                 extra = extra.float()
         return ops.routed_feed_forward(y, logits, self.correction, self.top, self.group_count, self.group_keep,
                                        self.w_gate_up, self.w_down, self.activation, extra=extra, rule=self.rule,
-                                       limit=self.limit)
+                                       limit=self.limit, weigh_input=self.weigh_input)

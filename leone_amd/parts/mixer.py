@@ -46,6 +46,11 @@ class GqaAttention(Part):
     request's last ``taps - 1`` projected rows.  ``distance_slopes`` (one number a query head): head h's score for a
     key at distance d is lowered by slopes[h] * d.  ``query_factor`` = (coef, every): the queries at position p count
     times 1 + coef * ln(floor((p + 1) / every) + 1).
+    ``talk`` (tensor name ``[q_heads, q_heads]``): the heads' scaled scores are mixed before the softmax, score_h <-
+    sum_g talk[h, g] score_g.  ``softcap``: scores become cap * tanh(score / cap).  ``sink`` (tensor name ``[q_heads]``): the
+    softmax's denominator also holds exp(sink_h).  ``value_position`` (name of a position part that covers the whole value):
+    values are turned by their own position when they are cached and a head's result is turned back by the position that
+    reads it.
     """
 
     graph_safe = True
@@ -98,14 +103,33 @@ class GqaAttention(Part):
                 "taps": int(c["taps"]), "weights": [c["q"], c["k"], c["v"]]}))
         if (self.bias_names or self.wide_norm) and self.shared_kv:
             raise ValueError("attention: biases and norms over a whole projection go with keys of the layer's own")
+        self.softcap = float(p["softcap"]) if p.get("softcap") is not None else None
+        if self.softcap is not None and not self.softcap > 0.0:
+            raise ValueError(f"attention: the scores' cap must be positive, found {self.softcap}")
+        if p.get("talk"):
+            self.names["talk"] = p["talk"]
+        if p.get("sink"):
+            self.names["sink"] = p["sink"]
+        self.value_position = (positions or {}).get(p["value_position"]) if p.get("value_position") else None
+        if p.get("value_position") and self.value_position is None:
+            raise ValueError(f"attention names position part {p['value_position']!r}, which the model does not define")
+        shaped = self.softcap is not None or "sink" in self.names or self.value_position is not None
+        if "talk" in self.names and (shaped or self.keep_first or self.slope_values is not None or self.query_factor is not None
+                                     or "gate" in self.names):
+            raise ValueError("attention: mixed scores go with a plain softmax: no cap, sink, turned values, slopes, query factor, "
+                             "kept first keys or gate")
+        if self.value_position is not None and rotation_of(self.value_position).rotary_dim != self.file_value_dim:
+            raise ValueError(f"attention: values of {self.file_value_dim} elements are turned whole")
+        if self.value_position is not None and self.shared_kv:
+            raise ValueError("attention: turned values go with keys and values of the layer's own")
         # a value size of its own, a gate, or anything between the projection and the heads: the projection carries
         # more than q, k and v of one size, or passes through kernels of its own
         self.general = (self.value_dim != self.head_dim or "gate" in self.names or self.shared_kv or bool(self.bias_names)
                         or self.wide_norm or self.conv is not None or self.slope_values is not None
-                        or self.query_factor is not None or self.padded)
-        if self.padded and (self.shared_kv or self.gate_each or (self.qk_norm_eps is not None and not self.wide_norm)):
+                        or self.query_factor is not None or self.padded or shaped or "talk" in self.names)
+        if self.padded and (self.shared_kv or self.gate_each):
             raise ValueError(f"attention: heads of {self.file_head_dim} and values of {self.file_value_dim} elements are filled up "
-                             f"to multiples of 8 and 2, which a norm a head, a gate an element and a borrowed cache do not allow")
+                             f"to multiples of 8 and 2, which a gate an element and a borrowed cache do not allow")
         if self.qk_norm_eps is not None:
             self.names.update(q_norm=p["q_norm"])
             if not self.shared_kv:
@@ -113,7 +137,7 @@ class GqaAttention(Part):
         self.position = (positions or {}).get(p.get("position")) if p.get("position") else None
         if p.get("position") and self.position is None:
             raise ValueError(f"attention names position part {p.get('position')!r}, which the model does not define")
-        self.w_qkv = self.w_o = self.q_gain = self.k_gain = self.bias = self.slopes = None
+        self.w_qkv = self.w_o = self.q_gain = self.k_gain = self.bias = self.slopes = self.talk = self.sinks = None
 
     def cache_need(self):
         keys = KvNeed(self.kv_heads, self.head_dim, self.retain_window,
@@ -147,6 +171,10 @@ class GqaAttention(Part):
             specs += [TensorSpec(self.bias_names["q"], (qw,), VECTOR, init=small),
                       TensorSpec(self.bias_names["k"], (kvw,), VECTOR, init=small),
                       TensorSpec(self.bias_names["v"], (vw,), VECTOR, init=small)]
+        if "talk" in self.names:
+            specs.append(TensorSpec(self.names["talk"], (self.q_heads, self.q_heads), VECTOR, init=("normal", 0.0, 0.3)))
+        if "sink" in self.names:
+            specs.append(TensorSpec(self.names["sink"], (self.q_heads,), VECTOR, init=("normal", 0.0, 1.0)))
         if self.conv is not None:       # the filters as the file has them: one row a channel of the heads' own sizes
             specs += [TensorSpec(name, (width, self.conv.taps), VECTOR) for name, width in zip(self.conv.names, (qw, kvw, vw))]
         return specs
@@ -178,6 +206,9 @@ class GqaAttention(Part):
             self.k_gain = self.q_gain if self.shared_kv else tensors.pop(self.names["k_norm"]).contiguous()
             if self.q_gain.dtype != self.k_gain.dtype:
                 self.q_gain, self.k_gain = self.q_gain.float(), self.k_gain.float()
+            if self.padded and not self.wide_norm:
+                self.q_gain = self._filled(self.q_gain, 1, d, self.head_dim).contiguous()
+                self.k_gain = self._filled(self.k_gain, 1, d, self.head_dim).contiguous()
             if self.wide_norm:
                 self.q_gain = self._filled(self.q_gain, self.q_heads, d, self.head_dim).contiguous()
                 self.k_gain = self._filled(self.k_gain, self.kv_heads, d, self.head_dim).contiguous()
@@ -190,6 +221,10 @@ class GqaAttention(Part):
                                              (self.head_dim, self.head_dim, self.value_dim)):
                 tensors[name] = self._filled(tensors[name], heads, size, to)
             self.conv.bind(tensors)
+        if "talk" in self.names:
+            self.talk = tensors.pop(self.names["talk"]).contiguous()
+        if "sink" in self.names:
+            self.sinks = tensors.pop(self.names["sink"]).float().contiguous()
         if self.slope_values is not None:
             self.slopes = torch.tensor(self.slope_values, dtype=torch.float32, device=self.w_o.device)
 
@@ -219,17 +254,23 @@ class GqaAttention(Part):
             if self.conv is not None:
                 # q, k and v pass their filters side by side in one launch; the gates' columns stay where they are
                 heads = self.conv.forward(proj[:, :qw + kw + vw], step, conv_state, torch.float32)
-            if self.bias is not None or self.wide_norm:
+            turn = rotation_of(self.value_position)
+            if turn.cos is not None and step.max_position >= turn.cos.shape[0]:
+                raise ValueError(f"position {step.max_position} is beyond the values' table of {turn.cos.shape[0]} positions")
+            if self.wide_norm:
                 # a span's mean is taken over the elements the projection has in the file, not over what fills it up
                 spans = [(0, qw, self.q_gain, self.q_heads * self.file_head_dim),
-                         (qw, kw, self.k_gain, self.kv_heads * self.file_head_dim)] if self.wide_norm else []
-                ops.bias_span_norm(heads, self.bias, spans, self.qk_norm_eps if self.wide_norm else 1.0, round_to=step.dtype)
+                         (qw, kw, self.k_gain, self.kv_heads * self.file_head_dim)]
+                ops.bias_span_norm(heads, self.bias, spans, self.qk_norm_eps, round_to=step.dtype)
             head_gains = (None, None) if self.wide_norm else (self.q_gain, self.k_gain)
             q = ops.qk_norm_rope_write(heads, self.q_heads, self.kv_heads, self.head_dim, head_gains[0], head_gains[1],
                                        self.qk_norm_eps if self.qk_norm_eps is not None else 1.0, rotation.cos, rotation.sin,
                                        step.positions, step.row_entry, cache.block_table, cache.k_pool, cache.v_pool,
                                        write_cache=cache.writes and not self.shared_kv, out_dtype=step.dtype,
-                                       pairing=rotation.pairing, value_dim=self.value_dim, queries_only=self.shared_kv)
+                                       pairing=rotation.pairing, value_dim=self.value_dim, queries_only=self.shared_kv,
+                                       bias=None if self.wide_norm else self.bias,
+                                       value_rotation=(turn.cos, turn.sin, turn.pairing) if turn.cos is not None else None,
+                                       norm_count=self.file_head_dim if self.padded and not self.wide_norm else 0)
             gate = None
             if "gate" in self.names:
                 gate = proj[:, self.q_heads * self.head_dim:] if self.shared_kv else \
@@ -283,12 +324,17 @@ class GqaAttention(Part):
         window = int(self.window or 0)
         group = self.q_heads // self.kv_heads
         max_blocks = cache.block_table.shape[1]
+        if self.talk is not None:
+            return ops.attention_rows_talk(q, cache.k_pool, cache.v_pool, self.talk, step.positions, step.row_entry,
+                                           cache.block_table, self.q_heads, self.scale, window)
+        turn = rotation_of(self.value_position)
+        shape = ops.ScoreShape(self.softcap, self.sinks, (turn.cos, turn.sin, turn.pairing) if turn.cos is not None else None)
         if self._rows_only() or \
                 not ops.decode_attention_supported(q.dtype, self.head_dim, cache.page_tokens, group, max_blocks):
             return ops.attention_rows(q, cache.k_pool, cache.v_pool, step.positions, step.row_entry,
                                       cache.block_table, self.q_heads, self.scale, window, gate=gate,
                                       keep_first=self.keep_first, gate_each=self.gate_each, slopes=self.slopes,
-                                      query_factor=self.query_factor)
+                                      query_factor=self.query_factor, shape=shape)
         first = 0
         out = torch.empty_like(q)
         tiled = step.tiled.get(self.row_tiling())
@@ -297,13 +343,13 @@ class GqaAttention(Part):
             ops.attention_prefill(q, out, cache.k_pool, cache.v_pool, step.positions, tiled.tiles,
                                   cache.block_table, self.q_heads, self.scale, window,
                                   mean_keys=tiled.mean_keys or step.max_position + 1, covered_rows=tiled.rows,
-                                  keep_first=self.keep_first, slopes=self.slopes, query_factor=self.query_factor)
+                                  keep_first=self.keep_first, slopes=self.slopes, query_factor=self.query_factor, shape=shape)
             first = tiled.rows
         if first < step.rows:
             ops.attention_decode(q[first:], cache.k_pool, cache.v_pool, step.positions[first:],
                                  step.row_entry[first:], cache.block_table, self.q_heads, self.scale, window,
                                  max_context=step.max_position + 1, out=out[first:], keep_first=self.keep_first,
-                                 slopes=self.slopes, query_factor=self.query_factor)
+                                 slopes=self.slopes, query_factor=self.query_factor, shape=shape)
         if gate is None:
             return out
         # a gate for every element is a gate a head of one element

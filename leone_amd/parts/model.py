@@ -268,7 +268,7 @@ class DecoderModel:
             pending = None
         elif isinstance(pending, ops.ScaledDelta):
             pending, scale = pending.rows, pending.scale
-        elif isinstance(pending, ops.NormedDelta):
+        elif isinstance(pending, (ops.NormedDelta, ops.MixedDelta)):
             pending = pending.materialize()
         ops.depth_mix(x, pending, scale, history, at + 2, self.depth_weights[at])
         return None
@@ -304,7 +304,7 @@ class DecoderModel:
             return None
         if isinstance(pending, ops.PreparedRows):
             pending = None                    # prepared for a norm that never ran: the stream is up to date
-        if isinstance(pending, ops.ScaledDelta) and not hasattr(self.final_norm, "gain"):
+        if isinstance(pending, (ops.ScaledDelta, ops.MixedDelta)) and not hasattr(self.final_norm, "gain"):
             pending = pending.materialize()
         if hasattr(self.final_norm, "lazy"):
             y = self.final_norm.lazy(x, pending, self.dtype, rows=step.want_rows)

@@ -16,7 +16,9 @@ class RmsNorm(Part):
 
     Reference: crates/leone/src/cpu.rs:1642-1663.  Parameters: ``size``, ``eps``, ``weight`` (tensor name).
     Optional: ``weight_offset`` (a number): the stored weight lies around zero and the gain is offset + weight; the
-    sum is made once, in float32, when the weights are bound, and the kernels see an ordinary gain.
+    sum is made once, in float32, when the weights are bound, and the kernels see an ordinary gain.  ``gain_factor`` (a
+    number): the gain is that many times what it would be (a factor on everything the norm's reader makes of it), made the
+    same way.  ``groups``: the row is split into so many equal consecutive parts, each divided by its own root mean square.
     """
 
     graph_safe = True
@@ -26,6 +28,10 @@ class RmsNorm(Part):
         self.eps = float(spec["eps"])
         self.weight_name = spec["weight"]
         self.weight_offset = float(spec["weight_offset"]) if spec.get("weight_offset") is not None else None
+        self.gain_factor = float(spec["gain_factor"]) if spec.get("gain_factor") is not None else None
+        self.groups = int(spec.get("groups") or 1)
+        if self.size % self.groups:
+            raise ValueError(f"rmsnorm: {self.size} elements cannot be normed in {self.groups} equal groups")
         self.gain: Optional[torch.Tensor] = None
 
     def tensor_specs(self) -> List[TensorSpec]:
@@ -37,11 +43,35 @@ class RmsNorm(Part):
         self.gain = tensors[self.weight_name].contiguous()
         if self.weight_offset is not None:
             self.gain = (self.gain.float() + self.weight_offset).contiguous()
+        if self.gain_factor is not None:
+            self.gain = (self.gain.float() * self.gain_factor).contiguous()
+
+    def add_norms(self, other, x: torch.Tensor, delta, out_dtype: torch.dtype) -> list:
+        """This norm's rows and ``other``'s, both of the stream after ``delta`` has been added: one kernel if the two norms
+        differ in their gains alone."""
+        if isinstance(other, RmsNorm) and (other.groups, other.eps, other.size) == (self.groups, self.eps, self.size):
+            return ops.branch_norm(x, self._terms(delta), [self.gain, other.gain], self.eps, self.groups, out_dtype)
+        return [self.add_norm(x, delta, out_dtype), other.add_norm(x, None, out_dtype)]
+
+    @staticmethod
+    def _terms(delta) -> list:
+        """A delta of any kind as the terms of a ``MixedDelta``."""
+        if delta is None or isinstance(delta, ops.PreparedRows):
+            return []
+        if isinstance(delta, ops.MixedDelta):
+            return delta.terms
+        if isinstance(delta, ops.ScaledDelta):
+            return [(delta.rows, delta.scale, None)]
+        if isinstance(delta, ops.NormedDelta):
+            delta = delta.materialize()
+        return [(delta, 1.0, None)]
 
     def add_norm(self, x: torch.Tensor, delta: Optional[torch.Tensor], out_dtype: torch.dtype,
                  rows: Optional[torch.Tensor] = None) -> torch.Tensor:
         if isinstance(delta, ops.PreparedRows):
             delta = None                      # the product that made it has added into the stream already
+        if self.groups > 1 or isinstance(delta, ops.MixedDelta):
+            return ops.branch_norm(x, self._terms(delta), [self.gain], self.eps, self.groups, out_dtype, rows)[0]
         if isinstance(delta, ops.ScaledDelta):
             # a sublayer's result that enters the stream times a factor: sum and norm in one kernel
             return ops.residual_norm(x, delta.rows, delta.scale, self.gain, self.eps, out_dtype, rows)
@@ -55,17 +85,21 @@ class RmsNorm(Part):
 
     def apply(self, rows: torch.Tensor, out_dtype: torch.dtype = torch.float32) -> torch.Tensor:
         """The norm of float32 rows that are no stream (nothing is added, nothing written back)."""
+        if self.groups > 1:
+            return ops.branch_norm(rows, [], [self.gain], self.eps, self.groups, out_dtype)[0]
         return ops.add_rmsnorm(rows, None, self.gain, self.eps, out_dtype)
 
     def add_behind(self, x: torch.Tensor, delta: Optional[torch.Tensor], out_dtype: Optional[torch.dtype]):
         """For a norm that stands behind its sublayer: x += norm(delta) in the float32 stream, and the new rows of
         the stream come back in ``out_dtype`` (what the next sublayer's products read; None: nothing comes back)."""
+        if self.groups > 1:
+            raise ValueError("a norm in groups does not stand behind a sublayer")
         return ops.add_normed(x, delta, self.gain, self.eps, out_dtype=out_dtype)
 
     def folded(self, out_dtype: torch.dtype):
         """(gain, eps, type) for a product that can leave this norm's operand behind when it adds into the
-        stream (``ops.linear(..., next_norm=)``)."""
-        return (self.gain, self.eps, out_dtype)
+        stream (``ops.linear(..., next_norm=)``); None for a norm in groups, which no product prepares."""
+        return None if self.groups > 1 else (self.gain, self.eps, out_dtype)
 
     def lazy(self, x: torch.Tensor, delta: Optional[torch.Tensor], out_dtype: torch.dtype,
              rows: Optional[torch.Tensor] = None):
@@ -75,7 +109,7 @@ class RmsNorm(Part):
             if rows is None and delta.gain is self.gain and delta.eps == self.eps and delta.dtype == out_dtype:
                 return delta
             delta = None                      # made for another norm: the stream itself is up to date
-        if delta is not None:
+        if delta is not None or self.groups > 1:
             return self.add_norm(x, delta, out_dtype, rows)
         return ops.NormedRows(x, self.gain, self.eps, out_dtype, rows)
 
@@ -116,7 +150,7 @@ class LayerNorm(Part):
         if isinstance(delta, ops.PreparedRows):
             delta = None
         delta_norm = None
-        if isinstance(delta, ops.ScaledDelta):
+        if isinstance(delta, (ops.ScaledDelta, ops.MixedDelta)):
             delta = delta.materialize()
         if isinstance(delta, ops.NormedDelta):
             behind = delta.norm

@@ -367,6 +367,70 @@ class StateSpaceMixer(Part):
         return ops.linear(y, self.w_o, out_dtype=torch.float32)
 
 
+@MIXERS.register("time_mix")
+class TimeMixMixer(Part):
+    """A matrix memory that reads the token before beside the token itself and makes its decays from it (RWKV).
+
+    With h' the token before (zeros at a sequence's start) each of r, k, v, g, w reads a mix of its own,
+    h + (h' - h) * mu.  r = W_r ., k = W_k ., v = W_v . (``heads`` of ``dim``), gate = silu(W_g .), decay
+    w = exp(-exp(W_w2 tanh(W_w1 .) + w0)) per head and key channel.  Per head o_t = (S + diag(u) k_t v_t^T)^T r_t, then
+    S <- diag(w_t) S + k_t v_t^T (float32, from zero); each head's o over its root mean square, times ``norm`` (all heads'
+    size), times the gate, then W_o.  The token before is part of the state.
+
+    Parameters: ``hidden``, ``heads``, ``dim``, ``rank`` (of the low-rank decay), ``eps``, ``mu`` (a dict with tensor names
+    ``r``, ``k``, ``v``, ``g``, ``w``) and tensor names ``r``, ``k``, ``v``, ``g``, ``o``, ``norm``, ``u``, ``w0``, ``w1``, ``w2``.
+    """
+
+    graph_safe = True
+    MIXES = ("r", "k", "v", "g", "w")
+
+    def __init__(self, spec: PartSpec, **_):
+        p = spec.params
+        self.hidden, self.heads, self.dim, self.rank = (int(p[k]) for k in ("hidden", "heads", "dim", "rank"))
+        self.eps = float(p["eps"])
+        _check_dim("time_mix", self.dim)
+        self.names = {k: p[k] for k in ("r", "k", "v", "g", "o", "norm", "u", "w0", "w1", "w2")}
+        self.mu_names = {k: p["mu"][k] for k in self.MIXES}
+        self.mu = self.w_in = self.w_low = self.w_o = self.norm = self.bonus = self.decay_base = self.decay_matrix = None
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        n, inner = self.names, self.heads * self.dim
+        return [TensorSpec(self.mu_names[k], (self.hidden,), VECTOR, init=("uniform", 0.0, 1.0)) for k in self.MIXES] + \
+            [TensorSpec(n[k], (inner, self.hidden), MATRIX) for k in ("r", "k", "v", "g")] + \
+            [TensorSpec(n["w1"], (self.rank, self.hidden), MATRIX), TensorSpec(n["w2"], (inner, self.rank), MATRIX),
+             # decays exp(-exp(-6 .. -1)): memories that reach from a few to hundreds of tokens back
+             TensorSpec(n["w0"], (inner,), VECTOR, init=("uniform", -6.0, -1.0)),
+             TensorSpec(n["u"], (self.heads, self.dim), VECTOR, init=("normal", 0.0, 0.5)),
+             TensorSpec(n["norm"], (inner,), VECTOR), TensorSpec(n["o"], (self.hidden, inner), MATRIX)]
+
+    def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
+        n = self.names
+        self.mu = torch.stack([tensors.pop(self.mu_names[k]) for k in self.MIXES]).contiguous()
+        self.w_in = [tensors.pop(n[k]).contiguous() for k in ("r", "k", "v", "g")]
+        self.w_low = tensors.pop(n["w1"]).contiguous()
+        self.decay_matrix, self.decay_base = tensors.pop(n["w2"]).contiguous(), tensors.pop(n["w0"]).contiguous()
+        self.bonus = tensors.pop(n["u"]).reshape(-1).contiguous()
+        self.norm, self.w_o = tensors.pop(n["norm"]).contiguous(), tensors.pop(n["o"]).contiguous()
+
+    def streamed_weights(self) -> List[torch.Tensor]:
+        return [*self.w_in, self.w_low, self.w_o]
+
+    def cache_need(self):
+        return {"before": StateNeed((self.hidden,), torch.float32),
+                "memory": StateNeed((self.heads, self.dim * self.dim), torch.float32)}
+
+    def forward(self, h: torch.Tensor, step: StepContext, cache) -> torch.Tensor:
+        before, memory = cache["before"], cache["memory"]
+        mixed = ops.token_mix(ops.materialize(h), self.mu, before.state, step, write_state=before.writes)
+        r, k, v, gate = (ops.linear(mixed[m], w, out_dtype=torch.float32) for m, w in enumerate(self.w_in))
+        low = ops.linear(mixed[4], self.w_low, out_dtype=torch.float32)
+        decay = ops.low_rank_decay(low, self.decay_matrix, self.decay_base)
+        o = ops.time_mix_scan(r, k, v, decay, self.bonus, memory.state, step, self.heads, self.dim, self.dim,
+                              write_state=memory.writes)
+        y = ops.head_norm_gate(o, self.heads, self.dim, self.eps, step.dtype, gain=self.norm, gate=gate, activation="silu")
+        return ops.linear(y, self.w_o, out_dtype=torch.float32)
+
+
 @MIXERS.register("parallel")
 class ParallelMixer(Part):
     """Several mixers side by side on the same input: each result is divided by its root mean square over the
@@ -415,11 +479,20 @@ class ParallelMixer(Part):
     def cache_need(self):
         return {name: b.cache_need() for name, b in self.branches.items()}
 
-    def forward(self, h: torch.Tensor, step: StepContext, cache) -> torch.Tensor:
+    def branch_results(self, h: torch.Tensor, step: StepContext, cache) -> list:
+        """The branches' results (float32) with the factors of their sum, for a caller that sums them itself."""
+        if self.weights is None:
+            return [(self.forward(h, step, cache), 1.0)]
+        return list(zip(self._results(h, step, cache), (self.weights[name] for name in self.branches)))
+
+    def _results(self, h: torch.Tensor, step: StepContext, cache) -> list:
         h = ops.materialize(h)
         results = [b.forward(h, step, cache.get(name)) for name, b in self.branches.items()]
         results = [r.sum(dim=0) if r.dim() == 3 else r for r in results]
-        results = [r if r.dtype == torch.float32 else r.float() for r in results]
+        return [r if r.dtype == torch.float32 else r.float() for r in results]
+
+    def forward(self, h: torch.Tensor, step: StepContext, cache) -> torch.Tensor:
+        results = self._results(h, step, cache)
         if self.weights is not None:
             return ops.weighted_mix(results, [self.weights[name] for name in self.branches])
         return ops.rms_mix(results, [self.gains[name] for name in self.branches], self.eps, self.scale)
