@@ -446,9 +446,31 @@ def nogidra_shape(width: int, layers: int, vocab: int, context: int) -> dict:
             "layers": [{**order[i % 3], "mlp": routed if i % 2 else dense} for i in range(layers)]}
 
 
-DESIGN_SHAPES = {"pamevik": pamevik_shape, "zukinex": zukinex_shape, "fosulix": fosulix_shape, "nogidra": nogidra_shape}
+def reverax_shape(width: int, layers: int, vocab: int, context: int) -> dict:
+    """Reverax at layer sizes that resemble published models of its kinds: by turns softmax attention whose heads' scores are
+    mixed (heads of 128, at most 16 of them, four query heads a key head, half a head rotated) and softmax attention with
+    turned values, capped scores and a sink (heads of 128 with four query heads a key head, half a head rotated, a window
+    of 1,024) beside a matrix memory (heads of 64 x 64 over the model's width, a decay of rank 64); norms in four groups;
+    the feed-forward by turns dense (3 x width) and 32 ungated experts of 3/8 width of which four are chosen."""
+    heads = width // 128
+    talking = {"type": "attention",
+               "mixer": {"heads": min(heads, 16), "kv_heads": max(min(heads, 16) // 4, 1), "dim": 128, "vdim": 128,
+                         "scale": 128 ** -0.5, "rot": {"dims": 64, "base": 1000000.0}}}
+    side = {"type": "parallel",
+            "mixer": {"left": {"heads": heads, "kv_heads": width // 512, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                               "softcap": 50.0, "rot": {"dims": 64, "base": 1000000.0}, "mask": {"size": 1024}},
+                      "right": {"heads": width // 64, "dim": 64, "decay_rank": 64}, "left_scale": 0.5, "right_scale": 0.5}}
+    dense = {"kind": "dense", "ff": 3 * width}
+    routed = {"kind": "moe", "expert": {"ff": 3 * width // 8}, "router": {"experts": 32, "top": 4}}
+    order = [{**talking, "mlp": dense}, {**side, "mlp": routed}, {**talking, "mlp": routed}, {**side, "mlp": dense}]
+    return {"architecture": "Reverax", "vocab": vocab, "width": width, "norm": {"eps": 1e-6, "groups": 4}, "logit_scale": 1.0,
+            "max_positions": max(4096, context + 64), "layers": [order[i % 4] for i in range(layers)]}
+
+
+DESIGN_SHAPES = {"pamevik": pamevik_shape, "zukinex": zukinex_shape, "fosulix": fosulix_shape, "nogidra": nogidra_shape,
+                 "reverax": reverax_shape}
 # The existing design whose kernels a design's own stand closest to: measured beside it, at the same sizes.
-DESIGN_NEIGHBOURS = {"nogidra": "fosulix"}
+DESIGN_NEIGHBOURS = {"nogidra": "fosulix", "reverax": "nogidra"}
 
 
 def state_bytes_per_request(model) -> int:
