@@ -38,6 +38,7 @@
 // For S^T the two 16-key halves of a tile are laid out so that lane (g, c)
 // ends up with the scores of keys 8g .. 8g+7 of the tile: exactly the k-slots
 // it has to supply as P^T for the second product.
+#include "attention_merge.h"
 #include "common.h"
 #include "leone_hip.h"
 #include "score_shape.h"
@@ -613,6 +614,13 @@ attention_reduce_kernel(const float* __restrict__ part_acc, const float* __restr
         out[rh * head_dim + d] = from_float<bf16_t>(num / den);
     }
 }
+
+void launch_attention_reduce(const float* part_acc, const float* part_ml, bf16_t* out, int rows, int q_heads, int head_dim, int splits,
+                             hipStream_t stream) {
+    attention_reduce_kernel<false><<<rows * q_heads, kReduceThreads, 0, stream>>>(part_acc, part_ml, out, head_dim, splits, nullptr,
+                                                                                q_heads, ScoreShape{});
+}
+int attention_reduce_max_splits() { return kMaxSplits; }
 
 // The four waves' partial results, and the page ids of a split (at most the whole block table).
 static size_t decode_smem_bytes(int head_dim, int group, int max_blocks) {

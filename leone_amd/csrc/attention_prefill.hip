@@ -34,6 +34,7 @@
 // the keys of a workgroup are cut into `splits` ranges of whole 64-key stages, one workgroup a range
 // (blockIdx.y), each writes its reference, sum and unnormalised accumulator per (row, head, range),
 // and a second kernel merges the ranges in order.
+#include "attention_merge.h"
 #include "common.h"
 #include "leone_hip.h"
 #include "prefill_order.h"
@@ -566,6 +567,13 @@ attention_prefill_merge_kernel(const float* __restrict__ part_acc, const float* 
         }
     }
 }
+
+void launch_attention_tile_merge(const float* part_acc, const float* part_ml, bf16_t* out, const int* tiles, int n_tiles, int q_heads,
+                                 int head_dim, int splits, hipStream_t stream) {
+    attention_prefill_merge_kernel<<<dim3(n_tiles * kMergeBlocksPerTile, q_heads), kMergeThreads, 0, stream>>>(
+        part_acc, part_ml, out, tiles, q_heads, head_dim, splits, nullptr, ScoreShape{});
+}
+int attention_tile_merge_max_splits() { return kMaxPrefillSplits; }
 
 template <int kD16, bool kShaped>
 static int launch_prefill(const void* q, void* out, const void* k_pool, const void* v_pool, const int* positions,

@@ -1,0 +1,795 @@
+// Attention whose heads' scores are mixed before the softmax, score_h <- sum_g talk[h, g] score_g, on the matrix cores,
+// bfloat16 with float scores: both kernels hold the scores of all query heads of a piece of work in one wave's registers,
+// in an order in which a float matrix instruction mixes them where they lie.
+//
+//   attention_talk_decode   one workgroup takes a query row, all its heads and one split of the keys; its four waves walk
+//       tiles of 32 keys.  S [heads x keys] = Q K^T with v_mfma_f32_16x16x32_bf16, the rows of the other kv heads'
+//       queries zero, so that every kv head's product adds into one tile of scores.  A lane (c, g) then holds key c and
+//       heads 4 g .. 4 g + 3, one a register: register r is the operand "heads 4 g + r" of v_mfma_f32_16x16x4_f32, and four
+//       of those are the mix.  The weights cross to the layout of O^T += V^T P^T through a wave's own piece of shared memory.
+//   attention_talk_prefill  one workgroup takes 16 consecutive rows of a request, all heads, and walks the keys 64 at a
+//       time, a wave 16 of them: S^T [keys x rows] of every head, so that a lane holds one row and four keys and every head
+//       a register: v_mfma_f32_4x4x1_16b_f32 with its first operand broadcast (a column of talk) mixes them, four
+//       heads an instruction.  The weights go to shared memory, and for O^T += V^T P^T a wave takes a quarter of the heads
+//       over all 64 keys.
+//
+// The softmax is that of the other kernels: powers of two against a reference that is a whole number, raised only when a
+// score outgrows it by 2^8; row sums over the rounded weights.  talk comes times scale * log2(e), in float.
+#include "attention_merge.h"
+#include "common.h"
+#include "leone_hip.h"
+
+#include <math.h>
+
+namespace leone {
+
+typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8;
+typedef __attribute__((__vector_size__(2 * sizeof(__bf16)))) __bf16 bf16x2;
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4;
+
+constexpr int kTalkThreads = 256;
+constexpr int kTalkWaves = 4;
+constexpr float kTalkRaise = 8.0f;
+constexpr float kLog2e = 1.4426950408889634f;
+
+__device__ inline bf16x8 tk_load(const bf16_t* p) { return __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(p)); }
+__device__ inline bf16x8 tk_zero() { return __builtin_bit_cast(bf16x8, uint4{0u, 0u, 0u, 0u}); }
+// Keeps the low or high half of every word where the key it belongs to is one that counts.
+__device__ inline bf16x8 tk_keep(bf16x8 v, int first_key, int lo, int n) {
+    uint4 raw = __builtin_bit_cast(uint4, v);
+    unsigned* w = reinterpret_cast<unsigned*>(&raw);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int e0 = first_key + 2 * i, e1 = e0 + 1;
+        unsigned mask = 0u;
+        if (e0 >= lo && e0 < n) mask |= 0x0000ffffu;
+        if (e1 >= lo && e1 < n) mask |= 0xffff0000u;
+        w[i] &= mask;
+    }
+    return __builtin_bit_cast(bf16x8, raw);
+}
+
+// ---- single rows -------------------------------------------------------------------------------------------------
+constexpr int kTalkRowStride = 40;         // elements from head to head of a wave's weights in shared memory (32 keys and room)
+
+struct TalkArgs {
+    const bf16_t* q;
+    const bf16_t* k_pool;
+    const bf16_t* v_pool;
+    AnyVec talk;
+    const int* positions;
+    const int* block_table;
+    int max_blocks;
+    float* part_acc;
+    float* part_ml;
+    bf16_t* out;
+    int q_heads, kv_heads, head_dim, v_dim, page_shift;
+    float to_log2;
+    int splits;
+};
+
+template <int kSize, int kHT>
+__global__ void __launch_bounds__(kTalkThreads, 1)
+attention_talk_decode_kernel(TalkArgs a, const int* __restrict__ row_entry, int window) {
+    constexpr int kSteps = kSize / 32;                   // 32-element steps of a key
+    constexpr int kVT = kSize / 16;                      // 16-element tiles of a value
+    constexpr int kRing = 4;                             // pieces of keys or values on their way
+    extern __shared__ float talk_lds[];
+    const int heads = a.q_heads, kv_heads = a.kv_heads, group = heads / kv_heads;
+    const int row = blockIdx.x, split = blockIdx.y;
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave), lane = threadIdx.x % kWave;
+    const int c = lane & 15, g = lane >> 4;
+    const int page_tokens = 1 << a.page_shift, page_mask = page_tokens - 1;
+    float* sm_acc = talk_lds;                                                            // [waves][heads][v_dim]
+    float* sm_m = sm_acc + kTalkWaves * heads * a.v_dim;                                 // [waves][16 kHT]
+    float* sm_l = sm_m + kTalkWaves * 16 * kHT;
+    bf16_t* weights = reinterpret_cast<bf16_t*>(sm_l + kTalkWaves * 16 * kHT);           // [waves][kHT][16][kTalkRowStride]
+    int* pages = reinterpret_cast<int*>(weights + kTalkWaves * kHT * 16 * kTalkRowStride);
+    bf16_t* mine = weights + wave * kHT * 16 * kTalkRowStride;
+
+    const int n = a.positions[row] + 1;
+    const int lo = (window > 0 && n - window > 0) ? n - window : 0;
+    const int t_begin = lo / 32, t_end = (n + 31) / 32;
+    const int per_split = (t_end - t_begin + a.splits - 1) / a.splits;
+    const int my_begin = t_begin + split * per_split;
+    const int my_end = my_begin + per_split < t_end ? my_begin + per_split : t_end;
+    const int* table = a.block_table + static_cast<long>(row_entry[row]) * a.max_blocks;
+    const int first_page = (my_begin * 32) >> a.page_shift;
+    if (my_begin < my_end) {
+        const int last_key = (my_end * 32 < n ? my_end * 32 : n) - 1;
+        const int count = (last_key >> a.page_shift) - first_page + 1;
+        for (int i = threadIdx.x; i < count; i += kTalkThreads) pages[i] = table[first_page + i];
+    }
+    __syncthreads();
+
+    // queries: row c of tile t is head 16 t + c, elements 32 s + 8 g ..; the mix's operands
+    bf16x8 qreg[kHT][kSteps];
+    int kv_of[kHT];                                       // the kv head of this lane's head (as a row and as a column)
+    float mix[kHT][kHT][4];
+#pragma unroll
+    for (int t = 0; t < kHT; ++t) {
+        const int h = 16 * t + c;
+        kv_of[t] = h < heads ? h / group : -1;
+        const bf16_t* from = a.q + (static_cast<long>(row) * heads + (h < heads ? h : 0)) * a.head_dim;
+#pragma unroll
+        for (int s = 0; s < kSteps; ++s) {
+            const int at = 32 * s + 8 * g;
+            qreg[t][s] = (h < heads && at < a.head_dim) ? tk_load(from + at) : tk_zero();
+        }
+#pragma unroll
+        for (int u = 0; u < kHT; ++u)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int in = 16 * u + 4 * g + r;
+                mix[t][u][r] = (h < heads && in < heads) ? load_any(a.talk, static_cast<long>(h) * heads + in) * a.to_log2 : 0.f;
+            }
+    }
+
+    float m_run[kHT][4], l_run[kHT][4];
+    floatx4 acc[kHT][kVT];
+#pragma unroll
+    for (int t = 0; t < kHT; ++t) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            m_run[t][r] = -INFINITY;
+            l_run[t][r] = 0.f;
+        }
+#pragma unroll
+        for (int dt = 0; dt < kVT; ++dt) acc[t][dt] = floatx4{0.f, 0.f, 0.f, 0.f};
+    }
+    bool unmapped = false;
+
+    // A wave's work is a list of pieces: for every tile the keys of each kv head, then the values of each.  Every call of
+    // `issue` gives the same number of loads (a piece that does not exist reads the pool's first page and is not used).
+    bf16x8 ring[kRing][kVT];
+    int ahead_tile = my_begin + wave, ahead_piece = 0;
+    auto issue = [&](bf16x8* to) {
+        const bool exists = ahead_tile < my_end;
+        const int key0 = exists ? ahead_tile * 32 : 0;
+        const bool keys = ahead_piece < kv_heads;
+        const int kvh = !exists ? 0 : keys ? ahead_piece : ahead_piece - kv_heads;
+        if (keys) {
+#pragma unroll
+            for (int half = 0; half < 2; ++half) {
+                const int key = key0 + 16 * half;             // sixteen keys lie in one page
+                int page = exists && key < n ? pages[(key >> a.page_shift) - first_page] : 0;
+                if (page < 0) page = 0;
+                const bf16_t* from = a.k_pool + (static_cast<long>(page) * kv_heads + kvh) * page_tokens * a.head_dim +
+                                     static_cast<long>((key & page_mask) + c) * 8;
+#pragma unroll
+                for (int s = 0; s < kSteps; ++s) {
+                    const int run = 32 * s + 8 * g < a.head_dim ? 4 * s + g : 0;
+                    to[half * kSteps + s] = tk_load(from + static_cast<long>(run) * page_tokens * 8);
+                }
+            }
+        } else {
+            const int key = key0 + 8 * g;
+            int page = exists && key < n ? pages[(key >> a.page_shift) - first_page] : 0;
+            if (page < 0) page = 0;
+            const bf16_t* from = a.v_pool + (static_cast<long>(page) * kv_heads + kvh) * page_tokens * a.v_dim +
+                                 static_cast<long>((key & page_mask) >> 3) * a.v_dim * 8;
+#pragma unroll
+            for (int dt = 0; dt < kVT; ++dt) {
+                const int d = 16 * dt + c < a.v_dim ? 16 * dt + c : 0;
+                to[dt] = tk_load(from + static_cast<long>(d) * 8);
+            }
+        }
+        if (++ahead_piece == 2 * kv_heads) {
+            ahead_piece = 0;
+            ahead_tile += kTalkWaves;
+        }
+    };
+
+    floatx4 sc[kHT][2];
+    bf16x8 pt[kHT];
+    int tile = my_begin + wave, piece = 0;
+    auto finish = [&](bf16x8* from) {
+        const int key0 = tile * 32;
+        const bool full = key0 >= lo && key0 + 32 <= n;
+        if (piece < kv_heads) {
+            if (piece == 0) {
+#pragma unroll
+                for (int t = 0; t < kHT; ++t) sc[t][0] = sc[t][1] = floatx4{0.f, 0.f, 0.f, 0.f};
+            }
+#pragma unroll
+            for (int t = 0; t < kHT; ++t) {
+                if ((piece + 1) * group <= 16 * t || piece * group >= 16 * (t + 1)) continue;       // no head of this kv head
+#pragma unroll
+                for (int s = 0; s < kSteps; ++s) {
+                    const bf16x8 rows = kv_of[t] == piece ? qreg[t][s] : tk_zero();
+                    sc[t][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(rows, from[s], sc[t][0], 0, 0, 0);
+                    sc[t][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(rows, from[kSteps + s], sc[t][1], 0, 0, 0);
+                }
+            }
+            if (piece == kv_heads - 1) {
+                // lane (c, g): scores of key c (and 16 + c) for heads 16 t + 4 g + r.  Mixed, masked, weighed.
+                floatx4 mixed[kHT][2];
+#pragma unroll
+                for (int t = 0; t < kHT; ++t)
+#pragma unroll
+                    for (int half = 0; half < 2; ++half) {
+                        floatx4 sum = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                        for (int u = 0; u < kHT; ++u)
+#pragma unroll
+                            for (int r = 0; r < 4; ++r)
+                                sum = __builtin_amdgcn_mfma_f32_16x16x4f32(mix[t][u][r], sc[u][half][r], sum, 0, 0, 0);
+                        const int key = key0 + 16 * half + c;
+                        if (!full && !(key >= lo && key < n)) sum = floatx4{-INFINITY, -INFINITY, -INFINITY, -INFINITY};
+                        mixed[t][half] = sum;
+                    }
+                if (pages[(key0 >> a.page_shift) - first_page] < 0 ||
+                    (key0 + 16 < n && pages[((key0 + 16) >> a.page_shift) - first_page] < 0))
+                    unmapped = true;                          // the result is poisoned below
+                bool raise = false;
+#pragma unroll
+                for (int t = 0; t < kHT; ++t)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r)
+                        raise = raise || fmaxf(mixed[t][0][r], mixed[t][1][r]) > m_run[t][r] + kTalkRaise;
+                if (__any(raise)) {
+#pragma unroll
+                    for (int t = 0; t < kHT; ++t) {
+                        float alpha[4];
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) {
+                            float top = fmaxf(mixed[t][0][r], mixed[t][1][r]);
+#pragma unroll
+                            for (int off = 1; off < 16; off <<= 1) top = fmaxf(top, __shfl_xor(top, off, kWave));
+                            const float m_new = fmaxf(m_run[t][r], ceilf(top));
+                            alpha[r] = m_new == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(m_run[t][r] - m_new);
+                            m_run[t][r] = m_new;
+                            l_run[t][r] *= alpha[r];
+                        }
+                        // the sums' columns are heads: column c's factor sits in the lanes of group c / 4, register c % 4
+                        float factor = 0.f;
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) {
+                            const float got = __shfl(alpha[r], (c >> 2) * 16, kWave);
+                            if ((c & 3) == r) factor = got;
+                        }
+#pragma unroll
+                        for (int dt = 0; dt < kVT; ++dt)
+#pragma unroll
+                            for (int r = 0; r < 4; ++r) acc[t][dt][r] *= factor;
+                    }
+                }
+#pragma unroll
+                for (int t = 0; t < kHT; ++t)
+#pragma unroll
+                    for (int half = 0; half < 2; ++half)
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) {
+                            const float ref = m_run[t][r] == -INFINITY ? 0.f : m_run[t][r];
+                            const uint16_t bits = bf16_bits_from_float(__builtin_amdgcn_exp2f(mixed[t][half][r] - ref));
+                            l_run[t][r] += __uint_as_float(static_cast<unsigned>(bits) << 16);
+                            mine[(t * 16 + 4 * g + r) * kTalkRowStride + 16 * half + c].bits = bits;
+                        }
+                __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+                __builtin_amdgcn_wave_barrier();
+#pragma unroll
+                for (int t = 0; t < kHT; ++t) pt[t] = tk_load(mine + (t * 16 + c) * kTalkRowStride + 8 * g);
+                __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+                __builtin_amdgcn_wave_barrier();
+            }
+        } else {
+            const int kvh = piece - kv_heads;
+            if (!full) {                                      // slots outside the keys may hold anything, even NaN
+#pragma unroll
+                for (int dt = 0; dt < kVT; ++dt) from[dt] = tk_keep(from[dt], key0 + 8 * g, lo, n);
+            }
+#pragma unroll
+            for (int t = 0; t < kHT; ++t) {
+                if ((kvh + 1) * group <= 16 * t || kvh * group >= 16 * (t + 1)) continue;
+                const bf16x8 columns = kv_of[t] == kvh ? pt[t] : tk_zero();
+#pragma unroll
+                for (int dt = 0; dt < kVT; ++dt) acc[t][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(from[dt], columns, acc[t][dt], 0, 0, 0);
+            }
+        }
+        if (++piece == 2 * kv_heads) {
+            piece = 0;
+            tile += kTalkWaves;
+        }
+    };
+
+    if (tile < my_end) {
+#pragma unroll
+        for (int i = 0; i < kRing; ++i) issue(ring[i]);
+        while (true) {
+            bool more = true;
+#pragma unroll
+            for (int i = 0; i < kRing; ++i) {
+                if (more) {
+                    finish(ring[i]);
+                    issue(ring[i]);
+                    more = tile < my_end;
+                }
+            }
+            if (!more) break;
+        }
+    }
+
+    // ---- merge the four waves
+#pragma unroll
+    for (int t = 0; t < kHT; ++t) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            float l = l_run[t][r];
+#pragma unroll
+            for (int off = 1; off < 16; off <<= 1) l += __shfl_xor(l, off, kWave);
+            if (unmapped) l = __builtin_nanf("");
+            if (c == 0) {
+                sm_m[wave * 16 * kHT + 16 * t + 4 * g + r] = m_run[t][r];
+                sm_l[wave * 16 * kHT + 16 * t + 4 * g + r] = l;
+            }
+        }
+        const int h = 16 * t + c;
+        if (h < heads) {
+#pragma unroll
+            for (int dt = 0; dt < kVT; ++dt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int d = 16 * dt + 4 * g + r;
+                    if (d < a.v_dim) sm_acc[(static_cast<long>(wave) * heads + h) * a.v_dim + d] = acc[t][dt][r];
+                }
+        }
+    }
+    __syncthreads();
+    for (int i = threadIdx.x; i < heads * a.v_dim; i += kTalkThreads) {
+        const int h = i / a.v_dim, d = i % a.v_dim;
+        float top = -INFINITY;
+#pragma unroll
+        for (int w = 0; w < kTalkWaves; ++w) top = fmaxf(top, sm_m[w * 16 * kHT + h]);
+        float num = 0.f, den = 0.f;
+        if (top != -INFINITY) {
+#pragma unroll
+            for (int w = 0; w < kTalkWaves; ++w) {
+                const float mw = sm_m[w * 16 * kHT + h];
+                const float weight = mw == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(mw - top);
+                num += sm_acc[(static_cast<long>(w) * heads + h) * a.v_dim + d] * weight;
+                den += sm_l[w * 16 * kHT + h] * weight;
+            }
+        }
+        const long rh = static_cast<long>(row) * heads + h;
+        if (a.splits == 1) {
+            a.out[rh * a.v_dim + d] = from_float<bf16_t>(num / den);
+            continue;
+        }
+        const long slot = rh * a.splits + split;
+        a.part_acc[slot * a.v_dim + d] = num;
+        if (d == 0) {
+            a.part_ml[slot * 2] = top;
+            a.part_ml[slot * 2 + 1] = den;
+        }
+    }
+}
+
+static size_t talk_decode_shared(int heads, int v_dim, int tiles, int max_blocks) {
+    return (static_cast<size_t>(kTalkWaves) * heads * v_dim + 2 * kTalkWaves * 16 * tiles) * sizeof(float) +
+           static_cast<size_t>(kTalkWaves) * tiles * 16 * kTalkRowStride * sizeof(bf16_t) + static_cast<size_t>(max_blocks) * sizeof(int);
+}
+
+constexpr size_t kTalkMostShared = 160 * 1024;
+
+// ---- tiles of rows -----------------------------------------------------------------------------------------------
+constexpr int kTalkRows = 16;
+constexpr int kTalkStage = 64;             // keys of a stage: sixteen a wave
+
+template <int kSize, int kHB>
+__host__ __device__ constexpr size_t talk_prefill_fixed() {
+    // queries [heads][kSize / 8 runs][16 rows], weights [heads][8 runs][16 rows] (16-byte runs), maxima [waves][heads][16], flags
+    return static_cast<size_t>(4 * kHB) * (kSize / 8) * 16 * 16 + static_cast<size_t>(4 * kHB) * 8 * 16 * 16 +
+           static_cast<size_t>(kTalkWaves) * 4 * kHB * 16 * 4 + 16;
+}
+
+// kHB: blocks of four heads (heads beyond q_heads are zero).  kLG: heads that share one load of keys.
+template <int kSize, int kHB, int kLG>
+__global__ void __launch_bounds__(kTalkThreads, 1)
+attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_tiles) {
+    constexpr int kH = 4 * kHB;
+    constexpr int kSteps = kSize / 32, kVT = kSize / 16, kRuns = kSize / 8;
+    constexpr int kLoads = kH / kLG;                         // loads of keys a stage
+    constexpr int kRing = kLoads < 4 ? kLoads : 4;
+    constexpr int kPG = kLG < kHB ? kLG : kHB;               // heads of a wave that share one load of values
+    constexpr int kMixRegs = (kH + 15) / 16;
+    extern __shared__ uint4 talk_shared[];
+    uint4* sq = talk_shared;                                 // [head][run][row]
+    uint4* sp = sq + kH * kRuns * 16;                        // [head][run of 8 keys][row]
+    float* smax = reinterpret_cast<float*>(sp + kH * 8 * 16);   // [wave][head][row]
+    int* flags = reinterpret_cast<int*>(smax + kTalkWaves * kH * 16);   // [2] raise, [2] unmapped
+    int* pages = flags + 4;
+
+    const int heads = a.q_heads, kv_heads = a.kv_heads, group = heads / kv_heads;
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave), lane = threadIdx.x % kWave, tid = threadIdx.x;
+    const int c = lane & 15, g = lane >> 4;
+    const int page_tokens = 1 << a.page_shift, page_mask = page_tokens - 1;
+    const int* my_tile = tiles + 3 * static_cast<long>(n_tiles - 1 - static_cast<int>(blockIdx.x));   // the longest first
+    const int entry = my_tile[0], row0 = my_tile[1], rows = my_tile[2];
+    if (rows <= 0) return;
+    const int p0 = a.positions[row0], p_last = p0 + rows - 1, n = p_last + 1;
+    const int row_pos = c < rows ? p0 + c : -1;              // -1: sees no key
+    const int split = blockIdx.y;
+    const int stages = (n + kTalkStage - 1) / kTalkStage;
+    const int share = (stages + a.splits - 1) / a.splits;
+    const int st_begin = split * share, st_end = st_begin + share < stages ? st_begin + share : stages;
+    if (st_begin >= st_end) {                                // more parts than stages: nothing of this one
+        for (int i = tid; i < rows * heads; i += kTalkThreads) {
+            const long slot = ((static_cast<long>(row0) + i / heads) * heads + i % heads) * a.splits + split;
+            a.part_ml[2 * slot] = -INFINITY;
+            a.part_ml[2 * slot + 1] = 0.f;
+        }
+        return;
+    }
+    const int key_begin = st_begin * kTalkStage, key_end = st_end * kTalkStage < n ? st_end * kTalkStage : n;
+    const int first_page = key_begin >> a.page_shift;
+    const int n_pages = ((key_end - 1) >> a.page_shift) - first_page + 1;
+    const int* table = a.block_table + static_cast<long>(entry) * a.max_blocks;
+    for (int i = tid; i < n_pages; i += kTalkThreads) pages[i] = table[first_page + i];
+    if (tid < 4) flags[tid] = 0;
+    for (int i = tid; i < kH * kRuns * 16; i += kTalkThreads) {
+        const int r = i % 16, run = (i / 16) % kRuns, h = i / (16 * kRuns);
+        sq[i] = (h < heads && r < rows && 8 * run < a.head_dim)
+                    ? *reinterpret_cast<const uint4*>(a.q + ((static_cast<long>(row0) + r) * heads + h) * a.head_dim + 8 * run)
+                    : uint4{0u, 0u, 0u, 0u};
+    }
+    // the mix, four output heads and sixteen input heads a register: lane 4 b + i holds talk[4 block + i][16 part + b]
+    float mix[kHB][kMixRegs];
+#pragma unroll
+    for (int b = 0; b < kHB; ++b)
+#pragma unroll
+        for (int part = 0; part < kMixRegs; ++part) {
+            const int to = 4 * b + (lane & 3), in = 16 * part + (lane >> 2);
+            mix[b][part] = (to < heads && in < heads) ? load_any(a.talk, static_cast<long>(to) * heads + in) * a.to_log2 : 0.f;
+        }
+    __syncthreads();
+
+    auto page_of = [&](int key) {                             // a page that is not there reads page 0 and poisons the result
+        const int page = key < n ? pages[(key >> a.page_shift) - first_page] : 0;
+        return page;
+    };
+    bf16x8 kx[kRing][kSteps];
+    auto fetch_keys = [&](int st, int load, bf16x8* to) {
+        const bool exists = st < st_end;
+        const int key = exists ? st * kTalkStage + 16 * wave : key_begin;
+        const int page = page_of(key);
+        int kvh = load * kLG / group;
+        kvh = kvh < kv_heads ? kvh : kv_heads - 1;
+        const bf16_t* from = a.k_pool + (static_cast<long>(page < 0 ? 0 : page) * kv_heads + kvh) * page_tokens * a.head_dim +
+                             static_cast<long>((key & page_mask) + c) * 8;
+#pragma unroll
+        for (int s = 0; s < kSteps; ++s) {
+            const int run = 32 * s + 8 * g < a.head_dim ? 4 * s + g : 0;
+            to[s] = tk_load(from + static_cast<long>(run) * page_tokens * 8);
+        }
+    };
+    bf16x8 vx[2][kVT];
+    auto fetch_values = [&](int st, int h) {
+        int kvh = h / group;
+        kvh = kvh < kv_heads ? kvh : kv_heads - 1;
+#pragma unroll
+        for (int ks = 0; ks < 2; ++ks) {
+            const int key = st * kTalkStage + 32 * ks + 8 * g;
+            const int page = page_of(key);
+            const bf16_t* from = a.v_pool + (static_cast<long>(page < 0 ? 0 : page) * kv_heads + kvh) * page_tokens * a.v_dim +
+                                 static_cast<long>((key & page_mask) >> 3) * a.v_dim * 8;
+#pragma unroll
+            for (int dt = 0; dt < kVT; ++dt) {
+                const int d = 16 * dt + c < a.v_dim ? 16 * dt + c : 0;
+                vx[ks][dt] = tk_load(from + static_cast<long>(d) * 8);
+            }
+        }
+    };
+
+    float m_ref[kH];
+#pragma unroll
+    for (int h = 0; h < kH; ++h) m_ref[h] = -INFINITY;
+    float l_run[kHB];
+    floatx4 acc[kHB][kVT];
+#pragma unroll
+    for (int w = 0; w < kHB; ++w) {
+        l_run[w] = 0.f;
+#pragma unroll
+        for (int dt = 0; dt < kVT; ++dt) acc[w][dt] = floatx4{0.f, 0.f, 0.f, 0.f};
+    }
+#pragma unroll
+    for (int i = 0; i < kRing; ++i) fetch_keys(st_begin, i, kx[i]);
+
+    for (int st = st_begin; st < st_end; ++st) {
+        // ---- S^T of every head: lane (c, g) gets row c's scores of keys 4 g + r of this wave's sixteen
+        floatx4 sc[kH];
+#pragma unroll
+        for (int load = 0; load < kLoads; ++load) {
+            bf16x8* keys = kx[load % kRing];
+#pragma unroll
+            for (int i = 0; i < kLG; ++i) {
+                const int h = load * kLG + i;
+                floatx4 sum = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int s = 0; s < kSteps; ++s)
+                    sum = __builtin_amdgcn_mfma_f32_16x16x32_bf16(keys[s], __builtin_bit_cast(bf16x8, sq[(h * kRuns + 4 * s + g) * 16 + c]), sum, 0, 0, 0);
+                sc[h] = sum;
+            }
+            // the ring's next piece: a later load of this stage, or one of the next stage's first
+            fetch_keys(load + kRing < kLoads ? st : st + 1, (load + kRing) % kLoads, keys);
+        }
+        fetch_values(st, wave * kHB);
+
+        // ---- mixed scores and weights of all heads
+        const int key0 = st * kTalkStage + 16 * wave + 4 * g;
+        const bool full = (st + 1) * kTalkStage <= p0 + 1;
+        uint2 packed[kH];
+        bool raise = false;
+        auto weigh = [&](bool maxima) {
+#pragma unroll
+            for (int b = 0; b < kHB; ++b) {
+                floatx4 d[4];                                 // d[r][i]: head 4 b + i, key 4 g + r
+#pragma unroll
+                for (int r = 0; r < 4; ++r) d[r] = floatx4{0.f, 0.f, 0.f, 0.f};
+#define LEONE_TALK_ONE(PART, I)                                                                                           \
+    if constexpr (16 * (PART) + (I) < kH) {                                                                               \
+        _Pragma("unroll") for (int r = 0; r < 4; ++r)                                                                     \
+            d[r] = __builtin_amdgcn_mfma_f32_4x4x1f32(mix[b][PART], sc[16 * (PART) + (I)][r], d[r], 4, I, 0);             \
+    }
+#define LEONE_TALK_FOUR(PART, I) LEONE_TALK_ONE(PART, I) LEONE_TALK_ONE(PART, I + 1) LEONE_TALK_ONE(PART, I + 2) LEONE_TALK_ONE(PART, I + 3)
+                LEONE_TALK_FOUR(0, 0) LEONE_TALK_FOUR(0, 4) LEONE_TALK_FOUR(0, 8) LEONE_TALK_FOUR(0, 12)
+                if constexpr (kMixRegs > 1) {
+                    LEONE_TALK_FOUR(1, 0) LEONE_TALK_FOUR(1, 4) LEONE_TALK_FOUR(1, 8) LEONE_TALK_FOUR(1, 12)
+                }
+#undef LEONE_TALK_FOUR
+#undef LEONE_TALK_ONE
+                if (!full) {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r)
+                        if (key0 + r > row_pos) d[r] = floatx4{-INFINITY, -INFINITY, -INFINITY, -INFINITY};
+                }
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int h = 4 * b + i;
+                    float top = fmaxf(fmaxf(d[0][i], d[1][i]), fmaxf(d[2][i], d[3][i]));
+                    if (maxima) {
+                        top = fmaxf(top, __shfl_xor(top, 16, kWave));
+                        top = fmaxf(top, __shfl_xor(top, 32, kWave));
+                        if (g == 0) smax[(wave * kH + h) * 16 + c] = top;
+                    } else {
+                        raise = raise || top > m_ref[h] + kTalkRaise;
+                        const float ref = m_ref[h] == -INFINITY ? 0.f : m_ref[h];
+                        uint16_t bits[4];
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) bits[r] = bf16_bits_from_float(__builtin_amdgcn_exp2f(d[r][i] - ref));
+                        packed[h].x = bits[0] | (static_cast<unsigned>(bits[1]) << 16);
+                        packed[h].y = bits[2] | (static_cast<unsigned>(bits[3]) << 16);
+                    }
+                }
+            }
+        };
+        int* flag = flags + (st & 1);
+        bool maxima = st == st_begin;                         // the first scores always raise the references
+        if (!maxima) {
+            weigh(false);
+            if (__any(raise) && lane == 0) *flag = 1;
+        }
+        __syncthreads();                                      // the weights of the stage before have been read
+        if (!maxima) maxima = *flag != 0;
+        if (maxima) {                                         // the same for the whole workgroup
+            weigh(true);
+            __syncthreads();
+            float own[kHB];
+#pragma unroll
+            for (int h = 0; h < kH; ++h) {
+                float top = smax[h * 16 + c];
+#pragma unroll
+                for (int w = 1; w < kTalkWaves; ++w) top = fmaxf(top, smax[(w * kH + h) * 16 + c]);
+                const float m_new = fmaxf(m_ref[h], ceilf(top));
+                const float alpha = m_new == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(m_ref[h] - m_new);
+                m_ref[h] = m_new;
+                if (h / kHB == wave) own[h % kHB] = alpha;
+            }
+#pragma unroll
+            for (int w = 0; w < kHB; ++w) {
+                l_run[w] *= own[w];
+#pragma unroll
+                for (int dt = 0; dt < kVT; ++dt)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) acc[w][dt][r] *= own[w];
+            }
+            weigh(false);
+        }
+        if (page_of(st * kTalkStage + 16 * wave) < 0) flags[2] = 1;
+        if (tid == 0) flags[(st & 1) ^ 1] = 0;                // the next stage's flag: it is set behind the barrier below
+#pragma unroll
+        for (int h = 0; h < kH; ++h)
+            reinterpret_cast<uint2*>(sp)[((h * 8 + 2 * wave + (g >> 1)) * 16 + c) * 2 + (g & 1)] = packed[h];
+        __syncthreads();
+
+        // ---- O^T += V^T P^T: this wave's heads over all of the stage's keys
+        const bool whole = (st + 1) * kTalkStage <= n;
+#pragma unroll
+        for (int w0 = 0; w0 < kHB; w0 += kPG) {
+            if (w0 > 0) fetch_values(st, wave * kHB + w0);
+            if (!whole) {                                     // slots behind the keys may hold anything, even NaN
+#pragma unroll
+                for (int ks = 0; ks < 2; ++ks)
+#pragma unroll
+                    for (int dt = 0; dt < kVT; ++dt) vx[ks][dt] = tk_keep(vx[ks][dt], st * kTalkStage + 32 * ks + 8 * g, 0, n);
+            }
+#pragma unroll
+            for (int i = 0; i < kPG; ++i) {
+                const int w = w0 + i, h = wave * kHB + w;
+#pragma unroll
+                for (int ks = 0; ks < 2; ++ks) {
+                    const uint4 raw = sp[(h * 8 + 4 * ks + g) * 16 + c];
+                    const bf16x8 pt = __builtin_bit_cast(bf16x8, raw);
+                    const unsigned pairs[4] = {raw.x, raw.y, raw.z, raw.w};
+#pragma unroll
+                    for (int j = 0; j < 4; ++j)
+                        l_run[w] = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2, pairs[j]), __builtin_bit_cast(bf16x2, 0x3f803f80u),
+                                                                   l_run[w], false);
+#pragma unroll
+                    for (int dt = 0; dt < kVT; ++dt) acc[w][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vx[ks][dt], pt, acc[w][dt], 0, 0, 0);
+                }
+            }
+        }
+    }
+    const bool poisoned = flags[2] != 0;                      // every write came before the last barrier
+#pragma unroll
+    for (int w = 0; w < kHB; ++w) {
+        const int h = wave * kHB + w;
+        float l = l_run[w];
+        l += __shfl_xor(l, 16, kWave);
+        l += __shfl_xor(l, 32, kWave);
+        if (poisoned) l = __builtin_nanf("");
+        if (h >= heads || c >= rows) continue;
+        const long rh = (static_cast<long>(row0) + c) * heads + h;
+        if (a.splits > 1) {
+            float ref = m_ref[0];
+#pragma unroll
+            for (int j = 1; j < kH; ++j)
+                if (j == h) ref = m_ref[j];
+            const long slot = rh * a.splits + split;
+            if (g == 0) {
+                a.part_ml[2 * slot] = ref;
+                a.part_ml[2 * slot + 1] = l;
+            }
+#pragma unroll
+            for (int dt = 0; dt < kVT; ++dt)
+                if (16 * dt + 4 * g < a.v_dim) *reinterpret_cast<floatx4*>(a.part_acc + slot * a.v_dim + 16 * dt + 4 * g) = acc[w][dt];
+            continue;
+        }
+        const float inv = 1.0f / l;
+#pragma unroll
+        for (int dt = 0; dt < kVT; ++dt) {
+            const int d = 16 * dt + 4 * g;
+            if (d >= a.v_dim) continue;
+            uint2 two;
+            two.x = bf16_bits_from_float(acc[w][dt][0] * inv) | (static_cast<unsigned>(bf16_bits_from_float(acc[w][dt][1] * inv)) << 16);
+            two.y = bf16_bits_from_float(acc[w][dt][2] * inv) | (static_cast<unsigned>(bf16_bits_from_float(acc[w][dt][3] * inv)) << 16);
+            *reinterpret_cast<uint2*>(a.out + rh * a.v_dim + d) = two;
+        }
+    }
+}
+
+static int raise_shared(const void* kernel, size_t bytes, size_t* allowed, const char* what) {
+    if (bytes <= *allowed) return 0;
+    const hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(bytes));
+    if (e != hipSuccess) {
+        set_error("%s: %zu bytes of shared memory were refused: %s", what, bytes, hipGetErrorString(e));
+        return 1;
+    }
+    *allowed = bytes;
+    return 0;
+}
+
+static int check_talk(const char* what, const TalkArgs& a, int page_tokens, int talk_dtype, int most_heads) {
+    LEONE_REQUIRE(a.q && a.out && a.k_pool && a.v_pool && a.talk.ptr && a.positions && a.block_table, "%s: null pointer", what);
+    LEONE_REQUIRE(talk_dtype == kF32 || talk_dtype == kBF16, "%s: unknown type of the mix", what);
+    LEONE_REQUIRE(a.q_heads > 0 && a.q_heads <= most_heads && a.kv_heads > 0 && a.q_heads % a.kv_heads == 0,
+                  "%s: %d query heads (at most %d) over %d kv heads", what, a.q_heads, most_heads, a.kv_heads);
+    LEONE_REQUIRE(a.head_dim > 0 && a.head_dim % 8 == 0 && a.head_dim <= 128 && a.v_dim > 0 && a.v_dim % 4 == 0 && a.v_dim <= 128,
+                  "%s: heads of %d (a multiple of 8 up to 128) and values of %d elements (a multiple of 4 up to 128)", what, a.head_dim, a.v_dim);
+    LEONE_REQUIRE(page_tokens >= 16 && (page_tokens & (page_tokens - 1)) == 0 && a.max_blocks > 0,
+                  "%s: page_tokens %d must be a power of two, at least 16", what, page_tokens);
+    LEONE_REQUIRE(a.splits >= 1 && (a.splits == 1 || (a.part_acc && a.part_ml)), "%s: %d splits need the workspace", what, a.splits);
+    return 0;
+}
+
+static int shift_of(int page_tokens) {
+    int shift = 0;
+    while ((1 << shift) < page_tokens) ++shift;
+    return shift;
+}
+
+}  // namespace leone
+
+using namespace leone;
+
+extern "C" int leone_attention_talk_tile_rows() { return kTalkRows; }
+
+// bfloat16, up to 32 query heads, heads of a multiple of 8 and values of a multiple of 4 elements up to 128, pages of a
+// power of two of at least 16 tokens.  Workspace for splits > 1: part_acc rows * q_heads * splits * v_dim floats, part_ml
+// rows * q_heads * splits * 2.
+extern "C" int leone_attention_talk_decode(const void* q, void* out, const void* k_pool, const void* v_pool, const void* talk,
+                                           int talk_dtype, const int* positions, const int* row_entry, const int* block_table,
+                                           int max_blocks, float* part_acc, float* part_ml, int rows, int q_heads, int kv_heads,
+                                           int head_dim, int v_dim, int page_tokens, float scale, int window, int splits,
+                                           hipStream_t stream) {
+    const TalkArgs a{static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pool), static_cast<const bf16_t*>(v_pool),
+                     AnyVec{talk, talk_dtype}, positions, block_table, max_blocks, part_acc, part_ml, static_cast<bf16_t*>(out),
+                     q_heads, kv_heads, head_dim, v_dim, shift_of(page_tokens), scale * kLog2e, splits};
+    if (check_talk("attention_talk_decode", a, page_tokens, talk_dtype, 32)) return 1;
+    LEONE_REQUIRE(row_entry && rows > 0 && window >= 0 && splits <= attention_reduce_max_splits(),
+                  "attention_talk_decode: rows %d, window %d, splits %d", rows, window, splits);
+    const int tiles = q_heads <= 16 ? 1 : 2;
+    const size_t shared = talk_decode_shared(q_heads, v_dim, tiles, max_blocks);
+    LEONE_REQUIRE(shared <= kTalkMostShared, "attention_talk_decode: %zu bytes of shared memory are too many", shared);
+    const int size = head_dim > v_dim ? head_dim : v_dim;
+#define LEONE_TALK_DECODE(SIZE, HT)                                                                                               \
+    do {                                                                                                                          \
+        static size_t allowed = 48 * 1024;                                                                                        \
+        if (raise_shared(reinterpret_cast<const void*>(&attention_talk_decode_kernel<SIZE, HT>), shared, &allowed,                \
+                         "attention_talk_decode"))                                                                                \
+            return 1;                                                                                                             \
+        attention_talk_decode_kernel<SIZE, HT><<<dim3(rows, splits), kTalkThreads, shared, stream>>>(a, row_entry, window);       \
+    } while (0)
+    if (size <= 32) {
+        if (tiles == 1) LEONE_TALK_DECODE(32, 1); else LEONE_TALK_DECODE(32, 2);
+    } else if (size <= 64) {
+        if (tiles == 1) LEONE_TALK_DECODE(64, 1); else LEONE_TALK_DECODE(64, 2);
+    } else {
+        if (tiles == 1) LEONE_TALK_DECODE(128, 1); else LEONE_TALK_DECODE(128, 2);
+    }
+#undef LEONE_TALK_DECODE
+    LEONE_LAUNCH_CHECK("attention_talk_decode");
+    if (splits > 1) {
+        launch_attention_reduce(part_acc, part_ml, static_cast<bf16_t*>(out), rows, q_heads, v_dim, splits, stream);
+        LEONE_LAUNCH_CHECK("attention_talk_decode merge");
+    }
+    return 0;
+}
+
+// tiles int32 [n_tiles, 3]: (entry, first row, rows) with at most leone_attention_talk_tile_rows() consecutive rows of one
+// request; up to 16 query heads, otherwise as above.  Workspace for splits > 1: part_acc covered rows * q_heads * splits *
+// v_dim floats, part_ml covered rows * q_heads * splits * 2, `covered rows` one more than the last row a tile names.
+extern "C" int leone_attention_talk_prefill(const void* q, void* out, const void* k_pool, const void* v_pool, const void* talk,
+                                            int talk_dtype, const int* positions, const int* tiles, int n_tiles,
+                                            const int* block_table, int max_blocks, float* part_acc, float* part_ml, int q_heads,
+                                            int kv_heads, int head_dim, int v_dim, int page_tokens, float scale, int splits,
+                                            hipStream_t stream) {
+    const TalkArgs a{static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pool), static_cast<const bf16_t*>(v_pool),
+                     AnyVec{talk, talk_dtype}, positions, block_table, max_blocks, part_acc, part_ml, static_cast<bf16_t*>(out),
+                     q_heads, kv_heads, head_dim, v_dim, shift_of(page_tokens), scale * kLog2e, splits};
+    if (check_talk("attention_talk_prefill", a, page_tokens, talk_dtype, 16)) return 1;
+    LEONE_REQUIRE(tiles && n_tiles > 0 && splits <= attention_tile_merge_max_splits(), "attention_talk_prefill: %d tiles, splits %d", n_tiles, splits);
+    const int size = head_dim > v_dim ? head_dim : v_dim;
+    const bool grouped = (q_heads / kv_heads) % 4 == 0;       // four neighbouring heads read the same keys
+#define LEONE_TALK_PREFILL(SIZE, HB, LG)                                                                                          \
+    do {                                                                                                                          \
+        static size_t allowed = 48 * 1024;                                                                                        \
+        const size_t shared = talk_prefill_fixed<SIZE, HB>() + static_cast<size_t>(max_blocks) * sizeof(int);                     \
+        LEONE_REQUIRE(shared <= kTalkMostShared, "attention_talk_prefill: %zu bytes of shared memory are too many", shared);      \
+        if (raise_shared(reinterpret_cast<const void*>(&attention_talk_prefill_kernel<SIZE, HB, LG>), shared, &allowed,           \
+                         "attention_talk_prefill"))                                                                               \
+            return 1;                                                                                                             \
+        attention_talk_prefill_kernel<SIZE, HB, LG><<<dim3(n_tiles, splits), kTalkThreads, shared, stream>>>(a, tiles, n_tiles);  \
+    } while (0)
+#define LEONE_TALK_SIZES(HB)                                                        \
+    if (size <= 64) {                                                               \
+        if (grouped) LEONE_TALK_PREFILL(64, HB, 4); else LEONE_TALK_PREFILL(64, HB, 1);  \
+    } else {                                                                        \
+        if (grouped) LEONE_TALK_PREFILL(128, HB, 4); else LEONE_TALK_PREFILL(128, HB, 1); \
+    }
+    if (q_heads <= 4) {
+        LEONE_TALK_SIZES(1)
+    } else if (q_heads <= 8) {
+        LEONE_TALK_SIZES(2)
+    } else {
+        LEONE_TALK_SIZES(4)
+    }
+#undef LEONE_TALK_SIZES
+#undef LEONE_TALK_PREFILL
+    LEONE_LAUNCH_CHECK("attention_talk_prefill");
+    if (splits > 1) {
+        launch_attention_tile_merge(part_acc, part_ml, static_cast<bf16_t*>(out), tiles, n_tiles, q_heads, v_dim, splits, stream);
+        LEONE_LAUNCH_CHECK("attention_talk_prefill merge");
+    }
+    return 0;
+}

@@ -414,6 +414,16 @@ int leone_attention_rows_talk(const void* q, void* out, const void* k_pool, cons
                               int talk_dtype, const int* positions, const int* row_entry, const int* block_table, int max_blocks,
                               int rows, int q_heads, int kv_heads, int head_dim, int v_dim, int page_tokens, float scale,
                               int window, hipStream_t stream);
+// The same on the matrix cores, bfloat16 (see attention_talk.hip): single rows with a window, and tiles of 16 rows of prompt portions.
+int leone_attention_talk_tile_rows();
+int leone_attention_talk_decode(const void* q, void* out, const void* k_pool, const void* v_pool, const void* talk, int talk_dtype,
+                                const int* positions, const int* row_entry, const int* block_table, int max_blocks,
+                                float* part_acc, float* part_ml, int rows, int q_heads, int kv_heads, int head_dim, int v_dim,
+                                int page_tokens, float scale, int window, int splits, hipStream_t stream);
+int leone_attention_talk_prefill(const void* q, void* out, const void* k_pool, const void* v_pool, const void* talk, int talk_dtype,
+                                 const int* positions, const int* tiles, int n_tiles, const int* block_table, int max_blocks,
+                                 float* part_acc, float* part_ml, int q_heads, int kv_heads, int head_dim, int v_dim,
+                                 int page_tokens, float scale, int splits, hipStream_t stream);
 // leone_qk_norm_rope_write for projections that still get a bias [all heads' columns], values that are turned by their
 // position, and heads of which only the first norm_count elements exist (the rest are zeros that do not count in a norm).
 int leone_qk_norm_rope_write_turned(const void* qkv, int qkv_dtype, int qkv_planes, long qkv_plane, void* q_out, void* k_pool,

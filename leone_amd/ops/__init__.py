@@ -382,6 +382,91 @@ def attention_rows_talk(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Ten
     return out
 
 
+TALK_TILE_ROWS = 16            # rows of a tile of ``attention_talk_prefill`` (checked against the library)
+TALK_MIN_ROWS = 16             # portions from so many rows on go there
+
+
+def talk_attention_supported(dtype: torch.dtype, q_heads: int, head_dim: int, value_dim: int, page_tokens: int, max_blocks: int = 0) -> dict:
+    """Which matrix-core kernels for mixed scores take this shape: {"decode": ..., "prompt": ...}; the others go to
+    ``attention_rows_talk``.  The prompt kernel's workgroup holds the scores and sums of 16 rows of every head."""
+    fits = (dtype == torch.bfloat16 and head_dim % 8 == 0 and value_dim % 4 == 0 and max(head_dim, value_dim) <= 128
+            and page_tokens >= 16 and page_tokens & (page_tokens - 1) == 0 and 4 * max_blocks <= 32 * 1024)
+    return {"decode": fits and q_heads <= 32, "prompt": fits and q_heads <= 16}
+
+
+def _talk_operands(q, k_pool, v_pool, talk, q_heads: int):
+    rows = q.shape[0]
+    pages, kv_heads, page_tokens, head_dim, value_dim = cache_dims_kv(k_pool, v_pool)
+    if q.shape[1] != q_heads * head_dim:
+        raise KernelError(f"attention: query width {q.shape[1]} is not {q_heads}*{head_dim}")
+    _dev(talk, "talk", None, (q_heads, q_heads))
+    return rows, kv_heads, page_tokens, head_dim, value_dim
+
+
+def attention_talk_decode(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, talk: torch.Tensor, positions: torch.Tensor,
+                          row_entry: torch.Tensor, block_table: torch.Tensor, q_heads: int, scale: float, window: int = 0,
+                          max_context: int = 1, splits: Optional[int] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``attention_rows_talk`` on the matrix cores (bfloat16; ``talk_attention_supported``), a row's keys cut into
+    ``splits`` parts.  ``max_context`` only steers their number."""
+    rows, kv_heads, page_tokens, head_dim, value_dim = _talk_operands(q, k_pool, v_pool, talk, q_heads)
+    if splits is None:
+        reach = min(max_context, window + 32) if window else max_context
+        splits = choose_splits(rows, 1, 1, reach, compute_units(q.device))     # one workgroup takes all heads of a row
+    if out is None:
+        out = torch.empty((rows, q_heads * value_dim), dtype=torch.bfloat16, device=q.device)
+    part_acc = part_ml = None
+    if splits > 1:
+        part_acc = torch.empty((rows * q_heads * splits * value_dim,), dtype=torch.float32, device=q.device)
+        part_ml = torch.empty((rows * q_heads * splits * 2,), dtype=torch.float32, device=q.device)
+    call("leone_attention_talk_decode", _dev(q, "attention q", torch.bfloat16),
+         _dev(out, "attention out", torch.bfloat16, (rows, q_heads * value_dim)), _dev(k_pool, "k pool", torch.bfloat16),
+         _dev(v_pool, "v pool", torch.bfloat16), _dev(talk, "talk"), _code(talk, "talk"),
+         _dev(positions, "positions", torch.int32, (rows,)), _dev(row_entry, "row map", torch.int32, (rows,)),
+         _dev(block_table, "block table", torch.int32), block_table.shape[1], _dev(part_acc, "partials"), _dev(part_ml, "partial sums"),
+         rows, q_heads, kv_heads, head_dim, value_dim, page_tokens, float(scale), int(window), int(splits), _stream())
+    return out
+
+
+def choose_talk_splits(tiles: int, mean_keys: int, units: int = 256) -> int:
+    """Into how many parts the keys of a tile of rows are cut: the number for which rounds of workgroups (one a compute
+    unit) x (stages of 64 keys a part + a start worth 3 + a merge worth 2) come out least."""
+    stages = max(1, -(-mean_keys // 64))
+    best = None
+    for splits in range(1, min(16, stages) + 1):
+        cost = (-(-tiles * splits // units) * (-(-stages // splits) + 3 + (2 if splits > 1 else 0)), splits)
+        if best is None or cost < best:
+            best = cost
+    return best[1]
+
+
+def attention_talk_prefill(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, talk: torch.Tensor,
+                           positions: torch.Tensor, tiles: torch.Tensor, block_table: torch.Tensor, q_heads: int, scale: float,
+                           mean_keys: int = 1, splits: Optional[int] = None, covered_rows: Optional[int] = None) -> torch.Tensor:
+    """``attention_rows_talk`` without a window for the rows that ``tiles`` (int32 [n, 3]: entry, first row, up to
+    TALK_TILE_ROWS consecutive rows of one request) covers; writes into ``out``."""
+    if library().leone_attention_talk_tile_rows() != TALK_TILE_ROWS:
+        raise KernelError("the kernel library was built for another tile size of mixed-score attention")
+    rows, kv_heads, page_tokens, head_dim, value_dim = _talk_operands(q, k_pool, v_pool, talk, q_heads)
+    if tiles.dim() != 2 or tiles.shape[1] != 3:
+        raise KernelError(f"attention_talk_prefill: tiles must be int32 [n, 3], found {tuple(tiles.shape)}")
+    if splits is None:
+        splits = choose_talk_splits(tiles.shape[0], mean_keys, compute_units(q.device))
+    part_acc = part_ml = None
+    if splits > 1:
+        covered = rows if covered_rows is None else covered_rows
+        if not 0 < covered <= rows:
+            raise KernelError(f"attention_talk_prefill: {covered} covered rows of {rows}")
+        part_acc = torch.empty((covered * q_heads * splits * value_dim,), dtype=torch.float32, device=q.device)
+        part_ml = torch.empty((covered * q_heads * splits * 2,), dtype=torch.float32, device=q.device)
+    call("leone_attention_talk_prefill", _dev(q, "attention q", torch.bfloat16),
+         _dev(out, "attention out", torch.bfloat16, (rows, q_heads * value_dim)), _dev(k_pool, "k pool", torch.bfloat16),
+         _dev(v_pool, "v pool", torch.bfloat16), _dev(talk, "talk"), _code(talk, "talk"),
+         _dev(positions, "positions", torch.int32, (rows,)), _dev(tiles, "tiles", torch.int32), tiles.shape[0],
+         _dev(block_table, "block table", torch.int32), block_table.shape[1], _dev(part_acc, "partials"), _dev(part_ml, "partial sums"),
+         q_heads, kv_heads, head_dim, value_dim, page_tokens, float(scale), int(splits), _stream())
+    return out
+
+
 def decode_attention_supported(dtype: torch.dtype, head_dim: int, page_tokens: int, group: int = 1,
                                max_blocks: int = 0) -> bool:
     """Whether the matrix-core kernel takes this case; otherwise ``attention_rows`` does."""

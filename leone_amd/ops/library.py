@@ -117,6 +117,10 @@ _PROTOTYPES = {
                                        c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, P],
     "leone_attention_rows_talk": [P, P, P, P, c_int, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
                                   c_int, P],
+    "leone_attention_talk_decode": [P, P, P, P, P, c_int, P, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
+                                    c_int, c_int, P],
+    "leone_attention_talk_prefill": [P, P, P, P, P, c_int, P, P, c_int, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_float,
+                                     c_int, P],
     "leone_qk_norm_rope_write_turned": [P, c_int, c_int, ctypes.c_long, P, P, P, c_int, P, P, c_int, c_float, P, P, c_int, c_int,
                                         c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, ctypes.c_long,
                                         P, c_int, P, P, c_int, c_int, c_int, P],
@@ -163,6 +167,8 @@ def library() -> ctypes.CDLL:
             lib.leone_gemm_rows_max_rows.argtypes = []
             lib.leone_gemm_rows_chunk.restype = c_int
             lib.leone_gemm_rows_chunk.argtypes = [c_int]
+            lib.leone_attention_talk_tile_rows.restype = c_int
+            lib.leone_attention_talk_tile_rows.argtypes = []
             lib.leone_moe_tile_pairs.restype = c_int
             lib.leone_moe_tile_pairs.argtypes = []
             lib.leone_latent_max_width.restype = c_int

@@ -57,6 +57,8 @@ OPERATIONS = {
     "leone_attention_decode_shaped": "attention",
     "leone_attention_prefill_shaped": "attention",
     "leone_attention_rows_talk": "attention",
+    "leone_attention_talk_decode": "attention",
+    "leone_attention_talk_prefill": "attention",
     "leone_qk_norm_rope_write_turned": "qknorm rope kv",
     "leone_branch_norm": "norm",
     "leone_token_mix": "token mix",

@@ -149,6 +149,8 @@ class GqaAttention(Part):
 
     def row_tiling(self) -> RowTiling:
         """The tiles of the prompt-attention kernel."""
+        if "talk" in self.names:
+            return RowTiling(ops.TALK_TILE_ROWS, 1, ops.TALK_MIN_ROWS)
         return RowTiling(ops.PREFILL_TILE_ROWS, ops.PREFILL_GROUP_TILES, ops.PREFILL_MIN_ROWS)
 
     def tensor_specs(self) -> List[TensorSpec]:
@@ -304,8 +306,12 @@ class GqaAttention(Part):
         split-KV matrix-core kernel that also makes the heads and writes the cache), "split_kv" (the same
         kernel behind the norm/rotation/write kernel) or "rows" (the float kernel for any shape and type);
         ``prompt`` (portions of at least ``ops.PREFILL_MIN_ROWS`` rows): "flash" (the matrix-core prompt
-        kernel), else what single tokens get."""
+        kernel), else what single tokens get.  Heads whose scores are mixed have kernels of their own ("talk_...")."""
         group = self.q_heads // self.kv_heads
+        if "talk" in self.names:
+            kernels = ops.talk_attention_supported(dtype, self.q_heads, self.head_dim, self.value_dim, page_tokens, max_blocks)
+            single = "talk_split_kv" if kernels["decode"] else "talk_rows"
+            return {"decode": single, "prompt": "talk_flash" if kernels["prompt"] and not self.window else single}
         if self._rows_only() or not ops.decode_attention_supported(dtype, self.head_dim, page_tokens, group, max_blocks):
             return {"decode": "rows", "prompt": "rows"}
         rotation = rotation_of(self.position)
@@ -325,8 +331,7 @@ class GqaAttention(Part):
         group = self.q_heads // self.kv_heads
         max_blocks = cache.block_table.shape[1]
         if self.talk is not None:
-            return ops.attention_rows_talk(q, cache.k_pool, cache.v_pool, self.talk, step.positions, step.row_entry,
-                                           cache.block_table, self.q_heads, self.scale, window)
+            return self._attend_talking(q, step, cache, window)
         turn = rotation_of(self.value_position)
         shape = ops.ScoreShape(self.softcap, self.sinks, (turn.cos, turn.sin, turn.pairing) if turn.cos is not None else None)
         if self._rows_only() or \
@@ -355,3 +360,24 @@ class GqaAttention(Part):
         # a gate for every element is a gate a head of one element
         return ops.head_gate(out, gate, self.q_heads * self.value_dim, 1) if self.gate_each else \
             ops.head_gate(out, gate, self.q_heads, self.value_dim)
+
+    def _attend_talking(self, q: torch.Tensor, step: StepContext, cache: KvCacheView, window: int) -> torch.Tensor:
+        """The same for heads whose scores are mixed."""
+        kernels = ops.talk_attention_supported(q.dtype, self.q_heads, self.head_dim, self.value_dim, cache.page_tokens,
+                                               cache.block_table.shape[1])
+        if not kernels["decode"]:
+            return ops.attention_rows_talk(q, cache.k_pool, cache.v_pool, self.talk, step.positions, step.row_entry,
+                                           cache.block_table, self.q_heads, self.scale, window)
+        out = torch.empty((q.shape[0], self.q_heads * self.value_dim), dtype=q.dtype, device=q.device)
+        first = 0
+        tiled = step.tiled.get(self.row_tiling())
+        if tiled is not None and tiled.rows and kernels["prompt"] and not window:
+            ops.attention_talk_prefill(q, out, cache.k_pool, cache.v_pool, self.talk, step.positions, tiled.tiles,
+                                       cache.block_table, self.q_heads, self.scale,
+                                       mean_keys=tiled.mean_keys or step.max_position + 1, covered_rows=tiled.rows)
+            first = tiled.rows
+        if first < step.rows:
+            ops.attention_talk_decode(q[first:], cache.k_pool, cache.v_pool, self.talk, step.positions[first:],
+                                      step.row_entry[first:], cache.block_table, self.q_heads, self.scale, window,
+                                      max_context=step.max_position + 1, out=out[first:])
+        return out

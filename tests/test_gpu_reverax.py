@@ -611,3 +611,68 @@ def test_all_three_attention_kernels_with_caps_sinks_and_turned_results(window, 
             ops.attention_prefill(flat_q, out, k_pool, v_pool, rows_at, tiles, table, q_heads, 1.0, window, mean_keys=300,
                                   splits=splits, shape=shape)
             close(out.float().view(len(positions), q_heads, dim), want, bound, f"prompt kernel, splits {splits}")
+
+
+def talking_reference(q, k, v, talk, positions, scale, window, group):
+    """Plain attention of single rows whose heads' scores are mixed before the softmax."""
+    out = torch.zeros(len(positions), q.shape[1], v.shape[2], dtype=F)
+    keys = torch.arange(k.shape[0])
+    for r, p in enumerate(positions):
+        see = (keys <= p) & ((p - keys < window) if window else torch.ones_like(keys, dtype=torch.bool))
+        score = torch.stack([(k[:, g // group].double() @ q[r, g].double()) * scale for g in range(q.shape[1])])
+        mixed = (talk.double() @ score).masked_fill(~see, float("-inf"))
+        weight = torch.softmax(mixed, dim=-1)
+        for head in range(q.shape[1]):
+            out[r, head] = weight[head] @ v[:, head // group].double()
+    return out
+
+
+@pytest.mark.parametrize("page_tokens", [16, 64])
+@pytest.mark.parametrize("q_heads,kv_heads,dim,vdim,window", [(4, 4, 64, 64, 0), (8, 2, 32, 32, 40), (16, 4, 128, 128, 0), (12, 3, 128, 96, 0),
+                                                              (5, 5, 24, 20, 0), (16, 16, 40, 64, 0), (24, 6, 128, 64, 0), (32, 8, 128, 128, 33),
+                                                              (1, 1, 128, 128, 0), (6, 3, 64, 128, 0), (8, 1, 128, 128, 0), (2, 2, 16, 4, 64)])
+def test_all_three_attention_kernels_with_mixed_scores(q_heads, kv_heads, dim, vdim, window, page_tokens):
+    """The row kernel (float32 and bfloat16), the split-KV kernel (rows one by one, and cut into several parts) and the prompt
+    kernel (portions that continue a request of 100 tokens, one of them of 5 rows, in one range of keys and in several)
+    against plain attention.  Every row's queries point along one key each, another one for every head: its own, the one
+    before, the first, one far back, keys on both sides of a page's and a stage's border; the mix has large entries off
+    its diagonal, so a head reads what others ask for; scores differ by tens, so references are raised along the way."""
+    from leone_amd import ops
+    n, first = 333, 100
+    k, v = planted(n, kv_heads, dim, vdim, 5 + dim)
+    gen = torch.Generator().manual_seed(q_heads)
+    talk = (0.5 * torch.eye(q_heads) + 0.7 * torch.randn(q_heads, q_heads, generator=gen) / math.sqrt(q_heads)).bfloat16()
+    positions = list(range(first, n))
+    q = torch.zeros(len(positions), q_heads, dim)
+    for r, i in enumerate(positions):
+        for head in range(q_heads):
+            kinds = [i, i - 1, 0, i // 2, 63, 64, 15, 16, i - window + 1, i - window]
+            j = min(max(kinds[(r + 3 * head) % (len(kinds) if window else 8)], 0), i)
+            key = k[j, head * kv_heads // q_heads].bfloat16().float()
+            q[r, head] = key / (key @ key) * (4.0 + 10.0 * (r % 3))
+    rows_at = torch.tensor(positions, dtype=torch.int32, device=DEV)
+    entry = torch.zeros(len(positions), dtype=torch.int32, device=DEV)
+    for dtype, bound in ((torch.float32, 2e-5), (torch.bfloat16, 1.5e-2)):
+        want = talking_reference(q.to(dtype).float(), k.to(dtype).float(), v.to(dtype).float(), talk.float(), positions, 1.0, window,
+                                 q_heads // kv_heads)
+        k_pool, v_pool, table = paged(k, v, page_tokens, dtype, 9)
+        flat_q = q.reshape(len(positions), -1).to(dtype).to(DEV)
+        on = talk.to(DEV)
+        out = ops.attention_rows_talk(flat_q, k_pool, v_pool, on, rows_at, entry, table, q_heads, 1.0, window)
+        close(out.float().view(len(positions), q_heads, vdim), want, bound, f"row kernel {dtype}")
+        if dtype == torch.float32:
+            continue
+        kernels = ops.talk_attention_supported(dtype, q_heads, dim, vdim, page_tokens)
+        assert kernels == {"decode": q_heads <= 32, "prompt": q_heads <= 16}
+        for splits in (None, 1, 3, 20):
+            one = ops.attention_talk_decode(flat_q, k_pool, v_pool, on, rows_at, entry, table, q_heads, 1.0, window, max_context=n,
+                                            splits=splits)
+            close(one.float().view(len(positions), q_heads, vdim), want, bound, f"split-KV kernel, splits {splits}")
+        if not kernels["prompt"] or window:
+            continue
+        cuts = [(0, 5)] + [(at, min(16, len(positions) - at)) for at in range(5, len(positions), 16)]
+        tiles = torch.tensor([(0, at, rows) for at, rows in cuts], dtype=torch.int32, device=DEV)
+        for splits in (None, 1, 2, 7):
+            out = torch.full((len(positions), q_heads * vdim), float("nan"), dtype=dtype, device=DEV)
+            ops.attention_talk_prefill(flat_q, out, k_pool, v_pool, on, rows_at, tiles, table, q_heads, 1.0, mean_keys=200, splits=splits)
+            close(out.float().view(len(positions), q_heads, vdim), want, bound, f"prompt kernel, splits {splits}")
