@@ -7,11 +7,11 @@
 //       queries zero, so that every kv head's product adds into one tile of scores.  A lane (c, g) then holds key c and
 //       heads 4 g .. 4 g + 3, one a register: register r is the operand "heads 4 g + r" of v_mfma_f32_16x16x4_f32, and four
 //       of those are the mix.  The weights cross to the layout of O^T += V^T P^T through a wave's own piece of shared memory.
-//   attention_talk_prefill  one workgroup takes 16 consecutive rows of a request, all heads, and walks the keys 64 at a
-//       time, a wave 16 of them: S^T [keys x rows] of every head, so that a lane holds one row and four keys and every head
+//   attention_talk_prefill  one workgroup takes 16 consecutive rows of a request, all heads, and walks the keys 64 or 128 at
+//       a time, a wave 16 of them: S^T [keys x rows] of every head, so that a lane holds one row and four keys and every head
 //       a register: v_mfma_f32_4x4x1_16b_f32 with its first operand broadcast (a column of talk) mixes them, four
-//       heads an instruction.  The weights go to shared memory, and for O^T += V^T P^T a wave takes a quarter of the heads
-//       over all 64 keys.
+//       heads an instruction.  The weights go to shared memory, and for O^T += V^T P^T a wave takes its share of the heads
+//       over all the stage's keys.
 //
 // The softmax is that of the other kernels: powers of two against a reference that is a whole number, raised only when a
 // score outgrows it by 2^8; row sums over the rounded weights.  talk comes times scale * log2(e), in float.
@@ -34,6 +34,11 @@ constexpr float kLog2e = 1.4426950408889634f;
 
 __device__ inline bf16x8 tk_load(const bf16_t* p) { return __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(p)); }
 __device__ inline bf16x8 tk_zero() { return __builtin_bit_cast(bf16x8, uint4{0u, 0u, 0u, 0u}); }
+// Two floats rounded to bfloat16, the first in the low half.
+__device__ inline unsigned tk_pack(float a, float b) {
+    const bf16x2 two = {static_cast<__bf16>(a), static_cast<__bf16>(b)};
+    return __builtin_bit_cast(unsigned, two);
+}
 // Keeps the low or high half of every word where the key it belongs to is one that counts.
 __device__ inline bf16x8 tk_keep(bf16x8 v, int first_key, int lo, int n) {
     uint4 raw = __builtin_bit_cast(uint4, v);
@@ -261,9 +266,9 @@ attention_talk_decode_kernel(TalkArgs a, const int* __restrict__ row_entry, int 
 #pragma unroll
                         for (int r = 0; r < 4; ++r) {
                             const float ref = m_run[t][r] == -INFINITY ? 0.f : m_run[t][r];
-                            const uint16_t bits = bf16_bits_from_float(__builtin_amdgcn_exp2f(mixed[t][half][r] - ref));
-                            l_run[t][r] += __uint_as_float(static_cast<unsigned>(bits) << 16);
-                            mine[(t * 16 + 4 * g + r) * kTalkRowStride + 16 * half + c].bits = bits;
+                            const __bf16 weight = static_cast<__bf16>(__builtin_amdgcn_exp2f(mixed[t][half][r] - ref));
+                            l_run[t][r] += static_cast<float>(weight);
+                            mine[(t * 16 + 4 * g + r) * kTalkRowStride + 16 * half + c].bits = __builtin_bit_cast(uint16_t, weight);
                         }
                 __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
                 __builtin_amdgcn_wave_barrier();
@@ -373,30 +378,38 @@ constexpr size_t kTalkMostShared = 160 * 1024;
 
 // ---- tiles of rows -----------------------------------------------------------------------------------------------
 constexpr int kTalkRows = 16;
-constexpr int kTalkStage = 64;             // keys of a stage: sixteen a wave
+// Waves of a workgroup: two a SIMD where there are heads enough for each to have its own.
+__host__ __device__ constexpr int talk_waves(int blocks) { return blocks == 1 ? 4 : 8; }
 
 template <int kSize, int kHB>
 __host__ __device__ constexpr size_t talk_prefill_fixed() {
-    // queries [heads][kSize / 8 runs][16 rows], weights [heads][8 runs][16 rows] (16-byte runs), maxima [waves][heads][16], flags
-    return static_cast<size_t>(4 * kHB) * (kSize / 8) * 16 * 16 + static_cast<size_t>(4 * kHB) * 8 * 16 * 16 +
-           static_cast<size_t>(kTalkWaves) * 4 * kHB * 16 * 4 + 16;
+    // queries [heads][kSize / 8 runs][16 rows], weights [heads][2 runs a wave][16 rows] (16-byte runs), maxima [waves][heads][16],
+    // references [heads][16], flags
+    return static_cast<size_t>(4 * kHB) * (kSize / 8) * 16 * 16 + static_cast<size_t>(4 * kHB) * 2 * talk_waves(kHB) * 16 * 16 +
+           static_cast<size_t>(talk_waves(kHB) + 1) * 4 * kHB * 16 * 4 + 16;
 }
 
 // kHB: blocks of four heads (heads beyond q_heads are zero).  kLG: heads that share one load of keys.
 template <int kSize, int kHB, int kLG>
-__global__ void __launch_bounds__(kTalkThreads, 1)
+__global__ void __launch_bounds__(talk_waves(kHB) * kWave, talk_waves(kHB) / 4)
 attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_tiles) {
     constexpr int kH = 4 * kHB;
     constexpr int kSteps = kSize / 32, kVT = kSize / 16, kRuns = kSize / 8;
     constexpr int kLoads = kH / kLG;                         // loads of keys a stage
-    constexpr int kRing = kLoads < 4 ? kLoads : 4;
-    constexpr int kPG = kLG < kHB ? kLG : kHB;               // heads of a wave that share one load of values
+    constexpr int kRing = kLoads < 2 ? kLoads : 2;
+    constexpr int kWaves = talk_waves(kHB), kThreads = kWaves * kWave;
+    constexpr int kStage = 16 * kWaves;                      // keys of a stage: sixteen a wave
+    constexpr int kHW = kH / kWaves;                         // heads of a wave in the second product
+    constexpr int kPG = kLG < kHW ? kLG : kHW;               // of these, how many share one load of values
+    constexpr int kHalves = kStage / 64;                     // the second product takes 64 keys at a time
+    constexpr int kPRuns = kStage / 8;
     constexpr int kMixRegs = (kH + 15) / 16;
     extern __shared__ uint4 talk_shared[];
     uint4* sq = talk_shared;                                 // [head][run][row]
     uint4* sp = sq + kH * kRuns * 16;                        // [head][run of 8 keys][row]
-    float* smax = reinterpret_cast<float*>(sp + kH * 8 * 16);   // [wave][head][row]
-    int* flags = reinterpret_cast<int*>(smax + kTalkWaves * kH * 16);   // [2] raise, [2] unmapped
+    float* smax = reinterpret_cast<float*>(sp + kH * kPRuns * 16);   // [wave][head][row]
+    float* sref = smax + kWaves * kH * 16;                      // [head][row]
+    int* flags = reinterpret_cast<int*>(sref + kH * 16);        // [2] raise, [2] unmapped
     int* pages = flags + 4;
 
     const int heads = a.q_heads, kv_heads = a.kv_heads, group = heads / kv_heads;
@@ -409,24 +422,25 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
     const int p0 = a.positions[row0], p_last = p0 + rows - 1, n = p_last + 1;
     const int row_pos = c < rows ? p0 + c : -1;              // -1: sees no key
     const int split = blockIdx.y;
-    const int stages = (n + kTalkStage - 1) / kTalkStage;
+    const int stages = (n + kStage - 1) / kStage;
     const int share = (stages + a.splits - 1) / a.splits;
     const int st_begin = split * share, st_end = st_begin + share < stages ? st_begin + share : stages;
     if (st_begin >= st_end) {                                // more parts than stages: nothing of this one
-        for (int i = tid; i < rows * heads; i += kTalkThreads) {
+        for (int i = tid; i < rows * heads; i += kThreads) {
             const long slot = ((static_cast<long>(row0) + i / heads) * heads + i % heads) * a.splits + split;
             a.part_ml[2 * slot] = -INFINITY;
             a.part_ml[2 * slot + 1] = 0.f;
         }
         return;
     }
-    const int key_begin = st_begin * kTalkStage, key_end = st_end * kTalkStage < n ? st_end * kTalkStage : n;
+    const int key_begin = st_begin * kStage, key_end = st_end * kStage < n ? st_end * kStage : n;
     const int first_page = key_begin >> a.page_shift;
     const int n_pages = ((key_end - 1) >> a.page_shift) - first_page + 1;
     const int* table = a.block_table + static_cast<long>(entry) * a.max_blocks;
-    for (int i = tid; i < n_pages; i += kTalkThreads) pages[i] = table[first_page + i];
+    for (int i = tid; i < n_pages; i += kThreads) pages[i] = table[first_page + i];
     if (tid < 4) flags[tid] = 0;
-    for (int i = tid; i < kH * kRuns * 16; i += kTalkThreads) {
+    for (int i = tid; i < kH * 16; i += kThreads) sref[i] = -INFINITY;
+    for (int i = tid; i < kH * kRuns * 16; i += kThreads) {
         const int r = i % 16, run = (i / 16) % kRuns, h = i / (16 * kRuns);
         sq[i] = (h < heads && r < rows && 8 * run < a.head_dim)
                     ? *reinterpret_cast<const uint4*>(a.q + ((static_cast<long>(row0) + r) * heads + h) * a.head_dim + 8 * run)
@@ -450,7 +464,7 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
     bf16x8 kx[kRing][kSteps];
     auto fetch_keys = [&](int st, int load, bf16x8* to) {
         const bool exists = st < st_end;
-        const int key = exists ? st * kTalkStage + 16 * wave : key_begin;
+        const int key = exists ? st * kStage + 16 * wave : key_begin;
         const int page = page_of(key);
         int kvh = load * kLG / group;
         kvh = kvh < kv_heads ? kvh : kv_heads - 1;
@@ -463,12 +477,12 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
         }
     };
     bf16x8 vx[2][kVT];
-    auto fetch_values = [&](int st, int h) {
+    auto fetch_values = [&](int st, int half, int h) {
         int kvh = h / group;
         kvh = kvh < kv_heads ? kvh : kv_heads - 1;
 #pragma unroll
         for (int ks = 0; ks < 2; ++ks) {
-            const int key = st * kTalkStage + 32 * ks + 8 * g;
+            const int key = st * kStage + 64 * half + 32 * ks + 8 * g;
             const int page = page_of(key);
             const bf16_t* from = a.v_pool + (static_cast<long>(page < 0 ? 0 : page) * kv_heads + kvh) * page_tokens * a.v_dim +
                                  static_cast<long>((key & page_mask) >> 3) * a.v_dim * 8;
@@ -480,13 +494,10 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
         }
     };
 
-    float m_ref[kH];
+    float l_run[kHW];
+    floatx4 acc[kHW][kVT];
 #pragma unroll
-    for (int h = 0; h < kH; ++h) m_ref[h] = -INFINITY;
-    float l_run[kHB];
-    floatx4 acc[kHB][kVT];
-#pragma unroll
-    for (int w = 0; w < kHB; ++w) {
+    for (int w = 0; w < kHW; ++w) {
         l_run[w] = 0.f;
 #pragma unroll
         for (int dt = 0; dt < kVT; ++dt) acc[w][dt] = floatx4{0.f, 0.f, 0.f, 0.f};
@@ -512,14 +523,16 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
             // the ring's next piece: a later load of this stage, or one of the next stage's first
             fetch_keys(load + kRing < kLoads ? st : st + 1, (load + kRing) % kLoads, keys);
         }
-        fetch_values(st, wave * kHB);
 
         // ---- mixed scores and weights of all heads
-        const int key0 = st * kTalkStage + 16 * wave + 4 * g;
-        const bool full = (st + 1) * kTalkStage <= p0 + 1;
+        const int key0 = st * kStage + 16 * wave + 4 * g;
+        const bool full = (st + 1) * kStage <= p0 + 1;
         uint2 packed[kH];
-        bool raise = false;
-        auto weigh = [&](bool maxima) {
+        int* flag = flags + (st & 1);
+        bool maxima = st == st_begin;                         // the first scores always raise the references
+        bool met = false;                                     // the workgroup has met behind the stage before
+        while (true) {                                        // every wave takes the same turns
+            bool raise = false;
 #pragma unroll
             for (int b = 0; b < kHB; ++b) {
                 floatx4 d[4];                                 // d[r][i]: head 4 b + i, key 4 g + r
@@ -542,98 +555,104 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
                     for (int r = 0; r < 4; ++r)
                         if (key0 + r > row_pos) d[r] = floatx4{-INFINITY, -INFINITY, -INFINITY, -INFINITY};
                 }
+                if (maxima) {
 #pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    const int h = 4 * b + i;
-                    float top = fmaxf(fmaxf(d[0][i], d[1][i]), fmaxf(d[2][i], d[3][i]));
-                    if (maxima) {
+                    for (int i = 0; i < 4; ++i) {
+                        float top = fmaxf(fmaxf(d[0][i], d[1][i]), fmaxf(d[2][i], d[3][i]));
                         top = fmaxf(top, __shfl_xor(top, 16, kWave));
                         top = fmaxf(top, __shfl_xor(top, 32, kWave));
-                        if (g == 0) smax[(wave * kH + h) * 16 + c] = top;
-                    } else {
-                        raise = raise || top > m_ref[h] + kTalkRaise;
-                        const float ref = m_ref[h] == -INFINITY ? 0.f : m_ref[h];
-                        uint16_t bits[4];
+                        if (g == 0) smax[(wave * kH + 4 * b + i) * 16 + c] = top;
+                    }
+                } else {
 #pragma unroll
-                        for (int r = 0; r < 4; ++r) bits[r] = bf16_bits_from_float(__builtin_amdgcn_exp2f(d[r][i] - ref));
-                        packed[h].x = bits[0] | (static_cast<unsigned>(bits[1]) << 16);
-                        packed[h].y = bits[2] | (static_cast<unsigned>(bits[3]) << 16);
+                    for (int i = 0; i < 4; ++i) {
+                        const int h = 4 * b + i;
+                        float ref = sref[h * 16 + c];
+                        raise = raise || fmaxf(fmaxf(d[0][i], d[1][i]), fmaxf(d[2][i], d[3][i])) > ref + kTalkRaise;
+                        ref = ref == -INFINITY ? 0.f : ref;
+                        packed[h].x = tk_pack(__builtin_amdgcn_exp2f(d[0][i] - ref), __builtin_amdgcn_exp2f(d[1][i] - ref));
+                        packed[h].y = tk_pack(__builtin_amdgcn_exp2f(d[2][i] - ref), __builtin_amdgcn_exp2f(d[3][i] - ref));
                     }
                 }
+                __builtin_amdgcn_sched_barrier(0);            // block by block: all of them at once do not fit the registers
             }
-        };
-        int* flag = flags + (st & 1);
-        bool maxima = st == st_begin;                         // the first scores always raise the references
-        if (!maxima) {
-            weigh(false);
-            if (__any(raise) && lane == 0) *flag = 1;
-        }
-        __syncthreads();                                      // the weights of the stage before have been read
-        if (!maxima) maxima = *flag != 0;
-        if (maxima) {                                         // the same for the whole workgroup
-            weigh(true);
+            if (!maxima) {
+                if (met) break;
+                if (__any(raise) && lane == 0) *flag = 1;
+                __syncthreads();                              // the weights of the stage before have been read
+                met = true;
+                if (*flag == 0) break;
+                maxima = true;
+                continue;
+            }
             __syncthreads();
-            float own[kHB];
+            met = true;
+            maxima = false;
+            // a wave raises the references of its own heads and carries its sums over
 #pragma unroll
-            for (int h = 0; h < kH; ++h) {
+            for (int w = 0; w < kHW; ++w) {
+                const int h = wave * kHW + w;
                 float top = smax[h * 16 + c];
 #pragma unroll
-                for (int w = 1; w < kTalkWaves; ++w) top = fmaxf(top, smax[(w * kH + h) * 16 + c]);
-                const float m_new = fmaxf(m_ref[h], ceilf(top));
-                const float alpha = m_new == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(m_ref[h] - m_new);
-                m_ref[h] = m_new;
-                if (h / kHB == wave) own[h % kHB] = alpha;
-            }
-#pragma unroll
-            for (int w = 0; w < kHB; ++w) {
-                l_run[w] *= own[w];
+                for (int v = 1; v < kWaves; ++v) top = fmaxf(top, smax[(v * kH + h) * 16 + c]);
+                const float before = sref[h * 16 + c];
+                const float m_new = fmaxf(before, ceilf(top));
+                const float alpha = m_new == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(before - m_new);
+                if (g == 0) sref[h * 16 + c] = m_new;
+                l_run[w] *= alpha;
 #pragma unroll
                 for (int dt = 0; dt < kVT; ++dt)
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) acc[w][dt][r] *= own[w];
+                    for (int r = 0; r < 4; ++r) acc[w][dt][r] *= alpha;
             }
-            weigh(false);
+            __syncthreads();
         }
-        if (page_of(st * kTalkStage + 16 * wave) < 0) flags[2] = 1;
+        if (page_of(st * kStage + 16 * wave) < 0) flags[2] = 1;
         if (tid == 0) flags[(st & 1) ^ 1] = 0;                // the next stage's flag: it is set behind the barrier below
+        fetch_values(st, 0, wave * kHW);
 #pragma unroll
         for (int h = 0; h < kH; ++h)
-            reinterpret_cast<uint2*>(sp)[((h * 8 + 2 * wave + (g >> 1)) * 16 + c) * 2 + (g & 1)] = packed[h];
+            reinterpret_cast<uint2*>(sp)[((h * kPRuns + 2 * wave + (g >> 1)) * 16 + c) * 2 + (g & 1)] = packed[h];
         __syncthreads();
 
         // ---- O^T += V^T P^T: this wave's heads over all of the stage's keys
-        const bool whole = (st + 1) * kTalkStage <= n;
 #pragma unroll
-        for (int w0 = 0; w0 < kHB; w0 += kPG) {
-            if (w0 > 0) fetch_values(st, wave * kHB + w0);
-            if (!whole) {                                     // slots behind the keys may hold anything, even NaN
+        for (int half = 0; half < kHalves; ++half) {
+            const int begin = st * kStage + 64 * half;
+            if (begin >= n) continue;                         // the same for the workgroup
+            const bool whole = begin + 64 <= n;
 #pragma unroll
-                for (int ks = 0; ks < 2; ++ks)
+            for (int w0 = 0; w0 < kHW; w0 += kPG) {
+                if (half + w0 > 0) fetch_values(st, half, wave * kHW + w0);
+                if (!whole) {                                 // slots behind the keys may hold anything, even NaN
 #pragma unroll
-                    for (int dt = 0; dt < kVT; ++dt) vx[ks][dt] = tk_keep(vx[ks][dt], st * kTalkStage + 32 * ks + 8 * g, 0, n);
-            }
+                    for (int ks = 0; ks < 2; ++ks)
 #pragma unroll
-            for (int i = 0; i < kPG; ++i) {
-                const int w = w0 + i, h = wave * kHB + w;
+                        for (int dt = 0; dt < kVT; ++dt) vx[ks][dt] = tk_keep(vx[ks][dt], begin + 32 * ks + 8 * g, 0, n);
+                }
 #pragma unroll
-                for (int ks = 0; ks < 2; ++ks) {
-                    const uint4 raw = sp[(h * 8 + 4 * ks + g) * 16 + c];
-                    const bf16x8 pt = __builtin_bit_cast(bf16x8, raw);
-                    const unsigned pairs[4] = {raw.x, raw.y, raw.z, raw.w};
+                for (int i = 0; i < kPG; ++i) {
+                    const int w = w0 + i, h = wave * kHW + w;
 #pragma unroll
-                    for (int j = 0; j < 4; ++j)
-                        l_run[w] = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2, pairs[j]), __builtin_bit_cast(bf16x2, 0x3f803f80u),
-                                                                   l_run[w], false);
+                    for (int ks = 0; ks < 2; ++ks) {
+                        const uint4 raw = sp[(h * kPRuns + 8 * half + 4 * ks + g) * 16 + c];
+                        const bf16x8 pt = __builtin_bit_cast(bf16x8, raw);
+                        const unsigned pairs[4] = {raw.x, raw.y, raw.z, raw.w};
 #pragma unroll
-                    for (int dt = 0; dt < kVT; ++dt) acc[w][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vx[ks][dt], pt, acc[w][dt], 0, 0, 0);
+                        for (int j = 0; j < 4; ++j)
+                            l_run[w] = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2, pairs[j]), __builtin_bit_cast(bf16x2, 0x3f803f80u),
+                                                                       l_run[w], false);
+#pragma unroll
+                        for (int dt = 0; dt < kVT; ++dt) acc[w][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vx[ks][dt], pt, acc[w][dt], 0, 0, 0);
+                    }
                 }
             }
         }
     }
     const bool poisoned = flags[2] != 0;                      // every write came before the last barrier
 #pragma unroll
-    for (int w = 0; w < kHB; ++w) {
-        const int h = wave * kHB + w;
+    for (int w = 0; w < kHW; ++w) {
+        const int h = wave * kHW + w;
         float l = l_run[w];
         l += __shfl_xor(l, 16, kWave);
         l += __shfl_xor(l, 32, kWave);
@@ -641,10 +660,7 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
         if (h >= heads || c >= rows) continue;
         const long rh = (static_cast<long>(row0) + c) * heads + h;
         if (a.splits > 1) {
-            float ref = m_ref[0];
-#pragma unroll
-            for (int j = 1; j < kH; ++j)
-                if (j == h) ref = m_ref[j];
+            const float ref = sref[h * 16 + c];
             const long slot = rh * a.splits + split;
             if (g == 0) {
                 a.part_ml[2 * slot] = ref;
@@ -661,8 +677,8 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
             const int d = 16 * dt + 4 * g;
             if (d >= a.v_dim) continue;
             uint2 two;
-            two.x = bf16_bits_from_float(acc[w][dt][0] * inv) | (static_cast<unsigned>(bf16_bits_from_float(acc[w][dt][1] * inv)) << 16);
-            two.y = bf16_bits_from_float(acc[w][dt][2] * inv) | (static_cast<unsigned>(bf16_bits_from_float(acc[w][dt][3] * inv)) << 16);
+            two.x = tk_pack(acc[w][dt][0] * inv, acc[w][dt][1] * inv);
+            two.y = tk_pack(acc[w][dt][2] * inv, acc[w][dt][3] * inv);
             *reinterpret_cast<uint2*>(a.out + rh * a.v_dim + d) = two;
         }
     }
@@ -769,7 +785,7 @@ extern "C" int leone_attention_talk_prefill(const void* q, void* out, const void
         if (raise_shared(reinterpret_cast<const void*>(&attention_talk_prefill_kernel<SIZE, HB, LG>), shared, &allowed,           \
                          "attention_talk_prefill"))                                                                               \
             return 1;                                                                                                             \
-        attention_talk_prefill_kernel<SIZE, HB, LG><<<dim3(n_tiles, splits), kTalkThreads, shared, stream>>>(a, tiles, n_tiles);  \
+        attention_talk_prefill_kernel<SIZE, HB, LG><<<dim3(n_tiles, splits), talk_waves(HB) * kWave, shared, stream>>>(a, tiles, n_tiles);  \
     } while (0)
 #define LEONE_TALK_SIZES(HB)                                                        \
     if (size <= 64) {                                                               \
