@@ -5,6 +5,8 @@
 //           norm  : X is the float32 residual stream; the operand is bf16(x * gain) and the result is
 //                   scaled by 1/sqrt(mean(x^2) + eps) per row afterwards, which is the same RMSNorm
 //                   (crates/leone/src/cpu.rs:1642-1663) because that factor is constant along a row
+//           planes : X is several bfloat16 [M,K] one behind the other, and every run of `plane_rows` rows of W reads the
+//                   next of them (products of several inputs against matrices that lie together, in one launch)
 //           prepared : X is bfloat16 [M,K] = bf16(x * gain), written by a product before (see `prepare`
 //                   below) together with partial sums of x^2, one for every 16 columns of a row; the
 //                   result is scaled by 1/sqrt(sum / K + eps) as for `norm`, and no kernel runs in between
@@ -54,6 +56,8 @@ struct FusedArgs {
     const void* next_gain;     // prepare: [N]
     int next_gain_dtype;
     int act;                   // gated: the gate's activation (GateAct)
+    int plane_rows = 0;        // plain: rows of W that read one plane of X, a multiple of 16 (0: there is one plane)
+    int planes = 1;
 };
 
 __device__ inline bf16x8 fz8() {
@@ -111,7 +115,12 @@ gemm_fused_kernel(FusedArgs a) {
     constexpr int kQuads = 8;                        // 16-byte loads a thread takes; the entry point checks that they suffice
     extern __shared__ float4 sums_of_squares[];      // [m * k / 64]
     const int quads = kIn == kInPrepared ? m * (k / 64) : 0;
-    const bf16_t* xb = static_cast<const bf16_t*>(a.x) + xrow_index * k + 16 * g;   // plain
+    long plane = 0;
+    if (kIn == kInPlain && a.plane_rows > 0) {
+        plane = n0 / a.plane_rows;
+        plane = plane < a.planes ? plane : a.planes - 1;
+    }
+    const bf16_t* xb = static_cast<const bf16_t*>(a.x) + (plane * m + xrow_index) * k + 16 * g;   // plain
     const float* xf = static_cast<const float*>(a.x) + xrow_index * k + 16 * g;     // norm
     floatx4 acc = {0.f, 0.f, 0.f, 0.f};
 
@@ -377,5 +386,23 @@ extern "C" int leone_gemm_fused_bf16(const void* x, int in_mode, const int* rows
     }
 #undef LEONE_FUSED_OUT
     LEONE_LAUNCH_CHECK("gemm_fused");
+    return 0;
+}
+
+// x bfloat16 [planes, m, k]: rows [p * plane_rows, (p + 1) * plane_rows) of w read plane p (the last plane serves all rows that
+// are left); y of out_dtype [m, n].  plane_rows a multiple of 16; m up to 16.
+extern "C" int leone_gemm_planes_bf16(const void* x, int planes, int plane_rows, const void* w, int w_tiled, void* y, int out_dtype,
+                                      int m, int n, int k, hipStream_t stream) {
+    LEONE_REQUIRE(x && w && y, "gemm_planes: null pointer");
+    LEONE_REQUIRE(!w_tiled || (k % 64 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0),
+                  "gemm_planes: tiled weights need K %d to be a multiple of 64", k);
+    LEONE_REQUIRE(m > 0 && m <= 16 && n > 0 && k > 0 && k % 8 == 0, "gemm_planes: %d rows (1..16), sizes %d x %d, K a multiple of 8", m, n, k);
+    LEONE_REQUIRE(planes >= 1 && plane_rows > 0 && plane_rows % 16 == 0, "gemm_planes: %d planes, %d rows each (a multiple of 16)", planes, plane_rows);
+    LEONE_REQUIRE(out_dtype == kF32 || out_dtype == kBF16, "gemm_planes: unknown output type");
+    FusedArgs a{};
+    a.x = x, a.w = static_cast<const bf16_t*>(w), a.y = y, a.m = m, a.n = n, a.k = k, a.plane_rows = plane_rows, a.planes = planes;
+    if (out_dtype == kF32) launch_fused<kInPlain, kOutStore, float>(a, w_tiled != 0, stream);
+    else launch_fused<kInPlain, kOutStore, bf16_t>(a, w_tiled != 0, stream);
+    LEONE_LAUNCH_CHECK("gemm_planes");
     return 0;
 }

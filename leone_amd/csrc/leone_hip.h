@@ -451,4 +451,10 @@ int leone_time_mix_scan(const float* r, const float* k, const float* v, long str
                         int bonus_dtype, int no_input, int accumulate, const int* segments, int n_segments, const float* state_in,
                         long in_stride, float* state_out, long out_stride, float* decay_product, float* out, int heads, int dim,
                         int vdim, hipStream_t stream);
+int leone_time_mix_read_rows();
+int leone_time_mix_read(const float* r, long stride, const float* decay, const int* segments, int n_segments, const float* state,
+                        long state_stride, float* out, int heads, int dim, int vdim, hipStream_t stream);
+// The weight-streaming product of several inputs against matrices that lie together (see gemm_fused.hip).
+int leone_gemm_planes_bf16(const void* x, int planes, int plane_rows, const void* w, int w_tiled, void* y, int out_dtype, int m,
+                           int n, int k, hipStream_t stream);
 }

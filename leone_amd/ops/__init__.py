@@ -899,13 +899,13 @@ def rows_ways(m: int, waves: int) -> int:
 def gemm_rows(x: torch.Tensor, weight: torch.Tensor, out_dtype: torch.dtype = torch.bfloat16,
               residual: Optional[torch.Tensor] = None, gated: bool = False, splits: Optional[int] = None,
               waves: Optional[int] = None, may_split: bool = True, ways: Optional[int] = None,
-              activation: str = "silu") -> Optional[torch.Tensor]:
+              activation: str = "silu", tiles: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """The weight-streaming product for up to ROWS_MAX rows of bfloat16 ``x``.  With ``residual`` and one
     range of K the product is added into that float32 tensor (None returned); with ``gated`` the weight is
     an interleaved gate/up weight and silu(gate) * up comes out.  With more than one range of K (``splits``;
     by default what ``rows_plan`` finds best, one if ``may_split`` is false or the product is gated) float32
     planes ``[splits, M, N]`` are returned whose sum, in order, is the product (with ``residual``: for the
-    caller to add)."""
+    caller to add).  ``tiles``: the weight's second copy where it is not kept under the weight itself."""
     m, k = x.shape
     n, k2 = weight.shape
     if k != k2:
@@ -939,7 +939,8 @@ def gemm_rows(x: torch.Tensor, weight: torch.Tensor, out_dtype: torch.dtype = to
                            4 if _gate_code(activation) == 1 else 2, torch.bfloat16)
     else:
         out, mode, kind = torch.empty((m, n), dtype=out_dtype, device=weight.device), 0, out_dtype
-    tiles = streamed_copy(weight) if _streamed else None
+    if tiles is None and _streamed:
+        tiles = streamed_copy(weight)
     with profile.span("gemm rows", weight):
         call("leone_gemm_rows_bf16", _dev(x, "gemm x", torch.bfloat16, (m, k)),
              _dev(weight if tiles is None else tiles, "gemm weight", torch.bfloat16), 0 if tiles is None else 1,
@@ -1154,6 +1155,36 @@ def linear(x, weight: torch.Tensor, out_dtype: Optional[torch.dtype] = None,
         if out_dtype != y.dtype:
             y = y.to(out_dtype)
     return swiglu(y, activation=activation) if gated else y
+
+
+def linear_planes(x: torch.Tensor, weight: torch.Tensor, rows_of) -> list:
+    """Products of several inputs ``x[planes, R, K]`` against matrices that lie one behind the other in ``weight[N, K]``
+    (``rows_of`` says how many rows each has): a list of float32 ``[R, rows_of[p]]`` = x[p] . weight_p^T, which may be slices
+    of one wider result.  Few bfloat16 rows against equal matrices of a multiple of 16 rows (the last may be smaller) are one
+    launch; otherwise a product each, as ``linear`` would make it."""
+    planes, rows, k = x.shape
+    rows_of = [int(r) for r in rows_of]
+    if len(rows_of) != planes or sum(rows_of) != weight.shape[0] or weight.shape[1] != k or x.dtype != weight.dtype:
+        raise KernelError(f"linear_planes: inputs {tuple(x.shape)} of {x.dtype} against {tuple(weight.shape)} of {weight.dtype} in {rows_of} rows")
+    starts = [sum(rows_of[:p]) for p in range(planes)]
+    tiles = streamed_copy(weight) if _streamed else None
+    if x.dtype == torch.bfloat16 and rows <= FUSED_ROWS and k % 8 == 0 and rows_of[0] % 16 == 0 \
+            and all(r == rows_of[0] for r in rows_of[:-1]) and rows_of[-1] <= rows_of[0]:
+        out = torch.empty((rows, weight.shape[0]), dtype=torch.float32, device=x.device)
+        with profile.span("gemv fused", weight):
+            call("leone_gemm_planes_bf16", _dev(x, "gemm x", torch.bfloat16), planes, rows_of[0],
+                 _dev(weight if tiles is None else tiles, "gemm weight", torch.bfloat16), 0 if tiles is None else 1,
+                 _dev(out, "gemm out"), F32, rows, weight.shape[0], k, _stream())
+        return [out[:, at:at + r] for at, r in zip(starts, rows_of)]
+    results = []
+    for p, (at, r) in enumerate(zip(starts, rows_of)):
+        part = weight[at:at + r]
+        if x.dtype == torch.bfloat16 and FUSED_ROWS < rows <= ROWS_MAX and k % 8 == 0 and tiles is not None and at % 16 == 0:
+            # the whole matrix's second copy is tiles of 16 rows: a part that begins at one has its own piece of it
+            results.append(gemm_rows(x[p], part, torch.float32, may_split=False, tiles=tiles[at // 16:-(-(at + r) // 16)]))
+        else:
+            results.append(linear(x[p], part, out_dtype=torch.float32))
+    return results
 
 
 def argmax(logits: torch.Tensor) -> torch.Tensor:
@@ -1938,7 +1969,13 @@ def time_mix_scan(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torc
              _dev(state_out, "state written"), state_out.stride(0) if state_out is not None else 0,
              _dev(product, "decay products"), _dev(out, "out"), heads, dim, vdim, _stream())
 
-    _walk_rows(step, walk, state, heads, dim, vdim, write_state)
+    def read(segments, work):
+        call("leone_time_mix_read", r_at, stride, _dev(decay, "decays", torch.float32, (rows, heads * dim)),
+             _dev(segments, "segments", torch.int32), segments.shape[0], _dev(work, "chunk states"), work.stride(0),
+             _dev(out, "out"), heads, dim, vdim, _stream())
+
+    fits = GATED_CHUNKS[0] <= library().leone_time_mix_read_rows()
+    _walk_rows(step, walk, state, heads, dim, vdim, write_state, read=read if fits else None)
     return out
 
 
@@ -1971,11 +2008,11 @@ def low_rank_decay(low: torch.Tensor, w2: torch.Tensor, w0: torch.Tensor) -> tor
     return out
 
 
-def _walk_rows(step, walk, state: torch.Tensor, heads: int, dim: int, vdim: int, write_state: bool) -> None:
+def _walk_rows(step, walk, state: torch.Tensor, heads: int, dim: int, vdim: int, write_state: bool, read=None) -> None:
     """A recurrence S <- diag(decay) S + ... over a step's rows: ``walk(segments, state read, state written, no_input=,
     accumulate=, product=)`` walks segments of rows in order.  Long portions go chunk by chunk side by side: every chunk
     from zeros (leaving what it wrote and the product of its decays), the chunks chained, every chunk again from the
-    state it starts from with nothing written into it."""
+    state it starts from with nothing written into it (by ``read(segments, states)`` if the recurrence has such a kernel)."""
     plan = chunk_plan(step, *GATED_CHUNKS)
     if plan is None:
         walk(entry_spans(step), state, state if write_state else None)
@@ -1987,7 +2024,10 @@ def _walk_rows(step, walk, state: torch.Tensor, heads: int, dim: int, vdim: int,
     call("leone_gated_chain", _dev(plan["links"], "links", torch.int32), plan["links"].shape[0], _dev(work, "work"),
          work.stride(0), _dev(product, "decay products"), _dev(state, "state"), state.stride(0), heads, dim, vdim,
          1 if write_state else 0, _stream())
-    walk(plan["again"], work, None, no_input=True, accumulate=True)
+    if read is not None:
+        read(plan["again"], work)
+    else:
+        walk(plan["again"], work, None, no_input=True, accumulate=True)
     if plan["short"].shape[0]:
         walk(plan["short"], state, state if write_state else None)
 

@@ -40,6 +40,7 @@ _PROTOTYPES = {
     "leone_gemm_f32": [P, P, P, c_int, c_int, c_int, P],
     "leone_gemm_fused_bf16": [P, c_int, P, P, c_int, c_float, P, c_int, P, c_int, c_int, c_int, c_int, c_int, P, P, P, P,
                               c_int, P],
+    "leone_gemm_planes_bf16": [P, c_int, c_int, P, c_int, P, c_int, c_int, c_int, c_int, P],
     "leone_gemm_rows_bf16": [P, P, c_int, P, c_int, c_int, c_int, c_int, c_int, c_int, ctypes.c_long, c_int, c_int, P],
     "leone_gemm_rows_shape_built": [c_int, c_int, c_int],
     "leone_argmax": [P, P, P, P, c_int, c_int, P],
@@ -129,6 +130,7 @@ _PROTOTYPES = {
     "leone_low_rank_decay": [P, ctypes.c_long, P, c_int, P, c_int, P, c_int, c_int, c_int, P],
     "leone_time_mix_scan": [P, P, P, ctypes.c_long, P, P, c_int, c_int, c_int, P, c_int, P, ctypes.c_long, P, ctypes.c_long, P, P,
                             c_int, c_int, c_int, P],
+    "leone_time_mix_read": [P, ctypes.c_long, P, P, c_int, P, ctypes.c_long, P, c_int, c_int, c_int, P],
     "leone_delta_chain": [P, c_int, P, ctypes.c_long, P, P, ctypes.c_long, c_int, c_int, c_int, c_int, P],
 }
 
@@ -169,6 +171,8 @@ def library() -> ctypes.CDLL:
             lib.leone_gemm_rows_chunk.argtypes = [c_int]
             lib.leone_attention_talk_tile_rows.restype = c_int
             lib.leone_attention_talk_tile_rows.argtypes = []
+            lib.leone_time_mix_read_rows.restype = c_int
+            lib.leone_time_mix_read_rows.argtypes = []
             lib.leone_moe_tile_pairs.restype = c_int
             lib.leone_moe_tile_pairs.argtypes = []
             lib.leone_latent_max_width.restype = c_int

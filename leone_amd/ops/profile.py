@@ -29,6 +29,7 @@ OPERATIONS = {
     "leone_attention_rows": "attention",
     "leone_attention_prefill": "attention",
     "leone_gemm_fused_bf16": "gemv fused",
+    "leone_gemm_planes_bf16": "gemv fused",
     "leone_gemm_rows_bf16": "gemm rows",
     "leone_gemm_f32": "gemm f32",
     "leone_swiglu": "swiglu",
@@ -64,6 +65,7 @@ OPERATIONS = {
     "leone_token_mix": "token mix",
     "leone_low_rank_decay": "low rank decay",
     "leone_time_mix_scan": "time mix scan",
+    "leone_time_mix_read": "time mix scan",
     "leone_route_topk": "router",
     "leone_moe_plan": "router",
     "leone_route_plan": "router",

@@ -391,7 +391,7 @@ class TimeMixMixer(Part):
         _check_dim("time_mix", self.dim)
         self.names = {k: p[k] for k in ("r", "k", "v", "g", "o", "norm", "u", "w0", "w1", "w2")}
         self.mu_names = {k: p["mu"][k] for k in self.MIXES}
-        self.mu = self.w_in = self.w_low = self.w_o = self.norm = self.bonus = self.decay_base = self.decay_matrix = None
+        self.mu = self.w_in = self.w_o = self.norm = self.bonus = self.decay_base = self.decay_matrix = None
 
     def tensor_specs(self) -> List[TensorSpec]:
         n, inner = self.names, self.heads * self.dim
@@ -406,14 +406,14 @@ class TimeMixMixer(Part):
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         n = self.names
         self.mu = torch.stack([tensors.pop(self.mu_names[k]) for k in self.MIXES]).contiguous()
-        self.w_in = [tensors.pop(n[k]).contiguous() for k in ("r", "k", "v", "g")]
-        self.w_low = tensors.pop(n["w1"]).contiguous()
+        # the five projections lie together: each reads a mix of its own, all of them are one launch for few rows
+        self.w_in = torch.cat([tensors.pop(n[k]) for k in ("r", "k", "v", "g", "w1")], dim=0).contiguous()
         self.decay_matrix, self.decay_base = tensors.pop(n["w2"]).contiguous(), tensors.pop(n["w0"]).contiguous()
         self.bonus = tensors.pop(n["u"]).reshape(-1).contiguous()
         self.norm, self.w_o = tensors.pop(n["norm"]).contiguous(), tensors.pop(n["o"]).contiguous()
 
     def streamed_weights(self) -> List[torch.Tensor]:
-        return [*self.w_in, self.w_low, self.w_o]
+        return [self.w_in, self.w_o]
 
     def cache_need(self):
         return {"before": StateNeed((self.hidden,), torch.float32),
@@ -422,8 +422,7 @@ class TimeMixMixer(Part):
     def forward(self, h: torch.Tensor, step: StepContext, cache) -> torch.Tensor:
         before, memory = cache["before"], cache["memory"]
         mixed = ops.token_mix(ops.materialize(h), self.mu, before.state, step, write_state=before.writes)
-        r, k, v, gate = (ops.linear(mixed[m], w, out_dtype=torch.float32) for m, w in enumerate(self.w_in))
-        low = ops.linear(mixed[4], self.w_low, out_dtype=torch.float32)
+        r, k, v, gate, low = ops.linear_planes(mixed, self.w_in, [self.heads * self.dim] * 4 + [self.rank])
         decay = ops.low_rank_decay(low, self.decay_matrix, self.decay_base)
         o = ops.time_mix_scan(r, k, v, decay, self.bonus, memory.state, step, self.heads, self.dim, self.dim,
                               write_state=memory.writes)

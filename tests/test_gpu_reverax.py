@@ -541,6 +541,28 @@ def test_token_mix_and_decays_against_torch(dtype_name):
         assert torch.allclose(got, want, atol=2e-6, rtol=1e-4), (rows, channels, rank)
 
 
+@pytest.mark.parametrize("rows", [1, 8, 16, 17, 40, 200])
+def test_products_of_several_inputs_against_matrices_that_lie_together(rows):
+    """One launch for few rows, a product each for more; with the second copies of the matrix the same bits."""
+    from leone_amd import ops
+    gen = torch.Generator().manual_seed(rows)
+    for k, parts, dtype in ((192, [32, 32, 32, 8], torch.bfloat16), (128, [48, 48, 48], torch.bfloat16), (72, [20, 20, 7], torch.bfloat16),
+                            (64, [16, 16], torch.float32), (128, [16, 40], torch.bfloat16)):
+        x = torch.randn(len(parts), rows, k, generator=gen).to(dtype)
+        w = (torch.randn(sum(parts), k, generator=gen) / math.sqrt(k)).to(dtype)
+        on_x, on_w = x.to(DEV), w.to(DEV)
+        got = [t.cpu() for t in ops.linear_planes(on_x, on_w, parts)]
+        at = 0
+        for p, n in enumerate(parts):
+            want = x[p].double() @ w[at:at + n].double().T
+            assert got[p].shape == (rows, n) and torch.allclose(got[p].double(), want, atol=2e-5, rtol=1e-5), (k, parts, p)
+            at += n
+        if dtype == torch.bfloat16 and k % 64 == 0:
+            assert ops.keep_streamed_copy(on_w) > 0
+            again = [t.cpu() for t in ops.linear_planes(on_x, on_w, parts)]
+            assert all(torch.equal(a, b) if rows <= 16 or rows > 128 else torch.allclose(a, b, atol=1e-5) for a, b in zip(got, again)), (k, parts)
+
+
 def shaped_reference(q, k, v, positions, scale, window, cap, sinks, turn, group):
     """Plain attention of single rows: q [rows, H, d] at ``positions`` against all keys k [n, G, d], values v [n, G, e] as they
     are cached; capped scores, a sink a head, results turned back by ``turn`` = (base, whether pairs are neighbours)."""
