@@ -8,10 +8,6 @@
 //                 dt_t = softplus(pre_t + bias),  f_t = exp(-exp(rate_log) * dt_t)  for every key channel of the head,
 //                 S_t = f_t S_(t-1) + (dt_t B_t) x_t^T,   o_t = S_t^T C_t + skip * x_t
 //                 with B and C shared by the heads of a group (head h reads group h / (heads / groups))
-//   time_mix_scan the same walk for a memory whose decays come ready made and whose current token counts by a weight of its
-//                 own until it is written: o_t = (S_(t-1) + diag(bonus) k_t v_t^T)^T r_t, then S_t = diag(w_t) S_(t-1) + k_t v_t^T
-//                 (the read-out of the old state plus v_t times the row's sum of bonus * k * r, which is made once a row)
-//   time_mix_read what a chunk's rows read of the state the chunk starts from, all rows at once (long portions of the same)
 //   gated_chain   chains the end states of chunks that were walked side by side (see below).
 //
 // The layout is that of the other matrix-memory recurrences: a workgroup of four waves owns a run of columns of one
@@ -36,8 +32,6 @@ constexpr int kGsTokens = 16;
 constexpr int kGsLaneRows = 32;      // key channels a lane holds
 constexpr int kGsThreads = 256;
 constexpr int kGsLaneCols = 2;       // columns a lane holds: every q and gate it reads serves both
-constexpr int kGsMixRows = 16;       // the time-mixing form: half the channels and twice the columns a lane, so that a value
-constexpr int kGsMixCols = 4;        // read from shared memory serves four columns
 constexpr int kGsMaxDim = 256;
 
 inline int gs_lane_groups(int dim) { return dim <= 32 ? 1 : dim <= 64 ? 2 : dim <= 128 ? 4 : 8; }
@@ -69,20 +63,12 @@ struct GatedScanArgs {
     long step_stride;
     int step_off;
     AnyVec step_bias, rate_log, skip;   // [heads] each
-    // the time-mixing form: r, k and v at proj, k_at and v_at (all of `stride`, head h at h * dim or h * vdim), the decays
-    // w at decay [rows, heads * dim]
-    const float* k_at = nullptr;
-    const float* v_at = nullptr;
-    const float* decay = nullptr;
-    AnyVec bonus{};                     // [heads * dim]
 };
 
-enum GsKind : int { kGsGated = 0, kGsStateSpace = 1, kGsTimeMix = 2 };
+enum GsKind : int { kGsGated = 0, kGsStateSpace = 1 };
 
 template <bool kTrack, int kKind>
 __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p, int groups) {
-    constexpr int kGsLaneRows = kKind == kGsTimeMix ? kGsMixRows : leone::kGsLaneRows;
-    constexpr int kGsLaneCols = kKind == kGsTimeMix ? kGsMixCols : leone::kGsLaneCols;
     extern __shared__ __align__(16) float gs_lds[];
     const int dkp = groups * kGsLaneRows;
     float* sq = gs_lds;                          // [kGsTokens][dkp]
@@ -115,7 +101,6 @@ __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p,
         for (int i = 0; i < kGsLaneRows; ++i) carried[i] = 1.f;
     }
 
-    __shared__ float s_now[kKind == kGsTimeMix ? kGsTokens : 1];   // the time-mixing form: a row's sum of bonus * k * r
     __shared__ float s_dt[kGsTokens], s_decay[kGsTokens];   // the state-space form: a row's step size and decay, made once
     for (int t0 = 0; t0 < n; t0 += kGsTokens) {
         const int here = min(kGsTokens, n - t0);
@@ -139,14 +124,6 @@ __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p,
                     fv = s_decay[t];
                     kv = p.no_input ? 0.f : s_dt[t] * base[p.k_off + shared_head * p.dim + i];
                 }
-            } else if (kKind == kGsTimeMix) {
-                if (i < p.dim) {
-                    const long r = first + t0 + t;
-                    const int ch = head * p.dim + i;
-                    qv = p.proj[r * p.stride + ch];
-                    fv = p.decay[r * p.heads * p.dim + ch];
-                    kv = p.no_input ? 0.f : p.k_at[r * p.stride + ch];
-                }
             } else if (i < p.dim) {
                 const float* base = p.proj + static_cast<long>(first + t0 + t) * p.stride;
                 const float qp = base[p.q_off + head * p.dim + i];
@@ -162,19 +139,6 @@ __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p,
             sk[idx] = kv;
         }
         __syncthreads();
-        if constexpr (kKind == kGsTimeMix) {
-            // sixteen threads a row
-            for (int t = tid / 16; t < here; t += blockDim.x / 16) {
-                float sum = 0.f;
-                if (!p.no_input)
-                    for (int i = tid % 16; i < p.dim; i += 16)
-                        sum = fmaf(load_any(p.bonus, head * p.dim + i) * sk[t * dkp + i], sq[t * dkp + i], sum);
-#pragma unroll
-                for (int off = 8; off > 0; off >>= 1) sum += __shfl_xor(sum, off, kWave);
-                if (tid % 16 == 0) s_now[t] = sum;
-            }
-            __syncthreads();
-        }
         if (col[0] < p.vdim) {                                  // the lanes of a column are in or out together
             for (int t = 0; t < here; ++t) {
                 const long row = first + t0 + t;
@@ -185,17 +149,15 @@ __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p,
 #pragma unroll
                 for (int c = 0; c < kGsLaneCols; ++c) {
                     acc[c] = 0.f;
-                    const float* v_row = kKind == kGsTimeMix ? p.v_at + row * p.stride : p.proj + row * p.stride + p.v_off;
-                    v[c] = (!p.no_input && col[c] < p.vdim) ? v_row[head * p.vdim + col[c]] : 0.f;
+                    v[c] = (!p.no_input && col[c] < p.vdim) ? p.proj[row * p.stride + p.v_off + head * p.vdim + col[c]] : 0.f;
                 }
 #pragma unroll
                 for (int i = 0; i < kGsLaneRows; ++i) {
                     const float f = ft[i], k = kt[i], q = qt[i];
 #pragma unroll
                     for (int c = 0; c < kGsLaneCols; ++c) {
-                        if constexpr (kKind == kGsTimeMix) acc[c] = fmaf(S[c][i], q, acc[c]);       // the state before this row
                         S[c][i] = fmaf(f, S[c][i], k * v[c]);
-                        if constexpr (kKind != kGsTimeMix) acc[c] = fmaf(S[c][i], q, acc[c]);
+                        acc[c] = fmaf(S[c][i], q, acc[c]);
                     }
                     if constexpr (kTrack) carried[i] *= f;
                 }
@@ -204,9 +166,7 @@ __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p,
                     for (int off = per_wave; off < kWave; off <<= 1) acc[c] += __shfl_xor(acc[c], off, kWave);
                     if (part == 0 && col[c] < p.vdim) {
                         float* dst = p.out + (row * p.heads + head) * p.vdim + col[c];
-                        const float read = kKind == kGsStateSpace ? fmaf(skip, v[c], acc[c])
-                                           : kKind == kGsTimeMix  ? fmaf(s_now[t], v[c], acc[c])
-                                                                  : acc[c];
+                        const float read = kKind == kGsStateSpace ? fmaf(skip, v[c], acc[c]) : acc[c];
                         *dst = p.accumulate ? *dst + read : read;
                     }
                 }
@@ -230,71 +190,6 @@ __global__ void __launch_bounds__(kGsThreads) gated_scan_kernel(GatedScanArgs p,
 #pragma unroll
         for (int i = 0; i < kGsLaneRows; ++i)
             if (ch0 + i < p.dim) to[static_cast<long>(ch0 + i) * p.vdim + col[c]] = S[c][i];
-    }
-}
-
-// What the rows of a chunk read of the state S the chunk starts from, for the time-mixing form: nothing is written into S on
-// the way, so row t reads S scaled by the product of the rows' decays before it, o_t += S^T (r_t * prod_(s < t) w_s), and
-// all rows are one product.  A workgroup takes a segment (up to kReadRows rows) and a head; the scaled r of all rows lie
-// channel by channel in shared memory, S comes by kReadDepth channels at a time, a thread holds 4 rows x 4 columns.
-constexpr int kReadRows = 64;
-constexpr int kReadCols = 64;
-constexpr int kReadDepth = 32;
-
-__global__ void __launch_bounds__(256)
-time_mix_read_kernel(const float* __restrict__ r, long stride, const float* __restrict__ decay, const GsSegment* __restrict__ segments,
-                     const float* __restrict__ state, long state_stride, float* __restrict__ out, int heads, int dim, int vdim) {
-    extern __shared__ __align__(16) float read_lds[];
-    float* scaled = read_lds;                                 // [dim][kReadRows]
-    float* s_state = scaled + dim * kReadRows;                // [kReadDepth][kReadCols]
-    const GsSegment seg = segments[blockIdx.x];
-    const int head = blockIdx.y, tid = threadIdx.x;
-    const int n = seg.end - seg.first;
-    if (seg.in < 0) return;
-    for (int i = tid; i < dim; i += 256) {
-        const float* rp = r + static_cast<long>(seg.first) * stride + head * dim + i;
-        const float* wp = decay + (static_cast<long>(seg.first) * heads + head) * dim + i;
-        float before = 1.f;
-#pragma unroll 8
-        for (int t = 0; t < kReadRows; ++t) {
-            const int at = t < n ? t : n - 1;                 // rows beyond the segment are not stored
-            scaled[i * kReadRows + t] = rp[at * stride] * before;
-            before *= wp[static_cast<long>(at) * heads * dim];
-        }
-    }
-    const int row0 = (tid / 16) * 4, col0 = (tid % 16) * 4;
-    const float* from = state + seg.in * state_stride + static_cast<long>(head) * dim * vdim;
-    for (int base = 0; base < vdim; base += kReadCols) {
-        float sum[4][4];
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-#pragma unroll
-            for (int j = 0; j < 4; ++j) sum[i][j] = 0.f;
-        for (int d0 = 0; d0 < dim; d0 += kReadDepth) {
-            __syncthreads();
-            for (int i = tid; i < kReadDepth * kReadCols; i += 256) {
-                const int d = d0 + i / kReadCols, c = base + i % kReadCols;
-                s_state[i] = (d < dim && c < vdim) ? from[static_cast<long>(d) * vdim + c] : 0.f;
-            }
-            __syncthreads();
-            const int depth = dim - d0 < kReadDepth ? dim - d0 : kReadDepth;
-            for (int d = 0; d < depth; ++d) {
-                const float4 a = *reinterpret_cast<const float4*>(scaled + (d0 + d) * kReadRows + row0);
-                const float4 b = *reinterpret_cast<const float4*>(s_state + d * kReadCols + col0);
-                const float av[4] = {a.x, a.y, a.z, a.w}, bv[4] = {b.x, b.y, b.z, b.w};
-#pragma unroll
-                for (int i = 0; i < 4; ++i)
-#pragma unroll
-                    for (int j = 0; j < 4; ++j) sum[i][j] = fmaf(av[i], bv[j], sum[i][j]);
-            }
-        }
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-#pragma unroll
-            for (int j = 0; j < 4; ++j) {
-                const int t = row0 + i, c = base + col0 + j;
-                if (t < n && c < vdim) out[((static_cast<long>(seg.first) + t) * heads + head) * vdim + c] += sum[i][j];
-            }
     }
 }
 
@@ -393,59 +288,6 @@ extern "C" int leone_state_space_scan(const float* xbc, long stride, int x_off, 
     if (gate_product) gated_scan_kernel<true, kGsStateSpace><<<grid, waves * kWave, shared, stream>>>(a, groups);
     else gated_scan_kernel<false, kGsStateSpace><<<grid, waves * kWave, shared, stream>>>(a, groups);
     LEONE_LAUNCH_CHECK("state_space_scan");
-    return 0;
-}
-
-// The time-mixing form.  r, k, v float [rows, stride] (heads * dim, heads * dim and heads * vdim columns), decay float
-// [rows, heads * dim], bonus [heads * dim] of bonus_dtype.  States, segments, products and out as for leone_gated_scan.
-extern "C" int leone_time_mix_scan(const float* r, const float* k, const float* v, long stride, const float* decay,
-                                   const void* bonus, int bonus_dtype, int no_input, int accumulate, const int* segments,
-                                   int n_segments, const float* state_in, long in_stride, float* state_out, long out_stride,
-                                   float* decay_product, float* out, int heads, int dim, int vdim, hipStream_t stream) {
-    LEONE_REQUIRE(r && k && v && decay && bonus && segments && out, "time_mix_scan: null pointer");
-    LEONE_REQUIRE(bonus_dtype == kF32 || bonus_dtype == kBF16, "time_mix_scan: unknown element type");
-    LEONE_REQUIRE(n_segments > 0 && heads > 0 && heads <= 65535 && dim > 0 && vdim > 0, "time_mix_scan: %d segments, %d heads of %d x %d",
-                  n_segments, heads, dim, vdim);
-    LEONE_REQUIRE(dim <= kGsMaxDim, "time_mix_scan: heads of %d key channels, the kernel takes up to %d", dim, kGsMaxDim);
-    const long per_slot = static_cast<long>(heads) * dim * vdim;
-    LEONE_REQUIRE((!state_in || in_stride >= per_slot) && (!state_out || out_stride >= per_slot),
-                  "time_mix_scan: states of %ld floats do not fit", per_slot);
-    LEONE_REQUIRE(stride >= static_cast<long>(heads) * (dim > vdim ? dim : vdim), "time_mix_scan: rows of %ld do not hold the heads", stride);
-    const AnyVec none{nullptr, bonus_dtype};
-    GatedScanArgs a{r, stride, 0, 0, 0, none, none, 0, no_input, accumulate, reinterpret_cast<const GsSegment*>(segments),
-                    state_in, in_stride, state_out, out_stride, decay_product, out, heads, dim, vdim, heads, 0, nullptr, 0, 0,
-                    none, none, none, k, v, decay, AnyVec{bonus, bonus_dtype}};
-    const int groups = dim <= 16 ? 1 : dim <= 32 ? 2 : dim <= 64 ? 4 : dim <= 128 ? 8 : 16;
-    const int per_wave = (kWave / groups) * kGsMixCols;          // as for the state-space form: no wave stands idle
-    const int waves = ceil_div(vdim, per_wave) < kGsThreads / kWave ? ceil_div(vdim, per_wave) : kGsThreads / kWave;
-    const dim3 grid(n_segments, heads, ceil_div(vdim, waves * per_wave));
-    const size_t shared = 3 * kGsTokens * groups * kGsMixRows * sizeof(float);
-    if (decay_product) gated_scan_kernel<true, kGsTimeMix><<<grid, waves * kWave, shared, stream>>>(a, groups);
-    else gated_scan_kernel<false, kGsTimeMix><<<grid, waves * kWave, shared, stream>>>(a, groups);
-    LEONE_LAUNCH_CHECK("time_mix_scan");
-    return 0;
-}
-
-extern "C" int leone_time_mix_read_rows() { return kReadRows; }
-
-// Adds to out what every segment's rows (at most leone_time_mix_read_rows() each) read of the state named by its third word.
-extern "C" int leone_time_mix_read(const float* r, long stride, const float* decay, const int* segments, int n_segments,
-                                   const float* state, long state_stride, float* out, int heads, int dim, int vdim, hipStream_t stream) {
-    LEONE_REQUIRE(r && decay && segments && state && out, "time_mix_read: null pointer");
-    LEONE_REQUIRE(n_segments > 0 && heads > 0 && heads <= 65535 && dim > 0 && dim <= kGsMaxDim && vdim > 0 &&
-                      stride >= static_cast<long>(heads) * dim && state_stride >= static_cast<long>(heads) * dim * vdim,
-                  "time_mix_read: %d segments, %d heads of %d x %d", n_segments, heads, dim, vdim);
-    const size_t shared = (static_cast<size_t>(dim) * kReadRows + kReadDepth * kReadCols) * sizeof(float);
-    static size_t allowed = 48 * 1024;
-    if (shared > allowed) {
-        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&time_mix_read_kernel), hipFuncAttributeMaxDynamicSharedMemorySize,
-                                                 static_cast<int>(shared));
-        LEONE_REQUIRE(e == hipSuccess, "time_mix_read: %zu bytes of shared memory were refused: %s", shared, hipGetErrorString(e));
-        allowed = shared;
-    }
-    time_mix_read_kernel<<<dim3(n_segments, heads), 256, shared, stream>>>(r, stride, decay, reinterpret_cast<const GsSegment*>(segments),
-                                                                           state, state_stride, out, heads, dim, vdim);
-    LEONE_LAUNCH_CHECK("time_mix_read");
     return 0;
 }
 

@@ -440,17 +440,16 @@ int leone_branch_norm(float* x, const void* const* term_rows, const int* term_pl
                       const float* term_factor, const void* const* term_scale, const int* term_scale_dtype, int terms,
                       const void* const* gains, const int* gain_dtypes, void* const* outs, int norms, int out_dtype, float eps,
                       int groups, const int* rows, int n_rows, int hidden, hipStream_t stream);
-// The token before beside the token itself, decays from a low-rank product, and the memory they drive (see time_mix.hip and
-// gated_scan.hip).
+// The token before beside the token itself, decays from a low-rank product, and the memory they drive (see time_mix.hip).
 int leone_token_mix(const void* h, int dtype, const void* mu, int mu_dtype, int mixes, const float* state, float* state_out,
                     const int* spans, int entries, const int* row_entry, void* out, int rows, int hidden, int single_rows,
                     hipStream_t stream);
 int leone_low_rank_decay(const float* low, long low_stride, const void* w2, int w2_dtype, const void* w0, int w0_dtype, float* out,
                          int rows, int channels, int rank, hipStream_t stream);
 int leone_time_mix_scan(const float* r, const float* k, const float* v, long stride, const float* decay, const void* bonus,
-                        int bonus_dtype, int no_input, int accumulate, const int* segments, int n_segments, const float* state_in,
-                        long in_stride, float* state_out, long out_stride, float* decay_product, float* out, int heads, int dim,
-                        int vdim, hipStream_t stream);
+                        int bonus_dtype, const int* segments, int n_segments, int single_rows, const float* state_in, long in_stride,
+                        float* state_out, long out_stride, float* decay_product, float* out, int heads, int dim, int vdim,
+                        hipStream_t stream);
 int leone_time_mix_read_rows();
 int leone_time_mix_read(const float* r, long stride, const float* decay, const int* segments, int n_segments, const float* state,
                         long state_stride, float* out, int heads, int dim, int vdim, hipStream_t stream);

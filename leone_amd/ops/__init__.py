@@ -1961,10 +1961,12 @@ def time_mix_scan(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torc
         raise KernelError(f"time_mix_scan: r, k and v lie {stride}, {k_stride} and {v_stride} elements apart from row to row")
     out = torch.empty((rows, heads * vdim), dtype=torch.float32, device=r.device)
 
-    def walk(segments, state_in, state_out, no_input=False, accumulate=False, product=None):
+    single_rows = bool(step.decode_only) and step.entry_slots.numel() == rows
+
+    def walk(segments, state_in, state_out, product=None):
         call("leone_time_mix_scan", r_at, k_at, v_at, stride, _dev(decay, "decays", torch.float32, (rows, heads * dim)),
-             _dev(bonus, "bonus", None, (heads * dim,)), _code(bonus, "bonus"), 1 if no_input else 0, 1 if accumulate else 0,
-             _dev(segments, "segments", torch.int32), segments.shape[0],
+             _dev(bonus, "bonus", None, (heads * dim,)), _code(bonus, "bonus"), _dev(segments, "segments", torch.int32),
+             segments.shape[0], 1 if single_rows else 0,
              _dev(state_in, "state read"), state_in.stride(0) if state_in is not None else 0,
              _dev(state_out, "state written"), state_out.stride(0) if state_out is not None else 0,
              _dev(product, "decay products"), _dev(out, "out"), heads, dim, vdim, _stream())
@@ -1974,8 +1976,8 @@ def time_mix_scan(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torc
              _dev(segments, "segments", torch.int32), segments.shape[0], _dev(work, "chunk states"), work.stride(0),
              _dev(out, "out"), heads, dim, vdim, _stream())
 
-    fits = GATED_CHUNKS[0] <= library().leone_time_mix_read_rows()
-    _walk_rows(step, walk, state, heads, dim, vdim, write_state, read=read if fits else None)
+    chunk = min(GATED_CHUNKS[0], library().leone_time_mix_read_rows())
+    _walk_rows(step, walk, state, heads, dim, vdim, write_state, read=read, chunks=(chunk, GATED_CHUNKS[1]))
     return out
 
 
@@ -2008,19 +2010,21 @@ def low_rank_decay(low: torch.Tensor, w2: torch.Tensor, w0: torch.Tensor) -> tor
     return out
 
 
-def _walk_rows(step, walk, state: torch.Tensor, heads: int, dim: int, vdim: int, write_state: bool, read=None) -> None:
+def _walk_rows(step, walk, state: torch.Tensor, heads: int, dim: int, vdim: int, write_state: bool, read=None,
+               chunks: Optional[tuple] = None) -> None:
     """A recurrence S <- diag(decay) S + ... over a step's rows: ``walk(segments, state read, state written, no_input=,
     accumulate=, product=)`` walks segments of rows in order.  Long portions go chunk by chunk side by side: every chunk
     from zeros (leaving what it wrote and the product of its decays), the chunks chained, every chunk again from the
-    state it starts from with nothing written into it (by ``read(segments, states)`` if the recurrence has such a kernel)."""
-    plan = chunk_plan(step, *GATED_CHUNKS)
+    state it starts from with nothing written into it (by ``read(segments, states)`` if the recurrence has such a kernel).
+    ``chunks``: rows of a chunk and the portions walked so, ``GATED_CHUNKS`` if not said."""
+    plan = chunk_plan(step, *(chunks or GATED_CHUNKS))
     if plan is None:
         walk(entry_spans(step), state, state if write_state else None)
         return
-    chunks = plan["chunks"]
-    work = torch.empty((chunks.shape[0], heads, dim * vdim), dtype=torch.float32, device=state.device)
-    product = torch.empty((chunks.shape[0], heads, dim), dtype=torch.float32, device=state.device)
-    walk(chunks, None, work, product=product)
+    listed = plan["chunks"]
+    work = torch.empty((listed.shape[0], heads, dim * vdim), dtype=torch.float32, device=state.device)
+    product = torch.empty((listed.shape[0], heads, dim), dtype=torch.float32, device=state.device)
+    walk(listed, None, work, product=product)
     call("leone_gated_chain", _dev(plan["links"], "links", torch.int32), plan["links"].shape[0], _dev(work, "work"),
          work.stride(0), _dev(product, "decay products"), _dev(state, "state"), state.stride(0), heads, dim, vdim,
          1 if write_state else 0, _stream())

@@ -128,7 +128,7 @@ _PROTOTYPES = {
     "leone_branch_norm": [P, P, P, P, P, P, P, c_int, P, P, P, c_int, c_int, c_float, c_int, P, c_int, c_int, P],
     "leone_token_mix": [P, c_int, P, c_int, c_int, P, P, P, c_int, P, P, c_int, c_int, c_int, P],
     "leone_low_rank_decay": [P, ctypes.c_long, P, c_int, P, c_int, P, c_int, c_int, c_int, P],
-    "leone_time_mix_scan": [P, P, P, ctypes.c_long, P, P, c_int, c_int, c_int, P, c_int, P, ctypes.c_long, P, ctypes.c_long, P, P,
+    "leone_time_mix_scan": [P, P, P, ctypes.c_long, P, P, c_int, P, c_int, c_int, P, ctypes.c_long, P, ctypes.c_long, P, P,
                             c_int, c_int, c_int, P],
     "leone_time_mix_read": [P, ctypes.c_long, P, P, c_int, P, ctypes.c_long, P, c_int, c_int, c_int, P],
     "leone_delta_chain": [P, c_int, P, ctypes.c_long, P, P, ctypes.c_long, c_int, c_int, c_int, c_int, P],

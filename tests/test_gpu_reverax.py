@@ -534,7 +534,7 @@ def test_token_mix_and_decays_against_torch(dtype_name):
                     assert torch.allclose(got[m, at:at + count], want, atol=1e-6 if dtype_name == "float32" else 2e-2), (hidden, e, m)
                 assert torch.equal(kept[slots[e]].cpu(), h[at + count - 1].float())
                 at += count
-    for rows, channels, rank in ((1, 300, 8), (9, 70, 5), (40, 512, 64), (3, 256, 33)):
+    for rows, channels, rank in ((1, 300, 8), (9, 70, 5), (40, 512, 64), (3, 256, 33), (70, 130, 64), (129, 300, 40), (200, 64, 7), (3, 128, 100)):
         low, w2, w0 = torch.randn(rows, rank + 3, generator=gen), torch.randn(channels, rank, generator=gen).to(dtype), torch.randn(channels, generator=gen).to(dtype)
         got = ops.low_rank_decay(low.to(DEV)[:, :rank], w2.to(DEV), w0.to(DEV)).cpu().double()
         want = torch.exp(-torch.exp(torch.tanh(low[:, :rank].double()) @ w2.double().T + w0.double()))
