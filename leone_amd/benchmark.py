@@ -448,13 +448,13 @@ def nogidra_shape(width: int, layers: int, vocab: int, context: int) -> dict:
 
 def reverax_shape(width: int, layers: int, vocab: int, context: int) -> dict:
     """Reverax at layer sizes that resemble published models of its kinds: by turns softmax attention whose heads' scores are
-    mixed (heads of 128, at most 16 of them, four query heads a key head, half a head rotated) and softmax attention with
+    mixed (heads of 128, four query heads a key head, half a head rotated) and softmax attention with
     turned values, capped scores and a sink (heads of 128 with four query heads a key head, half a head rotated, a window
     of 1,024) beside a matrix memory (heads of 64 x 64 over the model's width, a decay of rank 64); norms in four groups;
     the feed-forward by turns dense (3 x width) and 32 ungated experts of 3/8 width of which four are chosen."""
     heads = width // 128
     talking = {"type": "attention",
-               "mixer": {"heads": min(heads, 16), "kv_heads": max(min(heads, 16) // 4, 1), "dim": 128, "vdim": 128,
+               "mixer": {"heads": heads, "kv_heads": width // 512, "dim": 128, "vdim": 128,
                          "scale": 128 ** -0.5, "rot": {"dims": 64, "base": 1000000.0}}}
     side = {"type": "parallel",
             "mixer": {"left": {"heads": heads, "kv_heads": width // 512, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,

@@ -10,7 +10,8 @@
 //   attention_talk_prefill  one workgroup takes 16 consecutive rows of a request, all heads, and walks the keys 64 or 128 at
 //       a time, a wave 16 of them: S^T [keys x rows] of every head, so that a lane holds one row and four keys and every head
 //       a register: v_mfma_f32_4x4x1_16b_f32 with its first operand broadcast (a column of talk) mixes them, four
-//       heads an instruction.  The weights go to shared memory, and for O^T += V^T P^T a wave takes its share of the heads
+//       heads an instruction (more than 16 heads: two workgroups make half the results each, the scores come sixteen heads at
+//       a time and each sixteen add their part of the mix).  The weights go to shared memory, and for O^T += V^T P^T a wave takes its share of the heads
 //       over all the stage's keys.
 //
 // The softmax is that of the other kernels: powers of two against a reference that is a whole number, raised only when a
@@ -378,43 +379,55 @@ constexpr size_t kTalkMostShared = 160 * 1024;
 
 // ---- tiles of rows -----------------------------------------------------------------------------------------------
 constexpr int kTalkRows = 16;
-// Waves of a workgroup: two a SIMD where there are heads enough for each to have its own.
-__host__ __device__ constexpr int talk_waves(int blocks) { return blocks == 1 ? 4 : 8; }
+// A workgroup takes all heads' scores and makes the results of the heads in `blocks` blocks of four: of all of them, or, with
+// more than sixteen heads, of sixteen (another workgroup of the same rows makes the others).
+// Waves of a workgroup: two a SIMD where there are heads enough for each to have its own and their scores fit beside them.
+__host__ __device__ constexpr int talk_waves(int in_heads, int blocks) { return blocks == 1 || in_heads > 16 ? 4 : 8; }
+// Turns in which the weights pass through shared memory: two where the queries of all heads take most of it.
+__host__ __device__ constexpr int talk_turns(int size, int in_heads) { return in_heads > 16 && size > 64 ? 2 : 1; }
 
-template <int kSize, int kHB>
+template <int kSize, int kIn, int kHB>
 __host__ __device__ constexpr size_t talk_prefill_fixed() {
-    // queries [heads][kSize / 8 runs][16 rows], weights [heads][2 runs a wave][16 rows] (16-byte runs), maxima [waves][heads][16],
-    // references [heads][16], flags
-    return static_cast<size_t>(4 * kHB) * (kSize / 8) * 16 * 16 + static_cast<size_t>(4 * kHB) * 2 * talk_waves(kHB) * 16 * 16 +
-           static_cast<size_t>(talk_waves(kHB) + 1) * 4 * kHB * 16 * 4 + 16;
+    // queries [heads][kSize / 8 runs][16 rows], weights [heads of a turn][2 runs a wave][16 rows] (16-byte runs),
+    // maxima [waves][heads][16], references [heads][16], flags
+    return static_cast<size_t>(kIn) * (kSize / 8) * 16 * 16 +
+           static_cast<size_t>(4 * kHB / talk_turns(kSize, kIn)) * 2 * talk_waves(kIn, kHB) * 16 * 16 +
+           static_cast<size_t>(talk_waves(kIn, kHB) + 1) * 4 * kHB * 16 * 4 + 16;
 }
 
-// kHB: blocks of four heads (heads beyond q_heads are zero).  kLG: heads that share one load of keys.
-template <int kSize, int kHB, int kLG>
-__global__ void __launch_bounds__(talk_waves(kHB) * kWave, talk_waves(kHB) / 4)
+// kIn: heads whose scores are made (those beyond q_heads are zero).  kHB: blocks of four heads whose results are made, from
+// head 4 kHB blockIdx.z on.  kLG: heads that share one load of keys.
+template <int kSize, int kIn, int kHB, int kLG>
+__global__ void __launch_bounds__(talk_waves(kIn, kHB) * kWave, talk_waves(kIn, kHB) / 4)
 attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_tiles) {
     constexpr int kH = 4 * kHB;
     constexpr int kSteps = kSize / 32, kVT = kSize / 16, kRuns = kSize / 8;
-    constexpr int kLoads = kH / kLG;                         // loads of keys a stage
+    constexpr int kLoads = kIn / kLG;                        // loads of keys a stage
     constexpr int kRing = kLoads < 2 ? kLoads : 2;
-    constexpr int kWaves = talk_waves(kHB), kThreads = kWaves * kWave;
+    constexpr int kWaves = talk_waves(kIn, kHB), kThreads = kWaves * kWave;
     constexpr int kStage = 16 * kWaves;                      // keys of a stage: sixteen a wave
     constexpr int kHW = kH / kWaves;                         // heads of a wave in the second product
-    constexpr int kPG = kLG < kHW ? kLG : kHW;               // of these, how many share one load of values
+    constexpr int kTurns = talk_turns(kSize, kIn), kHT = kHW / kTurns;   // heads of a wave in a turn
+    constexpr int kPG = kLG < kHT ? kLG : kHT;               // of these, how many share one load of values
     constexpr int kHalves = kStage / 64;                     // the second product takes 64 keys at a time
     constexpr int kPRuns = kStage / 8;
-    constexpr int kMixRegs = (kH + 15) / 16;
+    constexpr int kMixRegs = (kIn + 15) / 16;
+    // More than sixteen heads: their scores come sixteen at a time, and the mixed ones are kept.  Otherwise the scores are
+    // kept, and mixed anew where references are raised.
+    constexpr bool kKeep = kIn > 16;
+    constexpr int kScores = kKeep ? 16 : kIn;
     extern __shared__ uint4 talk_shared[];
     uint4* sq = talk_shared;                                 // [head][run][row]
-    uint4* sp = sq + kH * kRuns * 16;                        // [head][run of 8 keys][row]
-    float* smax = reinterpret_cast<float*>(sp + kH * kPRuns * 16);   // [wave][head][row]
+    uint4* sp = sq + kIn * kRuns * 16;                       // [head of a turn][run of 8 keys][row]
+    float* smax = reinterpret_cast<float*>(sp + kH / kTurns * kPRuns * 16);   // [wave][head][row]
     float* sref = smax + kWaves * kH * 16;                      // [head][row]
     int* flags = reinterpret_cast<int*>(sref + kH * 16);        // [2] raise, [2] unmapped
     int* pages = flags + 4;
 
     const int heads = a.q_heads, kv_heads = a.kv_heads, group = heads / kv_heads;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave), lane = threadIdx.x % kWave, tid = threadIdx.x;
-    const int c = lane & 15, g = lane >> 4;
+    const int c = lane & 15, g = lane >> 4, out0 = kH * blockIdx.z;
+    auto head_of = [&](int w) { return w / kHT * (kH / kTurns) + wave * kHT + w % kHT; };   // this wave's heads, from out0 on
     const int page_tokens = 1 << a.page_shift, page_mask = page_tokens - 1;
     const int* my_tile = tiles + 3 * static_cast<long>(n_tiles - 1 - static_cast<int>(blockIdx.x));   // the longest first
     const int entry = my_tile[0], row0 = my_tile[1], rows = my_tile[2];
@@ -426,8 +439,9 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
     const int share = (stages + a.splits - 1) / a.splits;
     const int st_begin = split * share, st_end = st_begin + share < stages ? st_begin + share : stages;
     if (st_begin >= st_end) {                                // more parts than stages: nothing of this one
-        for (int i = tid; i < rows * heads; i += kThreads) {
-            const long slot = ((static_cast<long>(row0) + i / heads) * heads + i % heads) * a.splits + split;
+        for (int i = tid; i < rows * kH; i += kThreads) {
+            if (out0 + i % kH >= heads) continue;
+            const long slot = ((static_cast<long>(row0) + i / kH) * heads + out0 + i % kH) * a.splits + split;
             a.part_ml[2 * slot] = -INFINITY;
             a.part_ml[2 * slot + 1] = 0.f;
         }
@@ -440,19 +454,19 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
     for (int i = tid; i < n_pages; i += kThreads) pages[i] = table[first_page + i];
     if (tid < 4) flags[tid] = 0;
     for (int i = tid; i < kH * 16; i += kThreads) sref[i] = -INFINITY;
-    for (int i = tid; i < kH * kRuns * 16; i += kThreads) {
+    for (int i = tid; i < kIn * kRuns * 16; i += kThreads) {
         const int r = i % 16, run = (i / 16) % kRuns, h = i / (16 * kRuns);
         sq[i] = (h < heads && r < rows && 8 * run < a.head_dim)
                     ? *reinterpret_cast<const uint4*>(a.q + ((static_cast<long>(row0) + r) * heads + h) * a.head_dim + 8 * run)
                     : uint4{0u, 0u, 0u, 0u};
     }
-    // the mix, four output heads and sixteen input heads a register: lane 4 b + i holds talk[4 block + i][16 part + b]
+    // the mix, four output heads and sixteen input heads a register: lane 4 b + i holds talk[out0 + 4 block + i][16 part + b]
     float mix[kHB][kMixRegs];
 #pragma unroll
     for (int b = 0; b < kHB; ++b)
 #pragma unroll
         for (int part = 0; part < kMixRegs; ++part) {
-            const int to = 4 * b + (lane & 3), in = 16 * part + (lane >> 2);
+            const int to = out0 + 4 * b + (lane & 3), in = 16 * part + (lane >> 2);
             mix[b][part] = (to < heads && in < heads) ? load_any(a.talk, static_cast<long>(to) * heads + in) * a.to_log2 : 0.f;
         }
     __syncthreads();
@@ -478,7 +492,7 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
     };
     bf16x8 vx[2][kVT];
     auto fetch_values = [&](int st, int half, int h) {
-        int kvh = h / group;
+        int kvh = (out0 + h) / group;
         kvh = kvh < kv_heads ? kvh : kv_heads - 1;
 #pragma unroll
         for (int ks = 0; ks < 2; ++ks) {
@@ -494,6 +508,14 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
         }
     };
 
+    // where this lane's queries lie: an offset of a read reaches over sixteen heads and no further, so every sixteen have a
+    // start of their own, which the compiler must not turn back into one for every read
+    int q_at[kMixRegs];
+#pragma unroll
+    for (int part = 0; part < kMixRegs; ++part) {
+        q_at[part] = 16 * (16 * part * kRuns + g) + c;
+        if (part > 0) asm volatile("" : "+v"(q_at[part]));
+    }
     float l_run[kHW];
     floatx4 acc[kHW][kVT];
 #pragma unroll
@@ -507,7 +529,21 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
 
     for (int st = st_begin; st < st_end; ++st) {
         // ---- S^T of every head: lane (c, g) gets row c's scores of keys 4 g + r of this wave's sixteen
-        floatx4 sc[kH];
+        floatx4 sc[kScores];
+        floatx4 kept[kKeep ? kHB : 1][4];
+        if constexpr (kKeep) {
+#pragma unroll
+            for (int b = 0; b < kHB; ++b)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) kept[b][r] = floatx4{0.f, 0.f, 0.f, 0.f};
+        }
+#define LEONE_TALK_ONE(PART, I)                                                                                                   \
+    if constexpr (16 * (PART) + (I) < kIn) {                                                                                      \
+        _Pragma("unroll") for (int r = 0; r < 4; ++r)                                                                             \
+            d[r] = __builtin_amdgcn_mfma_f32_4x4x1f32(mix[b][PART], sc[(16 * (PART) + (I)) % kScores][r], d[r], 4, I, 0);         \
+    }
+#define LEONE_TALK_FOUR(PART, I) LEONE_TALK_ONE(PART, I) LEONE_TALK_ONE(PART, I + 1) LEONE_TALK_ONE(PART, I + 2) LEONE_TALK_ONE(PART, I + 3)
+#define LEONE_TALK_SIXTEEN(PART) LEONE_TALK_FOUR(PART, 0) LEONE_TALK_FOUR(PART, 4) LEONE_TALK_FOUR(PART, 8) LEONE_TALK_FOUR(PART, 12)
 #pragma unroll
         for (int load = 0; load < kLoads; ++load) {
             bf16x8* keys = kx[load % kRing];
@@ -517,11 +553,28 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
                 floatx4 sum = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
                 for (int s = 0; s < kSteps; ++s)
-                    sum = __builtin_amdgcn_mfma_f32_16x16x32_bf16(keys[s], __builtin_bit_cast(bf16x8, sq[(h * kRuns + 4 * s + g) * 16 + c]), sum, 0, 0, 0);
-                sc[h] = sum;
+                    sum = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                        keys[s], __builtin_bit_cast(bf16x8, sq[q_at[h / 16] + (h % 16 * kRuns + 4 * s) * 16]), sum, 0, 0, 0);
+                sc[h % kScores] = sum;
+                if constexpr (kKeep) __builtin_amdgcn_sched_barrier(0);      // or queries far ahead take the registers
             }
             // the ring's next piece: a later load of this stage, or one of the next stage's first
             fetch_keys(load + kRing < kLoads ? st : st + 1, (load + kRing) % kLoads, keys);
+            if constexpr (kKeep) {                            // sixteen heads' scores are there: their part of the mix
+                __builtin_amdgcn_sched_barrier(0);
+                if ((load + 1) * kLG % 16 == 0) {
+#pragma unroll
+                    for (int b = 0; b < kHB; ++b) {
+                        floatx4* d = kept[b];
+                        if (load * kLG / 16 == 0) {
+                            LEONE_TALK_SIXTEEN(0)
+                        } else {
+                            if constexpr (kMixRegs > 1) { LEONE_TALK_SIXTEEN(1) }
+                        }
+                    }
+                    __builtin_amdgcn_sched_barrier(0);
+                }
+            }
         }
 
         // ---- mixed scores and weights of all heads
@@ -537,19 +590,8 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
             for (int b = 0; b < kHB; ++b) {
                 floatx4 d[4];                                 // d[r][i]: head 4 b + i, key 4 g + r
 #pragma unroll
-                for (int r = 0; r < 4; ++r) d[r] = floatx4{0.f, 0.f, 0.f, 0.f};
-#define LEONE_TALK_ONE(PART, I)                                                                                           \
-    if constexpr (16 * (PART) + (I) < kH) {                                                                               \
-        _Pragma("unroll") for (int r = 0; r < 4; ++r)                                                                     \
-            d[r] = __builtin_amdgcn_mfma_f32_4x4x1f32(mix[b][PART], sc[16 * (PART) + (I)][r], d[r], 4, I, 0);             \
-    }
-#define LEONE_TALK_FOUR(PART, I) LEONE_TALK_ONE(PART, I) LEONE_TALK_ONE(PART, I + 1) LEONE_TALK_ONE(PART, I + 2) LEONE_TALK_ONE(PART, I + 3)
-                LEONE_TALK_FOUR(0, 0) LEONE_TALK_FOUR(0, 4) LEONE_TALK_FOUR(0, 8) LEONE_TALK_FOUR(0, 12)
-                if constexpr (kMixRegs > 1) {
-                    LEONE_TALK_FOUR(1, 0) LEONE_TALK_FOUR(1, 4) LEONE_TALK_FOUR(1, 8) LEONE_TALK_FOUR(1, 12)
-                }
-#undef LEONE_TALK_FOUR
-#undef LEONE_TALK_ONE
+                for (int r = 0; r < 4; ++r) d[r] = kKeep ? kept[kKeep ? b : 0][r] : floatx4{0.f, 0.f, 0.f, 0.f};
+                if constexpr (!kKeep) { LEONE_TALK_SIXTEEN(0) }
                 if (!full) {
 #pragma unroll
                     for (int r = 0; r < 4; ++r)
@@ -591,7 +633,7 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
             // a wave raises the references of its own heads and carries its sums over
 #pragma unroll
             for (int w = 0; w < kHW; ++w) {
-                const int h = wave * kHW + w;
+                const int h = head_of(w);
                 float top = smax[h * 16 + c];
 #pragma unroll
                 for (int v = 1; v < kWaves; ++v) top = fmaxf(top, smax[(v * kH + h) * 16 + c]);
@@ -609,41 +651,48 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
         }
         if (page_of(st * kStage + 16 * wave) < 0) flags[2] = 1;
         if (tid == 0) flags[(st & 1) ^ 1] = 0;                // the next stage's flag: it is set behind the barrier below
-        fetch_values(st, 0, wave * kHW);
-#pragma unroll
-        for (int h = 0; h < kH; ++h)
-            reinterpret_cast<uint2*>(sp)[((h * kPRuns + 2 * wave + (g >> 1)) * 16 + c) * 2 + (g & 1)] = packed[h];
-        __syncthreads();
-
+#undef LEONE_TALK_SIXTEEN
+#undef LEONE_TALK_FOUR
+#undef LEONE_TALK_ONE
         // ---- O^T += V^T P^T: this wave's heads over all of the stage's keys
 #pragma unroll
-        for (int half = 0; half < kHalves; ++half) {
-            const int begin = st * kStage + 64 * half;
-            if (begin >= n) continue;                         // the same for the workgroup
-            const bool whole = begin + 64 <= n;
+        for (int turn = 0; turn < kTurns; ++turn) {
+            if constexpr (kTurns > 1) __builtin_amdgcn_sched_barrier(0);     // or both turns' values are asked for at once
+            fetch_values(st, 0, head_of(turn * kHT));
+            if (turn > 0) __syncthreads();                    // the weights of the turn before have been read
 #pragma unroll
-            for (int w0 = 0; w0 < kHW; w0 += kPG) {
-                if (half + w0 > 0) fetch_values(st, half, wave * kHW + w0);
-                if (!whole) {                                 // slots behind the keys may hold anything, even NaN
+            for (int h = 0; h < kH / kTurns; ++h)
+                reinterpret_cast<uint2*>(sp)[((h * kPRuns + 2 * wave + (g >> 1)) * 16 + c) * 2 + (g & 1)] = packed[turn * (kH / kTurns) + h];
+            __syncthreads();
 #pragma unroll
-                    for (int ks = 0; ks < 2; ++ks)
+            for (int half = 0; half < kHalves; ++half) {
+                const int begin = st * kStage + 64 * half;
+                if (begin >= n) continue;                     // the same for the workgroup
+                const bool whole = begin + 64 <= n;
 #pragma unroll
-                        for (int dt = 0; dt < kVT; ++dt) vx[ks][dt] = tk_keep(vx[ks][dt], begin + 32 * ks + 8 * g, 0, n);
-                }
+                for (int w0 = 0; w0 < kHT; w0 += kPG) {
+                    if (half + w0 > 0) fetch_values(st, half, head_of(turn * kHT + w0));
+                    if (!whole) {                             // slots behind the keys may hold anything, even NaN
 #pragma unroll
-                for (int i = 0; i < kPG; ++i) {
-                    const int w = w0 + i, h = wave * kHW + w;
+                        for (int ks = 0; ks < 2; ++ks)
 #pragma unroll
-                    for (int ks = 0; ks < 2; ++ks) {
-                        const uint4 raw = sp[(h * kPRuns + 8 * half + 4 * ks + g) * 16 + c];
-                        const bf16x8 pt = __builtin_bit_cast(bf16x8, raw);
-                        const unsigned pairs[4] = {raw.x, raw.y, raw.z, raw.w};
+                            for (int dt = 0; dt < kVT; ++dt) vx[ks][dt] = tk_keep(vx[ks][dt], begin + 32 * ks + 8 * g, 0, n);
+                    }
 #pragma unroll
-                        for (int j = 0; j < 4; ++j)
-                            l_run[w] = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2, pairs[j]), __builtin_bit_cast(bf16x2, 0x3f803f80u),
-                                                                       l_run[w], false);
+                    for (int i = 0; i < kPG; ++i) {
+                        const int w = turn * kHT + w0 + i, h = wave * kHT + w0 + i;
 #pragma unroll
-                        for (int dt = 0; dt < kVT; ++dt) acc[w][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vx[ks][dt], pt, acc[w][dt], 0, 0, 0);
+                        for (int ks = 0; ks < 2; ++ks) {
+                            const uint4 raw = sp[(h * kPRuns + 8 * half + 4 * ks + g) * 16 + c];
+                            const bf16x8 pt = __builtin_bit_cast(bf16x8, raw);
+                            const unsigned pairs[4] = {raw.x, raw.y, raw.z, raw.w};
+#pragma unroll
+                            for (int j = 0; j < 4; ++j)
+                                l_run[w] = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2, pairs[j]),
+                                                                           __builtin_bit_cast(bf16x2, 0x3f803f80u), l_run[w], false);
+#pragma unroll
+                            for (int dt = 0; dt < kVT; ++dt) acc[w][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vx[ks][dt], pt, acc[w][dt], 0, 0, 0);
+                        }
                     }
                 }
             }
@@ -652,13 +701,13 @@ attention_talk_prefill_kernel(TalkArgs a, const int* __restrict__ tiles, int n_t
     const bool poisoned = flags[2] != 0;                      // every write came before the last barrier
 #pragma unroll
     for (int w = 0; w < kHW; ++w) {
-        const int h = wave * kHW + w;
+        const int h = head_of(w);
         float l = l_run[w];
         l += __shfl_xor(l, 16, kWave);
         l += __shfl_xor(l, 32, kWave);
         if (poisoned) l = __builtin_nanf("");
-        if (h >= heads || c >= rows) continue;
-        const long rh = (static_cast<long>(row0) + c) * heads + h;
+        if (out0 + h >= heads || c >= rows) continue;
+        const long rh = (static_cast<long>(row0) + c) * heads + out0 + h;
         if (a.splits > 1) {
             const float ref = sref[h * 16 + c];
             const long slot = rh * a.splits + split;
@@ -763,7 +812,7 @@ extern "C" int leone_attention_talk_decode(const void* q, void* out, const void*
 }
 
 // tiles int32 [n_tiles, 3]: (entry, first row, rows) with at most leone_attention_talk_tile_rows() consecutive rows of one
-// request; up to 16 query heads, otherwise as above.  Workspace for splits > 1: part_acc covered rows * q_heads * splits *
+// request; otherwise as above.  Workspace for splits > 1: part_acc covered rows * q_heads * splits *
 // v_dim floats, part_ml covered rows * q_heads * splits * 2, `covered rows` one more than the last row a tile names.
 extern "C" int leone_attention_talk_prefill(const void* q, void* out, const void* k_pool, const void* v_pool, const void* talk,
                                             int talk_dtype, const int* positions, const int* tiles, int n_tiles,
@@ -773,32 +822,35 @@ extern "C" int leone_attention_talk_prefill(const void* q, void* out, const void
     const TalkArgs a{static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pool), static_cast<const bf16_t*>(v_pool),
                      AnyVec{talk, talk_dtype}, positions, block_table, max_blocks, part_acc, part_ml, static_cast<bf16_t*>(out),
                      q_heads, kv_heads, head_dim, v_dim, shift_of(page_tokens), scale * kLog2e, splits};
-    if (check_talk("attention_talk_prefill", a, page_tokens, talk_dtype, 16)) return 1;
+    if (check_talk("attention_talk_prefill", a, page_tokens, talk_dtype, 32)) return 1;
     LEONE_REQUIRE(tiles && n_tiles > 0 && splits <= attention_tile_merge_max_splits(), "attention_talk_prefill: %d tiles, splits %d", n_tiles, splits);
     const int size = head_dim > v_dim ? head_dim : v_dim;
     const bool grouped = (q_heads / kv_heads) % 4 == 0;       // four neighbouring heads read the same keys
-#define LEONE_TALK_PREFILL(SIZE, HB, LG)                                                                                          \
+#define LEONE_TALK_PREFILL(SIZE, IN, HB, LG)                                                                                      \
     do {                                                                                                                          \
         static size_t allowed = 48 * 1024;                                                                                        \
-        const size_t shared = talk_prefill_fixed<SIZE, HB>() + static_cast<size_t>(max_blocks) * sizeof(int);                     \
+        const size_t shared = talk_prefill_fixed<SIZE, IN, HB>() + static_cast<size_t>(max_blocks) * sizeof(int);                 \
         LEONE_REQUIRE(shared <= kTalkMostShared, "attention_talk_prefill: %zu bytes of shared memory are too many", shared);      \
-        if (raise_shared(reinterpret_cast<const void*>(&attention_talk_prefill_kernel<SIZE, HB, LG>), shared, &allowed,           \
+        if (raise_shared(reinterpret_cast<const void*>(&attention_talk_prefill_kernel<SIZE, IN, HB, LG>), shared, &allowed,       \
                          "attention_talk_prefill"))                                                                               \
             return 1;                                                                                                             \
-        attention_talk_prefill_kernel<SIZE, HB, LG><<<dim3(n_tiles, splits), talk_waves(HB) * kWave, shared, stream>>>(a, tiles, n_tiles);  \
+        attention_talk_prefill_kernel<SIZE, IN, HB, LG><<<dim3(n_tiles, splits, ceil_div(q_heads, 4 * HB)),                       \
+                                                          talk_waves(IN, HB) * kWave, shared, stream>>>(a, tiles, n_tiles);       \
     } while (0)
-#define LEONE_TALK_SIZES(HB)                                                        \
-    if (size <= 64) {                                                               \
-        if (grouped) LEONE_TALK_PREFILL(64, HB, 4); else LEONE_TALK_PREFILL(64, HB, 1);  \
-    } else {                                                                        \
-        if (grouped) LEONE_TALK_PREFILL(128, HB, 4); else LEONE_TALK_PREFILL(128, HB, 1); \
+#define LEONE_TALK_SIZES(IN, HB)                                                            \
+    if (size <= 64) {                                                                       \
+        if (grouped) LEONE_TALK_PREFILL(64, IN, HB, 4); else LEONE_TALK_PREFILL(64, IN, HB, 1);    \
+    } else {                                                                                \
+        if (grouped) LEONE_TALK_PREFILL(128, IN, HB, 4); else LEONE_TALK_PREFILL(128, IN, HB, 1);  \
     }
     if (q_heads <= 4) {
-        LEONE_TALK_SIZES(1)
+        LEONE_TALK_SIZES(4, 1)
     } else if (q_heads <= 8) {
-        LEONE_TALK_SIZES(2)
+        LEONE_TALK_SIZES(8, 2)
+    } else if (q_heads <= 16) {
+        LEONE_TALK_SIZES(16, 4)
     } else {
-        LEONE_TALK_SIZES(4)
+        LEONE_TALK_SIZES(32, 4)
     }
 #undef LEONE_TALK_SIZES
 #undef LEONE_TALK_PREFILL

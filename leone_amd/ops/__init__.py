@@ -388,10 +388,11 @@ TALK_MIN_ROWS = 16             # portions from so many rows on go there
 
 def talk_attention_supported(dtype: torch.dtype, q_heads: int, head_dim: int, value_dim: int, page_tokens: int, max_blocks: int = 0) -> dict:
     """Which matrix-core kernels for mixed scores take this shape: {"decode": ..., "prompt": ...}; the others go to
-    ``attention_rows_talk``.  The prompt kernel's workgroup holds the scores and sums of 16 rows of every head."""
+    ``attention_rows_talk``.  The prompt kernel's workgroup holds 16 rows' queries of every head in shared memory, which
+    leaves room for the numbers of 2,560 pages."""
     fits = (dtype == torch.bfloat16 and head_dim % 8 == 0 and value_dim % 4 == 0 and max(head_dim, value_dim) <= 128
             and page_tokens >= 16 and page_tokens & (page_tokens - 1) == 0 and 4 * max_blocks <= 32 * 1024)
-    return {"decode": fits and q_heads <= 32, "prompt": fits and q_heads <= 16}
+    return {"decode": fits and q_heads <= 32, "prompt": fits and q_heads <= 32 and max_blocks <= 2560}
 
 
 def _talk_operands(q, k_pool, v_pool, talk, q_heads: int):
@@ -428,8 +429,9 @@ def attention_talk_decode(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
 
 
 def choose_talk_splits(tiles: int, mean_keys: int, units: int = 256) -> int:
-    """Into how many parts the keys of a tile of rows are cut: the number for which rounds of workgroups (one a compute
-    unit) x (stages of 64 keys a part + a start worth 3 + a merge worth 2) come out least."""
+    """Into how many parts the keys of a tile of rows are cut (a tile of more than 16 heads counts twice): the number for
+    which rounds of workgroups (one a compute unit) x (stages of 64 keys a part + a start worth 3 + a merge worth 2) come
+    out least."""
     stages = max(1, -(-mean_keys // 64))
     best = None
     for splits in range(1, min(16, stages) + 1):
@@ -450,7 +452,7 @@ def attention_talk_prefill(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Ten
     if tiles.dim() != 2 or tiles.shape[1] != 3:
         raise KernelError(f"attention_talk_prefill: tiles must be int32 [n, 3], found {tuple(tiles.shape)}")
     if splits is None:
-        splits = choose_talk_splits(tiles.shape[0], mean_keys, compute_units(q.device))
+        splits = choose_talk_splits(tiles.shape[0] * (1 if q_heads <= 16 else 2), mean_keys, compute_units(q.device))
     part_acc = part_ml = None
     if splits > 1:
         covered = rows if covered_rows is None else covered_rows
