@@ -10,9 +10,9 @@
 //   attention_talk_prefill  one workgroup takes 16 consecutive rows of a request, all heads, and walks the keys 64 or 128 at
 //       a time, a wave 16 of them: S^T [keys x rows] of every head, so that a lane holds one row and four keys and every head
 //       a register: v_mfma_f32_4x4x1_16b_f32 with its first operand broadcast (a column of talk) mixes them, four
-//       heads an instruction (more than 16 heads: two workgroups make half the results each, the scores come sixteen heads at
-//       a time and each sixteen add their part of the mix).  The weights go to shared memory, and for O^T += V^T P^T a wave takes its share of the heads
-//       over all the stage's keys.
+//       heads an instruction (more than 16 heads: two workgroups make half the results each, the scores come sixteen heads
+//       at a time and each sixteen add their part of the mix).  The weights go to shared memory, and for O^T += V^T P^T a
+//       wave takes its share of the heads over all the stage's keys.
 //
 // The softmax is that of the other kernels: powers of two against a reference that is a whole number, raised only when a
 // score outgrows it by 2^8; row sums over the rounded weights.  talk comes times scale * log2(e), in float.
