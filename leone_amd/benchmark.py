@@ -467,10 +467,31 @@ def reverax_shape(width: int, layers: int, vocab: int, context: int) -> dict:
             "max_positions": max(4096, context + 64), "layers": [order[i % 4] for i in range(layers)]}
 
 
+def sonulorn_shape(width: int, layers: int, vocab: int, context: int) -> dict:
+    """Sonulorn at layer sizes that resemble published models of its kinds, as many layer runs as ``layers``: linear attention
+    with fixed decays first and last (heads of 128 x 128 over the model's width), and between them a loop over two layers:
+    softmax attention within chunks of 1,024 positions (heads of 128, four query heads a key head, half a head rotated, a
+    gate for every element), and softmax attention over every key (the same heads behind convolutions of 4 taps) beside a
+    gated delta rule (heads of 128 x 128, two memories a q/k head, convolutions of 4 taps); feed-forwards of 3 x width."""
+    heads, passes = width // 128, (layers - 2) // 2
+    attention = {"heads": heads, "kv_heads": width // 512, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                 "rot": {"dims": 64, "base": 1000000.0}}
+    dense = {"kind": "dense", "ff": 3 * width, "limit": 7.0}
+    linear = {"type": "lightning", "mlp": dense,
+              "mixer": {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** (-1 - 8.0 * h / heads) for h in range(heads)]}}
+    chunked = {"type": "attention", "mlp": dense, "mixer": {**attention, "mask": {"size": 1024}}}
+    side = {"type": "parallel", "mlp": dense,
+            "mixer": {"left": {**attention, "conv": 4}, "left_scale": 0.5, "right_scale": 0.5,
+                      "right": {"heads": heads, "kv_heads": width // 256, "dim": 128, "vdim": 128, "conv": 4}}}
+    return {"architecture": "Sonulorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "max_positions": max(4096, context + 64), "layers": [linear, chunked, side, linear],
+            "loop": {"start": 1, "stop": 3, "times": passes}}
+
+
 DESIGN_SHAPES = {"pamevik": pamevik_shape, "zukinex": zukinex_shape, "fosulix": fosulix_shape, "nogidra": nogidra_shape,
-                 "reverax": reverax_shape}
+                 "reverax": reverax_shape, "sonulorn": sonulorn_shape}
 # The existing design whose kernels a design's own stand closest to: measured beside it, at the same sizes.
-DESIGN_NEIGHBOURS = {"nogidra": "fosulix", "reverax": "nogidra"}
+DESIGN_NEIGHBOURS = {"nogidra": "fosulix", "reverax": "nogidra", "sonulorn": "pamevik"}
 
 
 def state_bytes_per_request(model) -> int:

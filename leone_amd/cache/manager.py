@@ -14,7 +14,7 @@ fixed-size pages:
   no page is mapped);
 * ``reserve`` maps pages for the positions a step is about to write, in every
   group, all or nothing; ``commit`` advances the request's length and, for a
-  windowed group, hands back pages that no later query can reach; ``rollback``
+  windowed or chunked group, hands back pages that no later query can reach; ``rollback``
   undoes an uncommitted reservation; ``release`` returns everything a request
   holds, pages and state slot, at once;
 * a *state slot* is an index into per-request storage of fixed size, handed out
@@ -57,14 +57,23 @@ class CacheError(RuntimeError):
 @dataclass(frozen=True)
 class GroupSpec:
     """Pages of one group: ``window`` None keeps every position, else only the last ``window`` and, whatever the
-    window, the first ``keep_first`` (the pages that hold them are never handed back by a window that passes)."""
+    window, the first ``keep_first`` (the pages that hold them are never handed back by a window that passes).
+    ``chunk`` (of a group without a window): positions fall into chunks of so many, counted from 0, and a query reads keys
+    of its own chunk only; the pages of a chunk go back when the request has passed it."""
     num_pages: int
     page_tokens: int
     window: Optional[int] = None
     keep_first: int = 0
+    chunk: int = 0
 
     def kept_blocks(self) -> int:
         return 0 if self.window is None else -(-self.keep_first // self.page_tokens)
+
+    def first_readable(self, at: int) -> int:
+        """The first position that a query at position ``at``, or any later one, can read (kept first ones aside)."""
+        if self.chunk:
+            return at // self.chunk * self.chunk
+        return 0 if self.window is None else max(0, at - (self.window - 1))
 
 
 class RequestKeys:
@@ -121,7 +130,8 @@ class CacheManager:
         if max_requests <= 0 or max_context <= 0:
             raise ValueError("max_requests and max_context must be positive")
         for g in groups:
-            if g.num_pages <= 0 or g.page_tokens <= 0 or (g.window is not None and g.window <= 0) or g.keep_first < 0:
+            if g.num_pages <= 0 or g.page_tokens <= 0 or (g.window is not None and g.window <= 0) or g.keep_first < 0 \
+                    or g.chunk < 0 or (g.chunk and g.window is not None):
                 raise ValueError(f"invalid cache group {g}")
         self.groups = list(groups)
         self.max_requests = max_requests
@@ -137,6 +147,8 @@ class CacheManager:
         for i, g in enumerate(groups):
             if g.window is not None and g.keep_first:
                 self._checked(self._lib.leone_cache_set_keep_first(self.handle, i, g.keep_first))
+            if g.chunk:
+                self._checked(self._lib.leone_cache_set_chunk(self.handle, i, g.chunk))
         self._max_blocks = [self._lib.leone_cache_max_blocks(self.handle, g) for g in range(len(groups))]
         self._table_buffers = [(c_int * max(1, width))() for width in self._max_blocks]
 
@@ -309,7 +321,7 @@ class CacheManager:
                     holders[page] += 1
                 length = self.length(request)
                 total = length + self._checked(self._lib.leone_cache_pending(self.handle, self._key(request)))
-                first = 0 if g.window is None else max(0, length - (g.window - 1)) // g.page_tokens
+                first = g.first_readable(length) // g.page_tokens
                 if total:
                     for b in range(0, (total - 1) // g.page_tokens + 1):
                         if b < first and b >= g.kept_blocks():

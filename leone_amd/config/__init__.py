@@ -5,3 +5,4 @@ from .zukinex import ZukinexConfig
 from .fosulix import FosulixConfig
 from .nogidra import NogidraConfig
 from .reverax import ReveraxConfig
+from .sonulorn import SonulornConfig

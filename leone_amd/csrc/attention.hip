@@ -35,7 +35,7 @@ __global__ void attention_rows_kernel(const T* __restrict__ q, T* __restrict__ o
                                       const int* __restrict__ block_table, int max_blocks, int q_heads,
                                       int kv_heads, int head_dim, int v_dim, int page_tokens, float scale, int window,
                                       const float* __restrict__ gate, long gate_stride, int keep_first, int gate_each,
-                                      const float* __restrict__ slopes, float temp_coef, int temp_every, ScoreShape shape) {
+                                      const float* __restrict__ slopes, float temp_coef, int temp_every, ScoreShape shape, int chunk) {
     __shared__ float sm_m[kRowWaves];
     __shared__ float sm_l[kRowWaves];
     __shared__ float sm_acc[kRowWaves][kRowMaxHeadDim];
@@ -47,7 +47,7 @@ __global__ void attention_rows_kernel(const T* __restrict__ q, T* __restrict__ o
     const int kvh = head / (q_heads / kv_heads);
     const int pos = positions[row];
     const int* table = block_table + static_cast<long>(row_entry[row]) * max_blocks;
-    const int first = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+    const int first = first_key(pos, window, chunk);
     // a query that grows with its position: the factor 1 + coef * ln(floor((pos + 1) / every) + 1) rides on the scale
     if (temp_every > 0) scale *= 1.0f + temp_coef * logf(static_cast<float>((pos + 1) / temp_every + 1));
     // a head's scores are lowered by slope * distance
@@ -259,17 +259,20 @@ extern "C" int leone_attention_rows_biased(const void* q, void* out, const void*
     return leone_attention_rows_shaped(q, out, k_pool, v_pool, dtype, positions, row_entry, block_table, max_blocks, rows,
                                        q_heads, kv_heads, head_dim, v_dim, page_tokens, scale, window, gate, gate_stride,
                                        keep_first, gate_each, slopes, temp_coef, temp_every, 0.f, nullptr, nullptr, nullptr, 0,
-                                       0, stream);
+                                       0, 0, stream);
 }
 
-// The same with what score_shape.h describes: cap (0: none), sinks, and the tables that turn results back (null: none).
+// The same with what score_shape.h describes: cap (0: none), sinks, and the tables that turn results back (null: none);
+// chunk > 0 (no window, no kept first keys): a row sees the keys of its own chunk of so many positions only.
 extern "C" int leone_attention_rows_shaped(const void* q, void* out, const void* k_pool, const void* v_pool, int dtype,
                                            const int* positions, const int* row_entry, const int* block_table,
                                            int max_blocks, int rows, int q_heads, int kv_heads, int head_dim, int v_dim,
                                            int page_tokens, float scale, int window, const float* gate, long gate_stride,
                                            int keep_first, int gate_each, const float* slopes, float temp_coef,
                                            int temp_every, float cap, const float* sinks, const float* turn_cos,
-                                           const float* turn_sin, int turn_positions, int turn_pairing, hipStream_t stream) {
+                                           const float* turn_sin, int turn_positions, int turn_pairing, int chunk,
+                                           hipStream_t stream) {
+    if (check_mask("attention_rows", window, chunk, keep_first)) return 1;
     const ScoreShape shape{cap, sinks, turn_cos, turn_sin, turn_positions, turn_pairing};
     if (check_score_shape("attention_rows", shape, v_dim)) return 1;
     LEONE_REQUIRE(temp_every >= 0, "attention_rows: the query factor's period %d must not be negative", temp_every);
@@ -292,12 +295,12 @@ extern "C" int leone_attention_rows_shaped(const void* q, void* out, const void*
         attention_rows_kernel<float><<<grid, kRowThreads, 0, stream>>>(
             static_cast<const float*>(q), static_cast<float*>(out), static_cast<const float*>(k_pool),
             static_cast<const float*>(v_pool), positions, row_entry, block_table, max_blocks, q_heads, kv_heads,
-            head_dim, v_dim, page_tokens, scale, window, gate, gate_stride, keep_first, gate_each, slopes, temp_coef, temp_every, shape);
+            head_dim, v_dim, page_tokens, scale, window, gate, gate_stride, keep_first, gate_each, slopes, temp_coef, temp_every, shape, chunk);
     else
         attention_rows_kernel<bf16_t><<<grid, kRowThreads, 0, stream>>>(
             static_cast<const bf16_t*>(q), static_cast<bf16_t*>(out), static_cast<const bf16_t*>(k_pool),
             static_cast<const bf16_t*>(v_pool), positions, row_entry, block_table, max_blocks, q_heads, kv_heads,
-            head_dim, v_dim, page_tokens, scale, window, gate, gate_stride, keep_first, gate_each, slopes, temp_coef, temp_every, shape);
+            head_dim, v_dim, page_tokens, scale, window, gate, gate_stride, keep_first, gate_each, slopes, temp_coef, temp_every, shape, chunk);
     LEONE_LAUNCH_CHECK("attention_rows");
     return 0;
 }

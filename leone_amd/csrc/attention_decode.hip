@@ -139,7 +139,7 @@ attention_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__
                         const int* __restrict__ row_entry, const int* __restrict__ block_table, int max_blocks,
                         float* __restrict__ part_acc, float* __restrict__ part_ml, bf16_t* __restrict__ out,
                         int q_heads, int kv_heads, int page_shift, float to_log2, int window, int splits,
-                        FromProjection from, int keep_first, ScoreBias bias, ScoreShape shape) {
+                        FromProjection from, int keep_first, ScoreBias bias, ScoreShape shape, int chunk) {
     constexpr int kD = kD16 * 16;
     constexpr int kSteps = (kD16 + 1) / 2;           // 32-element steps of the q.k product
     extern __shared__ float smem[];                   // [waves][columns][kD] accumulators, then m and l
@@ -158,7 +158,7 @@ attention_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__
     const int page_mask = page_tokens - 1;
 
     const int n = positions[row] + 1;                                    // keys 0 .. n-1 exist
-    const int lo = (window > 0 && n - window > 0) ? n - window : 0;      // first key in reach
+    const int lo = first_key(n - 1, window, chunk);                      // first key in reach
     // this lane's column is query head kvh * group + col0 + c
     const float to_log2_row = bias.temp_every > 0
         ? to_log2 * (1.0f + bias.temp_coef * logf(static_cast<float>(n / bias.temp_every + 1))) : to_log2;
@@ -634,7 +634,7 @@ static void launch_decode(const void* q, const void* k_pool, const void* v_pool,
                           const int* row_entry, const int* block_table, int max_blocks, float* part_acc,
                           float* part_ml, void* out, int rows, int q_heads, int kv_heads, int page_shift, float scale,
                           int window, int splits, const FromProjection* from, int keep_first, ScoreBias bias,
-                          const ScoreShape& shape, hipStream_t stream) {
+                          const ScoreShape& shape, int chunk, hipStream_t stream) {
     const int group = q_heads / kv_heads;
     dim3 grid(rows, kv_heads * ((group + 15) / 16), splits);
     const size_t smem = decode_smem_bytes(kD16 * 16, group, max_blocks);
@@ -644,7 +644,7 @@ static void launch_decode(const void* q, const void* k_pool, const void* v_pool,
             attention_decode_kernel<kD16, true, false><<<grid, kDecodeThreads, smem, stream>>>(
                 nullptr, static_cast<const bf16_t*>(k_pool), static_cast<const bf16_t*>(v_pool), positions, row_entry,
                 block_table, max_blocks, part_acc, part_ml, static_cast<bf16_t*>(out), q_heads, kv_heads, page_shift,
-                to_log2, window, splits, *from, keep_first, bias, ScoreShape{});
+                to_log2, window, splits, *from, keep_first, bias, ScoreShape{}, chunk);
             return;
         }
     }
@@ -652,7 +652,7 @@ static void launch_decode(const void* q, const void* k_pool, const void* v_pool,
     attention_decode_kernel<kD16, false, SHAPED><<<grid, kDecodeThreads, smem, stream>>>(                                    \
         static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pool), static_cast<const bf16_t*>(v_pool),               \
         positions, row_entry, block_table, max_blocks, part_acc, part_ml, static_cast<bf16_t*>(out), q_heads, kv_heads,      \
-        page_shift, to_log2, window, splits, FromProjection{}, keep_first, bias, shape)
+        page_shift, to_log2, window, splits, FromProjection{}, keep_first, bias, shape, chunk)
     if (shape.any()) LEONE_DECODE_LAUNCH(true);
     else LEONE_DECODE_LAUNCH(false);
 #undef LEONE_DECODE_LAUNCH
@@ -662,7 +662,8 @@ static int decode_checked(const void* q, void* out, const void* k_pool, const vo
                           const int* row_entry, const int* block_table, int max_blocks, float* part_acc,
                           float* part_ml, int rows, int q_heads, int kv_heads, int head_dim, int page_tokens,
                           float scale, int window, int splits, const FromProjection* from, int keep_first,
-                          hipStream_t stream, ScoreBias bias = ScoreBias{}, const ScoreShape& shape = ScoreShape{}) {
+                          hipStream_t stream, ScoreBias bias = ScoreBias{}, const ScoreShape& shape = ScoreShape{}, int chunk = 0) {
+    if (check_mask("attention_decode", window, chunk, keep_first)) return 1;
     if (check_score_shape("attention_decode", shape, head_dim)) return 1;
     LEONE_REQUIRE(!from || !shape.any(), "attention_decode: capped scores, sinks and turned values come with finished queries");
     LEONE_REQUIRE(bias.temp_every >= 0, "attention_decode: the query factor's period %d must not be negative", bias.temp_every);
@@ -689,7 +690,7 @@ static int decode_checked(const void* q, void* out, const void* k_pool, const vo
 #define LEONE_DECODE_CASE(N)                                                                                      \
     case N:                                                                                                       \
         launch_decode<N>(q, k_pool, v_pool, positions, row_entry, block_table, max_blocks, part_acc, part_ml,     \
-                         out, rows, q_heads, kv_heads, page_shift, scale, window, splits, from, keep_first, bias, shape, stream); \
+                         out, rows, q_heads, kv_heads, page_shift, scale, window, splits, from, keep_first, bias, shape, chunk, stream); \
         break;
     switch (head_dim / 16) {
         LEONE_DECODE_CASE(1) LEONE_DECODE_CASE(2) LEONE_DECODE_CASE(3) LEONE_DECODE_CASE(4)
@@ -750,18 +751,20 @@ extern "C" int leone_attention_decode_biased(const void* q, void* out, const voi
                           ScoreBias{slopes, temp_coef, temp_every});
 }
 
-// The same with what score_shape.h describes: cap (0: none), sinks, and the tables that turn results back (null: none).
+// The same with what score_shape.h describes: cap (0: none), sinks, and the tables that turn results back (null: none);
+// chunk > 0 (no window, no kept first keys): a row sees the keys of its own chunk of so many positions only.
 extern "C" int leone_attention_decode_shaped(const void* q, void* out, const void* k_pool, const void* v_pool,
                                              const int* positions, const int* row_entry, const int* block_table,
                                              int max_blocks, float* part_acc, float* part_ml, int rows, int q_heads,
                                              int kv_heads, int head_dim, int page_tokens, float scale, int window,
                                              int splits, int keep_first, const float* slopes, float temp_coef,
                                              int temp_every, float cap, const float* sinks, const float* turn_cos,
-                                             const float* turn_sin, int turn_positions, int turn_pairing, hipStream_t stream) {
+                                             const float* turn_sin, int turn_positions, int turn_pairing, int chunk,
+                                             hipStream_t stream) {
     return decode_checked(q, out, k_pool, v_pool, positions, row_entry, block_table, max_blocks, part_acc, part_ml, rows,
                           q_heads, kv_heads, head_dim, page_tokens, scale, window, splits, nullptr, keep_first, stream,
                           ScoreBias{slopes, temp_coef, temp_every},
-                          ScoreShape{cap, sinks, turn_cos, turn_sin, turn_positions, turn_pairing});
+                          ScoreShape{cap, sinks, turn_cos, turn_sin, turn_positions, turn_pairing}, chunk);
 }
 
 // The same for a step in which every row is another request, taking the fused q/k/v projection instead of

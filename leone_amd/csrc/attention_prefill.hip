@@ -76,7 +76,7 @@ attention_prefill_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
                          const int* __restrict__ tiles, int n_groups, const int* __restrict__ block_table,
                          int max_blocks, int q_heads, int kv_heads, int page_shift, float scale, int window,
                          float* __restrict__ part_acc, float* __restrict__ part_ml, int splits, int keep_first,
-                         const float* __restrict__ slopes, float temp_coef, int temp_every, ScoreShape shape) {
+                         const float* __restrict__ slopes, float temp_coef, int temp_every, ScoreShape shape, int chunk) {
     constexpr int kD = kD16 * 16;
     constexpr int kRuns = kD / 8;                      // 16-byte runs of one key
     constexpr int kDT = (kD + 31) / 32;                // 32-row tiles of the second product's result
@@ -108,10 +108,10 @@ attention_prefill_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
     const int p0 = wave_rows > 0 ? positions[tile_row0] : 0;    // rows of a portion are consecutive positions
     const int p_last = p0 + wave_rows - 1;
     const int key_hi = wave_rows > 0 ? p_last + 1 : 0;          // keys the wave may read: [key_lo, key_hi)
-    const int key_lo = (window > 0 && p0 - window + 1 > 0) ? p0 - window + 1 : 0;
+    const int key_lo = first_key(p0, window, chunk);
     // A pass wholly inside [full_lo, full_hi) is visible to every row of the wave: no masks.
     const int full_hi = p0 + 1;
-    const int full_lo = (window > 0 && p_last - window + 1 > 0) ? p_last - window + 1 : 0;
+    const int full_lo = wave_rows > 0 ? first_key(p_last, window, chunk) : 0;
     if (lane == 0) {
         wave_lo[wave] = wave_rows > 0 ? key_lo : 0x7fffffff;
         wave_hi[wave] = key_hi;
@@ -164,6 +164,7 @@ attention_prefill_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
     // The Q^T operand and the row's own position.
     const bool row_ok = j < wave_rows;
     const int row_pos = row_ok ? p0 + j : -1;                                   // -1: the row sees no key
+    const int row_lo = row_ok ? first_key(row_pos, window, chunk) : 0;          // the first one it sees, kept ones aside
     // Scores that fall with the distance and queries that count more the further on they stand, both in units of the
     // raw dot product (the scale comes later): score = dot * row_factor - (slope / scale) * (row_pos - key).
     const bool biased = slopes != nullptr || temp_every > 0;                    // the same for the whole launch
@@ -347,11 +348,10 @@ attention_prefill_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
             }
         }
         if (!full) {                                           // the same for the whole wave
-            const int p_lo = (window > 0) ? row_pos - window + 1 : 0;
 #pragma unroll
             for (int v = 0; v < 16; ++v) {
                 const int key = key0 + 8 * h + (v & 7) + 16 * (v >> 3);
-                sc[v] = (key <= row_pos && (key >= p_lo || key < keep)) ? sc[v] : -INFINITY;
+                sc[v] = (key <= row_pos && (key >= row_lo || key < keep)) ? sc[v] : -INFINITY;
             }
         }
         float top = sc[0];
@@ -580,7 +580,7 @@ static int launch_prefill(const void* q, void* out, const void* k_pool, const vo
                           const int* tiles, int n_groups, const int* block_table, int max_blocks, int q_heads,
                           int kv_heads, int page_shift, float scale, int window, float* part_acc, float* part_ml,
                           int splits, int keep_first, const float* slopes, float temp_coef, int temp_every,
-                          const ScoreShape& shape, hipStream_t stream) {
+                          const ScoreShape& shape, int chunk, hipStream_t stream) {
     const size_t shared = 2 * static_cast<size_t>(stage_runs(16 * kD16)) * sizeof(uint4) + static_cast<size_t>(max_blocks) * sizeof(int);
     static size_t allowed = 48 * 1024;                 // what a kernel may use without asking
     if (shared > allowed) {
@@ -595,7 +595,7 @@ static int launch_prefill(const void* q, void* out, const void* k_pool, const vo
     attention_prefill_kernel<kD16, kShaped><<<dim3(n_groups * q_heads, splits), kPrefillThreads, shared, stream>>>(
         static_cast<const bf16_t*>(q), static_cast<bf16_t*>(out), static_cast<const bf16_t*>(k_pool),
         static_cast<const bf16_t*>(v_pool), positions, tiles, n_groups, block_table, max_blocks, q_heads, kv_heads,
-        page_shift, scale, window, part_acc, part_ml, splits, keep_first, slopes, temp_coef, temp_every, shape);
+        page_shift, scale, window, part_acc, part_ml, splits, keep_first, slopes, temp_coef, temp_every, shape, chunk);
     return 0;
 }
 
@@ -648,17 +648,19 @@ extern "C" int leone_attention_prefill_biased(const void* q, void* out, const vo
                                               hipStream_t stream) {
     return leone_attention_prefill_shaped(q, out, k_pool, v_pool, positions, tiles, n_groups, block_table, max_blocks, q_heads,
                                           kv_heads, head_dim, page_tokens, scale, window, part_acc, part_ml, splits, keep_first,
-                                          slopes, temp_coef, temp_every, 0.f, nullptr, nullptr, nullptr, 0, 0, stream);
+                                          slopes, temp_coef, temp_every, 0.f, nullptr, nullptr, nullptr, 0, 0, 0, stream);
 }
 
-// The same with what score_shape.h describes: cap (0: none), sinks, and the tables that turn results back (null: none).
+// The same with what score_shape.h describes: cap (0: none), sinks, and the tables that turn results back (null: none);
+// chunk > 0 (no window, no kept first keys): a row sees the keys of its own chunk of so many positions only.
 extern "C" int leone_attention_prefill_shaped(const void* q, void* out, const void* k_pool, const void* v_pool,
                                               const int* positions, const int* tiles, int n_groups, const int* block_table,
                                               int max_blocks, int q_heads, int kv_heads, int head_dim, int page_tokens,
                                               float scale, int window, float* part_acc, float* part_ml, int splits,
                                               int keep_first, const float* slopes, float temp_coef, int temp_every, float cap,
                                               const float* sinks, const float* turn_cos, const float* turn_sin,
-                                              int turn_positions, int turn_pairing, hipStream_t stream) {
+                                              int turn_positions, int turn_pairing, int chunk, hipStream_t stream) {
+    if (check_mask("attention_prefill", window, chunk, keep_first)) return 1;
     const ScoreShape shape{cap, sinks, turn_cos, turn_sin, turn_positions, turn_pairing};
     if (check_score_shape("attention_prefill", shape, head_dim)) return 1;
     LEONE_REQUIRE(temp_every >= 0, "attention_prefill: the query factor's period %d must not be negative", temp_every);
@@ -689,11 +691,11 @@ extern "C" int leone_attention_prefill_shaped(const void* q, void* out, const vo
                      ? launch_prefill<N, true>(q, out, k_pool, v_pool, positions, tiles, n_groups, block_table,    \
                                                max_blocks, q_heads, kv_heads, page_shift, scale, window, part_acc, \
                                                part_ml, splits, keep_first, slopes, temp_coef, temp_every, shape,  \
-                                               stream)                                                             \
+                                               chunk, stream)                                                      \
                      : launch_prefill<N, false>(q, out, k_pool, v_pool, positions, tiles, n_groups, block_table,   \
                                                 max_blocks, q_heads, kv_heads, page_shift, scale, window, part_acc, \
                                                 part_ml, splits, keep_first, slopes, temp_coef, temp_every, shape, \
-                                                stream);                                                           \
+                                                chunk, stream);                                                    \
         break;
     switch (head_dim / 16) {
         LEONE_PREFILL_CASE(1) LEONE_PREFILL_CASE(2) LEONE_PREFILL_CASE(3) LEONE_PREFILL_CASE(4)

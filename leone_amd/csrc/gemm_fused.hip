@@ -56,6 +56,7 @@ struct FusedArgs {
     const void* next_gain;     // prepare: [N]
     int next_gain_dtype;
     int act;                   // gated: the gate's activation (GateAct)
+    float limit = 0.f;         // gated: what that activation holds gate and up to
     int plane_rows = 0;        // plain: rows of W that read one plane of X, a multiple of 16 (0: there is one plane)
     int planes = 1;
 };
@@ -253,7 +254,7 @@ gemm_fused_kernel(FusedArgs a) {
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const float gate = sum[r];
-                out[r] = from_float<bf16_t>(gate_act(gate, a.act) * up[r]);
+                out[r] = from_float<bf16_t>(glu_value(gate, up[r], a.act, a.limit));
             }
         }
         return;
@@ -337,12 +338,12 @@ using namespace leone;
 // in_mode: 0 plain (x bfloat16 [m,k]), 1 norm (x float32 stream, optional rows, gain, eps), 2 prepared (x bfloat16
 // [m,k] and squares_in float32 [m, ceil(k / 16)] as an earlier call's out_mode 3 wrote them, eps).
 // out_mode: 0 store (y of out_dtype [m,n]), 1 residual (y float32 [m,n] += product), 2 gated (y bfloat16 [m,n/2]),
-// 4 gated with the tanh form of gelu on the gate instead of silu,
+// 4 gated with the tanh form of gelu on the gate instead of silu, 5 gated with gate and up held to `limit` (GateAct 2),
 // 3 prepare (as 1, and operand_out bfloat16 [m,n] = bf16(y * next_gain), squares_out float32 [m, ceil(n / 16)]).
 extern "C" int leone_gemm_fused_bf16(const void* x, int in_mode, const int* rows, const void* gain, int gain_dtype,
                                      float eps, const void* w, int w_tiled, void* y, int out_mode, int out_dtype, int m, int n,
                                      int k, const float* squares_in, void* operand_out, float* squares_out,
-                                     const void* next_gain, int next_gain_dtype, hipStream_t stream) {
+                                     const void* next_gain, int next_gain_dtype, float limit, hipStream_t stream) {
     LEONE_REQUIRE(x && w && y, "gemm_fused: null pointer");
     LEONE_REQUIRE(!w_tiled || (k % 64 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0),
                   "gemm_fused: tiled weights need K %d to be a multiple of 64", k);
@@ -357,16 +358,17 @@ extern "C" int leone_gemm_fused_bf16(const void* x, int in_mode, const int* rows
     LEONE_REQUIRE(in_mode != kInPrepared || (k % 64 == 0 && static_cast<long>(m) * (k / 64) <= 8 * 256 &&
                                              reinterpret_cast<uintptr_t>(squares_in) % 16 == 0),
                   "gemm_fused: the prepared input takes K %d a multiple of 64 with rows x K / 64 up to 2048", k);
-    LEONE_REQUIRE(out_mode >= kOutStore && out_mode <= kOutPrepare + 1, "gemm_fused: unknown output mode %d", out_mode);
-    const int act = out_mode == kOutPrepare + 1 ? kGateGeluTanh : kGateSilu;
-    if (out_mode == kOutPrepare + 1) out_mode = kOutGated;
+    LEONE_REQUIRE(out_mode >= kOutStore && out_mode <= kOutPrepare + 2, "gemm_fused: unknown output mode %d", out_mode);
+    const int act = out_mode == kOutPrepare + 1 ? kGateGeluTanh : out_mode == kOutPrepare + 2 ? kGateClampedSwish : kGateSilu;
+    if (out_mode > kOutPrepare) out_mode = kOutGated;
+    LEONE_REQUIRE(act != kGateClampedSwish || limit > 0.f, "gemm_fused: the clamped activation needs a positive limit, found %g", limit);
     LEONE_REQUIRE(out_mode != kOutGated || n % 16 == 0, "gemm_fused: gated output needs N %d to be a multiple of 16", n);
     LEONE_REQUIRE(out_mode != kOutStore || out_dtype == kF32 || out_dtype == kBF16, "gemm_fused: unknown output type");
     LEONE_REQUIRE(out_mode != kOutPrepare || (operand_out && squares_out && next_gain &&
                                               (next_gain_dtype == kF32 || next_gain_dtype == kBF16)),
                   "gemm_fused: the prepare output needs room for the operand and the sums, and the next gain");
     FusedArgs a{x, rows, gain, gain_dtype, eps, static_cast<const bf16_t*>(w), y, m, n, k,
-                squares_in, static_cast<bf16_t*>(operand_out), squares_out, next_gain, next_gain_dtype, act};
+                squares_in, static_cast<bf16_t*>(operand_out), squares_out, next_gain, next_gain_dtype, act, limit};
 #define LEONE_FUSED_OUT(IN)                                                                  \
     switch (out_mode) {                                                                      \
         case kOutStore:                                                                      \

@@ -49,6 +49,7 @@ struct RowsArgs {
     int m, n, k;
     int chunks_per_split;
     int act;           // gated: the gate's activation (GateAct)
+    float limit;       // gated: what that activation holds gate and up to
 };
 
 
@@ -251,7 +252,7 @@ gemm_rows_kernel(RowsArgs a) {
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
                     const float gate = acc[t][r];
-                    v[r] = gate_act(gate, a.act) * up[r];
+                    v[r] = glu_value(gate, up[r], a.act, a.limit);
                 }
                 uint2 packed;
                 packed.x = bf16_bits_from_float(v[0]) | (static_cast<uint32_t>(bf16_bits_from_float(v[1])) << 16);
@@ -372,15 +373,18 @@ extern "C" int leone_gemm_rows_shape_built(int m, int waves, int ways) {
 }
 
 extern "C" int leone_gemm_rows_bf16(const void* x, const void* w, int w_tiled, void* y, int out_mode, int out_dtype,
-                                    int m, int n, int k, int splits, long plane, int waves, int ways, hipStream_t stream) {
+                                    int m, int n, int k, int splits, long plane, int waves, int ways, float limit,
+                                    hipStream_t stream) {
     LEONE_REQUIRE(x && w && y, "gemm_rows: null pointer");
     LEONE_REQUIRE(!w_tiled || (k % 64 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0),
                   "gemm_rows: tiled weights need K %d to be a multiple of 64", k);
     LEONE_REQUIRE(m > 0 && m <= 128, "gemm_rows: rows %d must be in 1..128", m);
     LEONE_REQUIRE(n > 0 && k > 0 && k % 8 == 0, "gemm_rows: sizes %d x %d: K must be a positive multiple of 8", n, k);
-    LEONE_REQUIRE(out_mode >= kRowsStore && out_mode <= kRowsPlanes + 1, "gemm_rows: unknown output mode %d", out_mode);
-    const int act = out_mode == kRowsPlanes + 1 ? kGateGeluTanh : kGateSilu;     // 4: as 2 with the tanh form of gelu on the gate
-    if (out_mode == kRowsPlanes + 1) out_mode = kRowsGated;
+    LEONE_REQUIRE(out_mode >= kRowsStore && out_mode <= kRowsPlanes + 2, "gemm_rows: unknown output mode %d", out_mode);
+    // 4: as 2 with the tanh form of gelu on the gate; 5: as 2 with gate and up held to `limit` (GateAct 2)
+    const int act = out_mode == kRowsPlanes + 1 ? kGateGeluTanh : out_mode == kRowsPlanes + 2 ? kGateClampedSwish : kGateSilu;
+    if (out_mode > kRowsPlanes) out_mode = kRowsGated;
+    LEONE_REQUIRE(act != kGateClampedSwish || limit > 0.f, "gemm_rows: the clamped activation needs a positive limit, found %g", limit);
     LEONE_REQUIRE(out_mode != kRowsGated || n % 16 == 0, "gemm_rows: gated output needs N %d to be a multiple of 16", n);
     LEONE_REQUIRE(out_mode != kRowsStore || out_dtype == kF32 || out_dtype == kBF16, "gemm_rows: unknown output type");
     LEONE_REQUIRE(waves == 4 || waves == 6 || waves == 8, "gemm_rows: %d tiles of W a workgroup", waves);
@@ -393,7 +397,7 @@ extern "C" int leone_gemm_rows_bf16(const void* x, const void* w, int w_tiled, v
     const int per = ceil_div(chunks, splits);
     LEONE_REQUIRE(per * (splits - 1) < chunks, "gemm_rows: %d ranges of K would leave one empty (%d chunks)", splits, chunks);
     LEONE_REQUIRE(out_mode != kRowsPlanes || plane >= static_cast<long>(m) * n, "gemm_rows: planes overlap");
-    RowsArgs a{static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(w), y, plane, m, n, k, per, act};
+    RowsArgs a{static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(w), y, plane, m, n, k, per, act, limit};
     int status = 0;
 #define LEONE_ROWS_CASE(MT) \
     case MT: status = launch_rows_waves<MT>(a, out_mode, out_dtype, splits, waves, ways, w_tiled != 0, stream); break;

@@ -39,6 +39,14 @@ void CacheManager::set_keep_first(int g, int positions) {
     groups_[g].keep_first = positions;
 }
 
+void CacheManager::set_chunk(int g, int positions) {
+    if (g < 0 || g >= group_count()) throw CacheError("no cache group " + std::to_string(g));
+    if (positions < 0) throw std::invalid_argument("a chunk must not be negative");
+    if (positions > 0 && groups_[g].window != 0) throw std::invalid_argument("a cache group has a window or chunks, not both");
+    if (!requests_.empty()) throw CacheError("chunks are set before requests are admitted");
+    groups_[g].chunk = positions;
+}
+
 int CacheManager::max_blocks(int g) const {
     const int pt = groups_.at(g).page_tokens;
     return (max_context_ + pt - 1) / pt;
@@ -151,7 +159,7 @@ int CacheManager::fork(RequestKey parent, RequestKey child, int tokens) {
     for (int gi = 0; gi < group_count(); ++gi) {
         const GroupSpec& g = groups_[gi];
         const int blocks = shared / g.page_tokens;
-        const int first = g.window == 0 ? 0 : std::max(0, shared - (g.window - 1)) / g.page_tokens;
+        const int first = g.first_readable(shared) / g.page_tokens;
         const std::vector<int>& table = source.tables[gi];
         std::vector<int> pages(blocks, -1);
         for (int b = 0; b < blocks; ++b) {
@@ -188,8 +196,8 @@ void CacheManager::truncate(RequestKey request, int position) {
         if (position % g.page_tokens && keep <= size && table[keep - 1] >= 0 && refs_[gi][table[keep - 1]] > 1)
             throw CacheError("group " + std::to_string(gi) + ": the page holding position " + std::to_string(position) +
                              " is shared; truncate to a multiple of " + std::to_string(g.page_tokens));
-        if (g.window != 0) {
-            const int reach = std::max(0, position - (g.window - 1)) / g.page_tokens;
+        if (g.forgets()) {
+            const int reach = g.first_readable(position) / g.page_tokens;
             for (int b = 0; b < std::min(keep, size); ++b)
                 if ((b >= reach || b < g.kept_blocks()) && table[b] < 0)
                     throw CacheError("group " + std::to_string(gi) + ": keys before position " + std::to_string(position) +
@@ -245,11 +253,10 @@ void CacheManager::commit(RequestKey request, int tokens) {
     for (int gi = 0; gi < group_count(); ++gi) {
         const GroupSpec& g = groups_[gi];
         state.pending_blocks[gi].clear();
-        if (g.window == 0) continue;
-        // The next query sits at position `length` and reads keys >= length - window + 1.
-        const int reach = state.length - (g.window - 1);
+        if (!g.forgets()) continue;
+        // The next query sits at position `length` and reads keys from first_readable(length) on.
         std::vector<int>& table = state.tables[gi];
-        const int end = std::min(static_cast<int>(table.size()), std::max(0, reach) / g.page_tokens);
+        const int end = std::min(static_cast<int>(table.size()), g.first_readable(state.length) / g.page_tokens);
         for (int b = g.kept_blocks(); b < end; ++b)               // the kept first positions keep their pages
             if (table[b] >= 0) {
                 drop(gi, table[b]);

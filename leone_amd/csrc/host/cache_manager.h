@@ -8,8 +8,8 @@
 //   * a group is a set of layers with the same cache need; it has its own pages, free list and one
 //     block table per request (logical block -> page id, -1 where no page is mapped);
 //   * reserve maps pages for the positions a step is about to write, in every group, all or
-//     nothing; commit advances the request's length and, for a windowed group, hands back pages
-//     that no later query can reach; rollback undoes an uncommitted reservation; release returns
+//     nothing; commit advances the request's length and, for a windowed or chunked group, hands back
+//     pages that no later query can reach; rollback undoes an uncommitted reservation; release returns
 //     everything a request holds, pages and state slot, at once;
 //   * a state slot is an index into per-request storage of fixed size, handed out on admission
 //     and returned on release;
@@ -35,9 +35,20 @@ struct GroupSpec {
     int page_tokens;
     int window;   // 0: every position is kept; otherwise only the last `window`
     int keep_first = 0;   // of a windowed group: the first positions stay in sight whatever the window, so their pages stay
+    int chunk = 0;        // of a group without a window: positions fall into chunks of so many, counted from 0, and a query
+                          // reads keys of its own chunk only (0: no chunks)
 
     // Pages that hold the kept first positions (they are never handed back by a window that passes).
     int kept_blocks() const { return window == 0 ? 0 : (keep_first + page_tokens - 1) / page_tokens; }
+    // Whether keys leave sight for good at all.
+    bool forgets() const { return window != 0 || chunk != 0; }
+    // The first position that a query at position `at`, or any later one, can read (kept first positions aside).
+    int first_readable(int at) const {
+        if (chunk != 0) return at / chunk * chunk;
+        return window == 0 || at < window ? 0 : at - (window - 1);
+    }
+    // Most positions that are in sight ahead of a query at once (without a query's own).
+    int reach() const { return chunk != 0 ? chunk - 1 : window - 1; }
 };
 
 // A reservation needs more free pages than a group has; nothing was changed.
@@ -68,6 +79,8 @@ public:
     int max_blocks(int g) const;
     // The first `positions` positions of group g stay readable whatever its window (before any request is admitted).
     void set_keep_first(int g, int positions);
+    // Group g's queries read keys of their own chunk of `positions` positions only (before any request is admitted).
+    void set_chunk(int g, int positions);
     bool has(RequestKey request) const { return requests_.count(request) != 0; }
     std::vector<RequestKey> requests() const;   // every admitted request, ascending
     int length(RequestKey request) const { return get(request).length; }

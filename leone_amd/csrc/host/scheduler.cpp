@@ -57,11 +57,11 @@ Reject Scheduler::reject_reason(RequestKey request, int prompt, std::int64_t out
     for (int gi = 0; gi < cache_.group_count(); ++gi) {
         const GroupSpec& g = cache_.group(gi);
         std::int64_t need;
-        if (g.window == 0) {
+        if (!g.forgets()) {
             need = (held + g.page_tokens - 1) / g.page_tokens;
         } else {
             const std::int64_t portion = std::min(policy_.prefill_chunk_tokens, policy_.max_step_tokens);
-            const std::int64_t span = std::min<std::int64_t>(held, g.window - 1 + portion);
+            const std::int64_t span = std::min<std::int64_t>(held, g.reach() + portion);
             need = std::min<std::int64_t>((span + g.page_tokens - 1) / g.page_tokens + 1 + g.kept_blocks(),
                                           (held + g.page_tokens - 1) / g.page_tokens);
         }
@@ -266,7 +266,7 @@ bool Scheduler::room_for(int tokens) const {
     for (int gi = 0; gi < cache_.group_count(); ++gi) {
         const GroupSpec& g = cache_.group(gi);
         const std::int64_t span =
-            g.window == 0 ? tokens : std::min<std::int64_t>(tokens, g.window - 1 + policy_.prefill_chunk_tokens);
+            !g.forgets() ? tokens : std::min<std::int64_t>(tokens, g.reach() + policy_.prefill_chunk_tokens);
         const std::int64_t pages = std::min<std::int64_t>((span + g.page_tokens - 1) / g.page_tokens + g.kept_blocks(),
                                                           (tokens + g.page_tokens - 1) / g.page_tokens);
         if (pages > cache_.free_pages(gi)) return false;

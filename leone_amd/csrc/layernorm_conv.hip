@@ -238,6 +238,52 @@ __global__ void head_norm_gate_kernel(const float* __restrict__ o, const float* 
     for (int j = lane + kKept * kWave; j < vdim; j += kWave) finish(j, fetch(j));
 }
 
+// The same for runs too long for a wave: a workgroup a (row, head), the values kept in registers between the passes where they
+// fit, sums added in a fixed order.
+constexpr int kWideHeadFrom = 1024;                            // runs of more columns go here
+template <typename TOut, int kThreads>
+__global__ void __launch_bounds__(kThreads)
+head_norm_gate_wide_kernel(const float* __restrict__ o, const float* __restrict__ dot, const float* __restrict__ top, AnyVec gain,
+                           int gain_per_head, const float* __restrict__ gate, long gate_stride, int act, float eps,
+                           TOut* __restrict__ out, int heads, int vdim, int gate_first) {
+    __shared__ float scratch[kThreads / kWave];
+    const int row = blockIdx.x, head = blockIdx.y;
+    const long at = static_cast<long>(row) * heads + head;
+    const float* src = o + at * vdim;
+    const float under = dot ? fmaxf(fabsf(dot[at]), expf(-top[at])) + 1e-6f : 1.f;
+    const float* gate_row = gate ? gate + static_cast<long>(row) * gate_stride + static_cast<long>(head) * vdim : nullptr;
+    auto fetch = [&](int j) {
+        const float v = src[j] / under;
+        return (gate_first && gate_row) ? v * activate(gate_row[j], act) : v;
+    };
+    constexpr int kKept = 4;
+    float kept[kKept], open[kKept];
+    float ss = 0.f;
+#pragma unroll
+    for (int n = 0; n < kKept; ++n) {
+        const int j = threadIdx.x + n * kThreads;
+        kept[n] = j < vdim ? fetch(j) : 0.f;
+        open[n] = (gate_row && !gate_first && j < vdim) ? gate_row[j] : 0.f;     // asked for ahead of the sum
+        ss = fmaf(kept[n], kept[n], ss);
+    }
+    for (int j = threadIdx.x + kKept * kThreads; j < vdim; j += kThreads) {
+        const float v = fetch(j);
+        ss = fmaf(v, v, ss);
+    }
+    const float inv = 1.0f / sqrtf(block_sum<kThreads>(ss, scratch) / static_cast<float>(vdim) + eps);
+    TOut* dst = out + at * vdim;
+    auto finish = [&](int j, float v, float g) {
+        v *= inv;
+        if (gain.ptr) v *= load_any(gain, gain_per_head ? static_cast<long>(head) * vdim + j : j);
+        if (gate_row && !gate_first) v *= activate(g, act);
+        dst[j] = from_float<TOut>(v);
+    };
+#pragma unroll
+    for (int n = 0; n < kKept; ++n)
+        if (threadIdx.x + n * kThreads < static_cast<unsigned>(vdim)) finish(threadIdx.x + n * kThreads, kept[n], open[n]);
+    for (int j = threadIdx.x + kKept * kThreads; j < vdim; j += kThreads) finish(j, fetch(j), gate_row && !gate_first ? gate_row[j] : 0.f);
+}
+
 constexpr int kMaxBranches = 4;
 struct Branches {
     const float* rows[kMaxBranches];
@@ -409,6 +455,23 @@ extern "C" int leone_head_norm_gate_ordered(const float* o, const float* dot, co
     LEONE_REQUIRE(act >= kActNone && act <= kActSilu && eps > 0.f, "head_norm_gate: activation %d, eps %g", act, eps);
     LEONE_REQUIRE(rows <= 0x7fffffff && ceil_div(heads, 4) <= 65535, "head_norm_gate: too many heads");
     const AnyVec vg{gain, gain_dtype};
+    if (vdim > kWideHeadFrom) {
+        LEONE_REQUIRE(heads <= 65535, "head_norm_gate: too many heads");
+#define LEONE_WIDE_HEAD(T, THREADS)                                                                                           \
+    head_norm_gate_wide_kernel<T, THREADS><<<dim3(rows, heads), THREADS, 0, stream>>>(o, dot, top, vg, gain_per_head, gate, gate_stride, \
+                                                                                    act, eps, static_cast<T*>(out), heads, vdim, gate_first)
+        // few rows: a row in as few trips to memory as threads allow; many rows: more rows in flight a compute unit
+        if (out_dtype == kF32) {
+            if (rows >= kNormManyRows) LEONE_WIDE_HEAD(float, kNormThreadsMany);
+            else LEONE_WIDE_HEAD(float, kNormThreadsFew);
+        } else {
+            if (rows >= kNormManyRows) LEONE_WIDE_HEAD(bf16_t, kNormThreadsMany);
+            else LEONE_WIDE_HEAD(bf16_t, kNormThreadsFew);
+        }
+#undef LEONE_WIDE_HEAD
+        LEONE_LAUNCH_CHECK("head_norm_gate");
+        return 0;
+    }
     const dim3 grid(rows, ceil_div(heads, 4));
     if (out_dtype == kF32)
         head_norm_gate_kernel<float><<<grid, 4 * kWave, 0, stream>>>(o, dot, top, vg, gain_per_head, gate, gate_stride, act, eps,

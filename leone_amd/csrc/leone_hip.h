@@ -118,7 +118,7 @@ int leone_gemm_f32(const float* a, const float* b, float* c, int m, int n, int k
 int leone_gemm_fused_bf16(const void* x, int in_mode, const int* rows, const void* gain, int gain_dtype, float eps,
                           const void* w, int w_tiled, void* y, int out_mode, int out_dtype, int m, int n, int k,
                           const float* squares_in, void* operand_out, float* squares_out, const void* next_gain,
-                          int next_gain_dtype, hipStream_t stream);
+                          int next_gain_dtype, float limit, hipStream_t stream);
 
 // Y[M,N] = X[M,K] . W[N,K]^T for bfloat16 X and W, M in 1..leone_gemm_rows_max_rows(), K a multiple of 8: W is
 // streamed once, X goes through shared memory.  out_mode 0: y[M,N] of out_dtype; 1: y float32 [M,N] += product;
@@ -132,7 +132,7 @@ int leone_gemm_rows_max_rows();
 int leone_gemm_rows_chunk(int m);
 int leone_gemm_rows_shape_built(int m, int waves, int ways);
 int leone_gemm_rows_bf16(const void* x, const void* w, int w_tiled, void* y, int out_mode, int out_dtype, int m, int n, int k,
-                         int splits, long plane, int waves, int ways, hipStream_t stream);
+                         int splits, long plane, int waves, int ways, float limit, hipStream_t stream);
 
 // The vendor library's product for more rows than the kernels above take, Y[M,N] = X[M,K] . W[N,K]^T (or Y +=
 // with `accumulate`, Y float32), X and W bfloat16, Y of out_dtype, float accumulation, with the library's
@@ -263,7 +263,7 @@ int leone_exp_gates(const float* proj, long stride, int i_off, int f_off, const 
                     int bias_dtype, float cap, const int* spans, int entries, float* state, long slot_stride,
                     long head_stride, long top_at, int write_state, float* coef, float* top, int heads, hipStream_t stream);
 int leone_outer_scan(const float* proj, long stride, int q_off, int k_off, int v_off, const float* coef,
-                     const float* decay, int no_input, int accumulate, int norm_column, float q_scale, float k_scale,
+                     const float* decay, int no_input, int accumulate, int norm_column, float q_scale, float k_scale, int silu,
                      const float* cos_table, const float* sin_table, int rotary_dim, int table_positions,
                      const int* positions, const int* segments, int n_segments, const float* state_in, long in_stride,
                      float* state_out, long out_stride, long head_stride, float* decay_product, float* out, float* dot,
@@ -271,7 +271,7 @@ int leone_outer_scan(const float* proj, long stride, int q_off, int k_off, int v
 int leone_outer_chain(const int* links, int n_links, float* work, long work_stride, const float* product, float* state,
                       long slot_stride, long head_stride, int per_head, int heads, int write_state, hipStream_t stream);
 int leone_delta_scan(const float* qkv, long stride, int q_off, int k_off, int v_off, const float* beta,
-                     long beta_stride, const float* step, long step_stride, const void* rate_log,
+                     long beta_stride, const float* step, long step_stride, int per_head, const void* rate_log,
                      const void* step_bias, int vec_dtype, float q_scale, float unit_eps, int no_input, int accumulate,
                      const int* segments, int n_segments, const float* state_in, long in_stride, float* state_out,
                      long out_stride, float* transition, float* out, int heads, int kv_heads, int dim, int vdim,
@@ -280,11 +280,13 @@ int leone_delta_chain(const int* links, int n_links, float* work, long work_stri
                       long slot_stride, int heads, int dim, int vdim, int write_state, hipStream_t stream);
 
 // ---- a token table with a learned position table added, norms behind sublayers, kept first keys, routed experts ----
-// leone_embed, and place_table[positions[r], :] (of the table's type, [places, hidden]) added unscaled.
+// leone_embed, and place_table[positions[r], :] (of the table's type, [places, hidden], may be null) added unscaled; copy (float
+// [rows, hidden], may be null) receives the same rows once more.
 int leone_embed_placed(const void* table, int dtype, const int* tokens, float* out, int rows, int hidden, int vocab,
-                       float scale, const void* place_table, const int* positions, int places, hipStream_t stream);
-// gate_up as for leone_swiglu; act: 0 silu, 1 the tanh form of gelu on the gate.
-int leone_glu(const void* gate_up, void* out, int dtype, int rows, int ffn, int act, hipStream_t stream);
+                       float scale, const void* place_table, const int* positions, int places, float* copy, hipStream_t stream);
+// gate_up as for leone_swiglu; act: 0 silu, 1 the tanh form of gelu on the gate, 2 gate and up held to `limit`:
+// g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1).
+int leone_glu(const void* gate_up, void* out, int dtype, int rows, int ffn, int act, float limit, hipStream_t stream);
 // x[r] += rmsnorm(sum of the delta's planes)[r] * gain (delta float32, may be null); then y[r] = x[r] in y_dtype
 // (y may be null), or, with gain2, y[i] = rmsnorm(x[rows ? rows[i] : i]) * gain2 (with rows, x is not written).
 int leone_add_normed(float* x, const float* delta, int delta_planes, long delta_plane, const void* gain, int gain_dtype,
@@ -390,25 +392,26 @@ int leone_residual_norm(float* x, const float* delta, int planes, long plane, fl
 int leone_depth_mix(float* x, const float* delta, int planes, long plane, float scale, float* history, long slot_stride,
                     int count, const void* weight, int weight_dtype, long total, hipStream_t stream);
 // The attention kernels with a cap on the scores (0: none), a sink a head in the denominator and results turned back by the
-// row's own angles (null: none); see score_shape.h.
+// row's own angles (null: none); see score_shape.h.  chunk > 0 (no window, no kept first keys): a row sees the keys of its own
+// chunk of so many positions, counted from 0.
 int leone_attention_rows_shaped(const void* q, void* out, const void* k_pool, const void* v_pool, int dtype, const int* positions,
                                 const int* row_entry, const int* block_table, int max_blocks, int rows, int q_heads, int kv_heads,
                                 int head_dim, int v_dim, int page_tokens, float scale, int window, const float* gate,
                                 long gate_stride, int keep_first, int gate_each, const float* slopes, float temp_coef,
                                 int temp_every, float cap, const float* sinks, const float* turn_cos, const float* turn_sin,
-                                int turn_positions, int turn_pairing, hipStream_t stream);
+                                int turn_positions, int turn_pairing, int chunk, hipStream_t stream);
 int leone_attention_decode_shaped(const void* q, void* out, const void* k_pool, const void* v_pool, const int* positions,
                                   const int* row_entry, const int* block_table, int max_blocks, float* part_acc, float* part_ml,
                                   int rows, int q_heads, int kv_heads, int head_dim, int page_tokens, float scale, int window,
                                   int splits, int keep_first, const float* slopes, float temp_coef, int temp_every, float cap,
                                   const float* sinks, const float* turn_cos, const float* turn_sin, int turn_positions,
-                                  int turn_pairing, hipStream_t stream);
+                                  int turn_pairing, int chunk, hipStream_t stream);
 int leone_attention_prefill_shaped(const void* q, void* out, const void* k_pool, const void* v_pool, const int* positions,
                                    const int* tiles, int n_groups, const int* block_table, int max_blocks, int q_heads,
                                    int kv_heads, int head_dim, int page_tokens, float scale, int window, float* part_acc,
                                    float* part_ml, int splits, int keep_first, const float* slopes, float temp_coef,
                                    int temp_every, float cap, const float* sinks, const float* turn_cos, const float* turn_sin,
-                                   int turn_positions, int turn_pairing, hipStream_t stream);
+                                   int turn_positions, int turn_pairing, int chunk, hipStream_t stream);
 // Attention whose heads' scaled scores are mixed by talk [q_heads, q_heads] before the softmax.
 int leone_attention_rows_talk(const void* q, void* out, const void* k_pool, const void* v_pool, int dtype, const void* talk,
                               int talk_dtype, const int* positions, const int* row_entry, const int* block_table, int max_blocks,
@@ -440,6 +443,11 @@ int leone_branch_norm(float* x, const void* const* term_rows, const int* term_pl
                       const float* term_factor, const void* const* term_scale, const int* term_scale_dtype, int terms,
                       const void* const* gains, const int* gain_dtypes, void* const* outs, int norms, int out_dtype, float eps,
                       int groups, const int* rows, int n_rows, int hidden, hipStream_t stream);
+// x += the same sum; operand [n, 2 hidden] (out_dtype) = [x | first], and x becomes `next` (one vector for every row; null: zeros).
+int leone_stream_join(float* x, const void* const* term_rows, const int* term_planes, const long* term_plane,
+                      const float* term_factor, const void* const* term_scale, const int* term_scale_dtype, int terms,
+                      const float* first, const void* next, int next_dtype, void* operand, int out_dtype, int n_rows, int hidden,
+                      hipStream_t stream);
 // The token before beside the token itself, decays from a low-rank product, and the memory they drive (see time_mix.hip).
 int leone_token_mix(const void* h, int dtype, const void* mu, int mu_dtype, int mixes, const float* state, float* state_out,
                     const int* spans, int entries, const int* row_entry, void* out, int rows, int hidden, int single_rows,

@@ -6,8 +6,9 @@
 //                running maximum m_t = max(f_t + m_(t-1), i_t), a_t = exp(f_t + m_(t-1) - m_t),
 //                b_t = exp(i_t - m_t), together with the normaliser n_t = a_t n_(t-1) + b_t k_t carried as one
 //                more column of S (a value that is always 1), whose read-out n_t . q_t and m_t go out beside o
-//                for the division that follows.  Rotary positions on q and k if tables come.
-//   delta_scan   S <- g_t * S (g per key channel);  u = beta_t (v_t - S^T k_t);  S <- S + k_t u^T;  o_t = S^T q_t
+//                for the division that follows.  Rotary positions on q and k if tables come; q, k and v through silu first if
+//                asked for.
+//   delta_scan   S <- g_t * S (g per key channel, or one a head);  u = beta_t (v_t - S^T k_t);  S <- S + k_t u^T;  o_t = S^T q_t
 //                with q and k made unit vectors per head first.
 //
 // A workgroup of four waves owns a run of columns of one head of one segment (a request's rows in the step, or a
@@ -52,6 +53,7 @@ struct OuterScanArgs {
     int accumulate;             // read-outs are added to what out and dot hold
     int norm_column;            // one more column whose value is always 1 (the normaliser), read out into dot
     float q_scale, k_scale;
+    int silu;                   // q, k and v pass through silu first
     const float* cos_table;     // [table_positions, rot_half] or null
     const float* sin_table;
     int rot_half, table_positions;
@@ -68,11 +70,13 @@ struct OuterScanArgs {
     int heads, dim, vdim;
 };
 
-__device__ inline float rotated(const float* src, int i, int dim, const float* cos_row, const float* sin_row, int rot_half) {
-    const float x = src[i];
+__device__ inline float silu_if(float x, int silu) { return silu ? x / (1.0f + expf(-x)) : x; }
+
+__device__ inline float rotated(const float* src, int i, int silu, const float* cos_row, const float* sin_row, int rot_half) {
+    const float x = silu_if(src[i], silu);
     if (!cos_row || i >= 2 * rot_half) return x;
-    if (i < rot_half) return x * cos_row[i] - src[i + rot_half] * sin_row[i];
-    return x * cos_row[i - rot_half] + src[i - rot_half] * sin_row[i - rot_half];
+    if (i < rot_half) return x * cos_row[i] - silu_if(src[i + rot_half], silu) * sin_row[i];
+    return x * cos_row[i - rot_half] + silu_if(src[i - rot_half], silu) * sin_row[i - rot_half];
 }
 
 __device__ inline float soft_cap_f(float z, float cap) { return cap * tanhf(z / cap); }
@@ -186,8 +190,8 @@ __global__ void __launch_bounds__(kScanThreads) outer_scan_kernel(OuterScanArgs 
                 const float* c = p.cos_table ? p.cos_table + static_cast<long>(pos) * p.rot_half : nullptr;
                 const float* s = p.cos_table ? p.sin_table + static_cast<long>(pos) * p.rot_half : nullptr;
                 const float* base = p.proj + row * p.stride;
-                qv = rotated(base + p.q_off + head * p.dim, i, p.dim, c, s, p.rot_half) * p.q_scale;
-                if (!p.no_input) kv = rotated(base + p.k_off + head * p.dim, i, p.dim, c, s, p.rot_half) * p.k_scale;
+                qv = rotated(base + p.q_off + head * p.dim, i, p.silu, c, s, p.rot_half) * p.q_scale;
+                if (!p.no_input) kv = rotated(base + p.k_off + head * p.dim, i, p.silu, c, s, p.rot_half) * p.k_scale;
             }
             sq[idx] = qv;
             sk[idx] = kv;
@@ -221,7 +225,7 @@ __global__ void __launch_bounds__(kScanThreads) outer_scan_kernel(OuterScanArgs 
                     float bv[kLaneCols];
 #pragma unroll
                     for (int c = 0; c < kLaneCols; ++c) {
-                        const float v = is_value[c] ? p.proj[row * p.stride + p.v_off + head * p.vdim + col[c]] : 1.f;
+                        const float v = is_value[c] ? silu_if(p.proj[row * p.stride + p.v_off + head * p.vdim + col[c]], p.silu) : 1.f;
                         bv[c] = sb[t] * v;
                         acc[c] = 0.f;
                     }
@@ -293,10 +297,11 @@ struct DeltaScanArgs {
     int q_off, k_off, v_off;
     const float* beta;          // [rows, beta_stride]: pre-activation of the write strength, one a head
     long beta_stride;
-    const float* step;          // [rows, step_stride]: pre-activation of the step size, heads x dim
+    const float* step;          // [rows, step_stride]: pre-activation of the step size, heads x dim, or one a head
     long step_stride;
+    int per_head;               // one step size, and so one decay, a head
     AnyVec rate_log;            // [heads]: decay = exp(-exp(rate_log) * softplus(step + step_bias))
-    AnyVec step_bias;           // [heads * dim]
+    AnyVec step_bias;           // [heads * dim], per_head: [heads]
     float q_scale, unit_eps;
     int no_input;               // v is taken as 0: what a state carries through the rows, and what is read of it
     int accumulate;             // read-outs are added to what out holds
@@ -367,12 +372,15 @@ __global__ void __launch_bounds__(kScanThreads) delta_scan_kernel(DeltaScanArgs 
                 }
                 const float qinv = p.q_scale / sqrtf(qq + p.unit_eps);
                 const float kinv = 1.0f / sqrtf(kk + p.unit_eps);
+                const float head_decay = p.per_head
+                    ? expf(-rate * softplus_f(p.step[row * p.step_stride + head] + load_any(p.step_bias, head))) : 1.f;
                 for (int i = sub; i < dkp; i += kRowLanes) {
                     const bool in = i < p.dim;
                     sq[t * dkp + i] = in ? qs[i] * qinv : 0.f;
                     sk[t * dkp + i] = in ? ks[i] * kinv : 0.f;
                     const long ch = static_cast<long>(head) * p.dim + i;
-                    sg[t * dkp + i] = in ? expf(-rate * softplus_f(p.step[row * p.step_stride + ch] + load_any(p.step_bias, ch))) : 1.f;
+                    if (p.per_head) sg[t * dkp + i] = head_decay;
+                    else sg[t * dkp + i] = in ? expf(-rate * softplus_f(p.step[row * p.step_stride + ch] + load_any(p.step_bias, ch))) : 1.f;
                 }
                 if (sub == 0) sbeta[t] = 1.0f / (1.0f + expf(-p.beta[row * p.beta_stride + head]));
             }
@@ -509,7 +517,7 @@ extern "C" int leone_exp_gates(const float* proj, long stride, int i_off, int f_
 
 extern "C" int leone_outer_scan(const float* proj, long stride, int q_off, int k_off, int v_off, const float* coef,
                                 const float* decay, int no_input, int accumulate, int norm_column, float q_scale,
-                                float k_scale, const float* cos_table, const float* sin_table, int rotary_dim,
+                                float k_scale, int silu, const float* cos_table, const float* sin_table, int rotary_dim,
                                 int table_positions, const int* positions, const int* segments, int n_segments,
                                 const float* state_in, long in_stride, float* state_out, long out_stride, long head_stride,
                                 float* decay_product, float* out, float* dot, int heads, int dim, int vdim,
@@ -529,7 +537,7 @@ extern "C" int leone_outer_scan(const float* proj, long stride, int q_off, int k
     LEONE_REQUIRE(stride >= q_off + heads * dim && stride >= k_off + heads * dim && stride >= v_off + heads * vdim &&
                   q_off >= 0 && k_off >= 0 && v_off >= 0, "outer_scan: the projection's rows of %ld do not hold the named columns", stride);
     OuterScanArgs a{proj, stride, q_off, k_off, v_off, coef, decay, no_input, accumulate, norm_column, q_scale, k_scale,
-                    cos_table, sin_table, cos_table ? rotary_dim / 2 : 0, cos_table ? table_positions : 1, positions,
+                    silu, cos_table, sin_table, cos_table ? rotary_dim / 2 : 0, cos_table ? table_positions : 1, positions,
                     reinterpret_cast<const Segment*>(segments), state_in, in_stride, state_out, out_stride, head_stride,
                     decay_product, out, dot, heads, dim, vdim};
     const int groups = lane_groups(dim);
@@ -555,7 +563,7 @@ extern "C" int leone_outer_chain(const int* links, int n_links, float* work, lon
 }
 
 extern "C" int leone_delta_scan(const float* qkv, long stride, int q_off, int k_off, int v_off, const float* beta,
-                                long beta_stride, const float* step, long step_stride, const void* rate_log,
+                                long beta_stride, const float* step, long step_stride, int per_head, const void* rate_log,
                                 const void* step_bias, int vec_dtype, float q_scale, float unit_eps, int no_input,
                                 int accumulate, const int* segments, int n_segments, const float* state_in, long in_stride,
                                 float* state_out, long out_stride, float* transition, float* out, int heads, int kv_heads,
@@ -569,9 +577,9 @@ extern "C" int leone_delta_scan(const float* qkv, long stride, int q_off, int k_
     LEONE_REQUIRE((!state_in || in_stride >= per_slot) && (!state_out || out_stride >= per_slot),
                   "delta_scan: states of %ld floats do not fit", per_slot);
     LEONE_REQUIRE(q_off >= 0 && k_off >= 0 && v_off >= 0 && stride >= q_off + kv_heads * dim && stride >= k_off + kv_heads * dim &&
-                  stride >= v_off + heads * vdim && beta_stride >= heads && step_stride >= static_cast<long>(heads) * dim,
+                  stride >= v_off + heads * vdim && beta_stride >= heads && step_stride >= static_cast<long>(heads) * (per_head ? 1 : dim),
                   "delta_scan: rows too short for the named columns");
-    DeltaScanArgs a{qkv, stride, q_off, k_off, v_off, beta, beta_stride, step, step_stride, AnyVec{rate_log, vec_dtype},
+    DeltaScanArgs a{qkv, stride, q_off, k_off, v_off, beta, beta_stride, step, step_stride, per_head, AnyVec{rate_log, vec_dtype},
                     AnyVec{step_bias, vec_dtype}, q_scale, unit_eps, no_input, accumulate,
                     reinterpret_cast<const Segment*>(segments), state_in, in_stride, state_out, out_stride, transition, out,
                     heads, kv_heads, dim, vdim};

@@ -18,13 +18,19 @@ namespace leone {
 template <typename T>
 __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict__ tokens,
                              float* __restrict__ out, int hidden, int vocab, float scale,
-                             const T* __restrict__ place_table, const int* __restrict__ positions, int places) {
+                             const T* __restrict__ place_table, const int* __restrict__ positions, int places,
+                             float* __restrict__ copy) {
     const int row = blockIdx.x;
     const int token = tokens[row];
     float* dst = out + static_cast<long>(row) * hidden;
+    float* twin = copy ? copy + static_cast<long>(row) * hidden : nullptr;     // the same row once more
+    auto put = [&](int c, float v) {
+        dst[c] = v;
+        if (twin) twin[c] = v;
+    };
     if (token < 0 || token >= vocab) {
         // The host rejects such ids before the launch; never read outside the table.
-        for (int c = threadIdx.x; c < hidden; c += blockDim.x) dst[c] = __builtin_nanf("");
+        for (int c = threadIdx.x; c < hidden; c += blockDim.x) put(c, __builtin_nanf(""));
         return;
     }
     const T* src = table + static_cast<long>(token) * hidden;
@@ -32,10 +38,10 @@ __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict_
         // a learned vector of the row's position is added (not scaled); the host checks the bound
         const int pos = positions[row];
         const T* at = place_table + static_cast<long>(pos < places ? (pos < 0 ? 0 : pos) : places - 1) * hidden;
-        for (int c = threadIdx.x; c < hidden; c += blockDim.x) dst[c] = to_float(src[c]) * scale + to_float(at[c]);
+        for (int c = threadIdx.x; c < hidden; c += blockDim.x) put(c, to_float(src[c]) * scale + to_float(at[c]));
         return;
     }
-    for (int c = threadIdx.x; c < hidden; c += blockDim.x) dst[c] = to_float(src[c]) * scale;
+    for (int c = threadIdx.x; c < hidden; c += blockDim.x) put(c, to_float(src[c]) * scale);
 }
 
 // ---- a soft cap on logits -----------------------------------------------------
@@ -192,7 +198,7 @@ struct alignas(8 * sizeof(T)) Run8 {
 };
 template <typename T>
 __global__ void __launch_bounds__(256)
-swiglu_kernel(const T* __restrict__ gate_up, T* __restrict__ out, long rows, int ffn, int act) {
+swiglu_kernel(const T* __restrict__ gate_up, T* __restrict__ out, long rows, int ffn, int act, float limit) {
     const int groups = ffn / 8;
     const int group = blockIdx.x * blockDim.x + threadIdx.x;
     if (group >= groups) return;
@@ -203,8 +209,7 @@ swiglu_kernel(const T* __restrict__ gate_up, T* __restrict__ out, long rows, int
         Run8<T> y;
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
-            const float g = to_float(gate.v[i]);
-            y.v[i] = from_float<T>(gate_act(g, act) * to_float(up.v[i]));
+            y.v[i] = from_float<T>(glu_value(to_float(gate.v[i]), to_float(up.v[i]), act, limit));
         }
         *reinterpret_cast<Run8<T>*>(out + r * ffn + 8 * static_cast<long>(group)) = y;
     }
@@ -640,7 +645,7 @@ extern "C" int leone_soft_cap(float* x, long n, float cap, hipStream_t stream) {
 
 extern "C" int leone_embed_placed(const void* table, int dtype, const int* tokens, float* out, int rows,
                                   int hidden, int vocab, float scale, const void* place_table, const int* positions,
-                                  int places, hipStream_t stream) {
+                                  int places, float* copy, hipStream_t stream) {
     if (check_dtype(dtype, "embed")) return 1;
     LEONE_REQUIRE(table && tokens && out, "embed: null pointer");
     LEONE_REQUIRE(!place_table || (positions && places > 0), "embed: a position table needs the rows' positions");
@@ -648,17 +653,17 @@ extern "C" int leone_embed_placed(const void* table, int dtype, const int* token
     const int threads = hidden >= 1024 ? 256 : 64;
     if (dtype == kF32)
         embed_kernel<float><<<rows, threads, 0, stream>>>(static_cast<const float*>(table), tokens, out, hidden, vocab, scale,
-                                                          static_cast<const float*>(place_table), positions, places);
+                                                          static_cast<const float*>(place_table), positions, places, copy);
     else
         embed_kernel<bf16_t><<<rows, threads, 0, stream>>>(static_cast<const bf16_t*>(table), tokens, out, hidden, vocab, scale,
-                                                           static_cast<const bf16_t*>(place_table), positions, places);
+                                                           static_cast<const bf16_t*>(place_table), positions, places, copy);
     LEONE_LAUNCH_CHECK("embed");
     return 0;
 }
 
 extern "C" int leone_embed(const void* table, int dtype, const int* tokens, float* out, int rows,
                            int hidden, int vocab, float scale, hipStream_t stream) {
-    return leone_embed_placed(table, dtype, tokens, out, rows, hidden, vocab, scale, nullptr, nullptr, 0, stream);
+    return leone_embed_placed(table, dtype, tokens, out, rows, hidden, vocab, scale, nullptr, nullptr, 0, nullptr, stream);
 }
 
 template <typename TD, typename TG, typename TY>
@@ -719,10 +724,11 @@ extern "C" int leone_add_rmsnorm(float* x, const void* delta, int delta_dtype, i
     return 0;
 }
 
-// act: the gate's activation (GateAct: 0 silu, 1 the tanh form of gelu).
-extern "C" int leone_glu(const void* gate_up, void* out, int dtype, int rows, int ffn, int act, hipStream_t stream) {
+// act: the gate's activation (GateAct: 0 silu, 1 the tanh form of gelu, 2 gate and up held to `limit`).
+extern "C" int leone_glu(const void* gate_up, void* out, int dtype, int rows, int ffn, int act, float limit, hipStream_t stream) {
     if (check_dtype(dtype, "swiglu")) return 1;
-    LEONE_REQUIRE(act == kGateSilu || act == kGateGeluTanh, "glu: unknown activation %d", act);
+    LEONE_REQUIRE(act == kGateSilu || act == kGateGeluTanh || (act == kGateClampedSwish && limit > 0.f),
+                  "glu: unknown activation %d (limit %g)", act, limit);
     LEONE_REQUIRE(gate_up && out, "swiglu: null pointer");
     LEONE_REQUIRE(rows > 0 && ffn > 0 && ffn % 8 == 0, "swiglu: rows %d, width %d: the width must be a positive multiple of 8", rows, ffn);
     const uintptr_t run = 8 * (dtype == kF32 ? sizeof(float) : sizeof(bf16_t));
@@ -730,15 +736,15 @@ extern "C" int leone_glu(const void* gate_up, void* out, int dtype, int rows, in
                   "swiglu: input and output must be aligned to %d bytes", static_cast<int>(run));
     const dim3 grid(ceil_div(ffn / 8, 256), rows < 32768 ? rows : 32768);
     if (dtype == kF32)
-        swiglu_kernel<float><<<grid, 256, 0, stream>>>(static_cast<const float*>(gate_up), static_cast<float*>(out), rows, ffn, act);
+        swiglu_kernel<float><<<grid, 256, 0, stream>>>(static_cast<const float*>(gate_up), static_cast<float*>(out), rows, ffn, act, limit);
     else
-        swiglu_kernel<bf16_t><<<grid, 256, 0, stream>>>(static_cast<const bf16_t*>(gate_up), static_cast<bf16_t*>(out), rows, ffn, act);
+        swiglu_kernel<bf16_t><<<grid, 256, 0, stream>>>(static_cast<const bf16_t*>(gate_up), static_cast<bf16_t*>(out), rows, ffn, act, limit);
     LEONE_LAUNCH_CHECK("swiglu");
     return 0;
 }
 
 extern "C" int leone_swiglu(const void* gate_up, void* out, int dtype, int rows, int ffn, hipStream_t stream) {
-    return leone_glu(gate_up, out, dtype, rows, ffn, kGateSilu, stream);
+    return leone_glu(gate_up, out, dtype, rows, ffn, kGateSilu, 0.f, stream);
 }
 
 extern "C" int leone_rope_table(float* cos_out, float* sin_out, double theta, int rotary_dim,

@@ -5,6 +5,13 @@
 
 namespace leone {
 
+// The first key that a query at position pos sees: the last `window` positions (0: all), or, with chunks (chunk > 0, then no
+// window), the positions of pos's own chunk of so many, counted from position 0.
+__device__ inline int first_key(int pos, int window, int chunk) {
+    if (chunk > 0) return pos - pos % chunk;
+    return (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+}
+
 // Scores held to a cap (cap > 0: score = cap * tanh(score / cap), taken on the scaled score), a sink in the denominator
 // (sinks float [q_heads] or null: exp(sinks[h]) is added once, weighs no value and is neither scaled nor capped), and
 // values that were turned by their own position when they were cached: a head's result at position i is turned back by
@@ -37,6 +44,12 @@ __device__ inline float turned_back(float own, float partner, int d, int v_dim, 
     const long at = (pos < s.turn_positions ? pos : s.turn_positions - 1) * half + m;
     const float c = s.turn_cos[at], n = s.turn_sin[at];
     return turn_is_first(d, half, s.turn_pairing) ? own * c + partner * n : own * c - partner * n;
+}
+
+inline int check_mask(const char* what, int window, int chunk, int keep_first) {
+    LEONE_REQUIRE(window >= 0 && chunk >= 0, "%s: window %d and chunk %d must not be negative", what, window, chunk);
+    LEONE_REQUIRE(chunk == 0 || (window == 0 && keep_first == 0), "%s: keys are seen by chunks of %d or by a window, not both", what, chunk);
+    return 0;
 }
 
 inline int check_score_shape(const char* what, const ScoreShape& s, int v_dim) {

@@ -32,11 +32,14 @@ class PoolFigures:
     page_tokens: int
     window: int = 0
     keep_first: int = 0                      # of a windowed group: positions whose pages a passing window leaves alone
+    chunk: int = 0                           # of a group without a window: keys are read within chunks of so many positions
 
     def first_page(self, held: int) -> int:
         """The first page a request still holds once ``held`` positions are committed: the next row sits
-        at position ``held`` and reads keys from ``held - window + 1`` on; pages wholly before that have
+        at position ``held`` and reads keys from ``held - window + 1`` (or its chunk's first position) on; pages wholly before that have
         been given back (crates/leone/src/kv.rs keeps whole segments in the same way)."""
+        if self.chunk:
+            return (held - held % self.chunk) // self.page_tokens
         return 0 if self.window == 0 else max(0, held - (self.window - 1)) // self.page_tokens
 
     def pages_for(self, before: int, after: int) -> int:
@@ -257,7 +260,8 @@ def verify_events(events: Iterable[tuple], figures: RunFigures) -> TraceReport:
 def figures_of(scheduler) -> RunFigures:
     """The figures of a ``Scheduler`` (its policy and its cache manager's groups)."""
     cache = scheduler.cache
-    pools = [PoolFigures(spec.num_pages, spec.page_tokens, int(spec.window or 0), int(getattr(spec, "keep_first", 0) or 0))
+    pools = [PoolFigures(spec.num_pages, spec.page_tokens, int(spec.window or 0), int(getattr(spec, "keep_first", 0) or 0),
+                         int(getattr(spec, "chunk", 0) or 0))
              for spec in cache.groups]
     policy = scheduler.policy
     return RunFigures(pools, policy.max_live_requests, policy.max_step_tokens, policy.prefill_chunk_tokens)

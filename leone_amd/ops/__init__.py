@@ -115,8 +115,9 @@ def pack_values(v: torch.Tensor) -> torch.Tensor:
 
 def embed(table: torch.Tensor, tokens: torch.Tensor, out: Optional[torch.Tensor] = None,
           scale: float = 1.0, position_table: Optional[torch.Tensor] = None,
-          positions: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """out[r] = table[tokens[r]] * scale as float32.  Token ids must have been checked against the table.
+          positions: Optional[torch.Tensor] = None, copy: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """out[r] = table[tokens[r]] * scale as float32.  Token ids must have been checked against the table.  ``copy`` (float32
+    ``[rows, hidden]``) receives the same rows once more.
     With ``position_table`` ``[places, hidden]`` (a learned vector for every position, of the table's type)
     row r also gets position_table[positions[r]], unscaled; the caller checks positions against ``places``."""
     vocab, hidden = table.shape
@@ -130,11 +131,12 @@ def embed(table: torch.Tensor, tokens: torch.Tensor, out: Optional[torch.Tensor]
         call("leone_embed_placed", _dev(table, "embed table"), _code(table, "embed table"),
              _dev(tokens, "embed tokens", torch.int32, (rows,)), _dev(out, "embed out", torch.float32, (rows, hidden)),
              rows, hidden, vocab, float(scale), _dev(position_table, "position table"),
-             _dev(positions, "positions", torch.int32, (rows,)), position_table.shape[0], _stream())
+             _dev(positions, "positions", torch.int32, (rows,)), position_table.shape[0],
+             _dev(copy, "embed copy", torch.float32, (rows, hidden)), _stream())
         return out
-    call("leone_embed", _dev(table, "embed table"), _code(table, "embed table"),
+    call("leone_embed_placed", _dev(table, "embed table"), _code(table, "embed table"),
          _dev(tokens, "embed tokens", torch.int32, (rows,)), _dev(out, "embed out", torch.float32, (rows, hidden)),
-         rows, hidden, vocab, float(scale), _stream())
+         rows, hidden, vocab, float(scale), 0, 0, 0, _dev(copy, "embed copy", torch.float32, (rows, hidden)), _stream())
     return out
 
 
@@ -172,6 +174,8 @@ def add_rmsnorm(x: torch.Tensor, delta: Optional[torch.Tensor], gain: torch.Tens
 
 
 GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}     # what a gated feed-forward puts on its gate
+# ... and what stands on gate and up together: "clamped_swish" holds both to a limit (see ``glu_value``)
+GLU_ACTIVATIONS = {**GATE_ACTIVATIONS, "clamped_swish": 2}
 
 
 def _gate_code(activation: str) -> int:
@@ -181,8 +185,19 @@ def _gate_code(activation: str) -> int:
         raise KernelError(f"unknown gate activation {activation!r}; known: {', '.join(GATE_ACTIVATIONS)}") from None
 
 
-def swiglu(gate_up: torch.Tensor, out: Optional[torch.Tensor] = None, activation: str = "silu") -> torch.Tensor:
-    """act(gate) * up of rows that hold 8 gates, their 8 ups, and so on; ``activation`` names act."""
+def _glu_code(activation: str, limit: Optional[float]) -> int:
+    code = GLU_ACTIVATIONS.get(activation)
+    if code is None:
+        raise KernelError(f"unknown gate activation {activation!r}; known: {', '.join(GLU_ACTIVATIONS)}")
+    if code == 2 and not (limit is not None and limit > 0.0):
+        raise KernelError(f"the clamped activation needs a positive limit, found {limit!r}")
+    return code
+
+
+def swiglu(gate_up: torch.Tensor, out: Optional[torch.Tensor] = None, activation: str = "silu",
+           limit: Optional[float] = None) -> torch.Tensor:
+    """act(gate) * up of rows that hold 8 gates, their 8 ups, and so on; ``activation`` names act (``GLU_ACTIVATIONS``), ``limit``
+    belongs to "clamped_swish" alone."""
     rows, twice = gate_up.shape
     if twice % 2:
         raise KernelError("swiglu: input width must be even (gate columns, then up columns)")
@@ -190,7 +205,7 @@ def swiglu(gate_up: torch.Tensor, out: Optional[torch.Tensor] = None, activation
     if out is None:
         out = torch.empty((rows, ffn), dtype=gate_up.dtype, device=gate_up.device)
     call("leone_glu", _dev(gate_up, "swiglu in"), _dev(out, "swiglu out", gate_up.dtype, (rows, ffn)),
-         _code(gate_up, "swiglu in"), rows, ffn, _gate_code(activation), _stream())
+         _code(gate_up, "swiglu in"), rows, ffn, _glu_code(activation, limit), float(limit or 0.0), _stream())
     return out
 
 
@@ -336,7 +351,7 @@ def attention_rows(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, 
                    row_entry: torch.Tensor, block_table: torch.Tensor, q_heads: int, scale: float,
                    window: int = 0, out: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
                    keep_first: int = 0, gate_each: bool = False, slopes: Optional[torch.Tensor] = None,
-                   query_factor: Optional[tuple] = None, shape: Optional[ScoreShape] = None) -> torch.Tensor:
+                   query_factor: Optional[tuple] = None, shape: Optional[ScoreShape] = None, chunk: int = 0) -> torch.Tensor:
     """Each query row attends its request's cached keys up to its own position (the last ``window`` of them,
     and, whatever the window, those at positions below ``keep_first``).  The result has the values'
     size a head.  ``slopes`` float32 ``[q_heads]``: head h's score for the key at distance d is lowered by
@@ -344,7 +359,8 @@ def attention_rows(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, 
     1 + coef * ln(floor((p + 1) / every) + 1).  ``gate``: float32 ``[rows, >= q_heads]`` (a view into a wider row is fine, unit stride along the
     heads): head h of row r is multiplied by sigmoid(gate[r, h]); with ``gate_each`` the gate holds a value for
     every element of the result, ``[rows, >= q_heads * value_dim]``.  ``shape``: capped scores, sinks, results turned
-    back (``ScoreShape``; results are turned back before the gate)."""
+    back (``ScoreShape``; results are turned back before the gate).  ``chunk`` (without a window): a row sees the keys of its
+    own chunk of so many positions, counted from 0, only."""
     rows = q.shape[0]
     pages, kv_heads, page_tokens, head_dim, value_dim = cache_dims_kv(k_pool, v_pool)
     if q.shape[1] != q_heads * head_dim:
@@ -359,7 +375,7 @@ def attention_rows(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, 
          _dev(block_table, "block table", torch.int32), block_table.shape[1], rows, q_heads, kv_heads, head_dim,
          value_dim, page_tokens, float(scale), int(window), gate_at, gate_stride, int(keep_first),
          1 if (gate_each and gate is not None) else 0, _dev(slopes, "slopes", torch.float32, (q_heads,)), float(coef),
-         int(every), *(shape or _PLAIN_SCORES).args(q_heads, value_dim), _stream())
+         int(every), *(shape or _PLAIN_SCORES).args(q_heads, value_dim), int(chunk), _stream())
     return out
 
 
@@ -502,17 +518,18 @@ def attention_decode(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor
                      row_entry: torch.Tensor, block_table: torch.Tensor, q_heads: int, scale: float,
                      window: int = 0, max_context: int = 1, splits: Optional[int] = None,
                      out: Optional[torch.Tensor] = None, keep_first: int = 0, slopes: Optional[torch.Tensor] = None,
-                     query_factor: Optional[tuple] = None, shape: Optional[ScoreShape] = None) -> torch.Tensor:
+                     query_factor: Optional[tuple] = None, shape: Optional[ScoreShape] = None, chunk: int = 0) -> torch.Tensor:
     """Split-KV attention on the matrix cores (bfloat16).  ``max_context`` only steers the number of splits.
     ``keep_first``: keys at positions below it stay in sight of a windowed layer.  ``slopes`` and ``query_factor``
     as for ``attention_rows``: scores that fall with the distance, queries that count more the further on they stand.
-    ``shape``: capped scores, sinks, results turned back."""
+    ``shape``: capped scores, sinks, results turned back.  ``chunk`` as for ``attention_rows``."""
     rows = q.shape[0]
     pages, kv_heads, page_tokens, head_dim = cache_dims(k_pool, v_pool)
     if q.shape[1] != q_heads * head_dim:
         raise KernelError(f"attention: query width {q.shape[1]} is not {q_heads}*{head_dim}")
     if splits is None:
         reach = min(max_context, window + keep_first + 32) if window else max_context     # keys a row can see at most
+        reach = min(reach, chunk) if chunk else reach
         splits = choose_splits(rows, kv_heads, q_heads // kv_heads, reach, compute_units(q.device))
     if out is None:
         out = torch.empty_like(q)
@@ -528,7 +545,7 @@ def attention_decode(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor
          block_table.shape[1], _dev(part_acc, "partials"), _dev(part_ml, "partial sums"), rows, q_heads, kv_heads,
          head_dim, page_tokens, float(scale), int(window), int(splits), int(keep_first) if window else 0,
          _dev(slopes, "slopes", torch.float32, (q_heads,)), float(coef), int(every),
-         *(shape or _PLAIN_SCORES).args(q_heads, head_dim), _stream())
+         *(shape or _PLAIN_SCORES).args(q_heads, head_dim), int(chunk), _stream())
     return out
 
 
@@ -618,9 +635,9 @@ def attention_prefill(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, 
                       positions: torch.Tensor, tiles: torch.Tensor, block_table: torch.Tensor, q_heads: int,
                       scale: float, window: int = 0, mean_keys: int = 1, splits: Optional[int] = None,
                       covered_rows: Optional[int] = None, keep_first: int = 0, slopes: Optional[torch.Tensor] = None,
-                      query_factor: Optional[tuple] = None, shape: Optional[ScoreShape] = None) -> torch.Tensor:
-    """Attention for the rows that ``tiles`` covers; writes into ``out``.  ``slopes``, ``query_factor`` and
-    ``shape`` as for ``attention_rows``.
+                      query_factor: Optional[tuple] = None, shape: Optional[ScoreShape] = None, chunk: int = 0) -> torch.Tensor:
+    """Attention for the rows that ``tiles`` covers; writes into ``out``.  ``slopes``, ``query_factor``, ``shape`` and
+    ``chunk`` as for ``attention_rows``.
 
     ``tiles`` is int32 [n, 3]: (entry, first row, rows) with at most PREFILL_TILE_ROWS consecutive rows of one
     request each, PREFILL_GROUP_TILES to a group, all tiles of a group of the same entry, unused places with
@@ -643,7 +660,8 @@ def attention_prefill(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, 
     if keep_first:
         splits = 1
     if splits is None:
-        splits = choose_prefill_splits(groups, q_heads, mean_keys, window, compute_units(q.device))
+        # a group's rows lie in one chunk or two
+        splits = choose_prefill_splits(groups, q_heads, mean_keys, chunk or window, compute_units(q.device))
     part_acc = part_ml = None
     if splits > 1:
         covered = rows if covered_rows is None else covered_rows
@@ -659,7 +677,7 @@ def attention_prefill(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, 
          block_table.shape[1], q_heads, kv_heads, head_dim, page_tokens, float(scale), int(window),
          _dev(part_acc, "partials"), _dev(part_ml, "partial sums"), int(splits), keep_first,
          _dev(slopes, "slopes", torch.float32, (q_heads,)), float(coef), int(every),
-         *(shape or _PLAIN_SCORES).args(q_heads, head_dim), _stream())
+         *(shape or _PLAIN_SCORES).args(q_heads, head_dim), int(chunk), _stream())
     return out
 
 
@@ -788,7 +806,8 @@ def drop_streamed_copies() -> None:
 
 
 def gemm_fused(x, weight: torch.Tensor, out_dtype: torch.dtype = torch.bfloat16,
-               residual: Optional[torch.Tensor] = None, gated: bool = False, next_norm=None, activation: str = "silu"):
+               residual: Optional[torch.Tensor] = None, gated: bool = False, next_norm=None, activation: str = "silu",
+               limit: Optional[float] = None):
     """The product for at most 16 rows with its neighbours folded in: ``x`` may be ``NormedRows`` or
     ``PreparedRows``; with ``residual`` the product is added into that float32 tensor and None is returned;
     with ``gated`` the weight is an interleaved gate/up weight and silu(gate) * up comes out.  With
@@ -812,9 +831,9 @@ def gemm_fused(x, weight: torch.Tensor, out_dtype: torch.dtype = torch.bfloat16,
             operand = torch.empty((m, n), dtype=torch.bfloat16, device=weight.device)
             squares = torch.empty((m, -(-n // 16)), dtype=torch.float32, device=weight.device)
     elif gated:
-        # mode 4: the gated output with the tanh form of gelu on the gate
+        # modes 4 and 5: the gated output with the tanh form of gelu on the gate, and with gate and up held to a limit
         out, mode, out_dtype = (torch.empty((m, n // 2), dtype=torch.bfloat16, device=weight.device),
-                                4 if _gate_code(activation) == 1 else 2, torch.bfloat16)
+                                (2, 4, 5)[_glu_code(activation, limit)], torch.bfloat16)
     else:
         out, mode = torch.empty((m, n), dtype=out_dtype, device=weight.device), 0
     if prepared:
@@ -833,7 +852,7 @@ def gemm_fused(x, weight: torch.Tensor, out_dtype: torch.dtype = torch.bfloat16,
              _dev(out, "gemm out", out_dtype, (m, n // 2 if gated else n)), mode, _CODES[out_dtype], m, n, k,
              x.squares.data_ptr() if prepared else 0, _dev(operand, "operand out"), _dev(squares, "sums out"),
              _dev(next_norm[0], "next gain", None, (n,)) if next_norm is not None else 0,
-             _code(next_norm[0], "next gain") if next_norm is not None else 0, _stream())
+             _code(next_norm[0], "next gain") if next_norm is not None else 0, float(limit or 0.0), _stream())
     if next_norm is not None:
         return PreparedRows(residual, next_norm[0], next_norm[1], next_norm[2], operand, squares)
     return None if residual is not None else out
@@ -901,7 +920,8 @@ def rows_ways(m: int, waves: int) -> int:
 def gemm_rows(x: torch.Tensor, weight: torch.Tensor, out_dtype: torch.dtype = torch.bfloat16,
               residual: Optional[torch.Tensor] = None, gated: bool = False, splits: Optional[int] = None,
               waves: Optional[int] = None, may_split: bool = True, ways: Optional[int] = None,
-              activation: str = "silu", tiles: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+              activation: str = "silu", tiles: Optional[torch.Tensor] = None,
+              limit: Optional[float] = None) -> Optional[torch.Tensor]:
     """The weight-streaming product for up to ROWS_MAX rows of bfloat16 ``x``.  With ``residual`` and one
     range of K the product is added into that float32 tensor (None returned); with ``gated`` the weight is
     an interleaved gate/up weight and silu(gate) * up comes out.  With more than one range of K (``splits``;
@@ -938,7 +958,7 @@ def gemm_rows(x: torch.Tensor, weight: torch.Tensor, out_dtype: torch.dtype = to
         _dev(out, "gemm_rows stream", torch.float32, (m, n))
     elif gated:
         out, mode, kind = (torch.empty((m, n // 2), dtype=torch.bfloat16, device=weight.device),
-                           4 if _gate_code(activation) == 1 else 2, torch.bfloat16)
+                           (2, 4, 5)[_glu_code(activation, limit)], torch.bfloat16)
     else:
         out, mode, kind = torch.empty((m, n), dtype=out_dtype, device=weight.device), 0, out_dtype
     if tiles is None and _streamed:
@@ -947,7 +967,7 @@ def gemm_rows(x: torch.Tensor, weight: torch.Tensor, out_dtype: torch.dtype = to
         call("leone_gemm_rows_bf16", _dev(x, "gemm x", torch.bfloat16, (m, k)),
              _dev(weight if tiles is None else tiles, "gemm weight", torch.bfloat16), 0 if tiles is None else 1,
              _dev(out, "gemm out", kind), mode, _CODES[kind], m, n, k,
-             splits, plane, int(waves), int(ways), _stream())
+             splits, plane, int(waves), int(ways), float(limit or 0.0), _stream())
     return None if (residual is not None and splits == 1) else out
 
 
@@ -1091,12 +1111,12 @@ def _library_product(x: torch.Tensor, weight: torch.Tensor, out_dtype: torch.dty
 
 def linear(x, weight: torch.Tensor, out_dtype: Optional[torch.dtype] = None,
            residual: Optional[torch.Tensor] = None, gated: bool = False,
-           planes_ok: bool = False, next_norm=None, activation: str = "silu"):
+           planes_ok: bool = False, next_norm=None, activation: str = "silu", limit: Optional[float] = None):
     """x[R,K] . weight[N,K]^T, with optional neighbours.
 
     ``x`` is a tensor or ``NormedRows`` (a norm still to be done).  ``gated``: the weight is an
     interleaved gate/up weight and the result is act(gate) * up, ``[R, N/2]``, act being silu or what
-    ``activation`` names (``GATE_ACTIVATIONS``).  ``residual``: the caller
+    ``activation`` names (``GLU_ACTIVATIONS``; ``limit`` belongs to "clamped_swish").  ``residual``: the caller
     wants the product added into this float32 tensor; if the kernel in use can do that, it does and None
     is returned, otherwise the product is returned for the caller to add later, as float32 ``[R, N]`` or
     as a stack of planes ``[p, R, N]`` whose sum is meant (``add_rmsnorm`` takes either).
@@ -1126,12 +1146,12 @@ def linear(x, weight: torch.Tensor, out_dtype: Optional[torch.dtype] = None,
         if next_norm is not None and (residual is None or not prepared_fits(rows, weight.shape[0])
                                       or next_norm[2] != torch.bfloat16):
             next_norm = None
-        return gemm_fused(x, weight, out_dtype, residual, gated, next_norm, activation=activation)
+        return gemm_fused(x, weight, out_dtype, residual, gated, next_norm, activation=activation, limit=limit)
     x = materialize(x)
     if dtype == torch.bfloat16 and weight.is_cuda and k % 8 == 0 and rows <= ROWS_MAX \
             and (not gated or weight.shape[0] % 16 == 0):
         return gemm_rows(x, weight, out_dtype, residual, gated, may_split=planes_ok or residual is not None,
-                         activation=activation)
+                         activation=activation, limit=limit)
     if dtype == torch.float32:
         if out_dtype != torch.float32:
             raise KernelError("linear: the float32 path produces float32")
@@ -1156,7 +1176,7 @@ def linear(x, weight: torch.Tensor, out_dtype: Optional[torch.dtype] = None,
             y = _library_product(x, weight, torch.bfloat16, None)
         if out_dtype != y.dtype:
             y = y.to(out_dtype)
-    return swiglu(y, activation=activation) if gated else y
+    return swiglu(y, activation=activation, limit=limit) if gated else y
 
 
 def linear_planes(x: torch.Tensor, weight: torch.Tensor, rows_of) -> list:
@@ -1571,13 +1591,14 @@ def scan_max_dim() -> int:
 def outer_scan(proj: torch.Tensor, columns: dict, state: torch.Tensor, step, heads: int, dim: int, vdim: int, *,
                gates: Optional[dict] = None, decay: Optional[torch.Tensor] = None, q_scale: float = 1.0,
                k_scale: float = 1.0, cos: Optional[torch.Tensor] = None, sin: Optional[torch.Tensor] = None,
-               write_state: bool = True):
+               activation: Optional[str] = None, write_state: bool = True):
     """The matrix-memory recurrence S_t = a_t S_(t-1) + b_t k_t v_t^T, o_t = S_t^T q_t over every entry's rows,
     from and into ``state`` (float32 ``[slots, heads, dim * vdim]``, with ``gates`` ``dim * vdim + dim + 1``: the
     normaliser and the running maximum ride along).  ``proj`` is float32 ``[rows, width]``; ``columns`` names the
     first column of q, k and v (and, with ``gates``, of the input and forget gates' pre-activations "i", "f").
     ``gates`` = {"i_bias", "f_bias", "cap"}: exponential gates with a running maximum that starts at 0; else
-    ``decay`` (float32 ``[heads]``) with b = 1.  ``cos``/``sin``: rotary tables for q and k.
+    ``decay`` (float32 ``[heads]``) with b = 1.  ``cos``/``sin``: rotary tables for q and k.  ``activation`` "silu": q, k and v
+    pass through it first.
     Returns o float32 ``[rows, heads * vdim]`` and, with gates, (dot, top) for ``head_norm_gate``.
 
     Single tokens and short portions are walked row by row.  A long portion (``OUTER_CHUNKS``) is cut into chunks
@@ -1587,6 +1608,8 @@ def outer_scan(proj: torch.Tensor, columns: dict, state: torch.Tensor, step, hea
     per_head = dim * vdim + (dim + 1 if gates else 0)
     if state.dtype != torch.float32 or state.dim() != 3 or tuple(state.shape[1:]) != (heads, per_head) or not state.is_contiguous():
         raise KernelError(f"outer_scan: state {tuple(state.shape)} is not [slots, {heads}, {per_head}] float32")
+    if activation not in (None, "silu"):
+        raise KernelError(f"outer_scan: q, k and v pass as they are or through silu, not {activation!r}")
     spans = entry_spans(step)
     device = proj.device
     out = torch.empty((rows, heads * vdim), dtype=torch.float32, device=device)
@@ -1608,6 +1631,7 @@ def outer_scan(proj: torch.Tensor, columns: dict, state: torch.Tensor, step, hea
         call("leone_outer_scan", _dev(proj, "projection", torch.float32), width, columns["q"], columns["k"], columns["v"],
              _dev(coef, "coefficients"), _dev(decay, "decay", torch.float32, (heads,)) if decay is not None else 0,
              1 if no_input else 0, 1 if accumulate else 0, 1 if gates else 0, float(q_scale), float(k_scale),
+             1 if activation == "silu" else 0,
              _dev(cos, "rope cos", torch.float32), _dev(sin, "rope sin", torch.float32), rotary_dim,
              cos.shape[0] if cos is not None else 0, _dev(step.positions, "positions", torch.int32, (rows,)),
              _dev(segments, "segments", torch.int32), segments.shape[0],
@@ -1637,7 +1661,8 @@ def delta_scan(qkv: torch.Tensor, columns: dict, beta: torch.Tensor, step_size: 
                q_scale: float, unit_eps: float, write_state: bool = True) -> torch.Tensor:
     """The gated delta rule over every entry's rows: S <- g * S with g = exp(-exp(rate_log) * softplus(step_size +
     step_bias)) per head and key channel, u = sigmoid(beta) (v - S^T k), S <- S + k u^T, o = S^T q, with q and k
-    made unit vectors per head (x / sqrt(sum x^2 + unit_eps)) and q times ``q_scale``.  ``qkv`` float32 rows
+    made unit vectors per head (x / sqrt(sum x^2 + unit_eps)) and q times ``q_scale``.  With a ``step_bias`` of one value a head
+    there is one step size, and so one decay, a head (``step_size`` ``[rows, heads]``).  ``qkv`` float32 rows
     holding q and k (``kv_heads`` heads of ``dim``) and v (``heads`` of ``vdim``) at ``columns``; ``beta`` float32
     ``[rows, heads]`` and ``step_size`` ``[rows, heads * dim]`` may be slices of wider rows.  ``state`` float32
     ``[slots, heads, dim, vdim]``.  Returns o float32 ``[rows, heads * vdim]``.
@@ -1654,12 +1679,13 @@ def delta_scan(qkv: torch.Tensor, columns: dict, beta: torch.Tensor, step_size: 
     device = qkv.device
     out = torch.empty((rows, heads * vdim), dtype=torch.float32, device=device)
     beta_at, beta_stride = _strided_rows(beta, "delta_scan beta", rows, heads)
-    step_at, step_stride = _strided_rows(step_size, "delta_scan step", rows, heads * dim)
+    per_head = step_bias.numel() == heads and dim > 1
+    step_at, step_stride = _strided_rows(step_size, "delta_scan step", rows, heads if per_head else heads * dim)
 
     def walk(segments, state_in, state_out, no_input=False, accumulate=False, transition=None):
         call("leone_delta_scan", _dev(qkv, "q, k, v", torch.float32), qkv.shape[1], columns["q"], columns["k"], columns["v"],
-             beta_at, beta_stride, step_at, step_stride, _dev(rate_log, "rate", None, (heads,)),
-             _dev(step_bias, "step bias", None, (heads * dim,)), _code(rate_log, "rate"), float(q_scale), float(unit_eps),
+             beta_at, beta_stride, step_at, step_stride, 1 if per_head else 0, _dev(rate_log, "rate", None, (heads,)),
+             _dev(step_bias, "step bias", None, (heads if per_head else heads * dim,)), _code(rate_log, "rate"), float(q_scale), float(unit_eps),
              1 if no_input else 0, 1 if accumulate else 0, _dev(segments, "segments", torch.int32), segments.shape[0],
              _dev(state_in, "state read"), state_in.stride(0) if state_in is not None else 0,
              _dev(state_out, "state written"), state_out.stride(0) if state_out is not None else 0,
@@ -1719,7 +1745,7 @@ def add_normed(x: torch.Tensor, delta: Optional[torch.Tensor], gain: Optional[to
 
 ROUTER_SCORES = {"softmax": 0, "sigmoid": 1}     # how a router turns its logits into scores
 # what experts put on gate and up: a gate activation, or "clamped_swish" (gate and up held to a limit, see ``glu_value``)
-EXPERT_ACTIVATIONS = {**GATE_ACTIVATIONS, "clamped_swish": 2}      # of experts with a gate
+EXPERT_ACTIVATIONS = GLU_ACTIVATIONS                               # of experts with a gate
 PLAIN_ACTIVATIONS = {**GATE_ACTIVATIONS, "relu2": 3}                # of experts without one
 
 
@@ -2270,6 +2296,40 @@ class MixedDelta:
         return total
 
 
+def delta_terms(delta) -> list:
+    """What is still to be added to the stream, of any kind, as the terms of a ``MixedDelta``."""
+    if delta is None or isinstance(delta, PreparedRows):
+        return []
+    if isinstance(delta, MixedDelta):
+        return delta.terms
+    if isinstance(delta, ScaledDelta):
+        return [(delta.rows, delta.scale, None)]
+    if isinstance(delta, NormedDelta):
+        delta = delta.materialize()
+    return [(delta, 1.0, None)]
+
+
+def _at(array):
+    return ctypes.cast(array, ctypes.c_void_p)
+
+
+def _term_args(terms, n: int, hidden: int) -> tuple:
+    """The arguments that name up to ``BRANCH_TERMS`` results to a kernel, and what must live until it is launched."""
+    held = []
+    for delta, factor, scale in terms:
+        delta, planes, plane = _planes(delta, n, hidden, "result")
+        held.append((delta, planes, plane, float(factor), scale))
+    t = max(len(held), 1)
+    term_rows = (ctypes.c_void_p * t)(*[_dev(d, "result") for d, *_ in held])
+    term_planes = (ctypes.c_int * t)(*[p for _, p, *_ in held])
+    term_plane = (ctypes.c_long * t)(*[p for _, _, p, *_ in held])
+    factors = (ctypes.c_float * t)(*[f for *_, f, _ in held])
+    scales = (ctypes.c_void_p * t)(*[_dev(s, "result scale", None, (hidden,)) for *_, s in held])
+    scale_codes = (ctypes.c_int * t)(*[_code(s, "result scale") if s is not None else F32 for *_, s in held])
+    return ((_at(term_rows), _at(term_planes), _at(term_plane), _at(factors), _at(scales), _at(scale_codes), len(held)),
+            (held, term_rows, term_planes, term_plane, factors, scales, scale_codes))
+
+
 BRANCH_TERMS = 4          # results one call adds
 BRANCH_NORMS = 2          # norms it makes
 
@@ -2295,24 +2355,29 @@ def branch_norm(x: torch.Tensor, terms, gains, eps: float, groups: int, out_dtyp
     outs = [torch.empty((n_out, hidden), dtype=out_dtype, device=x.device) for _ in gains]
     if not terms and not gains:
         return outs
-    held = []
-    for delta, factor, scale in terms:
-        delta, planes, plane = _planes(delta, n, hidden, "result")
-        held.append((delta, planes, plane, float(factor), scale))
-    t, g = max(len(held), 1), max(len(gains), 1)
-    term_rows = (ctypes.c_void_p * t)(*[_dev(d, "result") for d, *_ in held])
-    term_planes = (ctypes.c_int * t)(*[p for _, p, *_ in held])
-    term_plane = (ctypes.c_long * t)(*[p for _, _, p, *_ in held])
-    factors = (ctypes.c_float * t)(*[f for *_, f, _ in held])
-    scales = (ctypes.c_void_p * t)(*[_dev(s, "result scale", None, (hidden,)) for *_, s in held])
-    scale_codes = (ctypes.c_int * t)(*[_code(s, "result scale") if s is not None else F32 for *_, s in held])
+    term_args, held = _term_args(terms, n, hidden)
+    g = max(len(gains), 1)
     gain_ptrs = (ctypes.c_void_p * g)(*[_dev(v, "gain", None, (hidden,)) for v in gains])
     gain_codes = (ctypes.c_int * g)(*[_code(v, "gain") for v in gains])
     out_ptrs = (ctypes.c_void_p * g)(*[_dev(y, "normed rows") for y in outs])
 
-    def at(array):
-        return ctypes.cast(array, ctypes.c_void_p)
-    call("leone_branch_norm", _dev(x, "stream", torch.float32), at(term_rows), at(term_planes), at(term_plane), at(factors),
-         at(scales), at(scale_codes), len(held), at(gain_ptrs), at(gain_codes), at(out_ptrs), len(gains), _CODES[out_dtype],
-         float(eps), int(groups), _dev(rows, "rows", torch.int32) if rows is not None else 0, n_out, hidden, _stream())
+    call("leone_branch_norm", _dev(x, "stream", torch.float32), *term_args, _at(gain_ptrs), _at(gain_codes), _at(out_ptrs),
+         len(gains), _CODES[out_dtype], float(eps), int(groups), _dev(rows, "rows", torch.int32) if rows is not None else 0, n_out, hidden, _stream())
     return outs
+
+
+def stream_join(x: torch.Tensor, terms, first: torch.Tensor, following: Optional[torch.Tensor], out_dtype: torch.dtype) -> torch.Tensor:
+    """The operand ``[n, 2 hidden]`` of a product that reads the stream beside ``first`` (float32 ``[n, hidden]``): the stream's
+    rows with ``terms`` (see ``MixedDelta``) added, then ``first``'s, in ``out_dtype``.  The stream ``x`` itself becomes
+    ``following`` (``[hidden]``, the same for every row; None: zeros), ready for that product to be added to it."""
+    n, hidden = x.shape
+    terms = list(terms)
+    while len(terms) > BRANCH_TERMS:
+        branch_norm(x, terms[:BRANCH_TERMS], [], 1.0, 1, out_dtype)
+        terms = terms[BRANCH_TERMS:]
+    term_args, held = _term_args(terms, n, hidden)
+    operand = torch.empty((n, 2 * hidden), dtype=out_dtype, device=x.device)
+    call("leone_stream_join", _dev(x, "stream", torch.float32), *term_args, _dev(first, "first rows", torch.float32, (n, hidden)),
+         _dev(following, "following rows", None, (hidden,)), _code(following, "following rows") if following is not None else F32,
+         _dev(operand, "operand"), _CODES[out_dtype], n, hidden, _stream())
+    return operand

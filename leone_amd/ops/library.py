@@ -39,9 +39,9 @@ _PROTOTYPES = {
                                 c_int, P],
     "leone_gemm_f32": [P, P, P, c_int, c_int, c_int, P],
     "leone_gemm_fused_bf16": [P, c_int, P, P, c_int, c_float, P, c_int, P, c_int, c_int, c_int, c_int, c_int, P, P, P, P,
-                              c_int, P],
+                              c_int, c_float, P],
     "leone_gemm_planes_bf16": [P, c_int, c_int, P, c_int, P, c_int, c_int, c_int, c_int, P],
-    "leone_gemm_rows_bf16": [P, P, c_int, P, c_int, c_int, c_int, c_int, c_int, c_int, ctypes.c_long, c_int, c_int, P],
+    "leone_gemm_rows_bf16": [P, P, c_int, P, c_int, c_int, c_int, c_int, c_int, c_int, ctypes.c_long, c_int, c_int, c_float, P],
     "leone_gemm_rows_shape_built": [c_int, c_int, c_int],
     "leone_argmax": [P, P, P, P, c_int, c_int, P],
     "leone_peak_read": [P, ctypes.c_long, P, c_int, P],
@@ -75,13 +75,13 @@ _PROTOTYPES = {
     "leone_head_gate": [P, c_int, P, ctypes.c_long, c_int, c_int, c_int, P],
     "leone_exp_gates": [P, ctypes.c_long, c_int, c_int, P, P, c_int, c_float, P, c_int, P, ctypes.c_long, ctypes.c_long,
                         ctypes.c_long, c_int, P, P, c_int, P],
-    "leone_outer_scan": [P, ctypes.c_long, c_int, c_int, c_int, P, P, c_int, c_int, c_int, c_float, c_float, P, P, c_int, c_int,
+    "leone_outer_scan": [P, ctypes.c_long, c_int, c_int, c_int, P, P, c_int, c_int, c_int, c_float, c_float, c_int, P, P, c_int, c_int,
                          P, P, c_int, P, ctypes.c_long, P, ctypes.c_long, ctypes.c_long, P, P, P, c_int, c_int, c_int, P],
     "leone_outer_chain": [P, c_int, P, ctypes.c_long, P, P, ctypes.c_long, ctypes.c_long, c_int, c_int, c_int, P],
-    "leone_delta_scan": [P, ctypes.c_long, c_int, c_int, c_int, P, ctypes.c_long, P, ctypes.c_long, P, P, c_int, c_float,
+    "leone_delta_scan": [P, ctypes.c_long, c_int, c_int, c_int, P, ctypes.c_long, P, ctypes.c_long, c_int, P, P, c_int, c_float,
                          c_float, c_int, c_int, P, c_int, P, ctypes.c_long, P, ctypes.c_long, P, P, c_int, c_int, c_int, c_int, P],
-    "leone_embed_placed": [P, c_int, P, P, c_int, c_int, c_int, c_float, P, P, c_int, P],
-    "leone_glu": [P, P, c_int, c_int, c_int, c_int, P],
+    "leone_embed_placed": [P, c_int, P, P, c_int, c_int, c_int, c_float, P, P, c_int, P, P],
+    "leone_glu": [P, P, c_int, c_int, c_int, c_int, c_float, P],
     "leone_add_normed": [P, P, c_int, ctypes.c_long, P, c_int, c_float, P, c_int, P, c_int, c_float, P, c_int, c_int, P],
     "leone_attention_rows_kept": [P, P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
                                   c_int, P, ctypes.c_long, c_int, c_int, P],
@@ -110,12 +110,13 @@ _PROTOTYPES = {
     "leone_latent_attention": [P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, P],
     "leone_residual_norm": [P, P, c_int, ctypes.c_long, c_float, P, c_int, c_float, P, c_int, P, c_int, c_int, P],
     "leone_depth_mix": [P, P, c_int, ctypes.c_long, c_float, P, ctypes.c_long, c_int, P, c_int, ctypes.c_long, P],
+    "leone_stream_join": [P, P, P, P, P, P, P, c_int, P, P, c_int, P, c_int, c_int, c_int, P],
     "leone_attention_rows_shaped": [P, P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
-                                    c_int, P, ctypes.c_long, c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, P],
+                                    c_int, P, ctypes.c_long, c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, c_int, P],
     "leone_attention_decode_shaped": [P, P, P, P, P, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
-                                      c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, P],
+                                      c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, c_int, P],
     "leone_attention_prefill_shaped": [P, P, P, P, P, P, c_int, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, P, P,
-                                       c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, P],
+                                       c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, c_int, P],
     "leone_attention_rows_talk": [P, P, P, P, c_int, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
                                   c_int, P],
     "leone_attention_talk_decode": [P, P, P, P, P, c_int, P, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_float,

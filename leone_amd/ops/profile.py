@@ -62,6 +62,7 @@ OPERATIONS = {
     "leone_attention_talk_prefill": "attention",
     "leone_qk_norm_rope_write_turned": "qknorm rope kv",
     "leone_branch_norm": "norm",
+    "leone_stream_join": "stream join",
     "leone_token_mix": "token mix",
     "leone_low_rank_decay": "low rank decay",
     "leone_time_mix_scan": "time mix scan",

@@ -80,6 +80,7 @@ class KvNeed:
     page_tokens: Optional[int] = None   # tokens a page of this group holds; None: the engine's choice
     value_dim: Optional[int] = None     # size of a value vector; None: the keys' size
     keep_first: int = 0                 # with a window: the first positions stay readable too (their pages are kept)
+    chunk: int = 0                      # without one: keys are read within chunks of so many positions, counted from 0 (0: no chunks)
 
     paged = True
 

@@ -323,7 +323,7 @@ class ParallelPreNormBlock(Part):
         x <- x + scale1 * mixer(norm1(x)) + scale2 * feed_forward(norm2(x))
 
     with learned vectors ``scale1`` and ``scale2`` (tensor names ``[hidden]``; None: no scale).  The second sublayer is there
-    only if ``feed_forward`` is given.  Parameters: ``hidden``, ``norm1``, ``mixer``, ``scale1`` and optionally ``norm2``,
+    only if ``feed_forward`` is given; without a ``norm2`` it reads what the mixer reads.  Parameters: ``hidden``, ``norm1``, ``mixer``, ``scale1`` and optionally ``norm2``,
     ``feed_forward``, ``scale2``.  The sublayers hand back float32.  Nothing is added here: the block hands on
     ``ops.MixedDelta`` (the branches of a mixer made of several as terms of their own), and the norms that run next
     make the sum, the stream's new rows and both norms of them in one kernel.
@@ -335,8 +335,6 @@ class ParallelPreNormBlock(Part):
         self.mixer = MIXERS.build(spec["mixer"], **context)
         self.feed_forward = FEED_FORWARDS.build(spec["feed_forward"], **context) if spec.get("feed_forward") is not None else None
         self.norm2 = NORMS.build(spec["norm2"], **context) if spec.get("norm2") is not None else None
-        if self.feed_forward is not None and self.norm2 is None:
-            raise ValueError("a parallel_prenorm block with a feed-forward needs norm2")
         self.scale_names = (spec.get("scale1"), spec.get("scale2") if self.feed_forward is not None else None)
         self.scales = [None, None]
 
@@ -372,8 +370,8 @@ class ParallelPreNormBlock(Part):
         return found
 
     def forward(self, x: torch.Tensor, pending, step: StepContext, cache: Optional[CacheView]):
-        if self.feed_forward is None:
-            y1, y2 = self.norm1.add_norm(x, pending, step.dtype), None
+        if self.feed_forward is None or self.norm2 is None:
+            y1 = y2 = self.norm1.add_norm(x, pending, step.dtype)
         elif hasattr(self.norm1, "add_norms"):
             y1, y2 = self.norm1.add_norms(self.norm2, x, pending, step.dtype)
         else:

@@ -20,33 +20,36 @@ class CausalConv(Part):
 
     Parameters: ``channels``, ``taps``, ``weights`` (tensor names, each ``[its channels, taps]``, laid side by
     side along the channels: projections that were fused into one product are convolved in one launch),
-    ``add_input`` (the residual form x + conv(x)), ``activation`` (None, "silu", "sigmoid").
+    ``add_input`` (the residual form x + conv(x)), ``activation`` (None, "silu", "sigmoid").  A single tap is a factor
+    a channel; the kernel's filters have two taps at least, so it gets a zero tap ahead of it when the weights are bound.
     """
 
     graph_safe = True
 
     def __init__(self, spec: PartSpec, **_):
-        self.taps = int(spec["taps"])
+        self.file_taps = int(spec["taps"])                       # as the tensors have them
+        self.taps = max(self.file_taps, 2)
         self.names: Sequence[str] = list(spec["weights"])
         self.widths: Sequence[int] = [int(c) for c in spec["channels"]] if isinstance(spec["channels"], (list, tuple)) \
             else [int(spec["channels"])]
         if len(self.names) != len(self.widths):
             raise ValueError("a causal convolution needs one channel count per weight")
-        if self.taps < 2:
-            raise ValueError(f"a causal convolution needs at least 2 taps, found {self.taps}")
+        if self.file_taps < 1:
+            raise ValueError(f"a causal convolution needs at least 1 tap, found {self.file_taps}")
         self.channels = sum(self.widths)
         self.add_input = bool(spec.get("add_input", False))
         self.activation = spec.get("activation")
         self.weight: Optional[torch.Tensor] = None
 
     def tensor_specs(self) -> List[TensorSpec]:
-        return [TensorSpec(name, (width, self.taps), VECTOR) for name, width in zip(self.names, self.widths)]
+        return [TensorSpec(name, (width, self.file_taps), VECTOR) for name, width in zip(self.names, self.widths)]
 
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         parts = [tensors.pop(name) for name in self.names]
         if len({p.dtype for p in parts}) > 1:
             parts = [p.float() for p in parts]
-        self.weight = torch.cat(parts, dim=0).contiguous()
+        weight = torch.cat(parts, dim=0)
+        self.weight = torch.nn.functional.pad(weight, (self.taps - self.file_taps, 0)).contiguous()
 
     def cache_need(self) -> StateNeed:
         return StateNeed((self.taps - 1, self.channels), torch.float32)

@@ -17,7 +17,8 @@ class SwiGluMlp(Part):
 
     Reference: crates/leone/src/runtime.rs:9283-9319, crates/leone/src/cpu.rs:892-907.
     Parameters: ``hidden``, ``intermediate`` and tensor names ``gate``, ``up``, ``down``.
-    Optional: ``activation`` (what stands on the gate instead of silu, a key of ``ops.GATE_ACTIVATIONS``),
+    Optional: ``activation`` (what stands on the gate instead of silu, a key of ``ops.GATE_ACTIVATIONS``, or "clamped_swish"
+    with ``limit``: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1), without biases),
     ``float_output`` (what is handed back comes in float32 whatever the engine's type), ``bias`` (a dict with tensor
     names ``gate``, ``up``, ``down``: all three projections add a bias; the products then hand on float32, the biases
     are added there, and the result comes in float32).
@@ -35,8 +36,12 @@ class SwiGluMlp(Part):
         if self.bias_names:
             self.fused_io = self.prepares_next = False      # its products hand on float32 for the biases to be added
         self.activation = str(p.get("activation") or "silu")
-        if self.activation not in ops.GATE_ACTIVATIONS:
-            raise ValueError(f"unknown gate activation {self.activation!r}; known: {', '.join(ops.GATE_ACTIVATIONS)}")
+        known = ops.GATE_ACTIVATIONS if self.bias_names else ops.GLU_ACTIVATIONS
+        if self.activation not in known:
+            raise ValueError(f"unknown gate activation {self.activation!r}; known: {', '.join(known)}")
+        self.limit = float(p["limit"]) if p.get("limit") is not None else None
+        if self.activation == "clamped_swish" and not (self.limit and self.limit > 0.0):
+            raise ValueError(f"the clamped activation needs a positive limit, found {self.limit!r}")
         self.float_output = bool(p.get("float_output", False))
         self.w_gate_up = self.w_down = None
 
@@ -57,7 +62,7 @@ class SwiGluMlp(Part):
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         # One product for gate and up: 8 gate rows, their 8 up rows, and so on (a pure re-layout), which
         # lets the activation be applied where the product is finished.  An intermediate size that is no
-        # multiple of 8 is filled up with zero rows; they give silu(0) * 0 = 0 and meet zero columns of
+        # multiple of 8 is filled up with zero rows; they give act(0) * 0 = 0 (or 0 * (0 + 1)) and meet zero columns of
         # the down projection, so the result is unchanged.
         gate, up, down = (tensors.pop(self.names[k]) for k in ("gate", "up", "down"))
         if self.bias_names:
@@ -90,7 +95,7 @@ class SwiGluMlp(Part):
             if out.dim() == 3:
                 out = out.sum(dim=0)
             return ops.add_bias(out, self.bias_out)
-        activated = ops.linear(y, self.w_gate_up, gated=True, activation=self.activation)
+        activated = ops.linear(y, self.w_gate_up, gated=True, activation=self.activation, limit=self.limit)
         return ops.linear(activated, self.w_down, residual=residual, next_norm=next_norm,
                           out_dtype=torch.float32 if self.float_output else None)
 
@@ -202,7 +207,7 @@ class RoutedGluMlp(Part):
         # the experts' size (the last filled up with zero rows, which add nothing), they stand behind the experts as
         # experts that every row takes with weight 1.
         self.always = 0
-        if self.gated and isinstance(self.shared, SwiGluMlp) and self.shared.activation == self.activation:
+        if self.gated and isinstance(self.shared, SwiGluMlp) and (self.shared.activation, self.shared.limit) == (self.activation, self.limit):
             shared = {k: tensors[self.shared.names[k]] for k in ("gate", "up", "down")}
             pieces = -(-self.shared.intermediate // self.intermediate)
             pad = pieces * self.intermediate - self.shared.intermediate

@@ -34,7 +34,8 @@ class GqaAttention(Part):
     projection's result comes in float32 whatever the engine's type).
     ``gate_each`` (with ``gate``): the gate is ``[q_heads * value_dim, hidden]``, one value for every element of
     the heads' results.  ``keep_first`` (with ``window``): keys at positions below it stay in sight whatever the
-    window, at their own positions.  ``shared_kv``: the layer has no key and value projections (and no key norm)
+    window, at their own positions.  ``chunk`` (instead of a window): positions fall into chunks of so many, counted from a
+    sequence's start, and a row sees the keys of its own chunk only.  ``shared_kv``: the layer has no key and value projections (and no key norm)
     and reads the cache another layer writes (its run names that layer's cache slot and does not write).
     ``retain_window`` / ``retain_first``: what the cache must keep if other layers with wider masks read it too
     (by default this layer's own ``window`` and ``keep_first``; ``retain_window`` 0: everything).
@@ -65,6 +66,9 @@ class GqaAttention(Part):
             raise ValueError(f"{self.q_heads} query heads cannot be grouped over {self.kv_heads} kv heads")
         self.qk_norm_eps = p.get("qk_norm_eps")
         self.window = p.get("window")
+        self.chunk = int(p.get("chunk") or 0)
+        if self.chunk < 0 or (self.chunk and (self.window or p.get("shared_kv") or p.get("talk"))):
+            raise ValueError("attention: chunks of keys go with no window, keys of the layer's own and scores that are not mixed")
         self.scale = float(p.get("scale", 1.0 / math.sqrt(self.head_dim)))
         self.shared_kv = bool(p.get("shared_kv", False))
         self.names = {k: p[k] for k in (("q", "o") if self.shared_kv else ("q", "k", "v", "o"))}
@@ -126,10 +130,10 @@ class GqaAttention(Part):
         # more than q, k and v of one size, or passes through kernels of its own
         self.general = (self.value_dim != self.head_dim or "gate" in self.names or self.shared_kv or bool(self.bias_names)
                         or self.wide_norm or self.conv is not None or self.slope_values is not None
-                        or self.query_factor is not None or self.padded or shaped or "talk" in self.names)
-        if self.padded and (self.shared_kv or self.gate_each):
+                        or self.query_factor is not None or self.padded or shaped or "talk" in self.names or self.chunk > 0)
+        if self.padded and self.shared_kv:
             raise ValueError(f"attention: heads of {self.file_head_dim} and values of {self.file_value_dim} elements are filled up "
-                             f"to multiples of 8 and 2, which a gate an element and a borrowed cache do not allow")
+                             f"to multiples of 8 and 2, which a borrowed cache does not allow")
         if self.qk_norm_eps is not None:
             self.names.update(q_norm=p["q_norm"])
             if not self.shared_kv:
@@ -142,7 +146,7 @@ class GqaAttention(Part):
     def cache_need(self):
         keys = KvNeed(self.kv_heads, self.head_dim, self.retain_window,
                       value_dim=self.value_dim if self.value_dim != self.head_dim else None,
-                      keep_first=self.retain_first if self.retain_window else 0)
+                      keep_first=self.retain_first if self.retain_window else 0, chunk=self.chunk)
         if self.conv is None:
             return keys
         return {"kv": keys, "conv": self.conv.cache_need()}
@@ -178,7 +182,7 @@ class GqaAttention(Part):
         if "sink" in self.names:
             specs.append(TensorSpec(self.names["sink"], (self.q_heads,), VECTOR, init=("normal", 0.0, 1.0)))
         if self.conv is not None:       # the filters as the file has them: one row a channel of the heads' own sizes
-            specs += [TensorSpec(name, (width, self.conv.taps), VECTOR) for name, width in zip(self.conv.names, (qw, kvw, vw))]
+            specs += [TensorSpec(name, (width, self.conv.file_taps), VECTOR) for name, width in zip(self.conv.names, (qw, kvw, vw))]
         return specs
 
     def _filled(self, rows: torch.Tensor, heads: int, size: int, to: int) -> torch.Tensor:
@@ -197,7 +201,8 @@ class GqaAttention(Part):
             fused += [self._filled(tensors.pop(self.names["k"]), self.kv_heads, d, self.head_dim),
                       self._filled(tensors.pop(self.names["v"]), self.kv_heads, e, self.value_dim)]
         if "gate" in self.names:
-            fused.append(tensors.pop(self.names["gate"]))      # the heads' gates ride along as further columns
+            gates = tensors.pop(self.names["gate"])            # the heads' gates ride along as further columns
+            fused.append(self._filled(gates, self.q_heads, e, self.value_dim) if self.gate_each else gates)
         self.w_qkv = torch.cat(fused, dim=0).contiguous()
         w_o = tensors.pop(self.names["o"])
         # zero columns of the output projection meet what the values' zero rows give
@@ -339,7 +344,7 @@ class GqaAttention(Part):
             return ops.attention_rows(q, cache.k_pool, cache.v_pool, step.positions, step.row_entry,
                                       cache.block_table, self.q_heads, self.scale, window, gate=gate,
                                       keep_first=self.keep_first, gate_each=self.gate_each, slopes=self.slopes,
-                                      query_factor=self.query_factor, shape=shape)
+                                      query_factor=self.query_factor, shape=shape, chunk=self.chunk)
         first = 0
         out = torch.empty_like(q)
         tiled = step.tiled.get(self.row_tiling())
@@ -348,13 +353,14 @@ class GqaAttention(Part):
             ops.attention_prefill(q, out, cache.k_pool, cache.v_pool, step.positions, tiled.tiles,
                                   cache.block_table, self.q_heads, self.scale, window,
                                   mean_keys=tiled.mean_keys or step.max_position + 1, covered_rows=tiled.rows,
-                                  keep_first=self.keep_first, slopes=self.slopes, query_factor=self.query_factor, shape=shape)
+                                  keep_first=self.keep_first, slopes=self.slopes, query_factor=self.query_factor, shape=shape,
+                                  chunk=self.chunk)
             first = tiled.rows
         if first < step.rows:
             ops.attention_decode(q[first:], cache.k_pool, cache.v_pool, step.positions[first:],
                                  step.row_entry[first:], cache.block_table, self.q_heads, self.scale, window,
                                  max_context=step.max_position + 1, out=out[first:], keep_first=self.keep_first,
-                                 slopes=self.slopes, query_factor=self.query_factor, shape=shape)
+                                 slopes=self.slopes, query_factor=self.query_factor, shape=shape, chunk=self.chunk)
         if gate is None:
             return out
         # a gate for every element is a gate a head of one element

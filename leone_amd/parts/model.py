@@ -32,6 +32,16 @@ class LayerRun:
         return hash((self.layer, self.cache, self.writes, tuple(sorted((self.borrow or {}).items()))))
 
 
+@dataclass(frozen=True)
+class StreamJoin:
+    """Ahead of the runs whose places in the schedule ``before`` lists, the stream becomes W [x; x0] + vectors[t]: x the stream,
+    x0 the embedding's output, W the tensor ``matrix`` ``[hidden, 2 hidden]`` (x's columns first) and t the place in ``before``
+    (``vectors`` ``[len(before), hidden]``).  Layers that run several times over begin every pass so."""
+    before: Sequence[int]
+    matrix: str
+    vectors: str
+
+
 @dataclass
 class ModelSpec:
     hidden_size: int
@@ -50,6 +60,7 @@ class ModelSpec:
     # One tensor name for every scheduled run (or None): behind run i the stream becomes the sum over j <= i + 1 of
     # weight_i[j] * X_j, with X_0 the embedding's output and X_(j+1) run j's own result; weight_i has i + 2 elements.
     depth_weights: Optional[Sequence[str]] = None
+    join: Optional["StreamJoin"] = None             # where runs start from the stream and the embedding's output together
 
 
 def default_schedule(n_layers: int) -> List[LayerRun]:
@@ -74,6 +85,15 @@ class DecoderModel:
                 raise ValueError(f"schedule names layer {run.layer}, the model has {len(self.layers)}")
         if spec.depth_weights is not None and len(spec.depth_weights) != len(self.schedule):
             raise ValueError(f"{len(spec.depth_weights)} depth weights for {len(self.schedule)} layer runs")
+        self.joins: Dict[int, int] = {}                   # run -> place among the joins
+        if spec.join is not None:
+            if spec.depth_weights is not None:
+                raise ValueError("a stream that is joined with the embedding's output is not re-mixed over depth as well")
+            self.joins = {int(run): t for t, run in enumerate(spec.join.before)}
+            if len(self.joins) != len(spec.join.before) or not all(0 <= run < len(self.schedule) for run in self.joins):
+                raise ValueError(f"the stream is joined ahead of runs {list(spec.join.before)}; the schedule has {len(self.schedule)}")
+        self.join_matrix: Optional[torch.Tensor] = None
+        self.join_vectors: List[torch.Tensor] = []
         self.depth_weights: Optional[List[torch.Tensor]] = None
         self.embedding: Optional[torch.Tensor] = None
         self.position_table: Optional[torch.Tensor] = None
@@ -95,10 +115,16 @@ class DecoderModel:
             specs += layer.tensor_specs()
         for at, name in enumerate(self.spec.depth_weights or ()):
             specs.append(TensorSpec(name, (at + 2,), VECTOR, init=("normal", 1.0 / (at + 2), 0.02)))     # about an average
+        specs += self._join_specs()
         specs += self.final_norm.tensor_specs()
         if self.spec.head is not None:
             specs.append(TensorSpec(self.spec.head, (self.spec.vocab_size, self.spec.hidden_size), MATRIX))
         return specs
+
+    def _join_specs(self) -> List[TensorSpec]:
+        join, hidden = self.spec.join, self.spec.hidden_size
+        return [] if join is None else [TensorSpec(join.matrix, (hidden, 2 * hidden), MATRIX),
+                                        TensorSpec(join.vectors, (len(join.before), hidden), VECTOR, init=("normal", 0.0, 0.02))]
 
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         tensors = dict(tensors)
@@ -110,6 +136,10 @@ class DecoderModel:
             layer.bind(tensors)
         if self.spec.depth_weights is not None:
             self.depth_weights = [tensors.pop(name).contiguous() for name in self.spec.depth_weights]
+        if self.spec.join is not None:
+            self.join_matrix = tensors.pop(self.spec.join.matrix).contiguous()
+            # one tensor a pass: a row of the table need not begin where the kernels' 16-byte reads may
+            self.join_vectors = [row.clone() for row in tensors.pop(self.spec.join.vectors)]
         self.final_norm.bind(tensors)
         for position in self.positions.values():
             position.prepare(self.spec.max_positions, self.device)
@@ -121,6 +151,8 @@ class DecoderModel:
     def streamed_weights(self) -> List[torch.Tensor]:
         """Every matrix a decode step streams through ``ops.linear``: the layers' and the head."""
         found = [w for layer in self.layers if hasattr(layer, "streamed_weights") for w in layer.streamed_weights()]
+        if self.join_matrix is not None:
+            found.append(self.join_matrix)
         if self.head is not None:
             found.append(self.head)
         return found
@@ -185,6 +217,8 @@ class DecoderModel:
         resident["norm"] = resident.get("norm", 0) + sum(nbytes(s) for s in self.final_norm.tensor_specs())
         if self.spec.depth_weights is not None:
             resident["depth"] = sum(nbytes(TensorSpec(name, (at + 2,), VECTOR)) for at, name in enumerate(self.spec.depth_weights))
+        if self.spec.join is not None:
+            resident["join"] = sum(nbytes(s) for s in self._join_specs())
         decode = dict(resident)
         decode["embed"] = resident["embed"] // self.spec.vocab_size * rows
         if "positions" in decode:
@@ -273,13 +307,22 @@ class DecoderModel:
         ops.depth_mix(x, pending, scale, history, at + 2, self.depth_weights[at])
         return None
 
+    def _join_stream(self, x: torch.Tensor, pending, first: torch.Tensor, t: int, step: StepContext):
+        """The stream with what is pending goes into the operand of the joining product beside ``first`` and becomes the pass's
+        vector; what comes back is that product, still to be added."""
+        operand = ops.stream_join(x, ops.delta_terms(pending), first, self.join_vectors[t], step.dtype)
+        return ops.linear(operand, self.join_matrix, out_dtype=torch.float32, planes_ok=True)
+
     # ---- forward ---------------------------------------------------------------
     def forward(self, tokens: torch.Tensor, step: StepContext, caches: Dict[int, CacheView]) -> Optional[torch.Tensor]:
         """Runs the step's rows through every scheduled layer; returns float32 logits of the wanted rows."""
         if self.position_table is not None and step.max_position >= self.position_table.shape[0]:
             raise ValueError(f"position {step.max_position} is beyond the position table of {self.position_table.shape[0]} rows")
-        x = ops.embed(self.embedding, tokens, scale=self.spec.embedding_scale or 1.0,
-                      position_table=self.position_table, positions=step.positions)
+        first = None
+        if self.joins:                        # the embedding's output is asked for again: the embedding writes it twice
+            first = torch.empty((tokens.numel(), self.spec.hidden_size), dtype=torch.float32, device=tokens.device)
+        x = ops.embed(self.embedding, tokens, scale=1.0 if self.spec.embedding_scale is None else self.spec.embedding_scale,
+                      position_table=self.position_table, positions=step.positions, copy=first)
         pending = None
         history = None
         if self.depth_weights is not None:
@@ -289,8 +332,10 @@ class DecoderModel:
         for at, run in enumerate(self.schedule):
             layer = self.layers[run.layer]
             cache = self._cache_of(run, layer, caches)
+            if at in self.joins:
+                pending = self._join_stream(x, pending, first, self.joins[at], step)
             # A block that can do so leaves the first norm of the block that runs next prepared.
-            after = self.layers[self.schedule[at + 1].layer] if at + 1 < len(self.schedule) else None
+            after = self.layers[self.schedule[at + 1].layer] if at + 1 < len(self.schedule) and at + 1 not in self.joins else None
             next_norm = after.entry_norm(step.dtype) if hasattr(after, "entry_norm") else None
             if next_norm is not None and getattr(layer, "prepares_next", False):
                 pending = layer.forward(x, pending, step, cache, next_norm=next_norm)

@@ -50,28 +50,15 @@ class RmsNorm(Part):
         """This norm's rows and ``other``'s, both of the stream after ``delta`` has been added: one kernel if the two norms
         differ in their gains alone."""
         if isinstance(other, RmsNorm) and (other.groups, other.eps, other.size) == (self.groups, self.eps, self.size):
-            return ops.branch_norm(x, self._terms(delta), [self.gain, other.gain], self.eps, self.groups, out_dtype)
+            return ops.branch_norm(x, ops.delta_terms(delta), [self.gain, other.gain], self.eps, self.groups, out_dtype)
         return [self.add_norm(x, delta, out_dtype), other.add_norm(x, None, out_dtype)]
-
-    @staticmethod
-    def _terms(delta) -> list:
-        """A delta of any kind as the terms of a ``MixedDelta``."""
-        if delta is None or isinstance(delta, ops.PreparedRows):
-            return []
-        if isinstance(delta, ops.MixedDelta):
-            return delta.terms
-        if isinstance(delta, ops.ScaledDelta):
-            return [(delta.rows, delta.scale, None)]
-        if isinstance(delta, ops.NormedDelta):
-            delta = delta.materialize()
-        return [(delta, 1.0, None)]
 
     def add_norm(self, x: torch.Tensor, delta: Optional[torch.Tensor], out_dtype: torch.dtype,
                  rows: Optional[torch.Tensor] = None) -> torch.Tensor:
         if isinstance(delta, ops.PreparedRows):
             delta = None                      # the product that made it has added into the stream already
         if self.groups > 1 or isinstance(delta, ops.MixedDelta):
-            return ops.branch_norm(x, self._terms(delta), [self.gain], self.eps, self.groups, out_dtype, rows)[0]
+            return ops.branch_norm(x, ops.delta_terms(delta), [self.gain], self.eps, self.groups, out_dtype, rows)[0]
         if isinstance(delta, ops.ScaledDelta):
             # a sublayer's result that enters the stream times a factor: sum and norm in one kernel
             return ops.residual_norm(x, delta.rows, delta.scale, self.gain, self.eps, out_dtype, rows)

@@ -95,6 +95,9 @@ class RetentionMixer(Part):
 
     Parameters: ``hidden``, ``heads``, ``dim``, ``vdim``, ``decay`` (one number a head), ``eps``, ``position``
     (name of a position part, or None) and tensor names ``q``, ``k``, ``v``, ``g``, ``o``.
+    Optional: ``activation`` "silu" (q, k and v pass through it behind their projections), ``k_scale`` (the keys' factor instead
+    of 1/sqrt(dim)), ``norm_span`` "heads" (the concatenated heads are divided by one root mean square, not each by its own),
+    ``norm`` (tensor name ``[heads * vdim]``: a gain behind the norm), ``gate`` (what stands on Wg h: "silu" or "sigmoid").
     """
 
     graph_safe = True
@@ -108,22 +111,31 @@ class RetentionMixer(Part):
         if len(self.decay_values) != self.heads:
             raise ValueError(f"retention: {len(self.decay_values)} decays for {self.heads} heads")
         self.names = {k: p[k] for k in ("q", "k", "v", "g", "o")}
+        self.activation, self.gate = p.get("activation"), str(p.get("gate") or "silu")
+        self.k_scale = float(p.get("k_scale", 1.0 / math.sqrt(self.dim)))
+        self.norm_span = str(p.get("norm_span") or "head")
+        if self.activation not in (None, "silu") or self.gate not in ("silu", "sigmoid") or self.norm_span not in ("head", "heads"):
+            raise ValueError(f"retention: activation {self.activation!r}, gate {self.gate!r}, norm span {self.norm_span!r}")
+        if p.get("norm"):
+            self.names["norm"] = p["norm"]
         self.position = (positions or {}).get(p.get("position")) if p.get("position") else None
         if p.get("position") and self.position is None:
             raise ValueError(f"retention names position part {p.get('position')!r}, which the model does not define")
         qk, vv = self.heads * self.dim, self.heads * self.vdim
         self.columns = {"q": 0, "k": qk, "v": 2 * qk, "g": 2 * qk + vv}
-        self.w_in = self.w_o = self.decay = None
+        self.w_in = self.w_o = self.decay = self.norm = None
 
     def tensor_specs(self) -> List[TensorSpec]:
         n, qk, vv = self.names, self.heads * self.dim, self.heads * self.vdim
         return [TensorSpec(n["q"], (qk, self.hidden), MATRIX), TensorSpec(n["k"], (qk, self.hidden), MATRIX),
                 TensorSpec(n["v"], (vv, self.hidden), MATRIX), TensorSpec(n["g"], (vv, self.hidden), MATRIX),
-                TensorSpec(n["o"], (self.hidden, vv), MATRIX)]
+                TensorSpec(n["o"], (self.hidden, vv), MATRIX)] + ([TensorSpec(n["norm"], (vv,), VECTOR)] if "norm" in n else [])
 
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         self.w_in = torch.cat([tensors.pop(self.names[k]) for k in ("q", "k", "v", "g")], dim=0).contiguous()
         self.w_o = tensors.pop(self.names["o"]).contiguous()
+        if "norm" in self.names:
+            self.norm = tensors.pop(self.names["norm"]).contiguous()
         self.decay = torch.tensor(self.decay_values, dtype=torch.float32, device=self.w_o.device)
 
     def streamed_weights(self) -> List[torch.Tensor]:
@@ -141,10 +153,11 @@ class RetentionMixer(Part):
             if step.max_position >= rotation.cos.shape[0]:
                 raise ValueError(f"position {step.max_position} is beyond the rotary table of {rotation.cos.shape[0]} positions")
         o, _ = ops.outer_scan(proj, self.columns, cache.state, step, self.heads, self.dim, self.vdim, decay=self.decay,
-                              k_scale=1.0 / math.sqrt(self.dim), cos=rotation.cos, sin=rotation.sin,
+                              k_scale=self.k_scale, cos=rotation.cos, sin=rotation.sin, activation=self.activation,
                               write_state=cache.writes)
-        y = ops.head_norm_gate(o, self.heads, self.vdim, self.eps, step.dtype, gate=proj[:, self.columns["g"]:],
-                               activation="silu")
+        heads, size = (self.heads, self.vdim) if self.norm_span == "head" else (1, self.heads * self.vdim)
+        y = ops.head_norm_gate(o, heads, size, self.eps, step.dtype, gain=self.norm, gate=proj[:, self.columns["g"]:],
+                               activation=self.gate)
         return ops.linear(y, self.w_o, out_dtype=torch.float32)
 
 
@@ -227,6 +240,81 @@ class ChannelDeltaMixer(Part):
                            self.vdim, q_scale=1.0 / math.sqrt(self.dim), unit_eps=self.UNIT_EPS, write_state=memory.writes)
         y = ops.head_norm_gate(o, self.heads, self.vdim, self.eps, step.dtype, gain=self.norm, gate=gate,
                                activation="sigmoid")
+        return ops.linear(y, self.w_o, out_dtype=torch.float32)
+
+
+@MIXERS.register("head_delta")
+class HeadDeltaMixer(Part):
+    """The gated delta rule with one decay per head.
+
+    q = Wq h, k = Wk h (``kv_heads`` heads of ``dim``; head h of the memory uses q/k head h // (heads / kv_heads)),
+    v = Wv h (``heads`` of ``vdim``); each through a short causal convolution and silu; q and k made unit vectors
+    per head (x / sqrt(sum x^2 + 1e-6)), q times dim^-1/2; beta = sigmoid(Wb h) and
+    g = exp(-exp(A_log) * softplus(Wa h + dt_bias)), one a head.  Per head: S <- g S; u = beta (v - S^T k); S <- S + k u^T;
+    o = S^T q.  Each head's o over its root mean square, times ``norm`` (size vdim, shared by the heads), times silu(Wg h),
+    then Wo.
+
+    Parameters: ``hidden``, ``heads``, ``kv_heads``, ``dim``, ``vdim``, ``taps``, ``eps`` and tensor names ``q``, ``k``, ``v``,
+    ``q_conv``, ``k_conv``, ``v_conv``, ``b``, ``a``, ``A_log``, ``dt_bias``, ``g``, ``norm``, ``o``.
+    """
+
+    graph_safe = True
+    UNIT_EPS = 1e-6
+
+    def __init__(self, spec: PartSpec, **context):
+        p = spec.params
+        self.hidden, self.heads, self.kv_heads, self.dim, self.vdim = (
+            int(p[k]) for k in ("hidden", "heads", "kv_heads", "dim", "vdim"))
+        if self.heads % self.kv_heads:
+            raise ValueError(f"head_delta: {self.heads} heads cannot be grouped over {self.kv_heads} q/k heads")
+        _check_dim("head_delta", self.dim)
+        self.eps = float(p["eps"])
+        self.names = {k: p[k] for k in ("q", "k", "v", "b", "a", "A_log", "dt_bias", "g", "norm", "o")}
+        qk, vv = self.kv_heads * self.dim, self.heads * self.vdim
+        self.conv = CONVS.build(PartSpec("causal_conv", {"channels": [qk, qk, vv], "taps": int(p["taps"]),
+                                                         "weights": [p["q_conv"], p["k_conv"], p["v_conv"]],
+                                                         "activation": "silu"}), **context)
+        self.conv_width = 2 * qk + vv
+        self.columns = {"q": 0, "k": qk, "v": 2 * qk, "g": self.conv_width, "b": self.conv_width + vv,
+                        "a": self.conv_width + vv + self.heads}
+        self.w_in = self.w_o = self.norm = self.rate_log = self.step_bias = None
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        n, qk, vv = self.names, self.kv_heads * self.dim, self.heads * self.vdim
+        return [TensorSpec(n["q"], (qk, self.hidden), MATRIX), TensorSpec(n["k"], (qk, self.hidden), MATRIX),
+                TensorSpec(n["v"], (vv, self.hidden), MATRIX), TensorSpec(n["g"], (vv, self.hidden), MATRIX),
+                TensorSpec(n["b"], (self.heads, self.hidden), MATRIX), TensorSpec(n["a"], (self.heads, self.hidden), MATRIX),
+                # rates exp(0 .. 1.5) of step sizes around softplus(-2 .. 0): memories that reach tens of tokens back
+                TensorSpec(n["A_log"], (self.heads,), VECTOR, init=("uniform", 0.0, 1.5)),
+                TensorSpec(n["dt_bias"], (self.heads,), VECTOR, init=("uniform", -2.0, 0.0)),
+                TensorSpec(n["norm"], (self.vdim,), VECTOR), TensorSpec(n["o"], (self.hidden, vv), MATRIX)] + self.conv.tensor_specs()
+
+    def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
+        # one product for everything that reads h: q, k, v, the output gate, write strengths and step sizes
+        self.w_in = torch.cat([tensors.pop(self.names[k]) for k in ("q", "k", "v", "g", "b", "a")], dim=0).contiguous()
+        self.w_o = tensors.pop(self.names["o"]).contiguous()
+        self.norm = tensors.pop(self.names["norm"]).contiguous()
+        self.rate_log, self.step_bias = (tensors.pop(self.names[k]).contiguous() for k in ("A_log", "dt_bias"))
+        if self.rate_log.dtype != self.step_bias.dtype:
+            self.rate_log, self.step_bias = self.rate_log.float(), self.step_bias.float()
+        self.conv.bind(tensors)
+
+    def streamed_weights(self) -> List[torch.Tensor]:
+        return [self.w_in, self.w_o]
+
+    def cache_need(self):
+        return {"conv": self.conv.cache_need(), "memory": StateNeed((self.heads, self.dim, self.vdim), torch.float32)}
+
+    def forward(self, h: torch.Tensor, step: StepContext, cache) -> torch.Tensor:
+        c = self.columns
+        proj = ops.linear(h, self.w_in, out_dtype=torch.float32)
+        qkv = self.conv.forward(proj[:, :self.conv_width], step, cache["conv"], torch.float32)
+        memory = cache["memory"]
+        o = ops.delta_scan(qkv, {"q": c["q"], "k": c["k"], "v": c["v"]}, proj[:, c["b"]:c["a"]], proj[:, c["a"]:],
+                           self.rate_log, self.step_bias, memory.state, step, self.heads, self.kv_heads, self.dim,
+                           self.vdim, q_scale=1.0 / math.sqrt(self.dim), unit_eps=self.UNIT_EPS, write_state=memory.writes)
+        y = ops.head_norm_gate(o, self.heads, self.vdim, self.eps, step.dtype, gain=self.norm,
+                               gate=proj[:, c["g"]:c["b"]], activation="silu")
         return ops.linear(y, self.w_o, out_dtype=torch.float32)
 
 
