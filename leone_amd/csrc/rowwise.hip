@@ -304,6 +304,8 @@ __global__ void qk_norm_rope_write_kernel(
     if (turn_values) {                           // the pairs are the values' own, over their whole size
         rotary_half = half;
         pairing = extra.v_pairing;
+    } else if (!is_q && !is_k) {                 // copied: the keys' rotated part may be longer than a value
+        rotary_half = 0;
     }
     // the two elements of pair p
     auto first = [&](int p) { return pairing == kPairHalfSplit && p < rotary_half ? p : 2 * p; };

@@ -67,7 +67,8 @@ def test_a_serving_scenario_with_one_layer(name):
 @pytest.mark.parametrize("design,operations", [("pamevik", {"outer scan", "delta scan", "layer norm"}),
                                                ("zukinex", {"router", "experts", "attention", "norm"}),
                                                ("nogidra", {"state space scan", "bias span norm", "attention", "experts"}),
-                                               ("reverax", {"time mix scan", "token mix", "attention", "experts", "norm"})])
+                                               ("reverax", {"time mix scan", "token mix", "attention", "experts", "norm"}),
+                                               ("sonulorn", {"delta scan", "outer scan", "attention", "stream join", "norm"})])
 def test_another_design_beside_its_closest_relative(capsys, design, operations):
     """``--design NAME``: one line with the design's decode and prompt figures and Qwen3's at equal width, depth
     and vocabulary beside them, each with a per-operation table; the headline workload is not run."""
