@@ -448,6 +448,16 @@ int leone_stream_join(float* x, const void* const* term_rows, const int* term_pl
                       const float* term_factor, const void* const* term_scale, const int* term_scale_dtype, int terms,
                       const float* first, const void* next, int next_dtype, void* operand, int out_dtype, int n_rows, int hidden,
                       hipStream_t stream);
+// Long portions through a matrix memory with one decay a head (fixed, or the delta rule's), chunk by chunk on the matrix cores
+// (see chunked_memory.hip); key channels up to leone_chunk_max_dim().
+int leone_chunk_rows();
+int leone_chunk_max_dim();
+long leone_chunk_workspace(int dim, int vdim, int delta);
+int leone_chunked_memory(const float* rows, long stride, int q_off, int k_off, int v_off, int silu, float q_scale, float k_scale,
+                         float unit_eps, const float* beta, long beta_stride, const float* step, long step_stride,
+                         const void* rate_log, const void* step_bias, int vec_dtype, const float* decay, const int* chunks,
+                         int n_chunks, const int* links, int n_links, float* workspace, float* state, long slot_stride,
+                         int write_state, float* out, int heads, int kv_heads, int dim, int vdim, hipStream_t stream);
 // The token before beside the token itself, decays from a low-rank product, and the memory they drive (see time_mix.hip).
 int leone_token_mix(const void* h, int dtype, const void* mu, int mu_dtype, int mixes, const float* state, float* state_out,
                     const int* spans, int entries, const int* row_entry, void* out, int rows, int hidden, int single_rows,

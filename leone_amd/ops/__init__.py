@@ -1588,6 +1588,37 @@ def scan_max_dim() -> int:
     return int(library().leone_scan_max_dim())
 
 
+MEMORY_CHUNKS_FROM = 128     # portions of at least so many rows go through a memory with one decay a head as ``chunked_memory``
+
+
+def chunked_memory_supported(dim: int) -> bool:
+    return dim <= library().leone_chunk_max_dim()
+
+
+def chunked_memory(rows: torch.Tensor, columns: dict, plan: dict, state: torch.Tensor, out: torch.Tensor, heads: int, kv_heads: int,
+                   dim: int, vdim: int, *, q_scale: float, k_scale: float, activation: Optional[str] = None,
+                   decay: Optional[torch.Tensor] = None, delta: Optional[tuple] = None, write_state: bool = True) -> None:
+    """The long portions of a step (``plan``: ``chunk_plan`` with chunks of ``leone_chunk_rows()`` rows) through a matrix memory
+    with one decay a head, chunk by chunk on the matrix cores in float: S <- g S + k u^T, o = S^T q, with ``decay`` (float32
+    ``[heads]``) and u = v, or the delta rule's u = beta (v - g S^T k): ``delta`` = (strengths' pre-activations ``[rows, >=
+    heads]``, step sizes' pre-activations likewise, rate_log and step_bias ``[heads]``, unit_eps).  Fills the portions' rows of
+    ``out`` and moves their states."""
+    chunks, links = plan["chunks"], plan["links"]
+    n, count = rows.shape[0], chunks.shape[0]
+    size = library().leone_chunk_workspace(dim, vdim, 1 if delta is not None else 0)
+    workspace = torch.empty((count * heads * size,), dtype=torch.float32, device=rows.device)
+    beta, step_size, rate_log, step_bias, unit_eps = delta if delta is not None else (None, None, None, None, 0.0)
+    beta_at, beta_stride = _strided_rows(beta, "write strengths", n, heads)
+    step_at, step_stride = _strided_rows(step_size, "step sizes", n, heads)
+    call("leone_chunked_memory", _dev(rows, "q, k, v", torch.float32), rows.shape[1], columns["q"], columns["k"], columns["v"],
+         1 if activation == "silu" else 0, float(q_scale), float(k_scale), float(unit_eps), beta_at, beta_stride, step_at, step_stride,
+         _dev(rate_log, "rate", None, (heads,)), _dev(step_bias, "step bias", None, (heads,)),
+         _code(rate_log, "rate") if rate_log is not None else F32,
+         _dev(decay, "decay", torch.float32, (heads,)) if delta is None else 0, _dev(chunks, "chunks", torch.int32), count,
+         _dev(links, "links", torch.int32), links.shape[0], _dev(workspace, "workspace"), _dev(state, "state", torch.float32),
+         state.stride(0), 1 if write_state else 0, _dev(out, "out", torch.float32, (n, heads * vdim)), heads, kv_heads, dim, vdim, _stream())
+
+
 def outer_scan(proj: torch.Tensor, columns: dict, state: torch.Tensor, step, heads: int, dim: int, vdim: int, *,
                gates: Optional[dict] = None, decay: Optional[torch.Tensor] = None, q_scale: float = 1.0,
                k_scale: float = 1.0, cos: Optional[torch.Tensor] = None, sin: Optional[torch.Tensor] = None,
@@ -1639,7 +1670,17 @@ def outer_scan(proj: torch.Tensor, columns: dict, state: torch.Tensor, step, hea
              _dev(state_out, "state written"), state_out.stride(0) if state_out is not None else 0, per_head,
              _dev(product, "decay products"), _dev(out, "out"), _dev(dot, "dot"), heads, dim, vdim, _stream())
 
-    plan = chunk_plan(step, *OUTER_CHUNKS)
+    plan = None
+    if not gates and cos is None and chunked_memory_supported(dim):
+        plan = chunk_plan(step, library().leone_chunk_rows(), MEMORY_CHUNKS_FROM)
+        if plan is not None:
+            chunked_memory(proj, columns, plan, state, out, heads, heads, dim, vdim, q_scale=q_scale, k_scale=k_scale,
+                           activation=activation, decay=decay, write_state=write_state)
+            if plan["short"].shape[0]:
+                walk(plan["short"], state, state if write_state else None)
+            return out, None
+    else:
+        plan = chunk_plan(step, *OUTER_CHUNKS)
     if plan is None:
         walk(spans, state, state if write_state else None)
     else:
@@ -1691,7 +1732,17 @@ def delta_scan(qkv: torch.Tensor, columns: dict, beta: torch.Tensor, step_size: 
              _dev(state_out, "state written"), state_out.stride(0) if state_out is not None else 0,
              _dev(transition, "transitions"), _dev(out, "out"), heads, kv_heads, dim, vdim, _stream())
 
-    plan = chunk_plan(step, *DELTA_CHUNKS)
+    plan = None
+    if per_head and chunked_memory_supported(dim):
+        plan = chunk_plan(step, library().leone_chunk_rows(), MEMORY_CHUNKS_FROM)
+        if plan is not None:
+            chunked_memory(qkv, columns, plan, state, out, heads, kv_heads, dim, vdim, q_scale=q_scale, k_scale=1.0,
+                           delta=(beta, step_size, rate_log, step_bias, unit_eps), write_state=write_state)
+            if plan["short"].shape[0]:
+                walk(plan["short"], state, state if write_state else None)
+            return out
+    else:
+        plan = chunk_plan(step, *DELTA_CHUNKS)
     if plan is None:
         walk(spans, state, state if write_state else None)
     else:

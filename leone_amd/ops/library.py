@@ -110,6 +110,8 @@ _PROTOTYPES = {
     "leone_latent_attention": [P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, P],
     "leone_residual_norm": [P, P, c_int, ctypes.c_long, c_float, P, c_int, c_float, P, c_int, P, c_int, c_int, P],
     "leone_depth_mix": [P, P, c_int, ctypes.c_long, c_float, P, ctypes.c_long, c_int, P, c_int, ctypes.c_long, P],
+    "leone_chunked_memory": [P, ctypes.c_long, c_int, c_int, c_int, c_int, c_float, c_float, c_float, P, ctypes.c_long, P, ctypes.c_long,
+                             P, P, c_int, P, P, c_int, P, c_int, P, P, ctypes.c_long, c_int, P, c_int, c_int, c_int, c_int, P],
     "leone_stream_join": [P, P, P, P, P, P, P, c_int, P, P, c_int, P, c_int, c_int, c_int, P],
     "leone_attention_rows_shaped": [P, P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
                                     c_int, P, ctypes.c_long, c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, c_int, P],
@@ -164,6 +166,12 @@ def library() -> ctypes.CDLL:
             lib.leone_sample_truncated_params.argtypes = []
             lib.leone_peak_mfma_flops.restype = ctypes.c_double
             lib.leone_peak_mfma_flops.argtypes = [c_int, c_int]
+            lib.leone_chunk_rows.restype = c_int
+            lib.leone_chunk_rows.argtypes = []
+            lib.leone_chunk_max_dim.restype = c_int
+            lib.leone_chunk_max_dim.argtypes = []
+            lib.leone_chunk_workspace.restype = ctypes.c_long
+            lib.leone_chunk_workspace.argtypes = [c_int, c_int, c_int]
             lib.leone_scan_max_dim.restype = c_int
             lib.leone_scan_max_dim.argtypes = []
             lib.leone_gemm_rows_max_rows.restype = c_int

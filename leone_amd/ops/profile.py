@@ -63,6 +63,7 @@ OPERATIONS = {
     "leone_qk_norm_rope_write_turned": "qknorm rope kv",
     "leone_branch_norm": "norm",
     "leone_stream_join": "stream join",
+    "leone_chunked_memory": "chunked memory",
     "leone_token_mix": "token mix",
     "leone_low_rank_decay": "low rank decay",
     "leone_time_mix_scan": "time mix scan",

@@ -63,14 +63,19 @@ def test_engine_agrees_with_plain_however_the_work_is_cut(cases, name, dtype_nam
     assert all(engine.cache.free_pages(g) == engine.cache.groups[g].num_pages for g in range(len(engine.cache.groups)))
 
 
+@pytest.mark.parametrize("how", ["products", "walks"])
 @pytest.mark.parametrize("schedule", ["whole", "portions", "mixed"])
 @pytest.mark.parametrize("name", ["A", "B"])
-def test_long_portions_of_the_memories_walked_in_chunks(cases, monkeypatch, name, schedule):
-    """With chunks of 8 rows from portions of 16 rows on, every longer portion is walked in chunks side by side and chained
-    (by a factor for the fixed decays, by a matrix for the delta rule); the results differ by rounding only."""
+def test_long_portions_of_the_memories_in_chunks(cases, monkeypatch, name, schedule, how):
+    """From portions of 16 rows on, the memories work in chunks: as products over chunks of 64 rows, or (what heads of more key
+    channels take) in chunks of 8 rows walked side by side and chained, by a factor for the fixed decays and by a matrix for
+    the delta rule.  The results differ by rounding only."""
     from leone_amd import ops
-    monkeypatch.setattr(ops, "OUTER_CHUNKS", (8, 16))
-    monkeypatch.setattr(ops, "DELTA_CHUNKS", (8, 16))
+    monkeypatch.setattr(ops, "MEMORY_CHUNKS_FROM", 16)
+    if how == "walks":
+        monkeypatch.setattr(ops, "chunked_memory_supported", lambda dim: False)
+        monkeypatch.setattr(ops, "OUTER_CHUNKS", (8, 16))
+        monkeypatch.setattr(ops, "DELTA_CHUNKS", (8, 16))
     folder, requests, expected = cases(name, "float32")
     steps = SCHEDULES[schedule](requests)
     engine = make_engine(folder, "float32", max_tokens=schedules.max_live_tokens(steps, 16), poison_freed=True)
@@ -392,6 +397,80 @@ def test_memories_reach_hundreds_of_tokens_back(which):
     assert float((want[200:] - without[200:]).abs().max()) > 0.05 * float(want[200:].abs().max())   # the mark is what is read
     err = su.relative_error(got.numpy(), want.numpy())
     assert err.max() <= 3e-5, (int(err.argmax()), float(err.max()))
+
+
+def memory_by_tokens(q, k, v, decay, beta, state):
+    """o_t = S_t^T q_t of one head, in float64: S <- g S + k u^T with u = v, or u = beta (v - g S^T k)."""
+    out = []
+    for t in range(q.shape[0]):
+        state = decay[t] * state
+        u = v[t] if beta is None else beta[t] * (v[t] - state.T @ k[t])
+        state = state + torch.outer(k[t], u)
+        out.append(state.T @ q[t])
+    return torch.stack(out), state
+
+
+@pytest.mark.parametrize("entries", [[(70, 0)], [(64, 5), (3, 0), (130, 0)], [(17, 3), (1, 9)], [(640, 0), (129, 7)]], ids=str)
+@pytest.mark.parametrize("heads,kv_heads,dim,vdim", [(2, 1, 32, 16), (3, 3, 7, 11), (4, 2, 128, 40), (1, 1, 65, 5), (2, 2, 100, 130), (1, 1, 136, 8)])
+@pytest.mark.parametrize("kind", ["delta", "fixed", "extreme"])
+def test_memories_with_one_decay_a_head_over_long_portions(monkeypatch, kind, heads, kv_heads, dim, vdim, entries):
+    """Portions of 16 rows and more as products over chunks of 64 rows (the largest heads: by walking), beside shorter ones, from
+    an empty and from a carried state; a fresh sequence does not read its slot.  Decays of nothing, nearly all and all."""
+    from leone_amd import ops
+    from leone_amd.parts.context import EntryInfo, StepContext
+    monkeypatch.setattr(ops, "MEMORY_CHUNKS_FROM", 16)
+    delta = kind != "fixed"
+    if not delta:
+        kv_heads = heads
+    gen = torch.Generator().manual_seed(5)
+    rows, kv = sum(count for count, _ in entries), kv_heads * dim
+    x = torch.randn(rows, 2 * kv + heads * vdim, generator=gen)
+    state = torch.randn(4, heads, dim, vdim, generator=gen)
+    strengths, steps_ = torch.randn(rows, heads, generator=gen), torch.randn(rows, heads, generator=gen)
+    rate_log, bias = torch.rand(heads, generator=gen) * 2 - 1, torch.rand(heads, generator=gen) * 5 - 6
+    if kind == "extreme":       # a step size of hundreds forgets everything, one of nothing keeps it; writes at full strength
+        steps_ = torch.where(torch.rand(rows, heads, generator=gen) < 0.1, 300.0, -40.0)
+        strengths = strengths * 20
+    fixed = torch.tensor([0.0, 0.97, 1.0][:heads] if heads <= 3 else [0.3, 0.9, 0.99, 1.0])
+    slots = [2, 0, 3][:len(entries)]
+    for slot, (count, start) in zip(slots, entries):
+        if start == 0:
+            state[slot] = float("nan")
+    infos, positions, owners = [], [], []
+    for i, (slot, (count, start)) in enumerate(zip(slots, entries)):
+        infos.append(EntryInfo(f"r{i}", slot, len(positions), count, start))
+        positions += range(start, start + count)
+        owners += [i] * count
+    step = StepContext(rows=rows, dtype=torch.float32, device=torch.device(DEV), positions=torch.tensor(positions, dtype=torch.int32, device=DEV),
+                       row_entry=torch.tensor(owners, dtype=torch.int32, device=DEV), entries=infos,
+                       entry_slots=torch.tensor(slots, dtype=torch.int32, device=DEV), want_rows=None)
+    dev_x, dev_state = x.to(DEV), state.to(DEV)
+    columns = {"q": 0, "k": kv, "v": 2 * kv}
+    if delta:
+        out = ops.delta_scan(dev_x, columns, strengths.to(DEV), steps_.to(DEV), rate_log.to(DEV), bias.to(DEV), dev_state, step, heads,
+                             kv_heads, dim, vdim, dim ** -0.5, 1e-6)
+    else:
+        out, _ = ops.outer_scan(dev_x, columns, dev_state.view(4, heads, dim * vdim), step, heads, dim, vdim, decay=fixed.to(DEV),
+                                activation="silu", k_scale=0.7)
+    out, dev_state, x = out.view(rows, heads, vdim).cpu().to(F), dev_state.cpu().to(F), x.to(F)
+    at = 0
+    for slot, (count, start) in zip(slots, entries):
+        span = slice(at, at + count)
+        at += count
+        for h in range(heads):
+            first = (h // (heads // kv_heads)) * dim
+            q, k, v = x[span, first:first + dim], x[span, kv + first:kv + first + dim], x[span, 2 * kv + h * vdim:2 * kv + (h + 1) * vdim]
+            before = torch.zeros(dim, vdim, dtype=F) if start == 0 else state[slot, h].to(F)
+            if delta:
+                q = q / torch.sqrt((q * q).sum(-1, keepdim=True) + 1e-6) * dim ** -0.5
+                k = k / torch.sqrt((k * k).sum(-1, keepdim=True) + 1e-6)
+                g = torch.exp(-torch.exp(rate_log[h].to(F)) * torch.nn.functional.softplus((steps_[span, h] + bias[h]).to(F)))
+                want, after = memory_by_tokens(q, k, v, g, torch.sigmoid(strengths[span, h].to(F)), before)
+            else:
+                q, k, v = (torch.nn.functional.silu(z) for z in (q, k, v))
+                want, after = memory_by_tokens(q, 0.7 * k, v, [float(fixed[h])] * count, None, before)
+            close(out[span, h], want, 2e-5, f"{kind} {slot} {h}")
+            close(dev_state[slot, h], after, 2e-5, f"{kind} {slot} {h} state")
 
 
 def key_query_value(heads, dim, vdim, width, sharp):
