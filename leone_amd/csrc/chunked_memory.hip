@@ -9,15 +9,15 @@
 // so with A_ti = beta_t (L_t / L_i) k_t.k_i (i < t) and M_ti = (L_t / L_i) q_t.k_i (i <= t), one row a token,
 //   (1 + A) U = diag(beta) V - diag(beta L) K S0,   O = diag(L) Q S0 + M U,   S_end = L_end S0 + (diag(L_end / L) K)^T U.
 // chunk_prepare makes everything that does not hold S0, all chunks and heads side by side: U0 and W, the solutions of the
-// triangular system for diag(beta) V and diag(beta L) K (forward substitution, a column a thread, the chunk's 64 values of a
-// column in registers), M, and Q and K with their decays.  chunk_walk then goes through a portion's chunks in order, a
-// workgroup a head and 16 columns of S: U = U0 - W S, O, S.  With fixed decays there is no system: U = V.
+// triangular system for diag(beta) V and diag(beta L) K (forward substitution, 16 rows at a time: the rows before leave them
+// as products), M, and Q and K with their decays.  chunk_walk then goes through a portion's chunks in order, a workgroup a head
+// and 16 columns of S: U = U0 - W S, O, S.  With fixed decays there is no system: U = V.
 //
 // Products are v_mfma_f32_16x16x4_f32.  Lane l = 16 g + c holds A[row c][k-slot g], B[k-slot g][column c] and rows 4 g + v of
 // column c of the result in register v.  Which inner element a k-slot stands for is free as long as both operands agree:
 // instruction v of a run of 16 takes element 4 g + v for slot g, so that an operand is one 16-byte read a lane, and a result
-// in registers (S, U) is the next product's second operand as it lies.  Decays travel as logarithms summed over the chunk, in double:
-// a row that forgets everything must not blur the small decays behind it.
+// in registers (S, U) is the next product's second operand as it lies.  Decays travel as logarithms summed over the chunk, in
+// double: a row that forgets everything must not blur the small decays behind it.
 #include "common.h"
 #include "leone_hip.h"
 
@@ -30,6 +30,7 @@ typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4;
 constexpr int kChunkRows = 64;
 constexpr int kChunkThreads = 256;
 constexpr int kChunkMaxDim = 128;       // key channels: two tiles of 16 a wave
+constexpr int kChunkTiles = 10;         // tiles of 16 x 16 of a chunk's rows by rows on and below the diagonal
 constexpr int kPartStride = 20;         // of a row of 16 in shared memory: rows four apart lie in banks of their own
 
 struct ChunkArgs {
@@ -47,10 +48,10 @@ struct ChunkArgs {
     const float* decay;         // fixed decays: [heads]
     const int* chunks;          // [chunks, 4]: first row, end, -, -
     const int* links;           // [links, 4]: state slot, whether the sequence starts here, first chunk, end
-    float* q_in;                // [chunks, heads, 64, dim_p]: q_t L_t
-    float* k_out;               // [chunks, heads, dim_p, 64]: k_t L_end / L_t
-    float* mix;                 // [chunks, heads, 64, 64]: M (tiles above the diagonal are not written)
-    float* solved_k;            // delta rule: [chunks, heads, 64, dim_p]: W
+    float* q_in;                // [chunks, heads, 64 x dim_p]: q_t L_t, in the order chunk_walk reads
+    float* k_out;               // [chunks, heads, dim_p x 64]: k_t L_end / L_t, likewise
+    float* mix;                 // [chunks, heads, 64 x 64]: M, likewise (tiles above the diagonal are not written)
+    float* solved_k;            // delta rule: [chunks, heads, 64 x dim_p]: W, likewise
     float* values;              // [chunks, heads, 64, vdim_p]: U0, or V
     float* total;               // [chunks, heads]: L_end
     float* state;               // [slots, heads, dim, vdim]
@@ -66,31 +67,49 @@ constexpr float kNothingLeft = -1e4f;   // a logarithm whose exponential is zero
 __device__ inline float between(double later, double earlier) { return expf(static_cast<float>(later - earlier)); }
 __device__ inline floatx4 mfma4(float a, float b, floatx4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
-template <bool kDelta>
-__global__ void __launch_bounds__(kChunkThreads, 1) chunk_prepare_kernel(ChunkArgs p) {
+// Where the four elements that a lane of chunk_walk reads at once stand in the chunk's rows: its operands lie in the order of
+// [wave][tile of rows][tile of channels][lane], so that a wave reads 1,024 bytes in a row.
+struct Place { int row, channel; };
+template <int kT>
+__device__ inline Place place_of(int idx) {
+    const int lane = idx % kWave, tile = idx / kWave;
+    return {16 * (tile / kT % 4) + (lane & 15), 16 * (tile / (4 * kT) * kT + tile % kT) + 4 * (lane >> 4)};
+}
+
+// kT: tiles of 16 key channels a wave of chunk_walk holds; 64 kT channels, the last ones zeros.
+template <bool kDelta, int kT>
+__global__ void __launch_bounds__(kChunkThreads, 2) chunk_prepare_kernel(ChunkArgs p) {
     extern __shared__ __align__(16) float chunk_lds[];
-    const int row_p = p.dim_p + 4;
+    constexpr int kDim = 64 * kT, row_p = kDim + 4;
     float* sq = chunk_lds;                              // [64][row_p]
     float* sk = sq + kChunkRows * row_p;
-    float* sa = sk + kChunkRows * row_p;                // [64][68]: A turned, column i of A at row i (delta rule only)
-    constexpr int kAStride = kChunkRows + 4;
+    float* sa = sk + kChunkRows * row_p;                // delta rule: -A in tiles of 16 x 16, those on and below the diagonal
     __shared__ double cum[kChunkRows];
-    __shared__ float strength[kChunkRows], q_norm[kChunkRows], k_norm[kChunkRows];
+    __shared__ float strength[kChunkRows], q_norm[kChunkRows], k_norm[kChunkRows], so_far[kChunkRows], to_end[kChunkRows];
     const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
     const int chunk = blockIdx.x, head = blockIdx.y, kvh = head / (p.heads / p.kv_heads);
     const int first = p.chunks[4 * chunk], n = p.chunks[4 * chunk + 1] - first;
     const long at = static_cast<long>(chunk) * p.heads + head;
+    const int block = blockIdx.z * kDim;        // delta rule: the value columns solved here; the first workgroup writes all the rest
 
-    for (int idx = tid; idx < kChunkRows * p.dim_p; idx += kChunkThreads) {
-        const int t = idx / p.dim_p, i = idx % p.dim_p;
-        float q = 0.f, k = 0.f;
-        if (t < n && i < p.dim) {
-            const float* base = p.rows + static_cast<long>(first + t) * p.stride + kvh * p.dim + i;
-            q = chunk_act(base[p.q_off], p.silu);
-            k = chunk_act(base[p.k_off], p.silu);
+    // reads in batches, of the last row or channel again where there is none, so that no read waits for the one before
+    constexpr int kBatch = 8;
+    static_assert(kChunkRows * kDim % (kBatch * kChunkThreads) == 0, "whole batches");
+    for (int from = tid; from < kChunkRows * kDim; from += kBatch * kChunkThreads) {
+        float q[kBatch], k[kBatch];
+#pragma unroll
+        for (int e = 0; e < kBatch; ++e) {
+            const int t = (from + e * kChunkThreads) / kDim, i = (from + e * kChunkThreads) % kDim;
+            const float* base = p.rows + static_cast<long>(first + min(t, n - 1)) * p.stride + kvh * p.dim + min(i, p.dim - 1);
+            q[e] = base[p.q_off], k[e] = base[p.k_off];
         }
-        sq[t * row_p + i] = q;
-        sk[t * row_p + i] = k;
+#pragma unroll
+        for (int e = 0; e < kBatch; ++e) {
+            const int t = (from + e * kChunkThreads) / kDim, i = (from + e * kChunkThreads) % kDim;
+            const bool there = t < n && i < p.dim;
+            sq[t * row_p + i] = there ? chunk_act(q[e], p.silu) : 0.f;
+            sk[t * row_p + i] = there ? chunk_act(k[e], p.silu) : 0.f;
+        }
     }
     if (wave == 0) {
         // the decays' logarithms summed up over the chunk; rows past its end decay nothing and write nothing
@@ -114,6 +133,8 @@ __global__ void __launch_bounds__(kChunkThreads, 1) chunk_prepare_kernel(ChunkAr
             if (lane >= off) l += before;
         }
         cum[lane] = l;
+        so_far[lane] = between(l, 0.);
+        to_end[lane] = between(__shfl(l, kWave - 1, kWave), l);
     }
     __syncthreads();
     {   // four lanes a row
@@ -135,18 +156,19 @@ __global__ void __launch_bounds__(kChunkThreads, 1) chunk_prepare_kernel(ChunkAr
         }
     }
     __syncthreads();
-    if (tid == 0) p.total[at] = between(cum[kChunkRows - 1], 0.);
+    if (tid == 0 && block == 0) p.total[at] = so_far[kChunkRows - 1];
 
     // k_t.k_i and q_t.k_i, the ten tiles of 16 x 16 on and below the diagonal shared out over the waves
     float* mix = p.mix + at * kChunkRows * kChunkRows;
     const int c = lane & 15, g = lane >> 4;
-    for (int pair = wave; pair < 10; pair += kChunkThreads / kWave) {
+    for (int pair = wave; pair < kChunkTiles; pair += kChunkThreads / kWave) {
         const int ti = pair < 1 ? 0 : pair < 3 ? 1 : pair < 6 ? 2 : 3, tj = pair - ti * (ti + 1) / 2;
         const float* rq = sq + (16 * ti + c) * row_p + 4 * g;
         const float* rk = sk + (16 * ti + c) * row_p + 4 * g;
         const float* ck = sk + (16 * tj + c) * row_p + 4 * g;
         floatx4 kk = {0.f, 0.f, 0.f, 0.f}, qk = {0.f, 0.f, 0.f, 0.f};
-        for (int d = 0; d < p.dim_p; d += 16) {
+#pragma unroll
+        for (int d = 0; d < kDim; d += 16) {
             const float4 b = *reinterpret_cast<const float4*>(ck + d), aq = *reinterpret_cast<const float4*>(rq + d);
             qk = mfma4(aq.x, b.x, qk);
             qk = mfma4(aq.y, b.y, qk);
@@ -165,54 +187,114 @@ __global__ void __launch_bounds__(kChunkThreads, 1) chunk_prepare_kernel(ChunkAr
         for (int v = 0; v < 4; ++v) {
             const int t = 16 * ti + 4 * g + v;
             const float decayed = t >= i ? between(cum[t], cum[i]) * k_norm[i] : 0.f;
-            mix[t * kChunkRows + i] = decayed * q_norm[t] * qk[v];
-            if (kDelta) sa[i * kAStride + t] = decayed * k_norm[t] * strength[t] * kk[v];
+            if (block == 0) mix[4 * ((ti * 4 + tj) * kWave + 16 * (c / 4) + 4 * g + v) + c % 4] = decayed * q_norm[t] * qk[v];
+            if (kDelta) sa[256 * pair + 16 * (4 * g + v) + c] = -decayed * k_norm[t] * strength[t] * kk[v];
         }
     }
-    float* q_in = p.q_in + at * kChunkRows * p.dim_p;
-    float* k_out = p.k_out + at * kChunkRows * p.dim_p;
-    for (int idx = tid; idx < kChunkRows * p.dim_p; idx += kChunkThreads) {
-        const int t = idx / p.dim_p, i = idx % p.dim_p;
-        q_in[idx] = sq[t * row_p + i] * q_norm[t] * between(cum[t], 0.);
-        const int kt = idx % kChunkRows, ki = idx / kChunkRows;
-        k_out[idx] = sk[kt * row_p + ki] * k_norm[kt] * between(cum[kChunkRows - 1], cum[kt]);
+    float* q_in = p.q_in + at * kChunkRows * kDim;
+    float* k_out = p.k_out + at * kChunkRows * kDim;
+    if (block == 0) {
+#pragma unroll 4
+        for (int idx = tid; idx < kChunkRows * kDim / 4; idx += kChunkThreads) {
+            const Place a = place_of<kT>(idx);
+            const float4 x = *reinterpret_cast<const float4*>(sq + a.row * row_p + a.channel);
+            const float f = q_norm[a.row] * so_far[a.row];
+            reinterpret_cast<float4*>(q_in)[idx] = float4{x.x * f, x.y * f, x.z * f, x.w * f};
+            const int ki = 16 * (idx / kWave / 4) + c, kt = 16 * (idx / kWave % 4) + 4 * g;
+            float4 y;
+            y.x = sk[kt * row_p + ki] * (k_norm[kt] * to_end[kt]);
+            y.y = sk[(kt + 1) * row_p + ki] * (k_norm[kt + 1] * to_end[kt + 1]);
+            y.z = sk[(kt + 2) * row_p + ki] * (k_norm[kt + 2] * to_end[kt + 2]);
+            y.w = sk[(kt + 3) * row_p + ki] * (k_norm[kt + 3] * to_end[kt + 3]);
+            reinterpret_cast<float4*>(k_out)[idx] = y;
+        }
     }
     float* values = p.values + at * kChunkRows * p.vdim_p;
     const float* v_base = p.rows + static_cast<long>(first) * p.stride + p.v_off + head * p.vdim;
+    const auto read_v = [&](int t, int j) { return v_base[min(t, n - 1) * p.stride + min(j, p.vdim - 1)]; };
+    const auto taken_v = [&](float v, int t, int j) { return t < n && j < p.vdim ? chunk_act(v, p.silu) : 0.f; };
     if constexpr (!kDelta) {
-        for (int idx = tid; idx < kChunkRows * p.vdim_p; idx += kChunkThreads) {
-            const int t = idx / p.vdim_p, j = idx % p.vdim_p;
-            values[idx] = (t < n && j < p.vdim) ? chunk_act(v_base[t * p.stride + j], p.silu) : 0.f;
+        constexpr int kRows = kChunkThreads / kWave, kEach = kChunkRows / kRows;
+        for (int j = lane; j < p.vdim_p; j += kWave) {
+            float v[kEach];
+#pragma unroll
+            for (int e = 0; e < kEach; ++e) v[e] = read_v(wave + kRows * e, j);
+#pragma unroll
+            for (int e = 0; e < kEach; ++e) values[(wave + kRows * e) * p.vdim_p + j] = taken_v(v[e], wave + kRows * e, j);
         }
     } else {
-        __syncthreads();
-        float* solved_k = p.solved_k + at * kChunkRows * p.dim_p;
-        for (int col = tid; col < p.dim_p + p.vdim_p; col += kChunkThreads) {
-            const bool is_key = col < p.dim_p;
-            const int j = is_key ? col : col - p.dim_p;
-            float x[kChunkRows];
+        float* solved_k = p.solved_k + at * kChunkRows * kDim;
+        __syncthreads();                    // M is made and K written: their places take the right sides, K and a block of V
+        for (int from = tid; from < kChunkRows * kDim; from += kBatch * kChunkThreads) {
+            float v[kBatch];
 #pragma unroll
-            for (int t = 0; t < kChunkRows; ++t) {
-                if (is_key) x[t] = strength[t] * between(cum[t], 0.) * k_norm[t] * sk[t * row_p + j];
-                else x[t] = (t < n && j < p.vdim) ? strength[t] * chunk_act(v_base[t * p.stride + j], p.silu) : 0.f;
+            for (int e = 0; e < kBatch; ++e) v[e] = read_v((from + e * kChunkThreads) / kDim, block + (from + e * kChunkThreads) % kDim);
+#pragma unroll
+            for (int e = 0; e < kBatch; ++e) {
+                const int t = (from + e * kChunkThreads) / kDim, i = (from + e * kChunkThreads) % kDim;
+                sk[t * row_p + i] *= strength[t] * so_far[t] * k_norm[t];
+                sq[t * row_p + i] = strength[t] * taken_v(v[e], t, block + i);
             }
+        }
+        __syncthreads();
+        static_assert(2 * kDim <= kChunkThreads, "a thread takes one column");
+        const bool is_key = tid >= kDim;
+        const int mine = is_key ? tid - kDim : tid;
+        float* column = (is_key ? sk : sq) + mine;
+        float* to = values + block + mine;
+        const bool stores = !is_key && block + mine < p.vdim_p;
+#pragma unroll 1
+        for (int b = 0; b < kChunkRows / 16; ++b) {
+            // 16 rows at a time: the solved rows leave them as products,
+            const float* tiles = sa + 256 * (b * (b + 1) / 2);
+            if (b > 0) {
+                for (int at16 = wave; at16 < 2 * kDim / 16; at16 += kChunkThreads / kWave) {
+                    float* x = (at16 < kDim / 16 ? sq + 16 * at16 : sk + 16 * at16 - kDim) + c;
+                    floatx4 sum;
 #pragma unroll
-            for (int i = 0; i < kChunkRows - 1; ++i) {
-                // row i is solved: it leaves every row behind it
+                    for (int v = 0; v < 4; ++v) sum[v] = x[(16 * b + 4 * g + v) * row_p];
+                    for (int s = 0; s < b; ++s) {
+                        const float4 a = *reinterpret_cast<const float4*>(tiles + 256 * s + 16 * c + 4 * g);
+                        const float* solved = x + (16 * s + 4 * g) * row_p;
+                        sum = mfma4(a.x, solved[0], sum);
+                        sum = mfma4(a.y, solved[row_p], sum);
+                        sum = mfma4(a.z, solved[2 * row_p], sum);
+                        sum = mfma4(a.w, solved[3 * row_p], sum);
+                    }
 #pragma unroll
-                for (int t4 = (i + 1) / 4; t4 < kChunkRows / 4; ++t4) {
-                    const float4 a = *reinterpret_cast<const float4*>(sa + i * kAStride + 4 * t4);
-                    if (4 * t4 > i) x[4 * t4] = fmaf(-a.x, x[i], x[4 * t4]);
-                    if (4 * t4 + 1 > i) x[4 * t4 + 1] = fmaf(-a.y, x[i], x[4 * t4 + 1]);
-                    if (4 * t4 + 2 > i) x[4 * t4 + 2] = fmaf(-a.z, x[i], x[4 * t4 + 2]);
-                    if (4 * t4 + 3 > i) x[4 * t4 + 3] = fmaf(-a.w, x[i], x[4 * t4 + 3]);
+                    for (int v = 0; v < 4; ++v) x[(16 * b + 4 * g + v) * row_p] = sum[v];
+                }
+                __syncthreads();
+            }
+            // then a column a thread among themselves
+            if (tid < 2 * kDim) {
+                float x[16];
+#pragma unroll
+                for (int t = 0; t < 16; ++t) x[t] = column[(16 * b + t) * row_p];
+#pragma unroll
+                for (int t = 1; t < 16; ++t)
+#pragma unroll
+                    for (int i4 = 0; 4 * i4 < t; ++i4) {
+                        const float4 a = *reinterpret_cast<const float4*>(tiles + 256 * b + 16 * t + 4 * i4);
+                        x[t] = fmaf(a.x, x[4 * i4], x[t]);
+                        if (4 * i4 + 1 < t) x[t] = fmaf(a.y, x[4 * i4 + 1], x[t]);
+                        if (4 * i4 + 2 < t) x[t] = fmaf(a.z, x[4 * i4 + 2], x[t]);
+                        if (4 * i4 + 3 < t) x[t] = fmaf(a.w, x[4 * i4 + 3], x[t]);
+                    }
+#pragma unroll
+                for (int t = 0; t < 16; ++t) {
+                    column[(16 * b + t) * row_p] = x[t];
+                    if (stores) to[(16 * b + t) * p.vdim_p] = x[t];
                 }
             }
-            float* to = is_key ? solved_k : values;
-            const int width = is_key ? p.dim_p : p.vdim_p;
-#pragma unroll
-            for (int t = 0; t < kChunkRows; ++t) to[t * width + j] = x[t];
+            __syncthreads();
         }
+        if (block == 0)
+#pragma unroll 4
+            for (int idx = tid; idx < kChunkRows * kDim / 4; idx += kChunkThreads) {
+                const Place a = place_of<kT>(idx);
+                reinterpret_cast<float4*>(solved_k)[idx] = *reinterpret_cast<const float4*>(sk + a.row * row_p + a.channel);
+            }
     }
 }
 
@@ -221,30 +303,36 @@ template <bool kDelta, int kT>
 struct ChunkOperands {
     float4 w[kDelta ? 4 : 1][kT], q[4][kT], k[kT][4], m[4];
     float u[4], total;
+    int first, end;
 };
 
 template <bool kDelta, int kT>
 __device__ inline void fetch_chunk(const ChunkArgs& p, int chunk, int head, int wave, int c, int g, int col, ChunkOperands<kDelta, kT>& o) {
     const long at = static_cast<long>(chunk) * p.heads + head;
-    const float* q_in = p.q_in + at * kChunkRows * p.dim_p + 16 * wave * kT + 4 * g;
-    const float* k_out = p.k_out + at * kChunkRows * p.dim_p + 4 * g;
+    constexpr int kDim = 64 * kT;
+    const int lane = 16 * g + c;
+    const float4* q_in = reinterpret_cast<const float4*>(p.q_in + at * kChunkRows * kDim) + wave * 4 * kT * kWave + lane;
+    const float4* k_out = reinterpret_cast<const float4*>(p.k_out + at * kChunkRows * kDim) + wave * 4 * kT * kWave + lane;
+    const float4* mix = reinterpret_cast<const float4*>(p.mix + at * kChunkRows * kChunkRows) + wave * 4 * kWave + lane;
 #pragma unroll
-    for (int t = 0; t < kT; ++t) {
+    for (int r = 0; r < 4; ++r)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
+        for (int t = 0; t < kT; ++t) {
             if constexpr (kDelta)
-                o.w[r][t] = *reinterpret_cast<const float4*>(p.solved_k + at * kChunkRows * p.dim_p + (16 * r + c) * p.dim_p + 16 * (wave * kT + t) + 4 * g);
-            o.q[r][t] = *reinterpret_cast<const float4*>(q_in + (16 * r + c) * p.dim_p + 16 * t);
-            o.k[t][r] = *reinterpret_cast<const float4*>(k_out + (16 * (wave * kT + t) + c) * kChunkRows + 16 * r);
+                o.w[r][t] = (reinterpret_cast<const float4*>(p.solved_k + at * kChunkRows * kDim) + wave * 4 * kT * kWave + lane)[(r * kT + t) * kWave];
+            o.q[r][t] = q_in[(r * kT + t) * kWave];
         }
-    }
-#pragma unroll
-    for (int s = 0; s < 4; ++s)
-        o.m[s] = s <= wave ? *reinterpret_cast<const float4*>(p.mix + at * kChunkRows * kChunkRows + (16 * wave + c) * kChunkRows + 16 * s + 4 * g)
-                           : float4{0.f, 0.f, 0.f, 0.f};
+    o.first = p.chunks[4 * chunk];
+    o.end = p.chunks[4 * chunk + 1];
+    o.total = p.total[at];
 #pragma unroll
     for (int v = 0; v < 4; ++v) o.u[v] = p.values[at * kChunkRows * p.vdim_p + (16 * wave + 4 * g + v) * p.vdim_p + col];
-    o.total = p.total[at];
+#pragma unroll
+    for (int s = 0; s < 4; ++s) o.m[s] = s <= wave ? mix[s * kWave] : float4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int t = 0; t < kT; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o.k[t][r] = k_out[(t * 4 + r) * kWave];
 }
 
 __device__ inline float element(const float4& f, int v) { return v == 0 ? f.x : v == 1 ? f.y : v == 2 ? f.z : f.w; }
@@ -274,7 +362,6 @@ __global__ void __launch_bounds__(kChunkThreads, 1) chunk_walk_kernel(ChunkArgs 
     for (int chunk = g0; chunk < g1; ++chunk) {
         const ChunkOperands<kDelta, kT> now = ahead;
         fetch_chunk<kDelta, kT>(p, chunk + 1 < g1 ? chunk + 1 : chunk, head, wave, c, g, col, ahead);
-        const int first = p.chunks[4 * chunk], n = p.chunks[4 * chunk + 1] - first;
         floatx4 ws[4], qs[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) ws[r] = qs[r] = floatx4{0.f, 0.f, 0.f, 0.f};
@@ -326,7 +413,7 @@ __global__ void __launch_bounds__(kChunkThreads, 1) chunk_walk_kernel(ChunkArgs 
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             const int t = 16 * wave + 4 * g + v;
-            if (t < n && col < p.vdim) p.out[(static_cast<long>(first + t) * p.heads + head) * p.vdim + col] = o[v];
+            if (now.first + t < now.end && col < p.vdim) p.out[(static_cast<long>(now.first + t) * p.heads + head) * p.vdim + col] = o[v];
         }
     }
     if (!p.write_state) return;
@@ -390,24 +477,27 @@ extern "C" int leone_chunked_memory(const float* rows, long stride, int q_off, i
     a.mix = a.values + each * a.vdim_p;
     a.solved_k = a.mix + each * kChunkRows;
     a.total = a.solved_k + (delta ? each * a.dim_p : 0);
-    const size_t shared = (2 * kChunkRows * (a.dim_p + 4) + (delta ? kChunkRows * (kChunkRows + 4) : 0)) * sizeof(float);
+    const size_t shared = (2 * kChunkRows * (a.dim_p + 4) + (delta ? kChunkTiles * 256 : 0)) * sizeof(float);
     static bool allowed = false;
     if (!allowed) {
-        const int most = (2 * kChunkRows * (kChunkMaxDim + 4) + kChunkRows * (kChunkRows + 4)) * sizeof(float);
-        for (const void* kernel : {reinterpret_cast<const void*>(&chunk_prepare_kernel<false>), reinterpret_cast<const void*>(&chunk_prepare_kernel<true>)}) {
+        const int most = (2 * kChunkRows * (kChunkMaxDim + 4) + kChunkTiles * 256) * sizeof(float);
+        for (const void* kernel : {reinterpret_cast<const void*>(&chunk_prepare_kernel<false, 1>), reinterpret_cast<const void*>(&chunk_prepare_kernel<false, 2>),
+                                   reinterpret_cast<const void*>(&chunk_prepare_kernel<true, 1>), reinterpret_cast<const void*>(&chunk_prepare_kernel<true, 2>)}) {
             const hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, most);
             LEONE_REQUIRE(e == hipSuccess, "chunked_memory: %d bytes of shared memory were refused: %s", most, hipGetErrorString(e));
         }
         allowed = true;
     }
-    const dim3 prepare(n_chunks, heads), walk(n_links, heads, a.vdim_p / 16);
+    const dim3 prepare(n_chunks, heads, delta ? ceil_div(a.vdim_p, a.dim_p) : 1), walk(n_links, heads, a.vdim_p / 16);
     if (delta) {
-        chunk_prepare_kernel<true><<<prepare, kChunkThreads, shared, stream>>>(a);
+        if (tiles == 1) chunk_prepare_kernel<true, 1><<<prepare, kChunkThreads, shared, stream>>>(a);
+        else chunk_prepare_kernel<true, 2><<<prepare, kChunkThreads, shared, stream>>>(a);
         LEONE_LAUNCH_CHECK("chunk_prepare");
         if (tiles == 1) chunk_walk_kernel<true, 1><<<walk, kChunkThreads, 0, stream>>>(a);
         else chunk_walk_kernel<true, 2><<<walk, kChunkThreads, 0, stream>>>(a);
     } else {
-        chunk_prepare_kernel<false><<<prepare, kChunkThreads, shared, stream>>>(a);
+        if (tiles == 1) chunk_prepare_kernel<false, 1><<<prepare, kChunkThreads, shared, stream>>>(a);
+        else chunk_prepare_kernel<false, 2><<<prepare, kChunkThreads, shared, stream>>>(a);
         LEONE_LAUNCH_CHECK("chunk_prepare");
         if (tiles == 1) chunk_walk_kernel<false, 1><<<walk, kChunkThreads, 0, stream>>>(a);
         else chunk_walk_kernel<false, 2><<<walk, kChunkThreads, 0, stream>>>(a);
