@@ -567,11 +567,23 @@ attention_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__
 constexpr int kReduceThreads = 128;
 constexpr int kMaxSplits = 256;
 
+// Gates on a finished result: float rows of pre-activations, one a head or one an element.
+struct ResultGate {
+    const float* values;
+    long stride;
+    int each;
+    __device__ float factor(long row_head, int d, int head_dim, int q_heads) const {
+        if (values == nullptr) return 1.0f;
+        const long row = row_head / q_heads, head = row_head % q_heads;
+        return 1.0f / (1.0f + expf(-values[row * stride + (each ? head * head_dim + d : head)]));
+    }
+};
+
 template <bool kShaped>
 __global__ void __launch_bounds__(kReduceThreads)
 attention_reduce_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
                         bf16_t* __restrict__ out, int head_dim, int splits, const int* __restrict__ positions, int q_heads,
-                        ScoreShape shape) {
+                        ScoreShape shape, ResultGate gate) {
     __shared__ float weight[kMaxSplits];
     __shared__ float wave_top[kReduceThreads / kWave];
     const long rh = blockIdx.x;                      // row * q_heads + head
@@ -602,8 +614,8 @@ attention_reduce_kernel(const float* __restrict__ part_acc, const float* __restr
                     v += acc[e] * weight[s];
                 }
                 u /= den, v /= den;
-                out[rh * head_dim + d] = from_float<bf16_t>(turned_back(u, v, d, head_dim, pos, shape));
-                out[rh * head_dim + e] = from_float<bf16_t>(turned_back(v, u, e, head_dim, pos, shape));
+                out[rh * head_dim + d] = from_float<bf16_t>(turned_back(u, v, d, head_dim, pos, shape) * gate.factor(rh, d, head_dim, q_heads));
+                out[rh * head_dim + e] = from_float<bf16_t>(turned_back(v, u, e, head_dim, pos, shape) * gate.factor(rh, e, head_dim, q_heads));
             }
             return;
         }
@@ -611,14 +623,14 @@ attention_reduce_kernel(const float* __restrict__ part_acc, const float* __restr
     for (int d = threadIdx.x; d < head_dim; d += kReduceThreads) {
         float num = 0.f;
         for (int s = 0; s < splits; ++s) num += part_acc[(rh * splits + s) * head_dim + d] * weight[s];
-        out[rh * head_dim + d] = from_float<bf16_t>(num / den);
+        out[rh * head_dim + d] = from_float<bf16_t>(num / den * gate.factor(rh, d, head_dim, q_heads));
     }
 }
 
 void launch_attention_reduce(const float* part_acc, const float* part_ml, bf16_t* out, int rows, int q_heads, int head_dim, int splits,
                              hipStream_t stream) {
     attention_reduce_kernel<false><<<rows * q_heads, kReduceThreads, 0, stream>>>(part_acc, part_ml, out, head_dim, splits, nullptr,
-                                                                                q_heads, ScoreShape{});
+                                                                                q_heads, ScoreShape{}, ResultGate{});
 }
 int attention_reduce_max_splits() { return kMaxSplits; }
 
@@ -662,7 +674,10 @@ static int decode_checked(const void* q, void* out, const void* k_pool, const vo
                           const int* row_entry, const int* block_table, int max_blocks, float* part_acc,
                           float* part_ml, int rows, int q_heads, int kv_heads, int head_dim, int page_tokens,
                           float scale, int window, int splits, const FromProjection* from, int keep_first,
-                          hipStream_t stream, ScoreBias bias = ScoreBias{}, const ScoreShape& shape = ScoreShape{}, int chunk = 0) {
+                          hipStream_t stream, ScoreBias bias = ScoreBias{}, const ScoreShape& shape = ScoreShape{}, int chunk = 0,
+                          const ResultGate& gate = ResultGate{}) {
+    LEONE_REQUIRE(!gate.values || gate.stride >= static_cast<long>(q_heads) * (gate.each ? head_dim : 1),
+                  "attention_decode: rows of %ld gates are too short", gate.stride);
     if (check_mask("attention_decode", window, chunk, keep_first)) return 1;
     if (check_score_shape("attention_decode", shape, head_dim)) return 1;
     LEONE_REQUIRE(!from || !shape.any(), "attention_decode: capped scores, sinks and turned values come with finished queries");
@@ -706,11 +721,14 @@ static int decode_checked(const void* q, void* out, const void* k_pool, const vo
     if (splits > 1) {                                 // a single split has written the result itself
         if (shape.any())
             attention_reduce_kernel<true><<<rows * q_heads, kReduceThreads, 0, stream>>>(
-                part_acc, part_ml, static_cast<bf16_t*>(out), head_dim, splits, positions, q_heads, shape);
+                part_acc, part_ml, static_cast<bf16_t*>(out), head_dim, splits, positions, q_heads, shape, gate);
         else
             attention_reduce_kernel<false><<<rows * q_heads, kReduceThreads, 0, stream>>>(
-                part_acc, part_ml, static_cast<bf16_t*>(out), head_dim, splits, positions, q_heads, shape);
+                part_acc, part_ml, static_cast<bf16_t*>(out), head_dim, splits, positions, q_heads, shape, gate);
         LEONE_LAUNCH_CHECK("attention_reduce");
+    } else if (gate.values) {
+        return gate.each ? leone_head_gate(out, kBF16, gate.values, gate.stride, rows, q_heads * head_dim, 1, stream)
+                         : leone_head_gate(out, kBF16, gate.values, gate.stride, rows, q_heads, head_dim, stream);
     }
     return 0;
 }
@@ -753,6 +771,7 @@ extern "C" int leone_attention_decode_biased(const void* q, void* out, const voi
 
 // The same with what score_shape.h describes: cap (0: none), sinks, and the tables that turn results back (null: none);
 // chunk > 0 (no window, no kept first keys): a row sees the keys of its own chunk of so many positions only.
+// gate (null: none): pre-activations of a gate a head, or (gate_each) of one for every element; the result times their sigmoid.
 extern "C" int leone_attention_decode_shaped(const void* q, void* out, const void* k_pool, const void* v_pool,
                                              const int* positions, const int* row_entry, const int* block_table,
                                              int max_blocks, float* part_acc, float* part_ml, int rows, int q_heads,
@@ -760,11 +779,11 @@ extern "C" int leone_attention_decode_shaped(const void* q, void* out, const voi
                                              int splits, int keep_first, const float* slopes, float temp_coef,
                                              int temp_every, float cap, const float* sinks, const float* turn_cos,
                                              const float* turn_sin, int turn_positions, int turn_pairing, int chunk,
-                                             hipStream_t stream) {
+                                             const float* gate, long gate_stride, int gate_each, hipStream_t stream) {
     return decode_checked(q, out, k_pool, v_pool, positions, row_entry, block_table, max_blocks, part_acc, part_ml, rows,
                           q_heads, kv_heads, head_dim, page_tokens, scale, window, splits, nullptr, keep_first, stream,
                           ScoreBias{slopes, temp_coef, temp_every},
-                          ScoreShape{cap, sinks, turn_cos, turn_sin, turn_positions, turn_pairing}, chunk);
+                          ScoreShape{cap, sinks, turn_cos, turn_sin, turn_positions, turn_pairing}, chunk, ResultGate{gate, gate_stride, gate_each});
 }
 
 // The same for a step in which every row is another request, taking the fused q/k/v projection instead of

@@ -405,7 +405,8 @@ int leone_attention_decode_shaped(const void* q, void* out, const void* k_pool, 
                                   int rows, int q_heads, int kv_heads, int head_dim, int page_tokens, float scale, int window,
                                   int splits, int keep_first, const float* slopes, float temp_coef, int temp_every, float cap,
                                   const float* sinks, const float* turn_cos, const float* turn_sin, int turn_positions,
-                                  int turn_pairing, int chunk, hipStream_t stream);
+                                  int turn_pairing, int chunk, const float* gate, long gate_stride, int gate_each,
+                                  hipStream_t stream);
 int leone_attention_prefill_shaped(const void* q, void* out, const void* k_pool, const void* v_pool, const int* positions,
                                    const int* tiles, int n_groups, const int* block_table, int max_blocks, int q_heads,
                                    int kv_heads, int head_dim, int page_tokens, float scale, int window, float* part_acc,

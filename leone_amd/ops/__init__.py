@@ -518,15 +518,17 @@ def attention_decode(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor
                      row_entry: torch.Tensor, block_table: torch.Tensor, q_heads: int, scale: float,
                      window: int = 0, max_context: int = 1, splits: Optional[int] = None,
                      out: Optional[torch.Tensor] = None, keep_first: int = 0, slopes: Optional[torch.Tensor] = None,
-                     query_factor: Optional[tuple] = None, shape: Optional[ScoreShape] = None, chunk: int = 0) -> torch.Tensor:
+                     query_factor: Optional[tuple] = None, shape: Optional[ScoreShape] = None, chunk: int = 0,
+                     gate: Optional[torch.Tensor] = None, gate_each: bool = False) -> torch.Tensor:
     """Split-KV attention on the matrix cores (bfloat16).  ``max_context`` only steers the number of splits.
     ``keep_first``: keys at positions below it stay in sight of a windowed layer.  ``slopes`` and ``query_factor``
     as for ``attention_rows``: scores that fall with the distance, queries that count more the further on they stand.
-    ``shape``: capped scores, sinks, results turned back.  ``chunk`` as for ``attention_rows``."""
+    ``shape``: capped scores, sinks, results turned back.  ``chunk``, ``gate`` and ``gate_each`` as for ``attention_rows``."""
     rows = q.shape[0]
     pages, kv_heads, page_tokens, head_dim = cache_dims(k_pool, v_pool)
     if q.shape[1] != q_heads * head_dim:
         raise KernelError(f"attention: query width {q.shape[1]} is not {q_heads}*{head_dim}")
+    gate_at, gate_stride = _strided_rows(gate, "attention gate", rows, q_heads * head_dim if gate_each else q_heads)
     if splits is None:
         reach = min(max_context, window + keep_first + 32) if window else max_context     # keys a row can see at most
         reach = min(reach, chunk) if chunk else reach
@@ -545,7 +547,7 @@ def attention_decode(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor
          block_table.shape[1], _dev(part_acc, "partials"), _dev(part_ml, "partial sums"), rows, q_heads, kv_heads,
          head_dim, page_tokens, float(scale), int(window), int(splits), int(keep_first) if window else 0,
          _dev(slopes, "slopes", torch.float32, (q_heads,)), float(coef), int(every),
-         *(shape or _PLAIN_SCORES).args(q_heads, head_dim), int(chunk), _stream())
+         *(shape or _PLAIN_SCORES).args(q_heads, head_dim), int(chunk), gate_at, gate_stride, 1 if gate_each else 0, _stream())
     return out
 
 

@@ -116,7 +116,7 @@ _PROTOTYPES = {
     "leone_attention_rows_shaped": [P, P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
                                     c_int, P, ctypes.c_long, c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, c_int, P],
     "leone_attention_decode_shaped": [P, P, P, P, P, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
-                                      c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, c_int, P],
+                                      c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, c_int, P, ctypes.c_long, c_int, P],
     "leone_attention_prefill_shaped": [P, P, P, P, P, P, c_int, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, P, P,
                                        c_int, c_int, P, c_float, c_int, c_float, P, P, P, c_int, c_int, c_int, P],
     "leone_attention_rows_talk": [P, P, P, P, c_int, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,

@@ -360,12 +360,13 @@ class GqaAttention(Part):
             ops.attention_decode(q[first:], cache.k_pool, cache.v_pool, step.positions[first:],
                                  step.row_entry[first:], cache.block_table, self.q_heads, self.scale, window,
                                  max_context=step.max_position + 1, out=out[first:], keep_first=self.keep_first,
-                                 slopes=self.slopes, query_factor=self.query_factor, shape=shape, chunk=self.chunk)
-        if gate is None:
-            return out
-        # a gate for every element is a gate a head of one element
-        return ops.head_gate(out, gate, self.q_heads * self.value_dim, 1) if self.gate_each else \
-            ops.head_gate(out, gate, self.q_heads, self.value_dim)
+                                 slopes=self.slopes, query_factor=self.query_factor, shape=shape, chunk=self.chunk,
+                                 gate=gate[first:] if gate is not None else None, gate_each=self.gate_each)
+        if gate is not None and first:
+            # the prompt kernel's rows; a gate for every element is a gate a head of one element
+            heads, each = (self.q_heads * self.value_dim, 1) if self.gate_each else (self.q_heads, self.value_dim)
+            ops.head_gate(out[:first], gate[:first], heads, each)
+        return out
 
     def _attend_talking(self, q: torch.Tensor, step: StepContext, cache: KvCacheView, window: int) -> torch.Tensor:
         """The same for heads whose scores are mixed."""

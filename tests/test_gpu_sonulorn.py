@@ -630,6 +630,12 @@ def test_all_three_attention_kernels_within_chunks(chunk, sunk, dim, page_tokens
             one = ops.attention_decode(flat_q, k_pool, v_pool, rows_at, entry, table, q_heads, 1.0, max_context=n,
                                        splits=splits, shape=shape, chunk=chunk)
             close(one.float().view(len(positions), q_heads, dim), want, bound, f"split-KV kernel, splits {splits}")
+            # gates on the result, as slices of wider rows: one a head, one an element
+            wide = 2 * torch.randn(len(positions), q_heads * dim + 3, generator=torch.Generator().manual_seed(8))
+            for each, factor in ((False, wide[:, 3:3 + q_heads, None]), (True, wide[:, 3:].reshape(len(positions), q_heads, dim))):
+                gated = ops.attention_decode(flat_q, k_pool, v_pool, rows_at, entry, table, q_heads, 1.0, max_context=n, splits=splits,
+                                             shape=shape, chunk=chunk, gate=wide.to(DEV)[:, 3:], gate_each=each)
+                close(gated.float().view(len(positions), q_heads, dim), want * torch.sigmoid(factor.double()), bound, f"gated, splits {splits}")
         tiles = ops.prefill_tiles([(0, 0, len(positions))]).to(DEV)
         for splits in (None, 1, 2):
             out = torch.full_like(flat_q, float("nan"))
