@@ -1590,7 +1590,7 @@ def scan_max_dim() -> int:
     return int(library().leone_scan_max_dim())
 
 
-MEMORY_CHUNKS_FROM = 128     # portions of at least so many rows go through a memory with one decay a head as ``chunked_memory``
+MEMORY_CHUNKS_FROM = 32     # portions of at least so many rows go through a memory with one decay a head as ``chunked_memory``
 
 
 def chunked_memory_supported(dim: int) -> bool:
