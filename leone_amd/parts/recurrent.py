@@ -248,8 +248,8 @@ class HeadDeltaMixer(Part):
     """The gated delta rule with one decay per head.
 
     q = Wq h, k = Wk h (``kv_heads`` heads of ``dim``; head h of the memory uses q/k head h // (heads / kv_heads)),
-    v = Wv h (``heads`` of ``vdim``); each through a short causal convolution and silu; q and k made unit vectors
-    per head (x / sqrt(sum x^2 + 1e-6)), q times dim^-1/2; beta = sigmoid(Wb h) and
+    v = Wv h (``heads`` of ``vdim``); all three convolved over the last rows, then silu; every head of q and k is
+    brought to length one (under the root 1e-6 is added), q shrinks by the root of dim; beta = sigmoid(Wb h) and
     g = exp(-exp(A_log) * softplus(Wa h + dt_bias)), one a head.  Per head: S <- g S; u = beta (v - S^T k); S <- S + k u^T;
     o = S^T q.  Each head's o over its root mean square, times ``norm`` (size vdim, shared by the heads), times silu(Wg h),
     then Wo.
